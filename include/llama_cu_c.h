@@ -29,6 +29,12 @@ lcu_model* lcu_model_create_synthetic(uint32_t dim, uint32_t multiple_of, uint32
 /* mapped_buffer(path + "/params") + llama_params::load + llama_partition::autopipe + llama_model::load
  * (main.cpp:24-57, llama_cu.cu:987-997) */
 lcu_model* lcu_model_load(const char* model_dir, int context_len);
+/* llama_model::open: a model directory of any family (config.json or params); dtype 0 = the family's own
+ * element type, 1 = bfloat16, 2 = fp32 (layered decoders).  lcu_model_load is dtype 0. */
+lcu_model* lcu_model_open(const char* model_dir, int context_len, int dtype);
+/* a model of the given config.json text with seeded pseudo-random weights */
+lcu_model* lcu_model_create_synthetic_config(const char* config_text, uint64_t seed, int dtype);
+int lcu_model_max_context(const lcu_model*);
 void lcu_model_destroy(lcu_model*);
 uint32_t lcu_model_ffn_dim(const lcu_model*);                      /* llama_params::ffn_dim */
 /* the model's llama_params fields (llama_cu.h:280-291); q_type 0 = fp16, 1 = uint8 */
@@ -51,6 +57,13 @@ size_t lcu_context_memory_usage(lcu_context*);                                  
 size_t lcu_context_tokens_left(lcu_context*);                                       /* tokens_left */
 /* next_token (llama_cu.h:380); -1 if the tokens do not fit the context or an id is out of range */
 int lcu_context_next_token(lcu_context*, const int16_t* tokens, int n);
+/* llama_context::forward: n int32 ids, fp32 logits [n_want][n_vocab] at places want of these tokens; returns the
+ * next token or -1 */
+int lcu_context_forward(lcu_context*, const int32_t* tokens, int n, const int32_t* want, int n_want, float* logits);
+/* layered decoders, for tests and tools: keep the residual stream [rows][width] after every layer of the
+ * calls that follow (one-token steps then run launch by launch), and read the last call's */
+int lcu_context_record_residual(lcu_context*, int enabled);
+int lcu_context_read_residual(lcu_context*, int layer, float* out, int rows);
 /* results of the last next_token call, fp16: logits and probabilities [n_vocab], the residual
  * stream after the last layer [n][dim] (rows = n of that call) */
 int lcu_context_read_logits(lcu_context*, uint16_t* out);

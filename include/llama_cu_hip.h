@@ -310,6 +310,115 @@ int lcu_fill_f16(void* out_dev, size_t n, uint16_t bits, void* stream);
  * stream's workspace. */
 int lcu_error_stats(void* out3_dev, const void* a_dev, const void* b_dev, size_t n, void* stream);
 
+/* ---- layered decoders: models built from a list of layers (no counterpart in the reference, whose only
+ * model is the LLaMA above).  Element type: activations and weights are bfloat16 or fp32; products
+ * accumulate in fp32; the residual stream, norms, router, gates, recurrent state, scores and softmax are
+ * fp32 whatever the element type.  Vectors (biases, norm weights, decays) are fp32.  Rows of activations
+ * and weights are padded with zeros to a multiple of 64 elements ("ld"), so every K is one. ---- */
+#define LCU_BF16 0
+#define LCU_F32 1
+
+/* out[M,N] (row stride ldo) = lhs[M,K] . w[N,K]^T + bias; columns below gelu_cols then pass through the tanh
+ * GELU.  Output of the element type, or fp32 when out_f32. */
+int lcu_linear(void* out_dev, int out_f32, int ldo, const void* lhs_dev, const void* w_dev, const void* bias_dev,
+               int gelu_cols, int dtype, int M, int K, int N, void* stream);
+
+/* clamped gated unit: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + up_shift) */
+typedef struct lcu_gate_params {
+  float limit, alpha, up_shift;
+} lcu_gate_params;
+/* out[M][N/2] = gated unit of lhs . w^T; w holds, in blocks of 64 rows, 32 gate rows and then the 32 up rows
+ * of the same outputs (N a multiple of 64) */
+int lcu_linear_gated(void* out_dev, int ldo, const void* lhs_dev, const void* w_dev, const lcu_gate_params* gate, int dtype,
+                     int M, int K, int N, void* stream);
+
+/* Mixture of experts.  lcu_router: per token the `top` experts with the largest scores sigmoid(z), z = w . h
+ * in fp32 (int32 [n][top], fp32 [n][top]), and sigmoid of row n_experts of w (one more row) when
+ * shared_gate_dev is given.  lcu_experts_plan sorts the choices by expert: row r of the sorted order is
+ * token row_token[r] with weight row_weight[r], choice k of token t lies at row inverse[t * top + k], and
+ * tiles of at most tile_rows rows of one expert are listed.  lcu_experts_up: gated unit of
+ * row_weight[r] * h[row_token[r]] through expert e's matrix (w_dev + e * expert_stride bytes);
+ * lcu_experts_down: the rows' second product, fp32.  Arrays of the plan are device memory: row_* and
+ * inverse n * top entries, tile_* max_tiles, expert_end n_experts, n_tiles one.  tile_rows is 64 or 128
+ * (bfloat16), 32 (fp32). */
+typedef struct lcu_expert_plan {
+  void* row_token_dev;
+  void* row_weight_dev;
+  void* inverse_dev;
+  void* tile_expert_dev;
+  void* tile_row_dev;
+  void* expert_end_dev;
+  void* n_tiles_dev;
+  int tile_rows;
+  int max_tiles;
+} lcu_expert_plan;
+int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const void* h_dev, const void* w_dev, int n_experts,
+               int top, int dtype, int n, int K, void* stream);
+int lcu_experts_plan(const lcu_expert_plan* plan, const void* expert_dev, const void* weight_dev, int n, int top, int n_experts,
+                     void* stream);
+int lcu_experts_up(void* out_dev, int ldo, const void* lhs_dev, const void* w_dev, size_t expert_stride,
+                   const lcu_gate_params* gate, const lcu_expert_plan* plan, int dtype, int n_tokens, int K, int N,
+                   void* stream);
+int lcu_experts_down(void* out_f32_dev, int ldo, const void* lhs_dev, const void* w_dev, size_t expert_stride,
+                     const lcu_expert_plan* plan, int dtype, int n_rows, int K, int N, void* stream);
+
+/* Row kernels; a row is `width` of ld elements, its RMS norm taken over `groups` equal consecutive parts.
+ * lcu_embed_pos_norm: x = norm(table[id] + pos_table[*start + row]) under w_embed, h = norm(x) under w_next
+ * (NULL: none).  lcu_residual_norm: m = the sublayer's fp32 rows, or per token the sum of its expert rows
+ * (inverse_dev, top) and shared_gate[row] times the shared expert's row; x += norm(m) under w_after; h =
+ * norm(x) under w_next.  lcu_group_norm: h[i] = norm(x[row_index[i]]). */
+int lcu_embed_pos_norm(void* x_dev, void* h_dev, const void* ids_i32_dev, int n_ids, const void* table_dev, int n_vocab,
+                       const void* pos_table_dev, int n_pos, const void* start_dev, const void* w_embed_dev,
+                       const void* w_next_dev, int dtype, int width, int ld, int groups, float eps, void* stream);
+int lcu_residual_norm(void* x_dev, void* h_dev, const void* out_f32_dev, const void* inverse_dev, int top,
+                      const void* shared_f32_dev, const void* shared_gate_dev, const void* w_after_dev,
+                      const void* w_next_dev, int dtype, int rows, int width, int ld, int groups, float eps, void* stream);
+int lcu_group_norm(void* h_dev, const void* x_f32_dev, const void* row_index_dev, const void* w_dev, int dtype, int rows,
+                   int width, int ld, int groups, float eps, void* stream);
+/* index = first maximum of n fp32 logits; probs = fp16(softmax(logits / temp)) */
+int lcu_softmax_argmax_f32(void* probs_f16_dev, void* out_index_dev, const void* logits_dev, int n, float temp, void* stream);
+
+/* Gated linear recurrence.  Channels lie block by block, each block padded to a multiple of 32.
+ * lcu_conv_causal: u[t] = bias + sum over taps of w[k] z[t - (taps - 1) + k] per channel (w fp32
+ * [taps][ld]); inputs before this call come from state [taps - 1][ld] (element type), which is then
+ * brought up to date.  lcu_gated_recurrence: r, i = sigmoid of the block-diagonal products of u (w
+ * [blocks][block_width][block_width]) plus bias, log a = decay r, S = a S + sqrt(1 - a^2) i u from the fp32
+ * state [ld], which is brought up to date; out = S * y.  scratch: lcu_gated_recurrence_scratch bytes. */
+int lcu_conv_causal(void* u_dev, const void* z_dev, int ldz, const void* w_dev, const void* bias_dev, void* state_dev, int taps,
+                    int dtype, int n, int channels, int ld, void* stream);
+size_t lcu_gated_recurrence_scratch(int n, int ld);
+int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, int ldy, const void* wr_dev, const void* wi_dev,
+                         const void* br_dev, const void* bi_dev, const void* decay_dev, void* state_dev, void* scratch_dev,
+                         int dtype, int n, int channels, int block_width, int ld, void* stream);
+
+/* Sliding-window attention with kept first tokens, grouped heads and a per-head distance bias: key j of
+ * position i is visible when j <= i and (i - j < window or j < keep), its score scale q.k - r1 ln(1 + r2
+ * (i - j)).  dk: head size padded to a multiple of 32 (at most 256); dv: value size padded to 32, 64, 128 or
+ * 256.  Caches [positions][kv_heads * dk] and [positions][kv_heads * dv]. */
+typedef struct lcu_window_params {
+  int heads, kv_heads, dk, dv, window, keep;
+  float scale;
+  const void* r1_dev; /* fp32 [heads] */
+  const void* r2_dev;
+} lcu_window_params;
+/* Rows q | k | v of a projection: k and v of row t into cache row *start + t.  v_mode 0: v as it is; 1: and
+ * a copy into v_first [n][v_cols]; 2: (1 - lambda) v + lambda v_first. */
+int lcu_kv_store(void* k_cache_dev, void* v_cache_dev, const void* qkv_dev, int ldq, int q_cols, int k_cols, int v_cols,
+                 void* v_first_dev, int v_mode, const void* lambda_dev, const void* start_dev, int max_positions, int dtype, int n,
+                 void* stream);
+int lcu_attention_windowed(void* out_dev, int ldo, const void* q_dev, int ldq, const void* k_cache_dev, const void* v_cache_dev,
+                           int start, const lcu_window_params* window, int dtype, int n, void* stream);
+/* one new token at position *pos_dev (bfloat16), the visible keys spread over the chip; arrived_dev: kv_heads
+ * uint32, zero before the first call (and left zero).  Uses the stream's workspace. */
+int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* k_cache_dev, const void* v_cache_dev,
+                                  const void* pos_dev, int max_positions, const lcu_window_params* window, void* arrived_dev,
+                                  void* stream);
+
+/* pseudo-random matrix (synthetic weights): mean + std * N(0, 1) (the hash of lcu_fill_normal_f16) into
+ * columns 0 .. cols - 1 of rows of ld elements */
+int lcu_fill_normal_matrix(void* out_dev, size_t rows, int cols, int ld, int dtype, uint64_t seed, uint64_t stream_id, float mean,
+                           float std, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

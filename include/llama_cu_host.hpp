@@ -176,7 +176,15 @@ struct LLAMA_CU_API llama_tokenizer {
   std::string key_;
 };
 
-struct llama_model_impl;
+struct llama_context;
+
+// Not in the reference: the element type a model computes in.  native: the one its family serves it in
+// (fp16 for LLaMA, bfloat16 for the layered decoders).
+enum class element_type : uint8_t {
+  native,
+  bf16,
+  f32,
+};
 
 // llama_cu.h:362-372
 struct LLAMA_CU_API llama_model {
@@ -186,6 +194,16 @@ struct LLAMA_CU_API llama_model {
   // wk 1, wv 2, wo 3, w1 4, w2 5, w3 6}) and whose norm weights are 1, quantised on the device when
   // params.q_type is uint8.  Used by tests and benchmarks, where no checkpoint exists.
   static std::unique_ptr<llama_model> create_synthetic(llama_params params, uint64_t seed, float weight_std);
+  // Not in the reference: the model in a directory, of any family.  A directory with a config.json is of the
+  // family its "architecture" names, with weights in model.safetensors; one with a `params` file is a LLaMA in
+  // the reference's format.  nullptr (and a message) when it cannot be read.
+  static std::unique_ptr<llama_model> open(std::string const& dir, int context_len = 2048,
+                                           element_type type = element_type::native);
+  // a model of the given config.json text with seeded pseudo-random weights
+  static std::unique_ptr<llama_model> create_synthetic(std::string const& config_text, uint64_t seed,
+                                                       element_type type = element_type::native);
+  virtual std::unique_ptr<llama_context> make_context(int context_len, float temperature) = 0;
+  virtual int max_context() const = 0;  // the longest context the family's kernels or position table cover
   virtual ~llama_model() {}
   llama_params params;
   llama_partition partition;
@@ -208,11 +226,23 @@ struct LLAMA_CU_API llama_context {
   // generator started at `seed` for the k-th token drawn; greedy() returns to the maximum.
   virtual void sample_with_seed(uint64_t seed) = 0;
   virtual void greedy() = 0;
+  // Not in the reference: next_token for ids of any width, which also gives the fp32 logits at places
+  // want[0 .. n_want) of these n tokens, [n_want][n_vocab].  Returns the next token, or -1 (nothing done) when
+  // the tokens do not fit the context, an id is outside the vocabulary or a place outside the call.
+  virtual int forward(const int32_t* tokens, int n, const int32_t* want, int n_want, float* logits) = 0;
 
  protected:
-  llama_context(llama_model_impl* model, int context_len, float temperature)
-      : model_(model), context_len_(context_len), temperature_(temperature) {}
-  llama_model_impl* model_;
+  llama_context(int context_len, float temperature) : context_len_(context_len), temperature_(temperature) {}
+  bool call_fits(const int32_t* tokens, int n, const int32_t* want, int n_want, int n_vocab) const {
+    if (n <= 0 || n > context_len_ - start_pos_ || n_want < 0) return false;
+    for (int i = 0; i < n; ++i) {
+      if (tokens[i] < 0 || tokens[i] >= n_vocab) return false;
+    }
+    for (int i = 0; i < n_want; ++i) {
+      if (want[i] < 0 || want[i] >= n) return false;
+    }
+    return true;
+  }
   int context_len_;
   int start_pos_{0};
   float temperature_;

@@ -1,5 +1,6 @@
 """ctypes binding of libllama_cu_amd.so (C ABI: include/llama_cu_hip.h, include/llama_cu_c.h)."""
 import ctypes as C
+import json
 import os
 
 import numpy as np
@@ -91,7 +92,30 @@ SIGNATURES = {
     "lcu_fill_normal_f16": (i32, [vp, sz, u64, u64, f32, vp]),
     "lcu_fill_f16": (i32, [vp, sz, u16, vp]),
     "lcu_error_stats": (i32, [vp, vp, vp, sz, vp]),
+    "lcu_linear": (i32, [vp, i32, i32, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "lcu_linear_gated": (i32, [vp, i32, vp, vp, vp, i32, i32, i32, i32, vp]),
+    "lcu_router": (i32, [vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "lcu_experts_plan": (i32, [vp, vp, vp, i32, i32, i32, vp]),
+    "lcu_experts_up": (i32, [vp, i32, vp, vp, sz, vp, vp, i32, i32, i32, i32, vp]),
+    "lcu_experts_down": (i32, [vp, i32, vp, vp, sz, vp, i32, i32, i32, i32, vp]),
+    "lcu_embed_pos_norm": (i32, [vp, vp, vp, i32, vp, i32, vp, i32, vp, vp, vp, i32, i32, i32, i32, f32, vp]),
+    "lcu_residual_norm": (i32, [vp, vp, vp, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
+    "lcu_group_norm": (i32, [vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
+    "lcu_softmax_argmax_f32": (i32, [vp, vp, vp, i32, f32, vp]),
+    "lcu_conv_causal": (i32, [vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "lcu_gated_recurrence_scratch": (sz, [i32, i32]),
+    "lcu_gated_recurrence": (i32, [vp, vp, vp, i32, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "lcu_kv_store": (i32, [vp, vp, vp, i32, i32, i32, i32, vp, i32, vp, vp, i32, i32, i32, vp]),
+    "lcu_attention_windowed": (i32, [vp, i32, vp, i32, vp, vp, i32, vp, i32, i32, vp]),
+    "lcu_attention_windowed_decode": (i32, [vp, vp, vp, vp, vp, i32, vp, vp, vp]),
+    "lcu_fill_normal_matrix": (i32, [vp, sz, i32, i32, i32, u64, u64, f32, f32, vp]),
     # llama_cu_c.h
+    "lcu_model_open": (vp, [C.c_char_p, i32, i32]),
+    "lcu_model_create_synthetic_config": (vp, [C.c_char_p, u64, i32]),
+    "lcu_model_max_context": (i32, [vp]),
+    "lcu_context_forward": (i32, [vp, vp, i32, vp, i32, vp]),
+    "lcu_context_record_residual": (i32, [vp, i32]),
+    "lcu_context_read_residual": (i32, [vp, i32, vp, i32]),
     "lcu_model_create_synthetic": (vp, [u32, u32, u32, u32, u32, f32, i32, i32, u64, f32]),
     "lcu_model_load": (vp, [C.c_char_p, i32]),
     "lcu_model_destroy": (None, [vp]),
@@ -162,6 +186,23 @@ def device_props(device=0):
     return p
 
 
+class GateParams(C.Structure):
+    """lcu_gate_params"""
+    _fields_ = [("limit", f32), ("alpha", f32), ("up_shift", f32)]
+
+
+class ExpertPlan(C.Structure):
+    """lcu_expert_plan"""
+    _fields_ = [(n, vp) for n in ("row_token", "row_weight", "inverse", "tile_expert", "tile_row", "expert_end", "n_tiles")] + \
+        [("tile_rows", i32), ("max_tiles", i32)]
+
+
+class WindowParams(C.Structure):
+    """lcu_window_params"""
+    _fields_ = [("heads", i32), ("kv_heads", i32), ("dk", i32), ("dv", i32), ("window", i32), ("keep", i32), ("scale", f32),
+                ("r1", vp), ("r2", vp)]
+
+
 class DeviceBuffer:
     """Owning device allocation (lcu_malloc / lcu_free)."""
 
@@ -213,10 +254,15 @@ class Model:
     """llama_model (synthetic weights or a model directory in the reference's file format)."""
 
     def __init__(self, dim=None, multiple_of=None, n_heads=None, n_layers=None, n_vocab=None, norm_eps=1e-6,
-                 q_type=0, qblock=128, seed=0, weight_std=0.02, path=None, context_len=2048):
+                 q_type=0, qblock=128, seed=0, weight_std=0.02, path=None, context_len=2048, config=None, dtype="native"):
+        """path: a model directory of any family; config: the dict of a config.json, weights synthetic; dtype
+        ("native", "bf16", "f32"): the element type of a model with a config.json."""
         L = lib()
+        kind = ("native", "bf16", "f32").index(dtype)
         if path is not None:
-            self.h = L.lcu_model_load(path.encode(), context_len)
+            self.h = L.lcu_model_open(path.encode(), context_len, kind)
+        elif config is not None:
+            self.h = L.lcu_model_create_synthetic_config(json.dumps(config).encode(), seed, kind)
         else:
             self.h = L.lcu_model_create_synthetic(dim, multiple_of, n_heads, n_layers, n_vocab, norm_eps, q_type,
                                                   qblock, seed, weight_std)
@@ -229,6 +275,7 @@ class Model:
         self.dim, self.multiple_of, self.n_heads, self.n_layers, self.n_vocab = d.value, m.value, h.value, l.value, v.value
         self.norm_eps, self.q_type, self.qblock = eps.value, qt.value, (qb.value or qblock)
         self.ffn = L.lcu_model_ffn_dim(self.h)
+        self.max_context = L.lcu_model_max_context(self.h)
 
     def tensor(self, stream_id, rows, cols):
         if self.q_type == 1:
@@ -278,6 +325,26 @@ class Context:
     def next_token(self, tokens):
         t = np.ascontiguousarray(tokens, dtype=np.int16)
         return lib().lcu_context_next_token(self.h, t.ctypes.data_as(vp), len(t))
+
+    def forward(self, tokens, want=()):
+        """(next token, fp32 logits [len(want), vocab] at these places of `tokens`)."""
+        t = np.ascontiguousarray(tokens, dtype=np.int32)
+        w = np.ascontiguousarray(want, dtype=np.int32)
+        out = np.empty((len(w), self.model.n_vocab), dtype=np.float32)
+        token = lib().lcu_context_forward(self.h, t.ctypes.data_as(vp), len(t), w.ctypes.data_as(vp), len(w),
+                                          out.ctypes.data_as(vp))
+        if token < 0:
+            raise LcuError("forward refused: tokens outside the vocabulary or the context, or a place outside the call")
+        return token, out
+
+    def record_residual(self, on=True):
+        check(lib().lcu_context_record_residual(self.h, 1 if on else 0), "record_residual")
+
+    def residual(self, layer, rows):
+        """The fp32 residual stream after a layer in the last call, [rows, width]."""
+        out = np.empty((rows, self.model.dim), dtype=np.float32)
+        check(lib().lcu_context_read_residual(self.h, layer, out.ctypes.data_as(vp), rows), "read_residual")
+        return out
 
     def clear_tokens(self):
         lib().lcu_context_clear_tokens(self.h)

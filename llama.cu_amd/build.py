@@ -10,10 +10,13 @@ LIB = os.path.join(PKG, "libllama_cu_amd.so")
 # W2 + norm launch compiled in (csrc/attention.hip, csrc/gemv.hip, -DLCU_PHASE_TIMELINE), read by timeline.py
 TIMELINE_LIB = os.path.join(PKG, "libllama_cu_amd_timeline.so")
 
-HIP_SOURCES = ["csrc/runtime.hip", "csrc/elementwise.hip", "csrc/gemv.hip", "csrc/gemm.hip", "csrc/attention.hip"]
-HOST_SOURCES = ["host/buffers.cpp", "host/params.cpp", "host/model.cpp", "host/batch.cpp", "host/tokenizer.cpp", "host/capi.cpp"]
+HIP_SOURCES = ["csrc/runtime.hip", "csrc/elementwise.hip", "csrc/gemv.hip", "csrc/gemm.hip", "csrc/attention.hip",
+               "csrc/linear.hip", "csrc/rownorm.hip", "csrc/recurrent.hip", "csrc/windowed.hip", "csrc/experts.hip"]
+HOST_SOURCES = ["host/buffers.cpp", "host/params.cpp", "host/model.cpp", "host/batch.cpp", "host/tokenizer.cpp", "host/capi.cpp",
+                "host/json.cpp", "host/safetensors.cpp", "host/registry.cpp", "host/rirulix.cpp", "host/layered_model.cpp",
+                "host/layered_context.cpp"]
 # command line programs linked against the library (found at run time next to bin/ through $ORIGIN)
-APPS = {"transform": "apps/transform.cpp", "llama_cu": "apps/llama_cu.cpp"}
+APPS = {"transform": "apps/transform.cpp", "llama_cu": "apps/llama_cu.cpp", "trace_run": "apps/trace_run.cpp"}
 BIN = os.path.join(PKG, "bin")
 
 COMMON = ["-O3", "-std=c++17", "-fPIC", "-I" + os.path.join(ROOT, "include"), "-I" + os.path.join(PKG, "csrc"),
@@ -23,7 +26,8 @@ COMMON = ["-O3", "-std=c++17", "-fPIC", "-I" + os.path.join(ROOT, "include"), "-
 DEVICE = ["--offload-arch=gfx950", "-ffp-contract=off", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
-def build(verbose=False):
+def build(verbose=False, apps=None):
+    """The library and the programs named in `apps` (default: all)."""
     objs = []
     os.makedirs(os.path.join(PKG, "build"), exist_ok=True)
     procs = []
@@ -49,6 +53,8 @@ def build(verbose=False):
     subprocess.check_call(cmd)
     os.makedirs(BIN, exist_ok=True)
     for name, src in APPS.items():
+        if apps is not None and name not in apps:
+            continue
         cmd = ["hipcc"] + COMMON + ["-x", "c++", os.path.join(PKG, src), "-o", os.path.join(BIN, name),
                "-L" + PKG, "-lllama_cu_amd", "-Wl,-rpath,$ORIGIN/.."]
         if verbose:
@@ -73,6 +79,7 @@ def build_timeline():
 
 
 if __name__ == "__main__":
-    print(build(verbose="-v" in sys.argv))
+    only = sys.argv[sys.argv.index("--only") + 1:] if "--only" in sys.argv else None  # --only PROGRAM...
+    print(build(verbose="-v" in sys.argv, apps=only))
     if "--timeline" in sys.argv:
         print(build_timeline())

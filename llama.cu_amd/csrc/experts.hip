@@ -1,0 +1,142 @@
+// Mixture of experts: router (scores, choice of the largest, gate of the shared expert) and the
+// plan that sorts the tokens' choices by expert for the grouped products (linear.hip).
+#include "linear.hpp"
+
+using namespace lcu;
+
+namespace {
+
+constexpr int MAX_EXPERTS = 512;
+
+// One workgroup per token: logit e = row e of w . h in fp32, then the `top` largest (ties: the smaller
+// index), their scores sigmoid(z), and sigmoid of the row behind the experts' (the shared gate).
+template <class T>
+__global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, float* __restrict__ weight,
+                                                     float* __restrict__ shared_gate, const T* __restrict__ h,
+                                                     const T* __restrict__ w, int n_experts, int top, int K) {
+  __shared__ float z[MAX_EXPERTS + 1];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t = blockIdx.x;
+  const T* ht = h + (size_t)t * K;
+  const int n_rows = n_experts + (shared_gate ? 1 : 0);
+  for (int e = wave; e < n_rows; e += 4) {
+    const T* we = w + (size_t)e * K;
+    float s = 0.0f;
+    for (int k = lane; k < K; k += WAVE) s = fmaf(to_f32(ht[k]), to_f32(we[k]), s);
+    s = wave_sum(s);
+    if (lane == 0) z[e] = s;
+  }
+  __syncthreads();
+  if (wave != 0) return;
+  if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
+  for (int k = 0; k < top; ++k) {
+    float best = -INFINITY;
+    int idx = 0x7fffffff;
+    for (int e = lane; e < n_experts; e += WAVE) {
+      const float v = z[e];
+      if (v > best || (v == best && e < idx)) {
+        best = v;
+        idx = e;
+      }
+    }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float ob = __shfl_xor(best, off, WAVE);
+      const int oi = __shfl_xor(idx, off, WAVE);
+      if (ob > best || (ob == best && oi < idx)) {
+        best = ob;
+        idx = oi;
+      }
+    }
+    if (idx >= n_experts) idx = k;  // no finite logit left
+    if (lane == 0) {
+      expert[(size_t)t * top + k] = idx;
+      weight[(size_t)t * top + k] = sigmoid_f32(best);
+      z[idx] = -INFINITY;
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+}
+
+// One workgroup: counts per expert, their prefix sums, each choice's sorted row, and the row tiles.
+__global__ __launch_bounds__(1024) void plan_kernel(const int* __restrict__ expert, const float* __restrict__ weight, int n, int top,
+                                                    int n_experts, int tile_rows, int* __restrict__ row_token,
+                                                    float* __restrict__ row_weight, int* __restrict__ inverse,
+                                                    int* __restrict__ tile_expert, int* __restrict__ tile_row,
+                                                    int* __restrict__ expert_end, int* __restrict__ n_tiles) {
+  __shared__ int count[MAX_EXPERTS], next[MAX_EXPERTS], first_tile[MAX_EXPERTS];
+  const int tid = threadIdx.x, rows = n * top;
+  for (int e = tid; e < n_experts; e += 1024) count[e] = 0;
+  __syncthreads();
+  for (int i = tid; i < rows; i += 1024) atomicAdd(&count[expert[i]], 1);
+  __syncthreads();
+  if (tid == 0) {
+    int at = 0, tiles = 0;
+    for (int e = 0; e < n_experts; ++e) {
+      next[e] = at;
+      first_tile[e] = tiles;
+      at += count[e];
+      tiles += (count[e] + tile_rows - 1) / tile_rows;
+    }
+    *n_tiles = tiles;
+  }
+  __syncthreads();
+  for (int e = tid; e < n_experts; e += 1024) {
+    const int begin = next[e], end = begin + count[e];
+    expert_end[e] = end;
+    for (int r = begin, tl = first_tile[e]; r < end; r += tile_rows, ++tl) {
+      tile_expert[tl] = e;
+      tile_row[tl] = r;
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < rows; i += 1024) {
+    const int r = atomicAdd(&next[expert[i]], 1);
+    row_token[r] = i / top;
+    row_weight[r] = weight[i];
+    inverse[i] = r;
+  }
+}
+
+}  // namespace
+
+extern "C" {
+
+int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const void* h_dev, const void* w_dev, int n_experts,
+               int top, int dtype, int n, int K, void* stream) {
+  LCU_REQUIRE(expert_dev && weight_dev && h_dev && w_dev, "lcu_router: null pointer");
+  LCU_REQUIRE(n_experts > 0 && n_experts <= MAX_EXPERTS && top > 0 && top <= n_experts && n >= 0 && K > 0,
+              "lcu_router: experts %d (at most %d), top %d", n_experts, MAX_EXPERTS, top);
+  LCU_REQUIRE(dtype == LCU_BF16 || dtype == LCU_F32, "lcu_router: element type %d", dtype);
+  if (n == 0) return LCU_OK;
+  hipStream_t st = as_stream(stream);
+  if (dtype == LCU_F32) {
+    router_kernel<float><<<n, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const float*)h_dev,
+                                            (const float*)w_dev, n_experts, top, K);
+  } else {
+    router_kernel<bf16_t><<<n, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev,
+                                             (const bf16_t*)w_dev, n_experts, top, K);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+int lcu_experts_plan(const lcu_expert_plan* plan, const void* expert_dev, const void* weight_dev, int n, int top, int n_experts,
+                     void* stream) {
+  LCU_REQUIRE(plan && expert_dev && weight_dev && plan->row_token_dev && plan->row_weight_dev && plan->inverse_dev &&
+                  plan->tile_expert_dev && plan->tile_row_dev && plan->expert_end_dev && plan->n_tiles_dev,
+              "lcu_experts_plan: null pointer");
+  LCU_REQUIRE(n >= 0 && top > 0 && n_experts > 0 && n_experts <= MAX_EXPERTS && plan->tile_rows > 0,
+              "lcu_experts_plan: n %d top %d experts %d", n, top, n_experts);
+  // every expert may end in a partial tile
+  LCU_REQUIRE((long)plan->max_tiles >= (long)n * top / plan->tile_rows + (n_experts < n * top ? n_experts : n * top),
+              "lcu_experts_plan: room for %d tiles", plan->max_tiles);
+  if (n == 0) return LCU_OK;
+  plan_kernel<<<1, 1024, 0, as_stream(stream)>>>((const int*)expert_dev, (const float*)weight_dev, n, top, n_experts, plan->tile_rows,
+                                                 (int*)plan->row_token_dev, (float*)plan->row_weight_dev, (int*)plan->inverse_dev,
+                                                 (int*)plan->tile_expert_dev, (int*)plan->tile_row_dev,
+                                                 (int*)plan->expert_end_dev, (int*)plan->n_tiles_dev);
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+}  // extern "C"

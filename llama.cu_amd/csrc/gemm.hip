@@ -25,6 +25,7 @@
 #include <type_traits>
 
 #include "common.hpp"
+#include "linear.hpp"
 
 using namespace lcu;
 
@@ -354,11 +355,20 @@ __device__ __forceinline__ void wait_vmcnt() {
 // SPLIT (few rows, so few tiles): the grid holds `splits` workgroups per tile, each taking a
 // contiguous run of the K stages and writing its fp32 sums to part[split][M][N];
 // splitk_reduce_kernel adds them in split order and applies the epilogue.
-template <int BM, int BN, int WM, int WN, int KS, int NS, bool U8, bool SPLIT = false>
+//
+// EP: what the accumulators become.  f16_epilogue is the fp16 output described above.  The bfloat16
+// epilogues (linear.hpp) take bfloat16 operands, which travel exactly like the fp16 ones, through
+// v_mfma_f32_32x32x16_bf16, and end in a bias, a GELU, or a clamped gate; GROUPED ones take the
+// rows of a tile and its weight matrix from a tile list on the device (experts_plan in experts.hip).
+struct f16_epilogue {
+  static constexpr bool BF16 = false, GROUPED = false, GATED = false;
+};
+
+template <int BM, int BN, int WM, int WN, int KS, int NS, bool U8, bool SPLIT = false, class EP = f16_epilogue>
 __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void gemm_dl_kernel(
     half_t* __restrict__ out0, const half_t* __restrict__ A, const void* __restrict__ W0, const half_t* __restrict__ S0,
     int M, int K, int N, int block, float beta, int tiles_m, int tiles_n, float* __restrict__ part, int splits,
-    more_matrices_t more) {
+    more_matrices_t more, EP ep) {
   constexpr int NG = WM * WN;                // wavefronts of one group
   constexpr int NW = NG * KS;                // wavefronts
   constexpr int BKS = BK * KS;               // K extent of a stage
@@ -414,7 +424,16 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
       part += (size_t)g * splits * M * N;  // each matrix has its own partial sums
     }
   }
-  const int m0 = tm * BM, n0 = tn * BN;
+  int m0 = tm * BM;
+  const int n0 = tn * BN;
+  if constexpr (EP::GROUPED) {
+    // the launch has as many row tiles as the list can ever hold; the ones past its end have nothing to do
+    if (tm >= *ep.n_tiles) return;
+    const int e = ep.tile_group[tm];
+    m0 = ep.tile_row[tm];
+    M = ep.group_end[e];
+    W = (const char*)W0 + (size_t)e * ep.group_stride;
+  }
 
   // beta != 0: the old values of the output tile, asked for now in 16-byte pieces (tile row c / (BN / 8), eight
   // columns from 8 (c % (BN / 8))) and handed to the lanes that need them through LDS after the last stage.
@@ -424,8 +443,8 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
   // registers that more pieces occupy through the K loop cost the 256 x 128 tile 5 % with beta = 0.
   constexpr int OC = BM * BN / 8 / THREADS;  // pieces per thread
   constexpr int OLD_LD = BN + 8;             // halves per tile row in LDS
-  constexpr bool OLD_PIECES = !SPLIT && OC <= 2;
-  static_assert(BM * BN / 8 % THREADS == 0 && BM * OLD_LD * 2 <= LDS_BYTES, "old tile staging");
+  constexpr bool OLD_PIECES = !SPLIT && !EP::BF16 && OC <= 2;
+  static_assert(!OLD_PIECES || (BM * BN / 8 % THREADS == 0 && BM * OLD_LD * 2 <= LDS_BYTES), "old tile staging");
   // 16-byte requests: rows of a multiple of 8 halves from a 16-byte aligned base (anything else keeps
   // the 2-byte reads of the epilogue)
   const bool old_by_pieces = OLD_PIECES && beta != 0.0f && N % 8 == 0 && (reinterpret_cast<uintptr_t>(out) & 15) == 0;
@@ -449,7 +468,11 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
   for (int j = 0; j < PA; ++j) {
     const int c = (wave + j * NW) * 64 + lane;
     const int row = c / CR, g = (c % CR) ^ ((row / RPB) % CR);
-    a_off[j] = ((uint32_t)min(m0 + row, M - 1) * (uint32_t)K + g * 8) * 2u;
+    int gm = min(m0 + row, M - 1);
+    if constexpr (EP::GROUPED) {
+      if (ep.row_index) gm = ep.row_index[gm];
+    }
+    a_off[j] = ((uint32_t)gm * (uint32_t)K + g * 8) * 2u;
   }
 #pragma unroll
   for (int j = 0; j < PB; ++j) {
@@ -603,7 +626,12 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
     for (int i = 0; i < TM; ++i) {
 #pragma unroll
       for (int j = 0; j < TN; ++j) {
-        acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_f16(fa[buf][i], fb[buf][j], acc[i][j], 0, 0, 0);
+        if constexpr (EP::BF16) {
+          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8_t, fa[buf][i]),
+                                                              __builtin_bit_cast(bf16x8_t, fb[buf][j]), acc[i][j], 0, 0, 0);
+        } else {
+          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_f16(fa[buf][i], fb[buf][j], acc[i][j], 0, 0, 0);
+        }
       }
     }
   };
@@ -739,6 +767,32 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
       __syncthreads();
     }
   }
+  if constexpr (EP::BF16) {
+    static_assert(!SPLIT && !U8, "bfloat16 operands: whole K range per workgroup");
+    if (group == 0) {
+#pragma unroll
+      for (int i = 0; i < TM; ++i) {
+#pragma unroll
+        for (int v = 0; v < 16; ++v) {
+          const int gm = m0 + wm + i * 32 + (v >> 2) * 8 + (lane >> 5) * 4 + (v & 3);
+          if (gm >= M) continue;
+          if constexpr (EP::GATED) {
+            // 32 columns of gate rows, then the 32 of the up rows they belong to: one lane holds both
+            static_assert(TN == 2, "a wavefront's columns are one gate / up pair of blocks");
+            const int hc = (n0 + wn) / 2 + (lane & 31);
+            if (n0 + wn < N) ep.store_gated(gm, hc, acc[i][0][v], acc[i][1][v]);
+          } else {
+#pragma unroll
+            for (int j = 0; j < TN; ++j) {
+              const int gn = n0 + wn + j * 32 + (lane & 31);
+              if (gn < N) ep.store(gm, gn, acc[i][j][v]);
+            }
+          }
+        }
+      }
+    }
+    return;
+  }
   // epilogue as in gemm_kernel (llama_cu.cu:208-215)
   if (group == 0) {
 #pragma unroll
@@ -846,7 +900,7 @@ int launch_dl(operands_t op, const half_t* A, int M, int K, int N, int block, fl
     }
   }
   kernel<<<tiles_m * tiles_n, 64 * WM * WN * KS, lds, st>>>(op.out, A, op.W, op.S, M, K, N, block, beta, tiles_m,
-                                                            tiles_n, nullptr, 1, op.more);
+                                                            tiles_n, nullptr, 1, op.more, f16_epilogue{});
   LCU_LAUNCH_CHECK();
   return LCU_OK;
 }
@@ -883,7 +937,7 @@ int launch_split(operands_t op, const half_t* A, int M, int K, int N, int block,
     }
   }
   kernel<<<tiles_m * tiles_n * splits, 64 * WM * WN * KS, lds, st>>>(op.out, A, op.W, op.S, M, K, N, block, beta, tiles_m,
-                                                                     tiles_n, part, splits, op.more);
+                                                                     tiles_n, part, splits, op.more, f16_epilogue{});
   LCU_LAUNCH_CHECK();
   if (leave) {  // the caller's own kernel adds the partial sums up (fused with what follows the product)
     leave->part = part;
@@ -1252,7 +1306,70 @@ int dispatch_gemm(operands_t op, const half_t* A, int M, int K, int N, int block
   return LCU_OK;
 }
 
+// ---- bfloat16 operands ----
+template <int BM, int BN, int WM, int WN, int KS, int NS, class EP>
+int launch_bf16(EP const& ep, const void* A, const void* W, int tiles_m, int M, int K, int N, hipStream_t st) {
+  constexpr int ROWB = BK * KS * 2;
+  constexpr size_t lds = (size_t)NS * (BM + BN) * ROWB;
+  static_assert(lds <= 160 * 1024, "rings do not fit LDS");
+  static_assert(KS == 1 || lds >= (size_t)BM * BN * 4 / 2, "LDS must hold one group's accumulators");
+  auto kernel = gemm_dl_kernel<BM, BN, WM, WN, KS, NS, false, false, EP>;
+  if constexpr (lds > 64 * 1024) {
+    static bool raised[16] = {};  // per device, once
+    int dev = 0;
+    LCU_HIP(hipGetDevice(&dev));
+    if (!raised[dev & 15]) {
+      LCU_HIP(hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+      raised[dev & 15] = true;
+    }
+  }
+  const int tiles_n = (N + BN - 1) / BN;
+  const more_matrices_t none{{nullptr, nullptr}, {nullptr, nullptr}, {nullptr, nullptr}, 0};
+  kernel<<<tiles_m * tiles_n, 64 * WM * WN * KS, lds, st>>>(nullptr, (const half_t*)A, W, nullptr, M, K, N, 0, 0.0f, tiles_m,
+                                                            tiles_n, nullptr, 1, none, ep);
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
 }  // namespace
+
+namespace lcu {
+
+// One product with every row of lhs: the tile choice of dispatch_gemm.  GATED tiles give a wavefront 64
+// columns (a 32-wide gate block and its up block).
+template <bool GATED>
+int gemm_bf16(linear_epilogue<false, GATED> const& ep, const void* A, const void* W, int M, int K, int N, hipStream_t st) {
+  const auto tm = [&](int bm) { return (M + bm - 1) / bm; };
+  const auto tn = [&](int bn) { return (long)((N + bn - 1) / bn); };
+  if (tm(256) * tn(128) >= 160) return launch_bf16<256, 128, 4, 2, 1, 3>(ep, A, W, tm(256), M, K, N, st);
+  if (tm(128) * tn(128) >= 256) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, tm(128), M, K, N, st);
+  if (tm(128) * tn(128) >= 160) return launch_bf16<128, 128, 4, 2, 1, 3>(ep, A, W, tm(128), M, K, N, st);
+  if constexpr (GATED) {
+    if (M > 64 && tm(128) * tn(64) > 128) return launch_bf16<128, 64, 4, 1, 1, 3>(ep, A, W, tm(128), M, K, N, st);
+    return launch_bf16<64, 64, 2, 1, 1, 3>(ep, A, W, tm(64), M, K, N, st);
+  } else {
+    if (tm(128) * tn(64) > 256) return launch_bf16<128, 64, 2, 2, 1, 3>(ep, A, W, tm(128), M, K, N, st);
+    if (M > 64 && K % 128 == 0 && tm(128) * tn(64) > 128) {
+      return launch_bf16<128, 64, 2, 2, 2, 3>(ep, A, W, tm(128), M, K, N, st);
+    }
+    return launch_bf16<64, 64, 2, 2, 1, 3>(ep, A, W, tm(64), M, K, N, st);
+  }
+}
+template int gemm_bf16<false>(linear_epilogue<false, false> const&, const void*, const void*, int, int, int, hipStream_t);
+template int gemm_bf16<true>(linear_epilogue<false, true> const&, const void*, const void*, int, int, int, hipStream_t);
+
+// Products of groups of rows with one matrix each, from the tile list in ep (row tiles of ep.tile_rows rows, at
+// most max_tiles of them).
+template <bool GATED>
+int gemm_bf16_grouped(linear_epilogue<true, GATED> const& ep, const void* A, const void* W, int max_tiles, int K, int N,
+                      hipStream_t st) {
+  if (ep.tile_rows == 128) return launch_bf16<128, 128, 2, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
+  return launch_bf16<64, 128, 2, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
+}
+template int gemm_bf16_grouped<false>(linear_epilogue<true, false> const&, const void*, const void*, int, int, int, hipStream_t);
+template int gemm_bf16_grouped<true>(linear_epilogue<true, true> const&, const void*, const void*, int, int, int, hipStream_t);
+
+}  // namespace lcu
 
 extern "C" {
 

@@ -1,0 +1,265 @@
+// Gated linear recurrence (Griffin's recurrent block): causal per-channel convolution, block-diagonal
+// gates, and the state S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t with log a_t = decay r_t.
+//
+// Channels are laid out block by block, each block padded with zeros to a multiple of 32 (a padded
+// channel's state stays 0); ld is the row stride, a multiple of 64.  Gates, decays and state are fp32.
+//
+// Several tokens: the recurrence is linear in S, so tokens are cut into chunks of 64.  The gate
+// kernel leaves a_t and the drive b_t of every token and, per chunk, the chunk's map S -> A S + B; one
+// thread per channel runs over the chunks' maps (carry), and then every chunk runs through its own
+// tokens from its incoming state (apply).
+#include "linear.hpp"
+
+using namespace lcu;
+
+namespace {
+
+constexpr int CHUNK = 64;   // tokens per chunk and per gate tile
+constexpr int GATE_N = 32;  // channels per gate tile
+
+// u[t][c] = bias[c] + sum_k w[k][c] z[t - (taps - 1) + k]; inputs before this call come from state
+// [taps - 1][ld], oldest first
+template <class T>
+__global__ __launch_bounds__(256) void conv_causal_kernel(T* __restrict__ u, const T* __restrict__ z, int ldz,
+                                                          const float* __restrict__ w, const float* __restrict__ bias,
+                                                          const T* __restrict__ state, int taps, int channels, int ld) {
+  const int c = blockIdx.x * 256 + threadIdx.x, t = blockIdx.y;
+  if (c >= channels) return;
+  float acc = bias[c];
+  for (int k = 0; k < taps; ++k) {
+    const int s = t - (taps - 1) + k;
+    const float v = s >= 0 ? to_f32(z[(size_t)s * ldz + c]) : to_f32(state[(size_t)(s + taps - 1) * ld + c]);
+    acc = fmaf(w[(size_t)k * ld + c], v, acc);
+  }
+  u[(size_t)t * ld + c] = (T)acc;
+}
+
+// the last taps - 1 inputs become the state; ascending order, so a short call shifts in place
+template <class T>
+__global__ __launch_bounds__(256) void conv_state_kernel(T* __restrict__ state, const T* __restrict__ z, int ldz, int n, int taps,
+                                                         int channels, int ld) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= channels) return;
+  for (int k = 0; k + 1 < taps; ++k) {
+    const int s = k + n - (taps - 1);
+    state[(size_t)k * ld + c] = s >= 0 ? z[(size_t)s * ldz + c] : state[(size_t)(k + n) * ld + c];
+  }
+}
+
+struct gate_args {
+  const void* wr;       // [blocks][bw][bw], rows and blocks padded
+  const void* wi;
+  const float* br;
+  const float* bi;
+  const float* decay;   // log a = decay * r
+  float* a;
+  float* b;
+  float* chunk_a;
+  float* chunk_b;
+  int n, bw, ld;
+};
+
+// One workgroup: 64 tokens x 32 channels of both gates.  Wavefront w multiplies 32 tokens (w & 1) by the
+// channels of gate w >> 1; both gates of a channel then meet in LDS, and every thread turns eight
+// consecutive tokens of one channel into a, b and their composite map.
+template <class T>
+__global__ __launch_bounds__(256) void gates_kernel(const T* __restrict__ u, gate_args p) {
+  __shared__ float gate[2][CHUNK][GATE_N + 1];
+  __shared__ float seg[2][8][GATE_N];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int t0 = blockIdx.y * CHUNK, c0 = blockIdx.x * GATE_N;  // c0: first channel of the tile, inside one block
+  const int blk = c0 / p.bw, j0 = c0 - blk * p.bw;
+  const int which = wave >> 1, rows0 = (wave & 1) * 32;
+  const T* W = (const T*)(which ? p.wi : p.wr) + ((size_t)blk * p.bw + j0) * p.bw;
+  const T* ub = u + (size_t)blk * p.bw;
+  if constexpr (sizeof(T) == 2) {
+    float16_t acc = (float16_t)(0.0f);
+    const T* ua = ub + (size_t)min(t0 + rows0 + (lane & 31), p.n - 1) * p.ld + (lane >> 5) * 8;
+    const T* wa = W + (size_t)(lane & 31) * p.bw + (lane >> 5) * 8;
+#pragma unroll 4
+    for (int k = 0; k < p.bw; k += 16) {
+      const bf16x8_t fa = *reinterpret_cast<const bf16x8_t*>(ua + k);
+      const bf16x8_t fb = *reinterpret_cast<const bf16x8_t*>(wa + k);
+      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa, fb, acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int v = 0; v < 16; ++v) gate[which][rows0 + (v >> 2) * 8 + (lane >> 5) * 4 + (v & 3)][lane & 31] = acc[v];
+  } else {
+    // fp32: lane (channel lane & 31, half lane >> 5) sums 16 tokens of its wavefront's 32
+    float acc[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) acc[i] = 0.0f;
+    for (int k = 0; k < p.bw; ++k) {
+      const float w = W[(size_t)(lane & 31) * p.bw + k];
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        acc[i] = fmaf(ub[(size_t)min(t0 + rows0 + (lane >> 5) * 16 + i, p.n - 1) * p.ld + k], w, acc[i]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) gate[which][rows0 + (lane >> 5) * 16 + i][lane & 31] = acc[i];
+  }
+  __syncthreads();
+  const int ch = tid & 31, s8 = tid >> 5, c = c0 + ch;
+  const float br = p.br[c], bi = p.bi[c], decay = p.decay[c];
+  float A = 1.0f, B = 0.0f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const int lt = s8 * 8 + e, t = t0 + lt;
+    if (t < p.n) {
+      const float r = sigmoid_f32(gate[0][lt][ch] + br), i = sigmoid_f32(gate[1][lt][ch] + bi);
+      const float log_a = decay * r;
+      const float a = expf(log_a);
+      const float b = sqrtf(-expm1f(2.0f * log_a)) * i * to_f32(u[(size_t)t * p.ld + c]);
+      p.a[(size_t)t * p.ld + c] = a;
+      p.b[(size_t)t * p.ld + c] = b;
+      A = a * A;
+      B = fmaf(a, B, b);
+    }
+  }
+  seg[0][s8][ch] = A;
+  seg[1][s8][ch] = B;
+  __syncthreads();
+  if (tid < GATE_N) {
+    A = 1.0f;
+    B = 0.0f;
+#pragma unroll
+    for (int s = 0; s < 8; ++s) {
+      B = fmaf(seg[0][s][tid], B, seg[1][s][tid]);
+      A = seg[0][s][tid] * A;
+    }
+    p.chunk_a[(size_t)blockIdx.y * p.ld + c0 + tid] = A;
+    p.chunk_b[(size_t)blockIdx.y * p.ld + c0 + tid] = B;
+  }
+}
+
+// chunk_a[k] <- the state that enters chunk k; state <- the state after the last chunk
+__global__ __launch_bounds__(64) void carry_kernel(float* __restrict__ chunk_a, const float* __restrict__ chunk_b,
+                                                   float* __restrict__ state, int chunks, int channels, int ld) {
+  const int c = blockIdx.x * 64 + threadIdx.x;
+  if (c >= channels) return;
+  float S = state[c];
+  for (int k0 = 0; k0 < chunks; k0 += 8) {
+    float A[8], B[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int k = min(k0 + e, chunks - 1);
+      A[e] = chunk_a[(size_t)k * ld + c];
+      B[e] = chunk_b[(size_t)k * ld + c];
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      if (k0 + e < chunks) {
+        chunk_a[(size_t)(k0 + e) * ld + c] = S;
+        S = fmaf(A[e], S, B[e]);
+      }
+    }
+  }
+  state[c] = S;
+}
+
+// out[t][c] = S_t * y[t][c] over one chunk
+template <class T>
+__global__ __launch_bounds__(256) void apply_kernel(T* __restrict__ out, const float* __restrict__ a, const float* __restrict__ b,
+                                                    const float* __restrict__ enter, const T* __restrict__ y, int ldy, int n,
+                                                    int channels, int ld) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= channels) return;
+  const int t0 = blockIdx.y * CHUNK, t1 = min(t0 + CHUNK, n);
+  float S = enter[(size_t)blockIdx.y * ld + c];
+  for (int t = t0; t < t1; t += 8) {
+    float av[8], bv[8], yv[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int s = min(t + e, t1 - 1);
+      av[e] = a[(size_t)s * ld + c];
+      bv[e] = b[(size_t)s * ld + c];
+      yv[e] = to_f32(y[(size_t)s * ldy + c]);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      if (t + e < t1) {
+        S = fmaf(av[e], S, bv[e]);
+        out[(size_t)(t + e) * ld + c] = (T)(S * yv[e]);
+      }
+    }
+  }
+}
+
+int check_channels(const char* who, int dtype, int n, int channels, int ld) {
+  LCU_REQUIRE(dtype == LCU_BF16 || dtype == LCU_F32, "%s: element type %d", who, dtype);
+  LCU_REQUIRE(n >= 0 && n <= 65535 && channels > 0 && ld >= channels && ld % 32 == 0, "%s: bad shape n %d channels %d ld %d", who, n,
+              channels, ld);
+  return LCU_OK;
+}
+
+}  // namespace
+
+extern "C" {
+
+int lcu_conv_causal(void* u_dev, const void* z_dev, int ldz, const void* w_dev, const void* bias_dev, void* state_dev, int taps,
+                    int dtype, int n, int channels, int ld, void* stream) {
+  LCU_REQUIRE(u_dev && z_dev && w_dev && bias_dev && (state_dev || taps == 1), "lcu_conv_causal: null pointer");
+  const int rc = check_channels("lcu_conv_causal", dtype, n, channels, ld);
+  if (rc) return rc;
+  LCU_REQUIRE(taps >= 1 && ldz >= channels, "lcu_conv_causal: taps %d, input stride %d", taps, ldz);
+  if (n == 0) return LCU_OK;
+  hipStream_t st = as_stream(stream);
+  const dim3 grid((channels + 255) / 256, n);
+  if (dtype == LCU_F32) {
+    conv_causal_kernel<float><<<grid, 256, 0, st>>>((float*)u_dev, (const float*)z_dev, ldz, (const float*)w_dev,
+                                                    (const float*)bias_dev, (const float*)state_dev, taps, channels, ld);
+    if (taps > 1) {
+      conv_state_kernel<float><<<grid.x, 256, 0, st>>>((float*)state_dev, (const float*)z_dev, ldz, n, taps, channels, ld);
+    }
+  } else {
+    conv_causal_kernel<bf16_t><<<grid, 256, 0, st>>>((bf16_t*)u_dev, (const bf16_t*)z_dev, ldz, (const float*)w_dev,
+                                                     (const float*)bias_dev, (const bf16_t*)state_dev, taps, channels, ld);
+    if (taps > 1) {
+      conv_state_kernel<bf16_t><<<grid.x, 256, 0, st>>>((bf16_t*)state_dev, (const bf16_t*)z_dev, ldz, n, taps, channels, ld);
+    }
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, int ldy, const void* wr_dev, const void* wi_dev,
+                         const void* br_dev, const void* bi_dev, const void* decay_dev, void* state_dev, void* scratch_dev,
+                         int dtype, int n, int channels, int block_width, int ld, void* stream) {
+  LCU_REQUIRE(out_dev && u_dev && y_dev && wr_dev && wi_dev && br_dev && bi_dev && decay_dev && state_dev && scratch_dev,
+              "lcu_gated_recurrence: null pointer");
+  const int rc = check_channels("lcu_gated_recurrence", dtype, n, channels, ld);
+  if (rc) return rc;
+  LCU_REQUIRE(block_width > 0 && block_width % GATE_N == 0 && channels % block_width == 0 && ldy >= channels,
+              "lcu_gated_recurrence: block width %d (a multiple of %d dividing %d channels), stride of y %d", block_width, GATE_N,
+              channels, ldy);
+  if (n == 0) return LCU_OK;
+  hipStream_t st = as_stream(stream);
+  const int chunks = (n + CHUNK - 1) / CHUNK;
+  float* a = (float*)scratch_dev;
+  float* b = a + (size_t)n * ld;
+  float* ca = b + (size_t)n * ld;
+  float* cb = ca + (size_t)chunks * ld;
+  const gate_args p{wr_dev, wi_dev, (const float*)br_dev, (const float*)bi_dev, (const float*)decay_dev, a, b, ca, cb, n,
+                    block_width, ld};
+  const dim3 tiles(channels / GATE_N, chunks), rows((channels + 255) / 256, chunks);
+  if (dtype == LCU_F32) {
+    gates_kernel<float><<<tiles, 256, 0, st>>>((const float*)u_dev, p);
+  } else {
+    gates_kernel<bf16_t><<<tiles, 256, 0, st>>>((const bf16_t*)u_dev, p);
+  }
+  carry_kernel<<<(channels + 63) / 64, 64, 0, st>>>(ca, cb, (float*)state_dev, chunks, channels, ld);
+  if (dtype == LCU_F32) {
+    apply_kernel<float><<<rows, 256, 0, st>>>((float*)out_dev, a, b, ca, (const float*)y_dev, ldy, n, channels, ld);
+  } else {
+    apply_kernel<bf16_t><<<rows, 256, 0, st>>>((bf16_t*)out_dev, a, b, ca, (const bf16_t*)y_dev, ldy, n, channels, ld);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+size_t lcu_gated_recurrence_scratch(int n, int ld) {
+  return ((size_t)2 * n + (size_t)2 * ((n + CHUNK - 1) / CHUNK)) * ld * sizeof(float);
+}
+
+}  // extern "C"

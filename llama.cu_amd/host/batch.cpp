@@ -226,6 +226,10 @@ struct llama_batch_context_impl final : public llama_batch_context {
             LLAMA_CU_MAX_CONTEXT);
     return nullptr;
   }
+  if (dynamic_cast<llama_model_impl*>(model) == nullptr) {
+    fprintf(stderr, "batched decode is available for LLaMA models only\n");
+    return nullptr;
+  }
   return std::make_unique<llama_batch_context_impl>(model, n_sequences, context_len, temperature);
 }
 

@@ -5,18 +5,22 @@
 #include <memory>
 #include <string>
 
+#include "layered_context.hpp"
 #include "model_impl.hpp"
 
 using namespace llama_cu;
 
 struct lcu_model {
   std::unique_ptr<llama_model> model;
-  llama_model_impl* impl() const { return static_cast<llama_model_impl*>(model.get()); }
+  // the LLaMA implementation, or nullptr for a model of another family
+  llama_model_impl* impl() const { return dynamic_cast<llama_model_impl*>(model.get()); }
 };
 
 struct lcu_context {
   std::unique_ptr<llama_context> context;
-  llama_context_impl* impl() const { return static_cast<llama_context_impl*>(context.get()); }
+  int n_vocab;
+  llama_context_impl* impl() const { return dynamic_cast<llama_context_impl*>(context.get()); }
+  layered_context_impl* layered() const { return dynamic_cast<layered_context_impl*>(context.get()); }
 };
 
 struct lcu_batch {
@@ -85,32 +89,34 @@ lcu_model* lcu_model_create_synthetic(uint32_t dim, uint32_t multiple_of, uint32
 }
 
 lcu_model* lcu_model_load(const char* model_dir, int context_len) {
-  if (!model_dir || lcu_init(0) != 0) {
-    return nullptr;
-  }
-  const std::string dir(model_dir);
-  mapped_buffer params_buf(dir + "/params");
-  llama_params p;
-  if (!params_buf.is_ok() || !p.load(params_buf)) {
-    fprintf(stderr, "Could not load params file\n");
-    return nullptr;
-  }
-  llama_partition partition;
-  partition.autopipe(p, (size_t)context_len);
-  if (!partition.is_valid()) {
-    fprintf(stderr, "Could not partition model\n");
-    return nullptr;
-  }
-  auto m = llama_model::load(p, partition, dir);
-  if (!m) {
-    return nullptr;
-  }
-  return new lcu_model{std::move(m)};
+  return lcu_model_open(model_dir, context_len, 0);
 }
+
+static element_type element_of(int dtype) {
+  return dtype == 2 ? element_type::f32 : dtype == 1 ? element_type::bf16 : element_type::native;
+}
+
+lcu_model* lcu_model_open(const char* model_dir, int context_len, int dtype) {
+  if (!model_dir || dtype < 0 || dtype > 2 || lcu_init(0) != 0) {
+    return nullptr;
+  }
+  auto m = llama_model::open(model_dir, context_len, element_of(dtype));
+  return m ? new lcu_model{std::move(m)} : nullptr;
+}
+
+lcu_model* lcu_model_create_synthetic_config(const char* config_text, uint64_t seed, int dtype) {
+  if (!config_text || dtype < 0 || dtype > 2 || lcu_init(0) != 0) {
+    return nullptr;
+  }
+  auto m = llama_model::create_synthetic(std::string(config_text), seed, element_of(dtype));
+  return m ? new lcu_model{std::move(m)} : nullptr;
+}
+
+int lcu_model_max_context(const lcu_model* m) { return m ? m->model->max_context() : -1; }
 
 void lcu_model_destroy(lcu_model* m) { delete m; }
 
-uint32_t lcu_model_ffn_dim(const lcu_model* m) { return m->model->params.ffn_dim(); }
+uint32_t lcu_model_ffn_dim(const lcu_model* m) { return m->impl() ? m->model->params.ffn_dim() : 0; }
 
 void lcu_model_describe(const lcu_model* m, uint32_t* dim, uint32_t* multiple_of, uint32_t* n_heads,
                         uint32_t* n_layers, uint32_t* n_vocab, float* norm_eps, int* q_type,
@@ -127,7 +133,7 @@ void lcu_model_describe(const lcu_model* m, uint32_t* dim, uint32_t* multiple_of
 }
 
 int lcu_model_read_tensor(const lcu_model* m, uint64_t stream_id, void* values, void* scales) {
-  weight_tensor const* t = m->impl()->tensor_by_stream(stream_id);
+  weight_tensor const* t = m->impl() ? m->impl()->tensor_by_stream(stream_id) : nullptr;
   if (!t || !values) {
     return -1;
   }
@@ -139,7 +145,7 @@ int lcu_model_read_tensor(const lcu_model* m, uint64_t stream_id, void* values, 
 }
 
 int lcu_model_tensor_ptr(const lcu_model* m, uint64_t stream_id, void** values_dev, void** scales_dev) {
-  weight_tensor const* t = m->impl()->tensor_by_stream(stream_id);
+  weight_tensor const* t = m->impl() ? m->impl()->tensor_by_stream(stream_id) : nullptr;
   if (!t || !values_dev) {
     return -1;
   }
@@ -152,6 +158,9 @@ int lcu_model_tensor_ptr(const lcu_model* m, uint64_t stream_id, void** values_d
 
 void* lcu_model_norm_ptr(const lcu_model* m, int which) {
   llama_model_impl* mi = m->impl();
+  if (!mi) {
+    return nullptr;
+  }
   if (which == -1) {
     return mi->norm.data();
   }
@@ -170,7 +179,7 @@ lcu_context* lcu_context_create(lcu_model* m, int context_len, float temperature
   if (!ctx) {
     return nullptr;  // context length beyond what the attention kernels cover
   }
-  return new lcu_context{std::move(ctx)};
+  return new lcu_context{std::move(ctx), (int)m->model->params.n_vocab};
 }
 
 void lcu_context_destroy(lcu_context* c) { delete c; }
@@ -182,9 +191,8 @@ int lcu_context_next_token(lcu_context* c, const int16_t* tokens, int n) {
   if (!c || !tokens || n <= 0 || (size_t)n > c->context->tokens_left()) {
     return -1;  // the reference asserts (llama_cu.cu:1074)
   }
-  const int vocab = (int)c->impl()->model()->params.n_vocab;
   for (int i = 0; i < n; ++i) {
-    if (tokens[i] < 0 || tokens[i] >= vocab) {
+    if (tokens[i] < 0 || tokens[i] >= c->n_vocab) {
       return -1;
     }
   }
@@ -192,19 +200,29 @@ int lcu_context_next_token(lcu_context* c, const int16_t* tokens, int n) {
   return c->context->next_token(v);
 }
 
+int lcu_context_forward(lcu_context* c, const int32_t* tokens, int n, const int32_t* want, int n_want, float* logits) {
+  if (!c || !tokens || (n_want > 0 && (!want || !logits))) {
+    return -1;
+  }
+  return c->context->forward(tokens, n, want, n_want, logits);
+}
+
 int lcu_context_read_logits(lcu_context* c, uint16_t* out) {
   auto* ci = c->impl();
-  return lcu_d2h(out, ci->logits().data(), ci->logits().size(), ci->stream());
+  return ci ? lcu_d2h(out, ci->logits().data(), ci->logits().size(), ci->stream()) : -1;
 }
 
 int lcu_context_read_probs(lcu_context* c, uint16_t* out) {
+  if (auto* ly = c->layered()) {
+    return lcu_d2h(out, ly->probs().data(), (size_t)c->n_vocab * 2, ly->stream());
+  }
   auto* ci = c->impl();
-  return lcu_d2h(out, ci->probs().data(), ci->probs().size(), ci->stream());
+  return ci ? lcu_d2h(out, ci->probs().data(), ci->probs().size(), ci->stream()) : -1;
 }
 
 int lcu_context_read_hidden(lcu_context* c, uint16_t* out, int rows) {
   auto* ci = c->impl();
-  if (rows <= 0 || rows > ci->last_n()) {
+  if (!ci || rows <= 0 || rows > ci->last_n()) {
     return -1;
   }
   return lcu_d2h(out, ci->hidden().data(), (size_t)rows * ci->model()->params.dim * 2, ci->stream());
@@ -212,7 +230,7 @@ int lcu_context_read_hidden(lcu_context* c, uint16_t* out, int rows) {
 
 int lcu_context_read_kv(lcu_context* c, int layer, uint16_t* k_out, uint16_t* v_out, int T) {
   auto* ci = c->impl();
-  if (layer < 0 || (size_t)layer >= ci->kv().size() || T <= 0 || T > ci->context_len()) {
+  if (!ci || layer < 0 || (size_t)layer >= ci->kv().size() || T <= 0 || T > ci->context_len()) {
     return -1;
   }
   const size_t bytes = (size_t)T * ci->model()->params.dim * 2;
@@ -221,9 +239,19 @@ int lcu_context_read_kv(lcu_context* c, int layer, uint16_t* k_out, uint16_t* v_
   return 0;
 }
 
-void* lcu_context_stream(lcu_context* c) { return c->impl()->stream(); }
+int lcu_context_record_residual(lcu_context* c, int enabled) {
+  if (!c->layered()) return -1;
+  c->layered()->record_residual(enabled != 0);
+  return 0;
+}
 
-int lcu_context_hand_over_fallbacks(lcu_context* c) { return c->impl()->hand_over_fallbacks(); }
+int lcu_context_read_residual(lcu_context* c, int layer, float* out, int rows) {
+  return c->layered() ? c->layered()->read_residual(layer, out, rows) : -1;
+}
+
+void* lcu_context_stream(lcu_context* c) { return c->layered() ? c->layered()->stream() : c->impl()->stream(); }
+
+int lcu_context_hand_over_fallbacks(lcu_context* c) { return c->impl() ? c->impl()->hand_over_fallbacks() : 0; }
 
 lcu_batch* lcu_batch_create(lcu_model* m, int n_sequences, int context_len, float temperature) {
   if (!m || n_sequences <= 0 || context_len <= 0 || !(temperature > 0.0f)) {
@@ -233,7 +261,7 @@ lcu_batch* lcu_batch_create(lcu_model* m, int n_sequences, int context_len, floa
   if (!ctx) {
     return nullptr;
   }
-  return new lcu_batch{std::move(ctx), (int)m->impl()->params.n_vocab};
+  return new lcu_batch{std::move(ctx), (int)m->model->params.n_vocab};
 }
 
 void lcu_batch_destroy(lcu_batch* b) { delete b; }
@@ -278,9 +306,9 @@ int lcu_batch_read_probs(lcu_batch* b, uint16_t* out) { return batch_context_rea
 
 void lcu_context_set_sampling(lcu_context* c, int enabled, uint64_t seed) {
   if (enabled) {
-    c->impl()->sample_with_seed(seed);
+    c->context->sample_with_seed(seed);
   } else {
-    c->impl()->greedy();
+    c->context->greedy();
   }
 }
 

@@ -234,7 +234,7 @@ static bool shapes_supported(llama_params const& p) {
 // context
 // ------------------------------------------------------------------------------------------------
 llama_context_impl::llama_context_impl(llama_model* model, int context_len, float temperature)
-    : llama_context(static_cast<llama_model_impl*>(model), context_len, temperature) {
+    : llama_context(context_len, temperature), model_(static_cast<llama_model_impl*>(model)) {
   device_structure_lock lock(device_structure_mutex());
   LCU_CHECK(lcu_init(0));
   LCU_CHECK(lcu_stream_create(&stream_));
@@ -425,7 +425,7 @@ void llama_context_impl::enqueue_layers(int n, bool first_norm_ready) {
 
 // final norm of the last row, logits, softmax with temperature, argmax: llama_cu.cu:1191-1209.
 // The reference normalises every row and uses the last one.
-void llama_context_impl::enqueue_head(int n) {
+void llama_context_impl::enqueue_logits(int row) {
   llama_params const& p = model_->params;
   const int dim = p.dim, vocab = p.n_vocab;
   const int block = p.q_type == quantization_type::uint8 ? p.quantization_block_size : 0;
@@ -433,14 +433,19 @@ void llama_context_impl::enqueue_head(int n) {
   if (block > 0) {
     // uint8 weights: the GEMV is bound by its vector instructions, and normalising the row in each of
     // its 16 000 workgroups costs more there (60 us) than a norm launch of its own (6 + 39 us)
-    LCU_CHECK(lcu_rmsnorm(t_norm_.data(), x + (size_t)(n - 1) * dim * 2, model_->norm.data(), 1, dim, p.norm_eps, stream_));
+    LCU_CHECK(lcu_rmsnorm(t_norm_.data(), x + (size_t)row * dim * 2, model_->norm.data(), 1, dim, p.norm_eps, stream_));
     LCU_CHECK(lcu_gemm_f16u8_nt(t_logits_.data(), t_norm_.data(), model_->output.data.data(),
                                 model_->output.scales.data(), 1, dim, vocab, block, 0.0f, stream_));
   } else {
-    LCU_CHECK(lcu_decode_logits(t_logits_.data(), x + (size_t)(n - 1) * dim * 2, model_->norm.data(),
+    LCU_CHECK(lcu_decode_logits(t_logits_.data(), x + (size_t)row * dim * 2, model_->norm.data(),
                                 model_->output.data.data(), model_->output.scales.data(), block, dim, vocab, p.norm_eps,
                                 stream_));
   }
+}
+
+void llama_context_impl::enqueue_head(int n) {
+  const int vocab = model_->params.n_vocab;
+  enqueue_logits(n - 1);
   // the first maximum of the fp16 probabilities is found on the device; 4 bytes go back to the host
   // and, next to it, the stream's count of hand-overs that did not arrive, for next_token's one copy back
   LCU_CHECK(lcu_softmax_argmax_status(t_probs_.data(), t_argmax_.data(), t_logits_.data(), vocab, temperature_,
@@ -602,15 +607,45 @@ short llama_context_impl::next_token(std::vector<short> const& new_tokens) {
   return (short)result.token;
 }
 
+int llama_context_impl::forward(const int32_t* tokens, int n, const int32_t* want, int n_want, float* logits) {
+  const int vocab = (int)model_->params.n_vocab;
+  if (!call_fits(tokens, n, want, n_want, vocab)) {
+    return -1;
+  }
+  const short token = next_token(std::vector<short>(tokens, tokens + n));
+  // the residual rows of the call are still there: the wanted ones go through the head one by one, the last
+  // row last, so that the logits and probabilities left behind are those of the next token
+  std::vector<uint16_t> row(vocab);
+  for (int i = 0; i < n_want; ++i) {
+    enqueue_logits(want[i]);
+    LCU_CHECK(lcu_d2h(row.data(), t_logits_.data(), (size_t)vocab * 2, stream_));
+    for (int v = 0; v < vocab; ++v) {
+      _Float16 h;
+      memcpy(&h, &row[v], 2);
+      logits[(size_t)i * vocab + v] = (float)h;
+    }
+  }
+  if (n_want > 0 && want[n_want - 1] != n - 1) {
+    enqueue_logits(n - 1);
+  }
+  return token;
+}
+
+std::unique_ptr<llama_context> llama_model_impl::make_context(int context_len, float temperature) {
+  return std::make_unique<llama_context_impl>(this, context_len, temperature);
+}
+
 /* static */ std::unique_ptr<llama_context> llama_context::create(llama_model* model, int context_len,
                                                                   float temperature) {
   // The reference leaves context_len free (llama_cu.h:376); the attention kernels here hold a row of
-  // scores per head in LDS, which bounds it.  Refused at creation, not in the middle of a generation.
-  if (model == nullptr || context_len <= 0 || context_len > LLAMA_CU_MAX_CONTEXT) {
-    fprintf(stderr, "unsupported context length %d (1..%d)\n", context_len, LLAMA_CU_MAX_CONTEXT);
+  // scores per head in LDS, which bounds it, and learned positions end somewhere.  Refused at creation, not
+  // in the middle of a generation.
+  const int most = model ? model->max_context() : LLAMA_CU_MAX_CONTEXT;
+  if (model == nullptr || context_len <= 0 || context_len > most) {
+    fprintf(stderr, "unsupported context length %d (1..%d)\n", context_len, most);
     return nullptr;
   }
-  return std::make_unique<llama_context_impl>(model, context_len, temperature);
+  return model->make_context(context_len, temperature);
 }
 
 }  // namespace llama_cu

@@ -34,6 +34,8 @@ struct llama_model_impl : public llama_model {
   bool load_impl(std::string const& path);
   void synthesize(uint64_t seed, float weight_std);
   weight_tensor const* tensor_by_stream(uint64_t stream_id) const;
+  std::unique_ptr<llama_context> make_context(int context_len, float temperature) override;
+  int max_context() const override { return LLAMA_CU_MAX_CONTEXT; }
   weight_tensor tok_embeddings;
   weight_tensor output;
   gpu_buffer norm;
@@ -48,6 +50,7 @@ struct llama_context_impl final : public llama_context {
   short next_token(std::vector<short> const& new_tokens) override;
   void sample_with_seed(uint64_t seed) override;
   void greedy() override;
+  int forward(const int32_t* tokens, int n, const int32_t* want, int n_want, float* logits) override;
 
   // read-back used by tests and tools
   llama_model_impl* model() const { return model_; }
@@ -74,6 +77,8 @@ struct llama_context_impl final : public llama_context {
   }
 
  private:
+  llama_model_impl* model_;
+  void enqueue_logits(int row);
   void matmul(void* out, const void* lhs, weight_tensor const& w, int M, float beta);
   void matmul_multi(void* const* outs, const void* lhs, weight_tensor const* const* ws, int count, int M);
   void enqueue_layers(int n, bool first_norm_ready = false);
