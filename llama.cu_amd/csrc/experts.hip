@@ -8,26 +8,9 @@ namespace {
 
 constexpr int MAX_EXPERTS = 512;
 
-// One workgroup per token: logit e = row e of w . h in fp32, then the `top` largest (ties: the smaller
-// index), their scores sigmoid(z), and sigmoid of the row behind the experts' (the shared gate).
-template <class T>
-__global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, float* __restrict__ weight,
-                                                     float* __restrict__ shared_gate, const T* __restrict__ h,
-                                                     const T* __restrict__ w, int n_experts, int top, int K) {
-  __shared__ float z[MAX_EXPERTS + 1];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t = blockIdx.x;
-  const T* ht = h + (size_t)t * K;
-  const int n_rows = n_experts + (shared_gate ? 1 : 0);
-  for (int e = wave; e < n_rows; e += 4) {
-    const T* we = w + (size_t)e * K;
-    float s = 0.0f;
-    for (int k = lane; k < K; k += WAVE) s = fmaf(to_f32(ht[k]), to_f32(we[k]), s);
-    s = wave_sum(s);
-    if (lane == 0) z[e] = s;
-  }
-  __syncthreads();
-  if (wave != 0) return;
-  if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
+// One wavefront: the `top` largest of z (LDS; ties: the smaller index), with their scores.  z is used up.
+__device__ __forceinline__ void choose(float* z, int n_experts, int top, int* __restrict__ expert, float* __restrict__ weight) {
+  const int lane = threadIdx.x & 63;
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
     int idx = 0x7fffffff;
@@ -49,12 +32,74 @@ __global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, f
     }
     if (idx >= n_experts) idx = k;  // no finite logit left
     if (lane == 0) {
-      expert[(size_t)t * top + k] = idx;
-      weight[(size_t)t * top + k] = sigmoid_f32(best);
+      expert[k] = idx;
+      weight[k] = sigmoid_f32(best);
       z[idx] = -INFINITY;
     }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
+}
+
+// One workgroup per token: logit e = row e of w . h in fp32, then the `top` largest (ties: the smaller
+// index), their scores sigmoid(z), and sigmoid of the row behind the experts' (the shared gate).
+template <class T>
+__global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, float* __restrict__ weight,
+                                                     float* __restrict__ shared_gate, const T* __restrict__ h,
+                                                     const T* __restrict__ w, int n_experts, int top, int K) {
+  __shared__ float z[MAX_EXPERTS + 1];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t = blockIdx.x;
+  const T* ht = h + (size_t)t * K;
+  const int n_rows = n_experts + (shared_gate ? 1 : 0);
+  for (int e = wave; e < n_rows; e += 4) {
+    const T* we = w + (size_t)e * K;
+    float s = 0.0f;
+    for (int k = lane; k < K; k += WAVE) s = fmaf(to_f32(ht[k]), to_f32(we[k]), s);
+    s = wave_sum(s);
+    if (lane == 0) z[e] = s;
+  }
+  __syncthreads();
+  if (wave != 0) return;
+  if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
+  choose(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
+}
+
+// One new token: a wavefront per row of w; the workgroup that arrives last (its counter goes back to zero)
+// chooses.
+__global__ __launch_bounds__(256) void router_step_kernel(int* __restrict__ expert, float* __restrict__ weight,
+                                                          float* __restrict__ shared_gate, const bf16_t* __restrict__ h,
+                                                          const bf16_t* __restrict__ w, int n_experts, int top, int K,
+                                                          float* __restrict__ logits, uint32_t* __restrict__ arrived) {
+  __shared__ float z[MAX_EXPERTS + 1];
+  __shared__ bool last;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int n_rows = n_experts + (shared_gate ? 1 : 0), e = blockIdx.x * 4 + wave;
+  if (e < n_rows) {
+    const bf16_t* we = w + (size_t)e * K;
+    float s = 0.0f;
+#pragma unroll 8
+    for (int k = lane * 8; k < K; k += WAVE * 8) {
+      const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(h + k), wv = *reinterpret_cast<const bf16x8_t*>(we + k);
+#pragma unroll
+      for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
+    }
+    s = wave_sum(s);
+    if (lane == 0) __hip_atomic_store(logits + e, s, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // every wavefront's logit is out before the barrier
+  __syncthreads();
+  if (tid == 0) {
+    last = __hip_atomic_fetch_add(arrived, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == gridDim.x - 1;
+    if (last) __hip_atomic_store(arrived, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!last) return;
+  for (int i = tid; i < n_rows; i += 256) z[i] = __hip_atomic_load(logits + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  __syncthreads();
+  if (wave != 0) return;
+  if (shared_gate && lane == 0) *shared_gate = sigmoid_f32(z[n_experts]);
+  choose(z, n_experts, top, expert, weight);
 }
 
 // One workgroup: counts per expert, their prefix sums, each choice's sorted row, and the row tiles.
@@ -116,6 +161,21 @@ int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const 
     router_kernel<bf16_t><<<n, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev,
                                              (const bf16_t*)w_dev, n_experts, top, K);
   }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+int lcu_decode_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const void* h_dev, const void* w_dev, int n_experts,
+                      int top, void* arrived_dev, int K, void* stream) {
+  LCU_REQUIRE(expert_dev && weight_dev && h_dev && w_dev && arrived_dev, "lcu_decode_router: null pointer");
+  LCU_REQUIRE(n_experts > 0 && n_experts <= MAX_EXPERTS && top > 0 && top <= n_experts && K > 0 && K % 64 == 0,
+              "lcu_decode_router: experts %d (at most %d), top %d, K %d", n_experts, MAX_EXPERTS, top, K);
+  hipStream_t st = as_stream(stream);
+  const workspace_t ws = workspace_for(st);
+  if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_decode_router: lcu_init has not run on this device");
+  router_step_kernel<<<(n_experts + 1 + 3) / 4, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev,
+                                                              (const bf16_t*)h_dev, (const bf16_t*)w_dev, n_experts, top, K,
+                                                              (float*)ws.ptr, (uint32_t*)arrived_dev);
   LCU_LAUNCH_CHECK();
   return LCU_OK;
 }

@@ -24,6 +24,8 @@
 // kernel-order flavour restates from measured samples): the dequantisation arithmetic, not HBM,
 // is what bounds this kernel on large matrices.
 #include "common.hpp"
+#include "linear.hpp"
+#include "rownorm.hpp"
 
 #include <type_traits>
 
@@ -121,8 +123,10 @@ __device__ __forceinline__ half2_t dequant2_fma(uint32_t biased, half2_t scale, 
 
 // ---- one batch in registers: U chunks of R rows of W (16 bytes per lane each), with the matching
 // pieces of x and, when x is to be normalised, of the norm weights ------------------------------
-template <bool U8, int R, int U, bool NORM>
+// BF: weights and x are bfloat16 instead of fp16 (they travel in the same registers)
+template <bool U8, int R, int U, bool NORM, bool BF = false>
 struct batch_t {
+  static_assert(!BF || (!U8 && !NORM), "bfloat16 rows: plain weights on a normalised x");
   static constexpr int VEC = U8 ? 16 : 8;          // elements of K per lane per chunk
   static constexpr int CHUNK = VEC * WAVE;         // elements of K covered by one load of a wavefront
   static constexpr int XV = VEC / 8;
@@ -215,6 +219,14 @@ struct batch_t {
                 a1[r] = __builtin_amdgcn_fdot2(hi, __builtin_bit_cast(half2_t, xw[2 * j + 1]), a1[r], false);
               }
             }
+          } else if constexpr (BF) {
+            // a bfloat16 is the upper half of the fp32 it stands for
+            const uint4_t xw = __builtin_bit_cast(uint4_t, xv[0]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              a0[r] = fmaf(__builtin_bit_cast(float, w[u][r][e] << 16), __builtin_bit_cast(float, xw[e] << 16), a0[r]);
+              a1[r] = fmaf(__builtin_bit_cast(float, w[u][r][e] & 0xffff0000u), __builtin_bit_cast(float, xw[e] & 0xffff0000u), a1[r]);
+            }
           } else {
             const half8_t wv = __builtin_bit_cast(half8_t, w[u][r]);
 #pragma unroll
@@ -239,9 +251,9 @@ struct batch_t {
 // statistics; run() does the rest (NB == 0: a loop that requests one batch ahead; NB > 0: the
 // batches summed in the same order, K <= NB * WAVES * U * CHUNK) and ends with the
 // cross-wavefront sum.
-template <bool U8, int R, int U, bool NORM, class Tasks, int NB = 0>
+template <bool U8, int R, int U, bool NORM, class Tasks, int NB = 0, bool BF = false>
 struct stream_t {
-  using batch = batch_t<U8, R, U, NORM>;
+  using batch = batch_t<U8, R, U, NORM, BF>;
   const Tasks tk;  // by value: a reference member kept the struct in scratch memory in some instantiations
   const half_t* x;
   const half_t* norm_w;
@@ -689,6 +701,280 @@ __global__ __launch_bounds__(GEMV_THREADS) void decode_proj_norm_kernel(
   PTL_MARK(2);
 }
 
+// ---- one new token of a layered decoder (bfloat16 weights, x already normalised) -----------------
+// Rows with a bias; what a finished row becomes is the epilogue's business.
+template <int R, class Epilogue>
+struct bf16_tasks {
+  const bf16_t* W;
+  int K, N;
+  Epilogue ep;
+  __device__ __forceinline__ void rows(int task, const uint8_t* (&rows)[R], const half_t* (&srow)[R]) const {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      rows[r] = row_ptr<false>(W, min(task * R + r, N - 1), K);
+      srow[r] = nullptr;
+    }
+  }
+  __device__ __forceinline__ void finish(int task, const float (&acc)[R]) const {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      if (task * R + r < N) ep(task * R + r, acc[r]);
+    }
+  }
+};
+
+// out[n] = acc + bias[n], fp32 (logits)
+struct store_f32_row {
+  float* out;
+  const float* bias;
+  __device__ __forceinline__ void operator()(int n, float v) const { out[n] = bias ? v + bias[n] : v; }
+};
+
+// The two branches of a recurrent block: rows below ld give y = gelu(.); the others the input of the
+// convolution, whose step is taken here: one thread owns a channel's row and its last inputs.
+struct conv_step_row {
+  bf16_t* y;
+  bf16_t* u;
+  bf16_t* state;  // [taps - 1][ld], oldest first
+  const float* bias;
+  const float* conv;  // [taps][ld]
+  const float* conv_bias;
+  int taps, ld;
+  __device__ __forceinline__ void operator()(int n, float v) const {
+    v += bias[n];
+    if (n < ld) {
+      y[n] = (bf16_t)gelu_tanh(v);
+      return;
+    }
+    const int c = n - ld;
+    const bf16_t z = (bf16_t)v;
+    float acc = conv_bias[c];
+    for (int k = 0; k + 1 < taps; ++k) {
+      acc = fmaf(conv[(size_t)k * ld + c], (float)state[(size_t)k * ld + c], acc);
+      state[(size_t)k * ld + c] = k + 2 < taps ? state[(size_t)(k + 1) * ld + c] : z;
+    }
+    acc = fmaf(conv[(size_t)(taps - 1) * ld + c], (float)z, acc);
+    u[c] = (bf16_t)acc;
+  }
+};
+
+// q | k | v rows of an attention layer: q to q_out, k and the (mixed) v to the caches' row of this position
+struct qkv_row {
+  bf16_t* q_out;
+  bf16_t* k_cache;
+  bf16_t* v_cache;
+  bf16_t* v_first;
+  const float* bias;
+  const float* lambda;
+  const int* pos_dev;
+  int q_cols, k_cols, v_cols, v_mode, max_pos;
+  __device__ __forceinline__ void operator()(int n, float v) const {
+    bf16_t b = (bf16_t)(v + bias[n]);
+    if (n < q_cols) {
+      q_out[n] = b;
+      return;
+    }
+    const size_t pos = min(max(*pos_dev, 0), max_pos - 1);
+    n -= q_cols;
+    if (n < k_cols) {
+      k_cache[pos * k_cols + n] = b;
+      return;
+    }
+    n -= k_cols;
+    if (n >= v_cols) return;  // padding rows
+    if (v_mode == 1) v_first[n] = b;
+    if (v_mode == 2) b = (bf16_t)((1.0f - *lambda) * (float)b + *lambda * (float)v_first[n]);
+    v_cache[pos * v_cols + n] = b;
+  }
+};
+
+template <int R, int U, class Epilogue>
+__global__ __launch_bounds__(GEMV_THREADS) void decode_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ W, int K,
+                                                                   int N, Epilogue ep) {
+  __shared__ float part[GEMV_WAVES * R];
+  const bf16_tasks<R, Epilogue> tk{W, K, N, ep};
+  stream_t<false, R, U, false, bf16_tasks<R, Epilogue>, 0, true> st(tk, reinterpret_cast<const half_t*>(x), nullptr, K, 0, blockIdx.x);
+  st.begin();
+  st.run(nullptr, 1.0f, part);
+}
+
+template <class Epilogue>
+int launch_decode_rows(const void* x, const void* W, int K, int N, Epilogue ep, hipStream_t st) {
+  const bf16_t* xb = (const bf16_t*)x;
+  const bf16_t* Wb = (const bf16_t*)W;
+  if (K > 4096) {
+    decode_rows_kernel<2, 2><<<(N + 1) / 2, GEMV_THREADS, 0, st>>>(xb, Wb, K, N, ep);
+  } else if (K > 2048) {
+    decode_rows_kernel<1, 2><<<N, GEMV_THREADS, 0, st>>>(xb, Wb, K, N, ep);
+  } else {
+    decode_rows_kernel<2, 1><<<(N + 1) / 2, GEMV_THREADS, 0, st>>>(xb, Wb, K, N, ep);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+// Hidden activations of the chosen experts and of the shared one: task = one hidden unit of one slot, i.e. a
+// gate row and an up row (32 rows apart in the packed matrix).  Slot s < top is expert choice[s] with its
+// input scaled by weight[s]; slot top is the shared expert.
+struct expert_slots {
+  const int* choice;
+  const float* weight;
+  const bf16_t* up;
+  const bf16_t* shared_up;
+  size_t up_stride;  // elements
+  bf16_t* hidden;    // [top][ld]
+  bf16_t* shared_hidden;
+  clamped_gate gate, shared_gate;
+  int top, ld, shared_ld, K;
+};
+
+template <int PAIRS>
+struct expert_up_tasks {
+  const bf16_t* W;
+  bf16_t* out;
+  clamped_gate gate;
+  float scale;
+  int K;
+  __device__ __forceinline__ void rows(int task, const uint8_t* (&rows)[2 * PAIRS], const half_t* (&srow)[2 * PAIRS]) const {
+#pragma unroll
+    for (int i = 0; i < PAIRS; ++i) {
+      const int j = task * PAIRS + i, at = j / 32 * 64 + j % 32;
+      rows[2 * i] = row_ptr<false>(W, at, K);
+      rows[2 * i + 1] = row_ptr<false>(W, at + 32, K);
+      srow[2 * i] = srow[2 * i + 1] = nullptr;
+    }
+  }
+  __device__ __forceinline__ void finish(int task, const float (&acc)[2 * PAIRS]) const {
+#pragma unroll
+    for (int i = 0; i < PAIRS; ++i) out[task * PAIRS + i] = (bf16_t)gate(acc[2 * i] * scale, acc[2 * i + 1] * scale);
+  }
+};
+
+template <int U>
+__global__ __launch_bounds__(GEMV_THREADS) void decode_experts_up_kernel(const bf16_t* __restrict__ h, expert_slots p) {
+  __shared__ float part[GEMV_WAVES * 2];
+  const int slot = min((int)blockIdx.x / p.ld, p.top), j = blockIdx.x - slot * p.ld;
+  const bool shared = slot == p.top;
+  const bf16_t* W = shared ? p.shared_up : p.up + (size_t)p.choice[slot] * p.up_stride;
+  const expert_up_tasks<1> tk{W, shared ? p.shared_hidden : p.hidden + (size_t)slot * p.ld, shared ? p.shared_gate : p.gate,
+                              shared ? 1.0f : p.weight[slot], p.K};
+  stream_t<false, 2, U, false, expert_up_tasks<1>, 0, true> st(tk, reinterpret_cast<const half_t*>(h), nullptr, p.K, 0, j);
+  st.begin();
+  st.run(nullptr, 1.0f, part);
+}
+
+// ---- a projection and what follows it: x += norm(projection), h = norm(x) ---------------------------
+// Workgroups compute rows of one or several products (slots: one for a mixer's output; the chosen experts
+// and the shared one for a feed-forward) and store them as fp32 at device scope.  The workgroup that arrives
+// last -- a counter says which, and is set back to zero by it -- adds the slots, normalises the sum, adds it to
+// the residual row, and normalises that for the next sublayer.  Nobody waits for anybody.
+struct projection_slots {
+  const bf16_t* W;
+  const bf16_t* lhs;          // row of slot s at lhs + s * K
+  const int* choice;          // slot s multiplies W + choice[s] * stride; NULL: W itself
+  size_t stride;              // elements
+  int K, slots;
+  const bf16_t* shared_W;     // one more slot, or NULL
+  const bf16_t* shared_lhs;
+  int shared_K;
+  const float* shared_gate;   // its factor
+  const float* bias;
+  float* part;                // [slots + 1][ld]
+};
+struct residual_step {
+  float* x;
+  bf16_t* h;
+  const float* w_after;
+  const float* w_next;  // NULL: no next sublayer
+  uint32_t* arrived;
+  row_shape rs;
+};
+
+struct store_part_row {
+  float* out;
+  const float* bias;
+  __device__ __forceinline__ void operator()(int n, float v) const {
+    __hip_atomic_store(out + n, bias ? v + bias[n] : v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+};
+
+template <int R, int U>
+__global__ __launch_bounds__(GEMV_THREADS) void decode_project_kernel(projection_slots p, residual_step r) {
+  extern __shared__ __attribute__((aligned(16))) float row[];  // rs.width floats (rounded up to 4), then the reduction scratch
+  __shared__ float part[GEMV_WAVES * R];
+  __shared__ bool last;
+  const int per_slot = (r.rs.width + R - 1) / R;
+  const int slot = blockIdx.x / per_slot, task = blockIdx.x - slot * per_slot;
+  {
+    const bool shared = slot == p.slots;
+    const int K = shared ? p.shared_K : p.K;
+    const bf16_t* W = shared ? p.shared_W : p.choice ? p.W + (size_t)p.choice[slot] * p.stride : p.W;
+    const bf16_t* x = shared ? p.shared_lhs : p.lhs + (size_t)slot * p.K;
+    const bf16_tasks<R, store_part_row> tk{W, K, r.rs.width, store_part_row{p.part + (size_t)slot * r.rs.ld, p.bias}};
+    stream_t<false, R, U, false, bf16_tasks<R, store_part_row>, 0, true> st(tk, reinterpret_cast<const half_t*>(x), nullptr, K, 0, task);
+    st.begin();
+    st.run(nullptr, 1.0f, part);
+  }
+  if (threadIdx.x == 0) {
+    // this thread stored the workgroup's rows, write-through; they are complete before the count goes up
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    last = __hip_atomic_fetch_add(r.arrived, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == gridDim.x - 1;
+    if (last) __hip_atomic_store(r.arrived, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!last) return;
+  const int W = r.rs.width, tid = threadIdx.x, total = p.slots + (p.shared_W ? 1 : 0);
+  // the slots' rows at device scope, 16 bytes per request (rows are padded to a multiple of 64 floats)
+  for (int c0 = 0; c0 < W; c0 += 4 * GEMV_THREADS * 4) {
+    float4_t sum[4];
+    int at[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      sum[j] = (float4_t)(0.0f);
+      at[j] = c0 + (j * GEMV_THREADS + tid) * 4;
+    }
+    for (int s = 0; s < total; ++s) {
+      const float* src = p.part + (size_t)s * r.rs.ld;
+      uint4_t v[4];
+      const auto word = [&](int j) { return reinterpret_cast<const uint64_t*>(src + (at[j] < r.rs.ld ? at[j] : 0)); };
+      load_word_pairs_device_scope(v, word(0), word(1), word(2), word(3));
+      const float f = s == p.slots ? *p.shared_gate : 1.0f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) sum[j] += f * __builtin_bit_cast(float4_t, v[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if (at[j] + e < W) row[at[j] + e] = sum[j][e];
+      }
+    }
+  }
+  float* scratch = row + W;
+  group_scale(row, r.rs, scratch, r.w_after);
+  for (int c = tid; c < W; c += GEMV_THREADS) {
+    row[c] += r.x[c];
+    r.x[c] = row[c];
+  }
+  if (r.w_next) {
+    group_scale(row, r.rs, scratch, r.w_next);
+    for (int c = tid; c < W; c += GEMV_THREADS) r.h[c] = (bf16_t)row[c];
+  }
+}
+
+int launch_project(const projection_slots& p, const residual_step& r, hipStream_t st) {
+  const int n = p.slots + (p.shared_W ? 1 : 0);
+  const size_t lds = row_lds_bytes(r.rs);
+  const int K = p.shared_W && p.shared_K > p.K ? p.shared_K : p.K;
+  if (K > 2048) {
+    decode_project_kernel<2, 2><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
+  } else {
+    decode_project_kernel<2, 1><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
 // calls f with the number of 16-byte pieces of x per thread (x_stage_t) that covers dim <= 24576
 template <class F>
 void with_x_pieces(int dim, F&& f) {
@@ -946,6 +1232,86 @@ int lcu_decode_logits(void* logits_dev, const void* x_dev, const void* norm_w_de
   }
   LCU_LAUNCH_CHECK();
   return LCU_OK;
+}
+
+// ---- one new token of a layered decoder ----
+
+int lcu_decode_linear(void* out_f32_dev, const void* x_dev, const void* w_dev, const void* bias_dev, int K, int N, void* stream) {
+  LCU_REQUIRE(out_f32_dev && x_dev && w_dev && K > 0 && K % 64 == 0 && N > 0, "lcu_decode_linear: bad arguments");
+  return launch_decode_rows(x_dev, w_dev, K, N, store_f32_row{(float*)out_f32_dev, (const float*)bias_dev}, as_stream(stream));
+}
+
+int lcu_decode_recurrent_in(void* y_dev, void* u_dev, void* conv_state_dev, const void* x_dev, const void* w_dev,
+                            const void* bias_dev, const void* conv_dev, const void* conv_bias_dev, int taps, int K, int ld,
+                            void* stream) {
+  LCU_REQUIRE(y_dev && u_dev && x_dev && w_dev && bias_dev && conv_dev && conv_bias_dev && (conv_state_dev || taps == 1) && taps >= 1 &&
+                  K > 0 && K % 64 == 0 && ld > 0,
+              "lcu_decode_recurrent_in: bad arguments");
+  return launch_decode_rows(x_dev, w_dev, K, 2 * ld,
+                            conv_step_row{(bf16_t*)y_dev, (bf16_t*)u_dev, (bf16_t*)conv_state_dev, (const float*)bias_dev,
+                                          (const float*)conv_dev, (const float*)conv_bias_dev, taps, ld},
+                            as_stream(stream));
+}
+
+int lcu_decode_kv(void* q_out_dev, void* k_cache_dev, void* v_cache_dev, const void* x_dev, const void* w_dev, const void* bias_dev,
+                  int q_cols, int k_cols, int v_cols, void* v_first_dev, int v_mode, const void* lambda_dev, const void* pos_dev,
+                  int max_positions, int K, void* stream) {
+  LCU_REQUIRE(q_out_dev && k_cache_dev && v_cache_dev && x_dev && w_dev && bias_dev && pos_dev && (v_mode == 0 || v_first_dev) &&
+                  (v_mode != 2 || lambda_dev) && v_mode >= 0 && v_mode <= 2 && K > 0 && K % 64 == 0 && max_positions > 0,
+              "lcu_decode_kv: bad arguments");
+  return launch_decode_rows(x_dev, w_dev, K, q_cols + k_cols + v_cols,
+                            qkv_row{(bf16_t*)q_out_dev, (bf16_t*)k_cache_dev, (bf16_t*)v_cache_dev, (bf16_t*)v_first_dev,
+                                    (const float*)bias_dev, (const float*)lambda_dev, (const int*)pos_dev, q_cols, k_cols, v_cols,
+                                    v_mode, max_positions},
+                            as_stream(stream));
+}
+
+int lcu_decode_experts_up(void* hidden_dev, void* shared_hidden_dev, const void* h_dev, const void* choice_dev,
+                          const void* weight_dev, const void* up_dev, size_t up_stride, const lcu_gate_params* gate,
+                          const void* shared_up_dev, const lcu_gate_params* shared_gate, int top, int ld, int shared_ld, int K,
+                          void* stream) {
+  LCU_REQUIRE(hidden_dev && h_dev && choice_dev && weight_dev && up_dev && gate && (!shared_up_dev || (shared_hidden_dev && shared_gate)),
+              "lcu_decode_experts_up: null pointer");
+  LCU_REQUIRE(top > 0 && ld > 0 && ld % 32 == 0 && (!shared_up_dev || (shared_ld > 0 && shared_ld % 32 == 0)) && K > 0 && K % 64 == 0 &&
+                  up_stride % 2 == 0,
+              "lcu_decode_experts_up: bad shape top %d ld %d %d K %d", top, ld, shared_ld, K);
+  const clamped_gate g{gate->limit, gate->alpha, gate->up_shift};
+  const clamped_gate sg = shared_up_dev ? clamped_gate{shared_gate->limit, shared_gate->alpha, shared_gate->up_shift} : g;
+  const expert_slots p{(const int*)choice_dev, (const float*)weight_dev, (const bf16_t*)up_dev, (const bf16_t*)shared_up_dev,
+                       up_stride / 2, (bf16_t*)hidden_dev, (bf16_t*)shared_hidden_dev, g, sg, top, ld, shared_ld, K};
+  const int grid = top * ld + (shared_up_dev ? shared_ld : 0);
+  if (K > 2048) {
+    decode_experts_up_kernel<2><<<grid, GEMV_THREADS, 0, as_stream(stream)>>>((const bf16_t*)h_dev, p);
+  } else {
+    decode_experts_up_kernel<1><<<grid, GEMV_THREADS, 0, as_stream(stream)>>>((const bf16_t*)h_dev, p);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+int lcu_decode_project_norm(void* x_dev, void* h_dev, const void* lhs_dev, const void* w_dev, const void* bias_dev, int K,
+                            const void* choice_dev, size_t stride, int slots, const void* shared_lhs_dev, const void* shared_w_dev,
+                            int shared_K, const void* shared_gate_dev, const void* w_after_dev, const void* w_next_dev,
+                            void* arrived_dev, int width, int ld, int groups, float eps, void* stream) {
+  LCU_REQUIRE(x_dev && lhs_dev && w_dev && w_after_dev && arrived_dev && (h_dev || !w_next_dev) &&
+                  (!shared_w_dev || (shared_lhs_dev && shared_gate_dev)),
+              "lcu_decode_project_norm: null pointer");
+  LCU_REQUIRE(K > 0 && K % 64 == 0 && slots > 0 && (slots == 1 || choice_dev) && (!shared_w_dev || (shared_K > 0 && shared_K % 64 == 0)) &&
+                  stride % 2 == 0,
+              "lcu_decode_project_norm: bad shape K %d %d slots %d", K, shared_K, slots);
+  LCU_REQUIRE(width > 0 && width <= ROW_MAX_WIDTH && ld >= width && ld % 64 == 0 && groups > 0 && width % groups == 0 &&
+                  groups <= ROW_MAX_GROUPS,
+              "lcu_decode_project_norm: bad row width %d ld %d groups %d", width, ld, groups);
+  hipStream_t st = as_stream(stream);
+  const workspace_t ws = workspace_for(st);
+  if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_decode_project_norm: lcu_init has not run on this device");
+  LCU_REQUIRE((size_t)(slots + 1) * ld * sizeof(float) <= ws.bytes, "lcu_decode_project_norm: %d slots do not fit the workspace", slots);
+  const projection_slots p{(const bf16_t*)w_dev, (const bf16_t*)lhs_dev, (const int*)choice_dev, stride / 2, K, slots,
+                           (const bf16_t*)shared_w_dev, (const bf16_t*)shared_lhs_dev, shared_K, (const float*)shared_gate_dev,
+                           (const float*)bias_dev, (float*)ws.ptr};
+  const residual_step r{(float*)x_dev, (bf16_t*)h_dev, (const float*)w_after_dev, (const float*)w_next_dev, (uint32_t*)arrived_dev,
+                        row_shape{width, ld, groups, eps}};
+  return launch_project(p, r, st);
 }
 
 #ifdef LCU_PHASE_TIMELINE

@@ -186,6 +186,38 @@ __global__ __launch_bounds__(256) void apply_kernel(T* __restrict__ out, const f
   }
 }
 
+// One new token: 16 lanes share a channel, whose two gate rows they multiply with the block's u; the first of
+// them takes the channel's step.
+__global__ __launch_bounds__(256) void recurrent_step_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ u,
+                                                             const bf16_t* __restrict__ y, float* __restrict__ state, gate_args p,
+                                                             int channels) {
+  const int sub = threadIdx.x & 15, c = blockIdx.x * 16 + (threadIdx.x >> 4);
+  if (c >= channels) return;  // whole groups of 16 lanes
+  const bf16_t* wr = (const bf16_t*)p.wr + (size_t)c * p.bw;
+  const bf16_t* wi = (const bf16_t*)p.wi + (size_t)c * p.bw;
+  const bf16_t* ub = u + c / p.bw * p.bw;
+  float r = 0.0f, i = 0.0f;
+#pragma unroll 4
+  for (int k = sub * 8; k < p.bw; k += 128) {
+    const bf16x8_t uv = *reinterpret_cast<const bf16x8_t*>(ub + k);
+    const bf16x8_t rv = *reinterpret_cast<const bf16x8_t*>(wr + k), iv = *reinterpret_cast<const bf16x8_t*>(wi + k);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      r = fmaf((float)rv[e], (float)uv[e], r);
+      i = fmaf((float)iv[e], (float)uv[e], i);
+    }
+  }
+  r = row16_sum(r);
+  i = row16_sum(i);
+  if (sub != 0) return;
+  r = sigmoid_f32(r + p.br[c]);
+  i = sigmoid_f32(i + p.bi[c]);
+  const float log_a = p.decay[c] * r;
+  const float S = fmaf(expf(log_a), state[c], sqrtf(-expm1f(2.0f * log_a)) * i * (float)u[c]);
+  state[c] = S;
+  out[c] = (bf16_t)(S * (float)y[c]);
+}
+
 int check_channels(const char* who, int dtype, int n, int channels, int ld) {
   LCU_REQUIRE(dtype == LCU_BF16 || dtype == LCU_F32, "%s: element type %d", who, dtype);
   LCU_REQUIRE(n >= 0 && n <= 65535 && channels > 0 && ld >= channels && ld % 32 == 0, "%s: bad shape n %d channels %d ld %d", who, n,
@@ -260,6 +292,26 @@ int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, in
 
 size_t lcu_gated_recurrence_scratch(int n, int ld) {
   return ((size_t)2 * n + (size_t)2 * ((n + CHUNK - 1) / CHUNK)) * ld * sizeof(float);
+}
+
+int lcu_decode_recurrent_step(void* out_dev, const void* u_dev, const void* y_dev, const void* wr_dev, const void* wi_dev,
+                              const void* br_dev, const void* bi_dev, const void* decay_dev, void* state_dev, int channels,
+                              int block_width, void* stream) {
+  LCU_REQUIRE(out_dev && u_dev && y_dev && wr_dev && wi_dev && br_dev && bi_dev && decay_dev && state_dev,
+              "lcu_decode_recurrent_step: null pointer");
+  LCU_REQUIRE(channels > 0 && block_width > 0 && block_width % 32 == 0 && channels % block_width == 0,
+              "lcu_decode_recurrent_step: block width %d of %d channels", block_width, channels);
+  gate_args p{};
+  p.wr = wr_dev;
+  p.wi = wi_dev;
+  p.br = (const float*)br_dev;
+  p.bi = (const float*)bi_dev;
+  p.decay = (const float*)decay_dev;
+  p.bw = block_width;
+  recurrent_step_kernel<<<channels / 16, 256, 0, as_stream(stream)>>>((bf16_t*)out_dev, (const bf16_t*)u_dev, (const bf16_t*)y_dev,
+                                                                      (float*)state_dev, p, channels);
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
 }
 
 }  // extern "C"

@@ -2,7 +2,7 @@
 // launch that adds a sublayer's result also normalises the next sublayer's input.
 #include "layered_context.hpp"
 
-#include <assert.h>
+#include <stdlib.h>
 #include <string.h>
 
 #include <algorithm>
@@ -20,7 +20,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   LCU_CHECK(lcu_stream_create(&stream_));
   layered_model_impl const& m = *model_;
   const size_t R = rows_, e = m.elem, ctx = context_len_;
-  size_t wide = 0, u = 0, rec = 0, scratch = 0, hidden = 0, shared = 0, expert_rows = 0, v_first = 0, experts = 0, tiles = 0;
+  size_t counters = 1, wide = 0, u = 0, rec = 0, scratch = 0, hidden = 0, shared = 0, expert_rows = 0, v_first = 0, experts = 0, tiles = 0;
   state_.resize(m.layers.size());
   for (size_t l = 0; l < m.layers.size(); ++l) {
     layer_params const& p = m.shape.layers[l];
@@ -36,6 +36,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
     } else {
       wide = std::max(wide, (size_t)w.attention.ldq);
       rec = std::max(rec, (size_t)w.attention.ldo);
+      counters = std::max(counters, (size_t)p.attention.kv_heads);
       if (w.attention.v_mode != 0) v_first = std::max(v_first, (size_t)w.attention.v_cols);
       state_[l].k = zeroed(ctx * w.attention.k_cols * e);
       state_[l].v = zeroed(ctx * w.attention.v_cols * e);
@@ -68,8 +69,12 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   t_tile_row_ = zeroed(tiles * 4);
   t_expert_end_ = zeroed(experts * 4);
   t_n_tiles_ = zeroed(4);
-  t_ids_ = zeroed(R * 4);
-  t_start_ = zeroed(4);
+  // the one-token attention kernel holds the heads of a group in registers
+  for (layer_params const& p : m.shape.layers) {
+    if (p.mixer == mixer_type::attention && p.attention.heads / p.attention.kv_heads > 16) fused_step_ = false;
+  }
+  t_arrived_ = zeroed(counters * 4);
+  t_step_ = zeroed((1 + R) * 4);
   t_probs_ = zeroed((size_t)m.shape.vocab * 2);
   t_index_ = zeroed(4);
   plan_ = lcu_expert_plan{t_row_token_.data(),   t_row_weight_.data(), t_inverse_.data(), t_tile_expert_.data(),
@@ -80,6 +85,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
 layered_context_impl::~layered_context_impl() {
   lcu_sync(stream_);
   device_structure_lock lock(device_structure_mutex());
+  lcu_graph_destroy(decode_graph_);
   lcu_stream_destroy(stream_);
 }
 
@@ -107,7 +113,7 @@ size_t layered_context_impl::context_memory_usage() {
   for (gpu_buffer const* b :
        {&t_x_, &t_h_, &t_m_, &t_wide_, &t_u_, &t_rec_, &t_scratch_, &t_hidden_, &t_shared_hidden_, &t_expert_out_, &t_shared_out_,
         &t_v_first_, &t_choice_, &t_weight_, &t_shared_gate_, &t_row_token_, &t_row_weight_, &t_inverse_, &t_tile_expert_,
-        &t_tile_row_, &t_expert_end_, &t_n_tiles_, &t_ids_, &t_start_, &t_want_, &t_head_in_, &t_logits_, &t_probs_, &t_index_}) {
+        &t_tile_row_, &t_expert_end_, &t_n_tiles_, &t_arrived_, &t_step_, &t_want_, &t_head_in_, &t_logits_, &t_probs_, &t_index_}) {
     count += b->size();
   }
   return count;
@@ -135,7 +141,7 @@ void layered_context_impl::attention(attention_weights const& w, attention_param
   const lcu_window_params window{p.heads, p.kv_heads, w.dk, w.dv, p.window, p.keep_first, p.scale, w.r1.data(), w.r2.data()};
   LCU_CHECK(lcu_linear(t_wide_.data(), 0, w.ldq, t_h_.data(), w.qkv.data(), w.qkv_bias.data(), 0, m.dtype, n, m.ld, w.ldq, stream_));
   LCU_CHECK(lcu_kv_store(s.k.data(), s.v.data(), t_wide_.data(), w.ldq, w.q_cols, w.k_cols, w.v_cols, t_v_first_.data(), w.v_mode,
-                         w.v_mix.data(), t_start_.data(), context_len_, m.dtype, n, stream_));
+                         w.v_mix.data(), start(), context_len_, m.dtype, n, stream_));
   LCU_CHECK(lcu_attention_windowed(t_rec_.data(), w.ldo, t_wide_.data(), w.ldq, s.k.data(), s.v.data(), start_pos_, &window,
                                    m.dtype, n, stream_));
   LCU_CHECK(lcu_linear(t_m_.data(), 1, m.ld, t_rec_.data(), w.out.data(), w.out_bias.data(), 0, m.dtype, n, w.ldo, m.shape.width,
@@ -165,8 +171,8 @@ void layered_context_impl::experts(experts_weights const& w, experts_params cons
 void layered_context_impl::enqueue_rows(int n) {
   layered_model_impl const& m = *model_;
   layered_params const& p = m.shape;
-  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), t_ids_.data(), n, m.embed.data(), p.vocab, m.pos.data(), p.max_positions,
-                               t_start_.data(), m.embed_norm.data(), next_norm(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps,
+  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), n, m.embed.data(), p.vocab, m.pos.data(), p.max_positions,
+                               start(), m.embed_norm.data(), next_norm(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps,
                                stream_));
   for (size_t l = 0; l < m.layers.size(); ++l) {
     layer_params const& q = p.layers[l];
@@ -196,6 +202,90 @@ void layered_context_impl::enqueue_rows(int n) {
   }
 }
 
+// x += norm(w . lhs + bias) and the next norm, one launch
+void layered_context_impl::project(const void* lhs, const void* w, const void* bias, int K, const void* w_after, const void* w_next) {
+  layered_params const& p = model_->shape;
+  LCU_CHECK(lcu_decode_project_norm(t_x_.data(), t_h_.data(), lhs, w, bias, K, nullptr, 0, 1, nullptr, nullptr, 0, nullptr, w_after,
+                                    w_next, t_arrived_.data(), p.width, model_->ld, p.norm_groups, p.norm_eps, stream_));
+}
+
+// One token: the launches of enqueue_rows fused around the weight streams.  A recurrent layer takes three
+// (both branches with the convolution, gates with the state, output with the norms), an attention layer three
+// (projections with the cache rows, attention, output with the norms), a feed-forward three (router, first
+// products, second products with the norms).  The last layer's norms end in the final one.
+void layered_context_impl::enqueue_one() {
+  layered_model_impl const& m = *model_;
+  layered_params const& p = m.shape;
+  const size_t n_layers = m.layers.size();
+  const auto norm_ahead = [&](size_t l) { return l < n_layers ? m.layers[l].norm1.data() : m.final_norm.data(); };
+  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), 1, m.embed.data(), p.vocab, m.pos.data(), p.max_positions,
+                               start(), m.embed_norm.data(), norm_ahead(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps,
+                               stream_));
+  for (size_t l = 0; l < n_layers; ++l) {
+    layer_params const& q = p.layers[l];
+    layer_weights const& L = m.layers[l];
+    layer_state& s = state_[l];
+    const void* after_mixer = q.has_mlp ? L.norm2.data() : norm_ahead(l + 1);
+    if (q.mixer == mixer_type::rglru) {
+      recurrence_weights const& w = L.recurrence;
+      LCU_CHECK(lcu_decode_recurrent_in(t_wide_.data(), t_u_.data(), s.conv.data(), t_h_.data(), w.yx.data(), w.yx_bias.data(),
+                                        w.conv.data(), w.conv_bias.data(), q.recurrence.taps, m.ld, w.ld, stream_));
+      LCU_CHECK(lcu_decode_recurrent_step(t_rec_.data(), t_u_.data(), t_wide_.data(), w.gate_r.data(), w.gate_i.data(), w.bias_r.data(),
+                                          w.bias_i.data(), w.decay.data(), s.s.data(), w.channels, w.block, stream_));
+      project(t_rec_.data(), w.out.data(), nullptr, w.ld, L.norm1b.data(), after_mixer);
+    } else {
+      attention_weights const& w = L.attention;
+      attention_params const& a = q.attention;
+      const lcu_window_params window{a.heads, a.kv_heads, w.dk, w.dv, a.window, a.keep_first, a.scale, w.r1.data(), w.r2.data()};
+      LCU_CHECK(lcu_decode_kv(t_wide_.data(), s.k.data(), s.v.data(), t_h_.data(), w.qkv.data(), w.qkv_bias.data(), w.q_cols, w.k_cols,
+                              w.v_cols, t_v_first_.data(), w.v_mode, w.v_mix.data(), start(), context_len_, m.ld, stream_));
+      LCU_CHECK(lcu_attention_windowed_decode(t_rec_.data(), t_wide_.data(), s.k.data(), s.v.data(), start(), context_len_,
+                                              &window, t_arrived_.data(), stream_));
+      project(t_rec_.data(), w.out.data(), w.out_bias.data(), w.ldo, L.norm1b.data(), after_mixer);
+    }
+    if (q.has_mlp) {
+      experts_weights const& w = L.mlp;
+      const bool shared = q.mlp.shared_ff > 0;
+      LCU_CHECK(lcu_decode_router(t_choice_.data(), t_weight_.data(), shared ? t_shared_gate_.data() : nullptr, t_h_.data(),
+                                  w.router.data(), q.mlp.experts, q.mlp.top, t_arrived_.data(), m.ld, stream_));
+      LCU_CHECK(lcu_decode_experts_up(t_hidden_.data(), t_shared_hidden_.data(), t_h_.data(), t_choice_.data(), t_weight_.data(),
+                                      w.up.data(), w.up_stride, &q.mlp.gate, w.shared_up.data(), &q.mlp.shared_gate, q.mlp.top, w.ld,
+                                      w.shared_ld, m.ld, stream_));
+      LCU_CHECK(lcu_decode_project_norm(t_x_.data(), t_h_.data(), t_hidden_.data(), w.down.data(), nullptr, w.ld, t_choice_.data(),
+                                        w.down_stride, q.mlp.top, t_shared_hidden_.data(), w.shared_down.data(), w.shared_ld,
+                                        t_shared_gate_.data(), L.norm2b.data(), norm_ahead(l + 1), t_arrived_.data(), p.width, m.ld,
+                                        p.norm_groups, p.norm_eps, stream_));
+    }
+  }
+  LCU_CHECK(lcu_decode_linear(t_logits_.data(), t_h_.data(), m.head.data(), nullptr, m.ld, p.vocab, stream_));
+  LCU_CHECK(lcu_softmax_argmax_f32(t_probs_.data(), t_index_.data(), t_logits_.data(), p.vocab, temperature_, stream_));
+}
+
+// The first step runs eagerly (and loads the kernels), the second is captured, every later one replays it.
+void layered_context_impl::step_one() {
+  device_structure_lock lock(device_structure_mutex());  // capture, instantiation, launch: see host_common.hpp
+  static const bool no_graph = getenv("LLAMA_CU_NO_GRAPH") != nullptr && atoi(getenv("LLAMA_CU_NO_GRAPH")) != 0;
+  if (!decode_graph_ && ++decode_calls_ >= 2 && !no_graph) {
+    LCU_CHECK(lcu_graph_begin_capture(stream_));
+    enqueue_one();
+    LCU_CHECK(lcu_graph_end_capture(stream_, &decode_graph_));
+  }
+  if (decode_graph_) {
+    LCU_CHECK(lcu_graph_launch(decode_graph_, stream_));
+  } else {
+    enqueue_one();
+  }
+}
+
+void layered_context_impl::drop_graph() {
+  if (decode_graph_) {
+    device_structure_lock lock(device_structure_mutex());
+    LCU_CHECK(lcu_graph_destroy(decode_graph_));
+    decode_graph_ = nullptr;
+  }
+  decode_calls_ = 0;
+}
+
 int layered_context_impl::read_residual(int layer, float* out, int rows) const {
   if (layer < 0 || (size_t)layer >= residual_.size()) return -1;
   const size_t count = (size_t)rows * model_->shape.width;
@@ -221,6 +311,7 @@ int layered_context_impl::forward(const int32_t* tokens, int n, const int32_t* w
     return -1;
   }
   if (recording_) residual_.assign(m.layers.size(), {});
+  const bool fused = n == 1 && m.dtype == LCU_BF16 && fused_step_ && !recording_;
   int token = -1;
   for (int at = 0; at < n; at += rows_) {
     const int count = std::min(rows_, n - at);
@@ -235,20 +326,31 @@ int layered_context_impl::forward(const int32_t* tokens, int n, const int32_t* w
     }
     if (ends) rows.push_back(count - 1);
     if ((int)rows.size() > want_cap_) {
+      drop_graph();  // it holds the address of the logits
       want_cap_ = (int)round_up(rows.size(), 64);
       t_want_ = zeroed((size_t)want_cap_ * 4);
       t_head_in_ = zeroed((size_t)want_cap_ * m.ld * m.elem);
       t_logits_ = zeroed((size_t)want_cap_ * vocab * 4);
     }
-    LCU_CHECK(lcu_h2d(t_ids_.data(), tokens + at, (size_t)count * 4, stream_));
-    LCU_CHECK(lcu_h2d(t_start_.data(), &start_pos_, 4, stream_));
-    LCU_CHECK(lcu_h2d(t_want_.data(), rows.data(), rows.size() * 4, stream_));
-    LCU_CHECK(lcu_sync(stream_));  // the host copies above may go away or change
-    enqueue_rows(count);
-    if (!rows.empty()) enqueue_head((int)rows.size());
+    if (at > 0) LCU_CHECK(lcu_sync(stream_));  // the host's copies of the previous pass are about to change
+    host_step_.assign(1, start_pos_);
+    host_step_.insert(host_step_.end(), tokens + at, tokens + at + count);
+    LCU_CHECK(lcu_h2d(t_step_.data(), host_step_.data(), host_step_.size() * 4, stream_));
+    if (!fused && !rows.empty()) {
+      host_want_ = rows;
+      LCU_CHECK(lcu_h2d(t_want_.data(), host_want_.data(), host_want_.size() * 4, stream_));
+    }
+    if (fused) {
+      step_one();
+    } else {
+      enqueue_rows(count);
+      if (!rows.empty()) enqueue_head((int)rows.size());
+      if (ends) {
+        const size_t last = (rows.size() - 1) * (size_t)vocab * 4;
+        LCU_CHECK(lcu_softmax_argmax_f32(t_probs_.data(), t_index_.data(), (char*)t_logits_.data() + last, vocab, temperature_, stream_));
+      }
+    }
     if (ends) {
-      const size_t last = (rows.size() - 1) * (size_t)vocab * 4;
-      LCU_CHECK(lcu_softmax_argmax_f32(t_probs_.data(), t_index_.data(), (char*)t_logits_.data() + last, vocab, temperature_, stream_));
       if (sampling_) {
         uint64_t z = sample_seed_ + ++samples_drawn_ * 0x9E3779B97F4A7C15ull;
         z = (z ^ (z >> 30)) * 0xBF58476D1CE4E5B9ull;
@@ -258,7 +360,8 @@ int layered_context_impl::forward(const int32_t* tokens, int n, const int32_t* w
       LCU_CHECK(lcu_d2h(&token, t_index_.data(), 4, stream_));
     }
     for (size_t i = 0; i < slots.size(); ++i) {  // consecutive rows of logits
-      LCU_CHECK(lcu_d2h(logits + (size_t)slots[i] * vocab, (char*)t_logits_.data() + i * (size_t)vocab * 4, (size_t)vocab * 4, stream_));
+      const size_t row = fused ? 0 : i;
+      LCU_CHECK(lcu_d2h(logits + (size_t)slots[i] * vocab, (char*)t_logits_.data() + row * vocab * 4, (size_t)vocab * 4, stream_));
     }
     start_pos_ += count;
   }

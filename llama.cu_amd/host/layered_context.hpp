@@ -26,7 +26,11 @@ struct layered_context_impl final : public llama_context {
     gpu_buffer conv, s;      // recurrence: the convolution's last inputs [taps - 1][ld], the fp32 state [ld]
   };
   gpu_buffer zeroed(size_t bytes);
-  void enqueue_rows(int n);                        // n > 1 tokens, or one in fp32
+  void enqueue_rows(int n);                        // n tokens, launch by launch
+  void enqueue_one();                              // one token in bfloat16: fused launches, position from t_step_
+  void step_one();                                 // enqueue_one, captured and replayed
+  void drop_graph();
+  void project(const void* lhs, const void* w, const void* bias, int K, const void* w_after, const void* w_next);
   void recurrence(recurrence_weights const& w, recurrence_params const& p, layer_state& s, int n);
   void attention(attention_weights const& w, attention_params const& p, layer_state& s, int n);
   void experts(experts_weights const& w, experts_params const& p, int n);
@@ -39,13 +43,21 @@ struct layered_context_impl final : public llama_context {
   gpu_buffer t_x_, t_h_, t_m_, t_wide_, t_u_, t_rec_, t_scratch_, t_hidden_, t_shared_hidden_, t_expert_out_, t_shared_out_;
   gpu_buffer t_v_first_, t_choice_, t_weight_, t_shared_gate_, t_row_token_, t_row_weight_, t_inverse_, t_tile_expert_,
       t_tile_row_, t_expert_end_, t_n_tiles_;
-  gpu_buffer t_ids_, t_start_, t_want_, t_head_in_, t_logits_, t_probs_, t_index_;
+  gpu_buffer t_step_, t_want_, t_head_in_, t_logits_, t_probs_, t_index_;
+  // t_step_: position of the pass's first token, then its ids (int32); the launches read both from here
+  void* start() const { return t_step_.data(); }
+  void* ids() const { return (char*)t_step_.data() + 4; }
+  std::vector<int32_t> host_step_, host_want_;
   int want_cap_{0};
   lcu_expert_plan plan_{};
+  bool fused_step_{true};                          // one-token steps in bfloat16 take enqueue_one
   bool recording_{false};
   std::vector<std::vector<float>> residual_;
   bool sampling_{false};
   uint64_t sample_seed_{0}, samples_drawn_{0};
+  void* decode_graph_{nullptr};
+  int decode_calls_{0};
+  gpu_buffer t_arrived_;                           // counters of the fused launches, zero between launches
   void* stream_{nullptr};
 };
 
