@@ -2,6 +2,7 @@
 """Headline benchmark: batch-1 greedy decode of a LLaMA-7B-shaped fp16 model on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload llama7b_fp16|llama30b_u8]
+    python bench.py --layered [w2048] [w4096]      # layered decoders beside the LLaMA of equal width
 
 A step is one decode step (one new token through all layers, logits, softmax, argmax, 4-byte
 read-back) after a 512-token prompt; weights are seeded random values of the model's shape
@@ -303,6 +304,91 @@ def batched_leg(P, model, cfg, sizes=(8, 32), prompt=64, steps=32, warmup=4):
     return out
 
 
+# Layered decoders (Rirulix) beside the LLaMA of the same width and active feed-forward width: two recurrent
+# layers to one attention layer, 16 experts of which a token uses two, and a shared expert.
+LAYERED = {
+    "w2048": dict(width=2048, layers=6, heads=16, kv_heads=4, ff=1408, shared_ff=2816, multiple_of=256),
+    "w4096": dict(width=4096, layers=6, heads=32, kv_heads=8, ff=2816, shared_ff=5376, multiple_of=256),
+}
+
+
+def layered_config(s, vocab=32000, context=4096):
+    mlp = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": s["ff"], "limit": 7.0},
+           "shared": {"ff": s["shared_ff"], "limit": 7.0}}
+    rec = {"type": "rglru", "mixer": {"width": s["width"], "blocks": s["width"] // 256, "conv": 4}, "mlp": mlp}
+    att = {"type": "attention", "mlp": mlp,
+           "mixer": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "v_mix": True,
+                     "mask": {"size": 1024, "keep_first": 64}}}
+    return {"architecture": "Rirulix", "width": s["width"], "vocab": vocab, "max_positions": context,
+            "norm": {"eps": 1e-5, "groups": 8}, "layers": [att if l % 3 == 2 else rec for l in range(s["layers"])]}
+
+
+def layered_bytes(s, vocab):
+    """Weight bytes a one-token step reads: every matrix but the experts not chosen."""
+    w = s["width"]
+    n_att = s["layers"] // 3
+    n_rec = s["layers"] - n_att
+    rec = 3 * w * w + 2 * w * 256
+    att = 2 * s["heads"] * 128 * w + 2 * s["kv_heads"] * 128 * w
+    mlp = 3 * w * (2 * s["ff"] + s["shared_ff"]) + 17 * w
+    return 2 * (n_rec * rec + n_att * att + s["layers"] * mlp + vocab * w)
+
+
+def throughput(B, ctx, vocab, prompts, steps, warmup):
+    """Prompt times (second call each) and the one-token step after the first of them."""
+    L = B.lib()
+    rng = np.random.default_rng(0)
+    out = {}
+    for n in prompts:
+        prompt = rng.integers(0, vocab, n).astype(np.int16)
+        ms = []
+        for _ in range(4):
+            ctx.clear_tokens()
+            B.check(L.lcu_sync(None))
+            t0 = time.perf_counter()
+            tok = ctx.next_token(prompt)
+            B.check(L.lcu_sync(None))
+            ms.append((time.perf_counter() - t0) * 1e3)
+        best = sorted(ms[1:])[1]
+        out["prefill_%d" % n] = dict(ms=round(best, 3), tok_s=round(n / best * 1e3, 0))
+        if n == prompts[0]:
+            for _ in range(warmup):
+                tok = ctx.next_token([tok])
+            t0 = time.perf_counter()
+            for _ in range(steps):
+                tok = ctx.next_token([tok])
+            dt = (time.perf_counter() - t0) / steps
+            out["decode"] = dict(ms_per_step=round(dt * 1e3, 4), tok_s=round(1.0 / dt, 1))
+    return out
+
+
+def layered_leg(P, name, steps, warmup, vocab=32000, families=("rirulix", "llama")):
+    B = P.binding
+    s = LAYERED[name]
+    out = {"layers": s["layers"], "width": s["width"]}
+    prompts = (512, 2048)
+    if "rirulix" in families:
+        model = P.Model(config=layered_config(s, vocab), seed=1)
+        ctx = P.Context(model, context_len=4096, temperature=0.8)
+        r = throughput(B, ctx, vocab, prompts, steps, warmup)
+        r["weight_bytes_per_token"] = layered_bytes(s, vocab)
+        r["decode"]["weight_gb_s"] = round(r["weight_bytes_per_token"] / r["decode"]["ms_per_step"] / 1e6, 1)
+        out["rirulix_bf16"] = r
+        ctx.close()
+        model.close()
+    if "llama" in families:
+        cfg = dict(dim=s["width"], multiple_of=s["multiple_of"], n_heads=s["heads"], n_layers=s["layers"], n_vocab=vocab, q_type=0)
+        model = P.Model(norm_eps=1e-6, seed=0, weight_std=0.02, **cfg)
+        ctx = P.Context(model, context_len=4096, temperature=0.8)
+        r = throughput(B, ctx, vocab, prompts, steps, warmup)
+        r["weight_bytes_per_token"] = int(weight_bytes(cfg, model.ffn))
+        r["decode"]["weight_gb_s"] = round(r["weight_bytes_per_token"] / r["decode"]["ms_per_step"] / 1e6, 1)
+        out["llama_fp16"] = r
+        ctx.close()
+        model.close()
+    return out
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -312,6 +398,10 @@ def main():
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
     ap.add_argument("--no-extra", action="store_true", help="skip the per-shape GEMV / GEMM legs")
     ap.add_argument("--no-batched", action="store_true", help="skip the batched-decode leg of the extra figures")
+    ap.add_argument("--layered", nargs="*", choices=sorted(LAYERED), metavar="SIZE",
+                    help="instead of the headline workload: prefill and decode throughput of layered decoders of these sizes "
+                         "(default: all) beside the LLaMA of equal width, as one JSON line")
+    ap.add_argument("--family", choices=("rirulix", "llama"), help="with --layered: this family only (for profiles)")
     ap.add_argument("--copy-calibration", action="store_true",
                     help="also run one 256 MiB device-to-device copy: a copy kernel of known size, against which "
                          "rocprofv3 FETCH_SIZE / WRITE_SIZE readings of the other kernels are scaled")
@@ -323,6 +413,13 @@ def main():
     P = load_package()
     B = P.binding
     B.init(0)
+    if args.layered is not None:
+        families = (args.family,) if args.family else ("rirulix", "llama")
+        sizes = args.layered or sorted(LAYERED)
+        print(json.dumps({"metric": "layered decoders: prefill and decode throughput", "data": "synthetic", "n_gpus": 1,
+                          "steps": args.steps, "warmup": args.warmup,
+                          "sizes": {n: layered_leg(P, n, args.steps, args.warmup, families=families) for n in sizes}}))
+        return
     cfg = WORKLOADS[args.workload]
     model, ctx, dec = decode_leg(P, cfg, args.steps, args.warmup)
     k_us, k_bytes = ffn_up_kernel_leg(P, cfg, model, ctx, 4 * cfg["n_layers"])

@@ -339,8 +339,8 @@ int lcu_linear_gated(void* out_dev, int ldo, const void* lhs_dev, const void* w_
  * tiles of at most tile_rows rows of one expert are listed.  lcu_experts_up: gated unit of
  * row_weight[r] * h[row_token[r]] through expert e's matrix (w_dev + e * expert_stride bytes);
  * lcu_experts_down: the rows' second product, fp32.  Arrays of the plan are device memory: row_* and
- * inverse n * top entries, tile_* max_tiles, expert_end n_experts, n_tiles one.  tile_rows is 64 or 128
- * (bfloat16), 32 (fp32). */
+ * inverse n * top entries, tile_* max_tiles, expert_end n_experts, n_tiles one.  tile_rows is 64, 128
+ * or 256 (bfloat16), 32 (fp32). */
 typedef struct lcu_expert_plan {
   void* row_token_dev;
   void* row_weight_dev;
@@ -363,7 +363,7 @@ int lcu_experts_down(void* out_f32_dev, int ldo, const void* lhs_dev, const void
                      const lcu_expert_plan* plan, int dtype, int n_rows, int K, int N, void* stream);
 
 /* Row kernels; a row is `width` of ld elements, its RMS norm taken over `groups` equal consecutive parts.
- * lcu_embed_pos_norm: x = norm(table[id] + pos_table[*start + row]) under w_embed, h = norm(x) under w_next
+ * Norm weights are fp32 vectors of ld entries.  lcu_embed_pos_norm: x = norm(table[id] + pos_table[*start + row]) under w_embed, h = norm(x) under w_next
  * (NULL: none).  lcu_residual_norm: m = the sublayer's fp32 rows, or per token the sum of its expert rows
  * (inverse_dev, top) and shared_gate[row] times the shared expert's row; x += norm(m) under w_after; h =
  * norm(x) under w_next.  lcu_group_norm: h[i] = norm(x[row_index[i]]). */
@@ -375,8 +375,9 @@ int lcu_residual_norm(void* x_dev, void* h_dev, const void* out_f32_dev, const v
                       const void* w_next_dev, int dtype, int rows, int width, int ld, int groups, float eps, void* stream);
 int lcu_group_norm(void* h_dev, const void* x_f32_dev, const void* row_index_dev, const void* w_dev, int dtype, int rows,
                    int width, int ld, int groups, float eps, void* stream);
-/* index = first maximum of n fp32 logits; probs = fp16(softmax(logits / temp)) */
-int lcu_softmax_argmax_f32(void* probs_f16_dev, void* out_index_dev, const void* logits_dev, int n, float temp, void* stream);
+/* index = first maximum of n fp32 values; probs = fp16(softmax(logits / temp)) of one row of n */
+int lcu_argmax_f32(void* out_index_dev, const void* values_dev, int n, void* stream);
+int lcu_softmax_f32(void* probs_f16_dev, const void* logits_dev, int n, float temp, void* stream);
 
 /* Gated linear recurrence.  Channels lie block by block, each block padded to a multiple of 32.
  * lcu_conv_causal: u[t] = bias + sum over taps of w[k] z[t - (taps - 1) + k] per channel (w fp32
@@ -408,14 +409,16 @@ int lcu_kv_store(void* k_cache_dev, void* v_cache_dev, const void* qkv_dev, int 
                  void* stream);
 int lcu_attention_windowed(void* out_dev, int ldo, const void* q_dev, int ldq, const void* k_cache_dev, const void* v_cache_dev,
                            int start, const lcu_window_params* window, int dtype, int n, void* stream);
-/* one new token at position *pos_dev (bfloat16), the visible keys spread over the chip; arrived_dev: kv_heads
- * uint32, zero before the first call (and left zero).  Uses the stream's workspace. */
+/* one new token at position *pos_dev (bfloat16), the visible keys spread over the chip; arrived_dev:
+ * kv_heads times LCU_ARRIVAL_BYTES, zero before the first call (and left zero).  Uses the stream's workspace. */
+#define LCU_ARRIVAL_BYTES (65 * 128)
 int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* k_cache_dev, const void* v_cache_dev,
                                   const void* pos_dev, int max_positions, const lcu_window_params* window, void* arrived_dev,
                                   void* stream);
 
-/* One new token, bfloat16, fused.  x is normalised already.  arrived_dev: a uint32 that is zero before the
- * call and after it (the workgroup that arrives last goes on with what follows; nobody waits).
+/* One new token, bfloat16, fused.  x is normalised already.  arrived_dev: LCU_ARRIVAL_BYTES of counters that
+ * are zero before the call and after it (the workgroup that arrives last goes on with what follows; nobody
+ * waits).
  *   lcu_decode_linear: fp32 out = w . x + bias
  *   lcu_decode_recurrent_in: rows y (GELU) and x of a recurrent block, the latter through the convolution
  *   lcu_decode_recurrent_step: gates and state of lcu_gated_recurrence for one token

@@ -101,7 +101,8 @@ SIGNATURES = {
     "lcu_embed_pos_norm": (i32, [vp, vp, vp, i32, vp, i32, vp, i32, vp, vp, vp, i32, i32, i32, i32, f32, vp]),
     "lcu_residual_norm": (i32, [vp, vp, vp, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
     "lcu_group_norm": (i32, [vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
-    "lcu_softmax_argmax_f32": (i32, [vp, vp, vp, i32, f32, vp]),
+    "lcu_argmax_f32": (i32, [vp, vp, i32, vp]),
+    "lcu_softmax_f32": (i32, [vp, vp, i32, f32, vp]),
     "lcu_conv_causal": (i32, [vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
     "lcu_gated_recurrence_scratch": (sz, [i32, i32]),
     "lcu_gated_recurrence": (i32, [vp, vp, vp, i32, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp]),

@@ -1,6 +1,7 @@
 // Mixture of experts: router (scores, choice of the largest, gate of the shared expert) and the
 // plan that sorts the tokens' choices by expert for the grouped products (linear.hip).
 #include "linear.hpp"
+#include "rownorm.hpp"
 
 using namespace lcu;
 
@@ -65,33 +66,88 @@ __global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, f
   choose(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
 }
 
-// One new token: a wavefront per row of w; the workgroup that arrives last (its counter goes back to zero)
-// chooses.
+// The same for bfloat16 operands on the matrix cores: one workgroup takes 16 tokens and all rows of w, its
+// wavefronts a quarter of K each, four tiles of 16 rows of w at a time; the quarters are added in LDS in
+// wavefront order, and every wavefront chooses for four of the tokens.
+constexpr int ROUTER_TOKENS = 16;
+__global__ __launch_bounds__(256) void router_tile_kernel(int* __restrict__ expert, float* __restrict__ weight,
+                                                          float* __restrict__ shared_gate, const bf16_t* __restrict__ h,
+                                                          const bf16_t* __restrict__ w, int n, int n_experts, int top, int K) {
+  extern __shared__ float zs[];  // [ROUTER_TOKENS][ldz]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t0 = blockIdx.x * ROUTER_TOKENS;
+  const int n_rows = n_experts + (shared_gate ? 1 : 0), ldz = (n_rows + 15) / 16 * 16 + 1;
+  const int col = lane & 15, quad = lane >> 4;
+  const int steps = K / 32, s0 = wave * steps / 4, s1 = (wave + 1) * steps / 4;
+  const bf16_t* a = h + (size_t)min(t0 + col, n - 1) * K + quad * 8;
+  for (int e0 = 0; e0 < n_rows; e0 += 64) {
+    float4_t acc[4];
+    const bf16_t* b[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      acc[j] = (float4_t)(0.0f);
+      b[j] = w + (size_t)min(e0 + j * 16 + col, n_rows - 1) * K + quad * 8;
+    }
+    const int tiles = min(4, (n_rows - e0 + 15) / 16);
+#pragma unroll 4
+    for (int s = s0; s < s1; ++s) {
+      const bf16x8_t fa = *reinterpret_cast<const bf16x8_t*>(a + s * 32);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if (j < tiles) {
+          const bf16x8_t fb = *reinterpret_cast<const bf16x8_t*>(b[j] + s * 32);
+          acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, fb, acc[j], 0, 0, 0);
+        }
+      }
+    }
+    for (int turn = 0; turn < 4; ++turn) {
+      if (wave == turn) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          if (j < tiles) {
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+              float* z = zs + (quad * 4 + v) * ldz + e0 + j * 16 + col;
+              *z = turn == 0 ? acc[j][v] : *z + acc[j][v];
+            }
+          }
+        }
+      }
+      __syncthreads();
+    }
+  }
+  for (int k = 0; k < ROUTER_TOKENS / 4; ++k) {
+    const int t = t0 + wave * (ROUTER_TOKENS / 4) + k;
+    if (t >= n) continue;
+    float* z = zs + (t - t0) * ldz;
+    if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
+    choose(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
+  }
+}
+
+// One new token: a workgroup per row of w; the one that arrives last chooses.
 __global__ __launch_bounds__(256) void router_step_kernel(int* __restrict__ expert, float* __restrict__ weight,
                                                           float* __restrict__ shared_gate, const bf16_t* __restrict__ h,
                                                           const bf16_t* __restrict__ w, int n_experts, int top, int K,
                                                           float* __restrict__ logits, uint32_t* __restrict__ arrived) {
   __shared__ float z[MAX_EXPERTS + 1];
+  __shared__ float part[4];
   __shared__ bool last;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int n_rows = n_experts + (shared_gate ? 1 : 0), e = blockIdx.x * 4 + wave;
-  if (e < n_rows) {
-    const bf16_t* we = w + (size_t)e * K;
-    float s = 0.0f;
-#pragma unroll 8
-    for (int k = lane * 8; k < K; k += WAVE * 8) {
-      const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(h + k), wv = *reinterpret_cast<const bf16x8_t*>(we + k);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n_rows = gridDim.x;
+  const bf16_t* we = w + (size_t)blockIdx.x * K;
+  float s = 0.0f;
+#pragma unroll 4
+  for (int k = tid * 8; k < K; k += 256 * 8) {
+    const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(h + k), wv = *reinterpret_cast<const bf16x8_t*>(we + k);
 #pragma unroll
-      for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
-    }
-    s = wave_sum(s);
-    if (lane == 0) __hip_atomic_store(logits + e, s, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
   }
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // every wavefront's logit is out before the barrier
+  s = wave_sum(s);
+  if (lane == 0) part[wave] = s;
   __syncthreads();
   if (tid == 0) {
-    last = __hip_atomic_fetch_add(arrived, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == gridDim.x - 1;
-    if (last) __hip_atomic_store(arrived, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    __hip_atomic_store(logits + blockIdx.x, (part[0] + part[1]) + (part[2] + part[3]), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the logit is out before the count goes up
+    last = arrives_last(arrived, blockIdx.x, gridDim.x);
   }
   __syncthreads();
   if (!last) return;
@@ -149,7 +205,7 @@ extern "C" {
 int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const void* h_dev, const void* w_dev, int n_experts,
                int top, int dtype, int n, int K, void* stream) {
   LCU_REQUIRE(expert_dev && weight_dev && h_dev && w_dev, "lcu_router: null pointer");
-  LCU_REQUIRE(n_experts > 0 && n_experts <= MAX_EXPERTS && top > 0 && top <= n_experts && n >= 0 && K > 0,
+  LCU_REQUIRE(n_experts > 0 && n_experts <= MAX_EXPERTS && top > 0 && top <= n_experts && n >= 0 && K > 0 && K % 64 == 0,
               "lcu_router: experts %d (at most %d), top %d", n_experts, MAX_EXPERTS, top);
   LCU_REQUIRE(dtype == LCU_BF16 || dtype == LCU_F32, "lcu_router: element type %d", dtype);
   if (n == 0) return LCU_OK;
@@ -158,8 +214,9 @@ int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const 
     router_kernel<float><<<n, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const float*)h_dev,
                                             (const float*)w_dev, n_experts, top, K);
   } else {
-    router_kernel<bf16_t><<<n, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev,
-                                             (const bf16_t*)w_dev, n_experts, top, K);
+    const size_t lds = (size_t)ROUTER_TOKENS * ((n_experts + 1 + 15) / 16 * 16 + 1) * sizeof(float);
+    router_tile_kernel<<<(n + ROUTER_TOKENS - 1) / ROUTER_TOKENS, 256, lds, st>>>(
+        (int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev, (const bf16_t*)w_dev, n, n_experts, top, K);
   }
   LCU_LAUNCH_CHECK();
   return LCU_OK;
@@ -173,7 +230,7 @@ int lcu_decode_router(void* expert_dev, void* weight_dev, void* shared_gate_dev,
   hipStream_t st = as_stream(stream);
   const workspace_t ws = workspace_for(st);
   if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_decode_router: lcu_init has not run on this device");
-  router_step_kernel<<<(n_experts + 1 + 3) / 4, 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev,
+  router_step_kernel<<<n_experts + (shared_gate_dev ? 1 : 0), 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev,
                                                               (const bf16_t*)h_dev, (const bf16_t*)w_dev, n_experts, top, K,
                                                               (float*)ws.ptr, (uint32_t*)arrived_dev);
   LCU_LAUNCH_CHECK();

@@ -1341,15 +1341,16 @@ template <bool GATED>
 int gemm_bf16(linear_epilogue<false, GATED> const& ep, const void* A, const void* W, int M, int K, int N, hipStream_t st) {
   const auto tm = [&](int bm) { return (M + bm - 1) / bm; };
   const auto tn = [&](int bn) { return (long)((N + bn - 1) / bn); };
+  if (M <= 64) return launch_bf16<64, 64, 2, GATED ? 1 : 2, 1, 3>(ep, A, W, tm(64), M, K, N, st);
   if (tm(256) * tn(128) >= 160) return launch_bf16<256, 128, 4, 2, 1, 3>(ep, A, W, tm(256), M, K, N, st);
   if (tm(128) * tn(128) >= 256) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, tm(128), M, K, N, st);
   if (tm(128) * tn(128) >= 160) return launch_bf16<128, 128, 4, 2, 1, 3>(ep, A, W, tm(128), M, K, N, st);
   if constexpr (GATED) {
-    if (M > 64 && tm(128) * tn(64) > 128) return launch_bf16<128, 64, 4, 1, 1, 3>(ep, A, W, tm(128), M, K, N, st);
+    if (tm(128) * tn(64) > 128) return launch_bf16<128, 64, 4, 1, 1, 3>(ep, A, W, tm(128), M, K, N, st);
     return launch_bf16<64, 64, 2, 1, 1, 3>(ep, A, W, tm(64), M, K, N, st);
   } else {
     if (tm(128) * tn(64) > 256) return launch_bf16<128, 64, 2, 2, 1, 3>(ep, A, W, tm(128), M, K, N, st);
-    if (M > 64 && K % 128 == 0 && tm(128) * tn(64) > 128) {
+    if (K % 128 == 0 && tm(128) * tn(64) > 128) {
       return launch_bf16<128, 64, 2, 2, 2, 3>(ep, A, W, tm(128), M, K, N, st);
     }
     return launch_bf16<64, 64, 2, 2, 1, 3>(ep, A, W, tm(64), M, K, N, st);
@@ -1363,7 +1364,8 @@ template int gemm_bf16<true>(linear_epilogue<false, true> const&, const void*, c
 template <bool GATED>
 int gemm_bf16_grouped(linear_epilogue<true, GATED> const& ep, const void* A, const void* W, int max_tiles, int K, int N,
                       hipStream_t st) {
-  if (ep.tile_rows == 128) return launch_bf16<128, 128, 2, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
+  if (ep.tile_rows == 256) return launch_bf16<256, 128, 4, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
+  if (ep.tile_rows == 128) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, max_tiles, 0, K, N, st);
   return launch_bf16<64, 128, 2, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
 }
 template int gemm_bf16_grouped<false>(linear_epilogue<true, false> const&, const void*, const void*, int, int, int, hipStream_t);

@@ -23,11 +23,11 @@
 // the instruction aligns and cuts its three addends in a way of its own, which the oracle's
 // kernel-order flavour restates from measured samples): the dequantisation arithmetic, not HBM,
 // is what bounds this kernel on large matrices.
+#include <type_traits>
+
 #include "common.hpp"
 #include "linear.hpp"
 #include "rownorm.hpp"
-
-#include <type_traits>
 
 using namespace lcu;
 
@@ -866,7 +866,7 @@ __global__ __launch_bounds__(GEMV_THREADS) void decode_experts_up_kernel(const b
 // ---- a projection and what follows it: x += norm(projection), h = norm(x) ---------------------------
 // Workgroups compute rows of one or several products (slots: one for a mixer's output; the chosen experts
 // and the shared one for a feed-forward) and store them as fp32 at device scope.  The workgroup that arrives
-// last -- a counter says which, and is set back to zero by it -- adds the slots, normalises the sum, adds it to
+// last (arrives_last) adds the slots, normalises the sum, adds it to
 // the residual row, and normalises that for the next sublayer.  Nobody waits for anybody.
 struct projection_slots {
   const bf16_t* W;
@@ -898,9 +898,10 @@ struct store_part_row {
   }
 };
 
-template <int R, int U>
+template <int R, int U, int NV>
 __global__ __launch_bounds__(GEMV_THREADS) void decode_project_kernel(projection_slots p, residual_step r) {
-  extern __shared__ __attribute__((aligned(16))) float row[];  // rs.width floats (rounded up to 4), then the reduction scratch
+  static_assert(GEMV_THREADS == ROW_THREADS, "the last workgroup normalises the row");
+  extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float part[GEMV_WAVES * R];
   __shared__ bool last;
   const int per_slot = (r.rs.width + R - 1) / R;
@@ -918,47 +919,48 @@ __global__ __launch_bounds__(GEMV_THREADS) void decode_project_kernel(projection
   if (threadIdx.x == 0) {
     // this thread stored the workgroup's rows, write-through; they are complete before the count goes up
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    last = __hip_atomic_fetch_add(r.arrived, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == gridDim.x - 1;
-    if (last) __hip_atomic_store(r.arrived, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    last = arrives_last(r.arrived, blockIdx.x, gridDim.x);
   }
   __syncthreads();
   if (!last) return;
-  const int W = r.rs.width, tid = threadIdx.x, total = p.slots + (p.shared_W ? 1 : 0);
-  // the slots' rows at device scope, 16 bytes per request (rows are padded to a multiple of 64 floats)
-  for (int c0 = 0; c0 < W; c0 += 4 * GEMV_THREADS * 4) {
-    float4_t sum[4];
-    int at[4];
+  const int total = p.slots + (p.shared_W ? 1 : 0);
+  row_t<NV> m, t;
+  load_row(t, r.w_after, r.rs);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      sum[j] = (float4_t)(0.0f);
-      at[j] = c0 + (j * GEMV_THREADS + tid) * 4;
-    }
-    for (int s = 0; s < total; ++s) {
-      const float* src = p.part + (size_t)s * r.rs.ld;
+  for (int j = 0; j < NV; ++j) m.v[j] = (float4_t)(0.0f);
+  for (int s = 0; s < total; ++s) {
+    // device scope, 16 bytes per request, four requests per statement
+    const float* src = p.part + (size_t)s * r.rs.ld;
+    const float f = s == p.slots ? *p.shared_gate : 1.0f;
+#pragma unroll
+    for (int j = 0; j < NV; j += 4) {
       uint4_t v[4];
-      const auto word = [&](int j) { return reinterpret_cast<const uint64_t*>(src + (at[j] < r.rs.ld ? at[j] : 0)); };
+      const auto word = [&](int k) {
+        const int c = m.column(j + k);
+        return reinterpret_cast<const uint64_t*>(src + (j + k < NV && c < r.rs.width ? c : 0));
+      };
       load_word_pairs_device_scope(v, word(0), word(1), word(2), word(3));
-      const float f = s == p.slots ? *p.shared_gate : 1.0f;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) sum[j] += f * __builtin_bit_cast(float4_t, v[j]);
-    }
+      for (int k = 0; k < 4; ++k) {
+        if (j + k < NV) {
+          const float4_t x = __builtin_bit_cast(float4_t, v[k]);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        if (at[j] + e < W) row[at[j] + e] = sum[j][e];
+          for (int e = 0; e < 4; ++e) {
+            if (m.column(j + k) + e < r.rs.width) m.v[j + k][e] += f * x[e];
+          }
+        }
       }
     }
   }
-  float* scratch = row + W;
-  group_scale(row, r.rs, scratch, r.w_after);
-  for (int c = tid; c < W; c += GEMV_THREADS) {
-    row[c] += r.x[c];
-    r.x[c] = row[c];
-  }
+  scale_row(m, r.rs, lds, t);
+  load_row(t, r.x, r.rs);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) m.v[j] += t.v[j];
+  store_row(r.x, m, r.rs);
   if (r.w_next) {
-    group_scale(row, r.rs, scratch, r.w_next);
-    for (int c = tid; c < W; c += GEMV_THREADS) r.h[c] = (bf16_t)row[c];
+    load_row(t, r.w_next, r.rs);
+    scale_row(m, r.rs, lds, t);
+    store_row(r.h, m, r.rs);
   }
 }
 
@@ -966,11 +968,13 @@ int launch_project(const projection_slots& p, const residual_step& r, hipStream_
   const int n = p.slots + (p.shared_W ? 1 : 0);
   const size_t lds = row_lds_bytes(r.rs);
   const int K = p.shared_W && p.shared_K > p.K ? p.shared_K : p.K;
-  if (K > 2048) {
-    decode_project_kernel<2, 2><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
-  } else {
-    decode_project_kernel<2, 1><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
-  }
+  with_row_pieces(r.rs.ld, [&](auto nv) {
+    if (K > 2048) {
+      decode_project_kernel<2, 2, decltype(nv)::value><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
+    } else {
+      decode_project_kernel<2, 1, decltype(nv)::value><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
+    }
+  });
   LCU_LAUNCH_CHECK();
   return LCU_OK;
 }

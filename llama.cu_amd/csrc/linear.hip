@@ -115,7 +115,7 @@ void set_plan(EP& ep, const lcu_expert_plan* plan, const void* row_index, size_t
 
 bool plan_ok(const lcu_expert_plan* p, int dtype) {
   return p && p->tile_expert_dev && p->tile_row_dev && p->expert_end_dev && p->n_tiles_dev && p->row_token_dev &&
-         p->max_tiles > 0 && (dtype == LCU_F32 ? p->tile_rows == FM : (p->tile_rows == 64 || p->tile_rows == 128));
+         p->max_tiles > 0 && (dtype == LCU_F32 ? p->tile_rows == FM : (p->tile_rows == 64 || p->tile_rows == 128 || p->tile_rows == 256));
 }
 
 }  // namespace

@@ -9,6 +9,7 @@
 // thread per channel runs over the chunks' maps (carry), and then every chunk runs through its own
 // tokens from its incoming state (apply).
 #include "linear.hpp"
+#include "rownorm.hpp"
 
 using namespace lcu;
 
@@ -18,20 +19,32 @@ constexpr int CHUNK = 64;   // tokens per chunk and per gate tile
 constexpr int GATE_N = 32;  // channels per gate tile
 
 // u[t][c] = bias[c] + sum_k w[k][c] z[t - (taps - 1) + k]; inputs before this call come from state
-// [taps - 1][ld], oldest first
+// [taps - 1][ld], oldest first.  A thread takes four channels of CONV_T tokens.
+constexpr int CONV_T = 8;
 template <class T>
 __global__ __launch_bounds__(256) void conv_causal_kernel(T* __restrict__ u, const T* __restrict__ z, int ldz,
                                                           const float* __restrict__ w, const float* __restrict__ bias,
-                                                          const T* __restrict__ state, int taps, int channels, int ld) {
-  const int c = blockIdx.x * 256 + threadIdx.x, t = blockIdx.y;
+                                                          const T* __restrict__ state, int taps, int n, int channels, int ld) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 4, t0 = blockIdx.y * CONV_T;
   if (c >= channels) return;
-  float acc = bias[c];
+  float4_t acc[CONV_T];
+  const float4_t b = load4(bias + c);
+#pragma unroll
+  for (int e = 0; e < CONV_T; ++e) acc[e] = b;
   for (int k = 0; k < taps; ++k) {
-    const int s = t - (taps - 1) + k;
-    const float v = s >= 0 ? to_f32(z[(size_t)s * ldz + c]) : to_f32(state[(size_t)(s + taps - 1) * ld + c]);
-    acc = fmaf(w[(size_t)k * ld + c], v, acc);
+    const float4_t wk = load4(w + (size_t)k * ld + c);
+#pragma unroll
+    for (int e = 0; e < CONV_T; ++e) {
+      const int s = min(t0 + e, n - 1) - (taps - 1) + k;
+      const float4_t v = load4(s >= 0 ? z + (size_t)s * ldz + c : state + (size_t)(s + taps - 1) * ld + c);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[e][i] = fmaf(wk[i], v[i], acc[e][i]);
+    }
   }
-  u[(size_t)t * ld + c] = (T)acc;
+#pragma unroll
+  for (int e = 0; e < CONV_T; ++e) {
+    if (t0 + e < n) store4(u + (size_t)(t0 + e) * ld + c, acc[e]);
+  }
 }
 
 // the last taps - 1 inputs become the state; ascending order, so a short call shifts in place
@@ -45,6 +58,15 @@ __global__ __launch_bounds__(256) void conv_state_kernel(T* __restrict__ state, 
     state[(size_t)k * ld + c] = s >= 0 ? z[(size_t)s * ldz + c] : state[(size_t)(k + n) * ld + c];
   }
 }
+
+// sqrt(1 - a^2) for a = exp(log_a), log_a <= 0, without cancellation: 1 - e^x by its series near 0
+__device__ __forceinline__ float drive_factor(float log_a, float a) {
+  const float x = 2.0f * log_a;
+  const float series = -x * (1.0f + x * (1.0f / 2) * (1.0f + x * (1.0f / 3) * (1.0f + x * (1.0f / 4) * (1.0f + x * (1.0f / 5) * (1.0f + x * (1.0f / 6))))));
+  return __builtin_amdgcn_sqrtf(x > -0.25f ? series : 1.0f - a * a);
+}
+// fp32 gates of the bfloat16 element type: the machine's exponential, reciprocal and square root (1 ulp each)
+__device__ __forceinline__ float sigmoid_fast(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
 
 struct gate_args {
   const void* wr;       // [blocks][bw][bw], rows and blocks padded
@@ -107,10 +129,16 @@ __global__ __launch_bounds__(256) void gates_kernel(const T* __restrict__ u, gat
   for (int e = 0; e < 8; ++e) {
     const int lt = s8 * 8 + e, t = t0 + lt;
     if (t < p.n) {
-      const float r = sigmoid_f32(gate[0][lt][ch] + br), i = sigmoid_f32(gate[1][lt][ch] + bi);
-      const float log_a = decay * r;
-      const float a = expf(log_a);
-      const float b = sqrtf(-expm1f(2.0f * log_a)) * i * to_f32(u[(size_t)t * p.ld + c]);
+      float a, b;
+      if constexpr (sizeof(T) == 2) {
+        const float log_a = decay * sigmoid_fast(gate[0][lt][ch] + br);
+        a = __expf(log_a);
+        b = drive_factor(log_a, a) * sigmoid_fast(gate[1][lt][ch] + bi) * to_f32(u[(size_t)t * p.ld + c]);
+      } else {
+        const float log_a = decay * sigmoid_f32(gate[0][lt][ch] + br);
+        a = expf(log_a);
+        b = sqrtf(-expm1f(2.0f * log_a)) * sigmoid_f32(gate[1][lt][ch] + bi) * to_f32(u[(size_t)t * p.ld + c]);
+      }
       p.a[(size_t)t * p.ld + c] = a;
       p.b[(size_t)t * p.ld + c] = b;
       A = a * A;
@@ -234,21 +262,21 @@ int lcu_conv_causal(void* u_dev, const void* z_dev, int ldz, const void* w_dev, 
   LCU_REQUIRE(u_dev && z_dev && w_dev && bias_dev && (state_dev || taps == 1), "lcu_conv_causal: null pointer");
   const int rc = check_channels("lcu_conv_causal", dtype, n, channels, ld);
   if (rc) return rc;
-  LCU_REQUIRE(taps >= 1 && ldz >= channels, "lcu_conv_causal: taps %d, input stride %d", taps, ldz);
+  LCU_REQUIRE(taps >= 1 && ldz >= channels && ldz % 4 == 0 && channels % 4 == 0, "lcu_conv_causal: taps %d, input stride %d", taps, ldz);
   if (n == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
-  const dim3 grid((channels + 255) / 256, n);
+  const dim3 grid((channels / 4 + 255) / 256, (n + CONV_T - 1) / CONV_T), columns((channels + 255) / 256);
   if (dtype == LCU_F32) {
     conv_causal_kernel<float><<<grid, 256, 0, st>>>((float*)u_dev, (const float*)z_dev, ldz, (const float*)w_dev,
-                                                    (const float*)bias_dev, (const float*)state_dev, taps, channels, ld);
+                                                    (const float*)bias_dev, (const float*)state_dev, taps, n, channels, ld);
     if (taps > 1) {
-      conv_state_kernel<float><<<grid.x, 256, 0, st>>>((float*)state_dev, (const float*)z_dev, ldz, n, taps, channels, ld);
+      conv_state_kernel<float><<<columns, 256, 0, st>>>((float*)state_dev, (const float*)z_dev, ldz, n, taps, channels, ld);
     }
   } else {
     conv_causal_kernel<bf16_t><<<grid, 256, 0, st>>>((bf16_t*)u_dev, (const bf16_t*)z_dev, ldz, (const float*)w_dev,
-                                                     (const float*)bias_dev, (const bf16_t*)state_dev, taps, channels, ld);
+                                                     (const float*)bias_dev, (const bf16_t*)state_dev, taps, n, channels, ld);
     if (taps > 1) {
-      conv_state_kernel<bf16_t><<<grid.x, 256, 0, st>>>((bf16_t*)state_dev, (const bf16_t*)z_dev, ldz, n, taps, channels, ld);
+      conv_state_kernel<bf16_t><<<columns, 256, 0, st>>>((bf16_t*)state_dev, (const bf16_t*)z_dev, ldz, n, taps, channels, ld);
     }
   }
   LCU_LAUNCH_CHECK();

@@ -1,4 +1,4 @@
-// Grouped RMS norm of one row held in LDS by one workgroup.
+// Grouped RMS norm of one row by one 256-thread workgroup.
 #pragma once
 #include "common.hpp"
 
@@ -8,6 +8,7 @@ constexpr int ROW_THREADS = 256;
 constexpr int ROW_WAVES = ROW_THREADS / WAVE;
 constexpr int ROW_MAX_WIDTH = 12288;
 constexpr int ROW_MAX_GROUPS = 2048;
+constexpr int ROW_PIECE = WAVE * 4;  // columns a wavefront holds per register piece
 
 struct row_shape {
   int width, ld, groups;  // elements of a row, row stride in memory, equal consecutive parts
@@ -23,44 +24,148 @@ struct sublayer_rows {
   const float* shared_gate;
 };
 
-inline size_t row_lds_bytes(const row_shape& rs) {
-  return ((size_t)rs.width + (rs.groups > ROW_WAVES ? rs.groups : ROW_WAVES)) * sizeof(float);
+// A row spread over the workgroup's registers: piece j of thread t holds the four columns from
+// (t + 256 j) * 4.  Columns at or beyond the width hold zeros.
+template <int NV>
+struct row_t {
+  float4_t v[NV];
+  static __device__ __forceinline__ int column(int j) { return (int)(threadIdx.x + ROW_THREADS * j) * 4; }
+};
+
+__device__ __forceinline__ float4_t load4(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
+__device__ __forceinline__ float4_t load4(const bf16_t* p) {
+  typedef uint32_t uint2_t __attribute__((ext_vector_type(2)));
+  const uint2_t u = *reinterpret_cast<const uint2_t*>(p);
+  float4_t r;
+  r[0] = __builtin_bit_cast(float, u[0] << 16);
+  r[1] = __builtin_bit_cast(float, u[0] & 0xffff0000u);
+  r[2] = __builtin_bit_cast(float, u[1] << 16);
+  r[3] = __builtin_bit_cast(float, u[1] & 0xffff0000u);
+  return r;
+}
+__device__ __forceinline__ void store4(float* p, float4_t v) { *reinterpret_cast<float4_t*>(p) = v; }
+__device__ __forceinline__ void store4(bf16_t* p, float4_t v) {
+  typedef bf16_t bf16x4_t __attribute__((ext_vector_type(4)));
+  *reinterpret_cast<bf16x4_t*>(p) = __builtin_convertvector(v, bf16x4_t);
 }
 
-// row[c] <- row[c] / sqrt(mean of its part's squares + eps) * w[c].  Starts and ends with every thread's
-// writes to row visible to the workgroup.  A part is summed by one wavefront, or by several when there are
-// fewer parts than wavefronts.
-__device__ __forceinline__ void group_scale(float* row, const row_shape& rs, float* scratch, const float* __restrict__ w) {
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int part = rs.width / rs.groups;
+// Rows have a padded stride (a multiple of 64 elements), so whole pieces up to ld may be read and written;
+// vectors of the width (norm weights) are padded by their owners to ld too.
+template <int NV, class T>
+__device__ __forceinline__ void load_row(row_t<NV>& r, const T* p, const row_shape& rs) {
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = r.column(j);
+    r.v[j] = c < rs.ld ? load4(p + c) : (float4_t)(0.0f);
+  }
+}
+template <int NV, class T>
+__device__ __forceinline__ void store_row(T* p, const row_t<NV>& r, const row_shape& rs) {
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = r.column(j);
+    if (c < rs.ld) store4(p + c, r.v[j]);
+  }
+}
+
+// LDS a workgroup needs for scale_row
+inline size_t row_lds_bytes(const row_shape& rs) {
+  const size_t quads = (size_t)rs.ld / 4;                        // general form: a partial sum per four columns ...
+  const size_t pieces = (rs.ld + ROW_PIECE - 1) / ROW_PIECE;     // ... or one per piece of a wavefront
+  const bool whole = rs.width % rs.groups == 0 && (rs.width / rs.groups) % ROW_PIECE == 0;
+  return ((whole ? pieces : quads * 4) + rs.groups) * sizeof(float);
+}
+
+// row <- row / sqrt(mean of its part's squares + eps) * w.  Parts that are whole pieces of a wavefront (256
+// columns) are summed in registers; other sizes go through LDS column by column.  `lds` may be reused right
+// after an earlier call.
+template <int NV>
+__device__ __forceinline__ void scale_row(row_t<NV>& r, const row_shape& rs, float* lds, const row_t<NV>& w) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, part = rs.width / rs.groups;
+  if (part % ROW_PIECE == 0) {
+    float* piece = lds;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const float4_t q = r.v[j] * r.v[j];
+      const float s = wave_sum((q[0] + q[1]) + (q[2] + q[3]));
+      if (lane == 0 && r.column(j) < rs.ld) piece[j * ROW_WAVES + wave] = s;
+    }
+    __syncthreads();
+    const int per = part / ROW_PIECE;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int g = __builtin_amdgcn_readfirstlane((j * ROW_WAVES + wave) / per);
+      if (g < rs.groups) {
+        float total = 0.0f;
+        for (int k = 0; k < per; ++k) total += piece[g * per + k];
+        r.v[j] *= (1.0f / sqrtf(total / (float)part + rs.eps)) * w.v[j];
+      }
+    }
+    __syncthreads();
+    return;
+  }
+  float* sq = lds;                     // [ld] squares
+  float* inv = lds + rs.ld;            // [groups]
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = r.column(j);
+    if (c < rs.ld) store4(sq + c, r.v[j] * r.v[j]);
+  }
   __syncthreads();
-  if (rs.groups >= ROW_WAVES) {
-    for (int g = wave; g < rs.groups; g += ROW_WAVES) {
-      float s = 0.0f;
-      for (int i = lane; i < part; i += WAVE) s = fmaf(row[g * part + i], row[g * part + i], s);
-      s = wave_sum(s);
-      if (lane == 0) scratch[g] = 1.0f / sqrtf(s / (float)part + rs.eps);
-    }
-    __syncthreads();
-    for (int c = threadIdx.x; c < rs.width; c += ROW_THREADS) row[c] = row[c] * scratch[c / part] * w[c];
-  } else {
-    const int share = ROW_WAVES / rs.groups;  // wavefronts of a part
+  for (int g = wave; g < rs.groups; g += ROW_WAVES) {
     float s = 0.0f;
-    if (wave < share * rs.groups) {
-      const float* p = row + (wave / share) * part;
-      for (int i = (wave % share) * WAVE + lane; i < part; i += share * WAVE) s = fmaf(p[i], p[i], s);
-    }
+    for (int i = lane; i < part; i += WAVE) s += sq[g * part + i];
     s = wave_sum(s);
-    if (lane == 0) scratch[wave] = s;
-    __syncthreads();
-    for (int c = threadIdx.x; c < rs.width; c += ROW_THREADS) {
-      const int g = c / part;
-      float total = 0.0f;
-      for (int k = 0; k < share; ++k) total += scratch[g * share + k];
-      row[c] = row[c] * (1.0f / sqrtf(total / (float)part + rs.eps)) * w[c];
+    if (lane == 0) inv[g] = 1.0f / sqrtf(s / (float)part + rs.eps);
+  }
+  __syncthreads();
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int c = r.column(j) + e;
+      r.v[j][e] = c < rs.width ? r.v[j][e] * inv[c / part] * w.v[j][e] : 0.0f;
     }
   }
   __syncthreads();
+}
+
+// calls f with the number of pieces per thread that covers the row stride
+template <class F>
+void with_row_pieces(int ld, F&& f) {
+  if (ld <= 1024) {
+    f(std::integral_constant<int, 1>{});
+  } else if (ld <= 2048) {
+    f(std::integral_constant<int, 2>{});
+  } else if (ld <= 4096) {
+    f(std::integral_constant<int, 4>{});
+  } else if (ld <= 8192) {
+    f(std::integral_constant<int, 8>{});
+  } else {
+    f(std::integral_constant<int, 12>{});
+  }
+}
+
+// ---- which workgroup arrives last -------------------------------------------------------------------
+// Counters of a launch whose last workgroup goes on with the others' results: ARRIVAL_LANES first-level
+// counters, 128 bytes apart, and one behind them that counts full ones (thousands of workgroups adding to one
+// word would queue for it).  All are zero before the launch and after it.
+constexpr int ARRIVAL_LANES = 64;
+constexpr int ARRIVAL_STRIDE = 32;  // words
+constexpr int ARRIVAL_WORDS = (ARRIVAL_LANES + 1) * ARRIVAL_STRIDE;
+
+// Called by one thread after the workgroup's device-scope stores are complete.
+__device__ __forceinline__ bool arrives_last(uint32_t* counters, uint32_t block, uint32_t blocks) {
+  const uint32_t lane = block % ARRIVAL_LANES;
+  const uint32_t mine = blocks / ARRIVAL_LANES + (lane < blocks % ARRIVAL_LANES ? 1u : 0u);
+  uint32_t* c = counters + lane * ARRIVAL_STRIDE;
+  if (__hip_atomic_fetch_add(c, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != mine - 1) return false;
+  __hip_atomic_store(c, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  uint32_t* top = counters + ARRIVAL_LANES * ARRIVAL_STRIDE;
+  const uint32_t full = blocks < ARRIVAL_LANES ? blocks : ARRIVAL_LANES;
+  if (__hip_atomic_fetch_add(top, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != full - 1) return false;
+  __hip_atomic_store(top, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  return true;
 }
 
 }  // namespace lcu

@@ -10,6 +10,7 @@
 #include <algorithm>
 
 #include "linear.hpp"
+#include "rownorm.hpp"
 
 using namespace lcu;
 
@@ -253,7 +254,21 @@ int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, 
 // Workgroup (kv head, slice of the visible keys): 16 lanes share a key row and score it for every query
 // head of the group (the row is read once for all of them); then the slice's maximum, sum and weighted
 // values per head go to part[kv head][slice][head][dv + 2], and the last workgroup of a kv head to arrive
-// adds the slices up.  Nobody waits: the last one is known by a counter, which it sets back to zero.
+// adds the slices up (arrives_last).  Nobody waits.
+__device__ __forceinline__ float load_device(const float* p) {
+  return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+}
+// eight loads at device scope in flight together (see load_words_device_scope)
+__device__ __forceinline__ void load8_device(float (&o)[8], const float* const (&p)[8]) {
+  asm volatile(
+      "global_load_dword %0, %8, off sc0 sc1\n\tglobal_load_dword %1, %9, off sc0 sc1\n\t"
+      "global_load_dword %2, %10, off sc0 sc1\n\tglobal_load_dword %3, %11, off sc0 sc1\n\t"
+      "global_load_dword %4, %12, off sc0 sc1\n\tglobal_load_dword %5, %13, off sc0 sc1\n\t"
+      "global_load_dword %6, %14, off sc0 sc1\n\tglobal_load_dword %7, %15, off sc0 sc1\n\ts_waitcnt vmcnt(0)"
+      : "=&v"(o[0]), "=&v"(o[1]), "=&v"(o[2]), "=&v"(o[3]), "=&v"(o[4]), "=&v"(o[5]), "=&v"(o[6]), "=&v"(o[7])
+      : "v"(p[0]), "v"(p[1]), "v"(p[2]), "v"(p[3]), "v"(p[4]), "v"(p[5]), "v"(p[6]), "v"(p[7])
+      : "memory");
+}
 constexpr int DEC_MAX_SLICE = 256;   // keys of a slice
 constexpr int DEC_MAX_GROUP = 16;    // query heads per kv head
 
@@ -345,31 +360,49 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restric
     const float o = (ov[c] + ov[rd + c]) + (ov[2 * rd + c] + ov[3 * rd + c]);
     __hip_atomic_store(pg + (c / p.dv) * (p.dv + 2) + c % p.dv, o, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
-  __threadfence();
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // every wavefront's stores are out before the count goes up
   __syncthreads();
-  if (tid == 0) {
-    const uint32_t before = __hip_atomic_fetch_add(arrived + g, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
-    last = before == (uint32_t)slices - 1;
-    if (last) __hip_atomic_store(arrived + g, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  }
+  if (tid == 0) last = arrives_last(arrived + (size_t)g * ARRIVAL_WORDS, slice, slices);
   __syncthreads();
   if (!last) return;
-  __threadfence();
+  // factor and share of every slice, per head; then the columns
   const float* all = part + (size_t)g * slices * R * (p.dv + 2);
+  float* sm = sc;              // [R][slices]: maxima, then factors (a slice is at most DEC_MAX_SLICE keys, and so are the slices)
+  float* sl = dec_lds;         // [R]: sums (q is done with)
+  for (int c = tid; c < R * slices; c += 256) {
+    const int r = c / slices, s = c % slices;
+    sm[r * DEC_MAX_SLICE + s] = load_device(all + ((size_t)s * R + r) * (p.dv + 2) + p.dv);
+  }
+  __syncthreads();
+  for (int r = wave; r < R; r += 4) {
+    float m = -1e30f;
+    for (int s = lane; s < slices; s += WAVE) m = fmaxf(m, sm[r * DEC_MAX_SLICE + s]);
+    m = wave_max_dpp(m);
+    float l = 0.0f;
+    for (int s = lane; s < slices; s += WAVE) {
+      const float f = expf(sm[r * DEC_MAX_SLICE + s] - m);
+      l += f * load_device(all + ((size_t)s * R + r) * (p.dv + 2) + p.dv + 1);
+      sm[r * DEC_MAX_SLICE + s] = f;
+    }
+    l = wave_sum(l);
+    if (lane == 0) sl[r] = l;
+  }
+  __syncthreads();
   for (int c = tid; c < R * p.dv; c += 256) {
     const int r = c / p.dv, e = c % p.dv;
-    float m = -1e30f, l = 0.0f, o = 0.0f;
-    for (int s = 0; s < slices; ++s) {
-      const float* ps = all + ((size_t)s * R + r) * (p.dv + 2);
-      const float ms = __hip_atomic_load(ps + p.dv, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      const float ls = __hip_atomic_load(ps + p.dv + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      const float os = __hip_atomic_load(ps + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      const float mn = fmaxf(m, ms), was = expf(m - mn), now = expf(ms - mn);
-      l = l * was + ls * now;
-      o = o * was + os * now;
-      m = mn;
+    float o = 0.0f;
+    for (int s0 = 0; s0 < slices; s0 += 8) {
+      float v[8];
+      const float* at[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) at[k] = all + ((size_t)min(s0 + k, slices - 1) * R + r) * (p.dv + 2) + e;
+      load8_device(v, at);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        if (s0 + k < slices) o = fmaf(sm[r * DEC_MAX_SLICE + s0 + k], v[k], o);
+      }
     }
-    out[(size_t)(g * R + r) * p.dv + e] = (bf16_t)(o / l);
+    out[(size_t)(g * R + r) * p.dv + e] = (bf16_t)(o / sl[r]);
   }
 }
 
@@ -471,7 +504,7 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
   slices = std::max(slices, (most + DEC_MAX_SLICE - 1) / DEC_MAX_SLICE);
   const size_t need = (size_t)window->heads * slices * (window->dv + 2) * sizeof(float);
   const size_t lds = ((size_t)R * (window->dk + DEC_MAX_SLICE + 4 * window->dv)) * sizeof(float);
-  LCU_REQUIRE(need <= ws.bytes && slices <= 65535, "lcu_attention_windowed_decode: %d slices do not fit the workspace", slices);
+  LCU_REQUIRE(need <= ws.bytes && slices <= DEC_MAX_SLICE, "lcu_attention_windowed_decode: %d slices do not fit the workspace", slices);
   LCU_REQUIRE(lds <= 128 * 1024, "lcu_attention_windowed_decode: %d heads of %d / %d per kv head", R, window->dk, window->dv);
   static bool raised[16] = {};
   int dev = 0;

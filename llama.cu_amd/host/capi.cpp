@@ -214,7 +214,7 @@ int lcu_context_read_logits(lcu_context* c, uint16_t* out) {
 
 int lcu_context_read_probs(lcu_context* c, uint16_t* out) {
   if (auto* ly = c->layered()) {
-    return lcu_d2h(out, ly->probs().data(), (size_t)c->n_vocab * 2, ly->stream());
+    return ly->read_probs(out);
   }
   auto* ci = c->impl();
   return ci ? lcu_d2h(out, ci->probs().data(), ci->probs().size(), ci->stream()) : -1;

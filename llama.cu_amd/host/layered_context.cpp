@@ -73,7 +73,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   for (layer_params const& p : m.shape.layers) {
     if (p.mixer == mixer_type::attention && p.attention.heads / p.attention.kv_heads > 16) fused_step_ = false;
   }
-  t_arrived_ = zeroed(counters * 4);
+  t_arrived_ = zeroed(counters * LCU_ARRIVAL_BYTES);
   t_step_ = zeroed((1 + R) * 4);
   t_probs_ = zeroed((size_t)m.shape.vocab * 2);
   t_index_ = zeroed(4);
@@ -258,7 +258,7 @@ void layered_context_impl::enqueue_one() {
     }
   }
   LCU_CHECK(lcu_decode_linear(t_logits_.data(), t_h_.data(), m.head.data(), nullptr, m.ld, p.vocab, stream_));
-  LCU_CHECK(lcu_softmax_argmax_f32(t_probs_.data(), t_index_.data(), t_logits_.data(), p.vocab, temperature_, stream_));
+  LCU_CHECK(lcu_argmax_f32(t_index_.data(), t_logits_.data(), p.vocab, stream_));
 }
 
 // The first step runs eagerly (and loads the kernels), the second is captured, every later one replays it.
@@ -300,6 +300,10 @@ void layered_context_impl::enqueue_head(int n_rows) {
   layered_params const& p = m.shape;
   LCU_CHECK(lcu_group_norm(t_head_in_.data(), t_x_.data(), t_want_.data(), m.final_norm.data(), m.dtype, n_rows, p.width, m.ld,
                            p.norm_groups, p.norm_eps, stream_));
+  if (n_rows == 1 && m.dtype == LCU_BF16) {
+    LCU_CHECK(lcu_decode_linear(t_logits_.data(), t_head_in_.data(), m.head.data(), nullptr, m.ld, p.vocab, stream_));
+    return;
+  }
   LCU_CHECK(lcu_linear(t_logits_.data(), 1, p.vocab, t_head_in_.data(), m.head.data(), nullptr, 0, m.dtype, n_rows, m.ld, p.vocab,
                        stream_));
 }
@@ -346,12 +350,13 @@ int layered_context_impl::forward(const int32_t* tokens, int n, const int32_t* w
       enqueue_rows(count);
       if (!rows.empty()) enqueue_head((int)rows.size());
       if (ends) {
-        const size_t last = (rows.size() - 1) * (size_t)vocab * 4;
-        LCU_CHECK(lcu_softmax_argmax_f32(t_probs_.data(), t_index_.data(), (char*)t_logits_.data() + last, vocab, temperature_, stream_));
+        LCU_CHECK(lcu_argmax_f32(t_index_.data(), (float*)t_logits_.data() + (rows.size() - 1) * (size_t)vocab, vocab, stream_));
       }
     }
     if (ends) {
+      last_logits_row_ = fused ? 0 : rows.size() - 1;
       if (sampling_) {
+        LCU_CHECK(lcu_softmax_f32(t_probs_.data(), last_logits(), vocab, temperature_, stream_));
         uint64_t z = sample_seed_ + ++samples_drawn_ * 0x9E3779B97F4A7C15ull;
         z = (z ^ (z >> 30)) * 0xBF58476D1CE4E5B9ull;
         z = (z ^ (z >> 27)) * 0x94D049BB133111EBull;
@@ -366,6 +371,13 @@ int layered_context_impl::forward(const int32_t* tokens, int n, const int32_t* w
     start_pos_ += count;
   }
   return token;
+}
+
+int layered_context_impl::read_probs(uint16_t* out) {
+  if (t_logits_.size() == 0) return -1;  // no call yet
+  const int vocab = model_->shape.vocab;
+  LCU_CHECK(lcu_softmax_f32(t_probs_.data(), last_logits(), vocab, temperature_, stream_));
+  return lcu_d2h(out, t_probs_.data(), (size_t)vocab * 2, stream_);
 }
 
 short layered_context_impl::next_token(std::vector<short> const& new_tokens) {

@@ -15,7 +15,8 @@ struct layered_context_impl final : public llama_context {
   void greedy() override;
 
   void* stream() const { return stream_; }
-  gpu_buffer& probs() { return t_probs_; }
+  // fp16 softmax(logits / temperature) of the last call's last token
+  int read_probs(uint16_t* out);
   void record_residual(bool on) { recording_ = on; }
   int read_residual(int layer, float* out, int rows) const;
 
@@ -48,6 +49,8 @@ struct layered_context_impl final : public llama_context {
   void* start() const { return t_step_.data(); }
   void* ids() const { return (char*)t_step_.data() + 4; }
   std::vector<int32_t> host_step_, host_want_;
+  size_t last_logits_row_{0};
+  float* last_logits() const { return (float*)t_logits_.data() + last_logits_row_ * model_->shape.vocab; }
   int want_cap_{0};
   lcu_expert_plan plan_{};
   bool fused_step_{true};                          // one-token steps in bfloat16 take enqueue_one

@@ -89,7 +89,7 @@ struct loader {
     return t;
   }
   gpu_buffer vector(std::string const& name, size_t n) {
-    std::vector<float> v(n, 0.0f);
+    std::vector<float> v(round_up(n, 64), 0.0f);  // padded like the rows they scale
     put_vector(v, *get(name, {n}), [](size_t i) { return i; });
     return upload_vector(v);
   }
@@ -335,7 +335,8 @@ bool layered_model_impl::shapes_supported() const {
   };
   const auto linear = [&](size_t rows, size_t cols, size_t ld) { return matrix(rows, cols, ld, 1.0f / sqrtf((float)cols)); };
   const auto vector = [&](size_t n, float mean, float std) {
-    gpu_buffer b(n * 4);
+    gpu_buffer b(round_up(n, 64) * 4);
+    LCU_CHECK(lcu_memset(b.data(), 0, b.size(), nullptr));
     LCU_CHECK(lcu_fill_normal_matrix(b.data(), 1, (int)n, (int)n, LCU_F32, seed, ++stream, mean, std, nullptr));
     return b;
   };
