@@ -364,8 +364,9 @@ int lcu_experts_down(void* out_f32_dev, int ldo, const void* lhs_dev, const void
 
 /* Row kernels; a row is `width` of ld elements, its RMS norm taken over `groups` equal consecutive parts.
  * Norm weights are fp32 vectors of ld entries.  lcu_embed_pos_norm: x = norm(table[id] + pos_table[*start + row]) under w_embed, h = norm(x) under w_next
- * (NULL: none).  lcu_residual_norm: m = the sublayer's fp32 rows, or per token the sum of its expert rows
- * (inverse_dev, top) and shared_gate[row] times the shared expert's row; x += norm(m) under w_after; h =
+ * (NULL: none).  lcu_residual_norm: m = per token the sum of `top` fp32 rows of out (rows
+ * inverse[token * top + k], or token * top + k when inverse is NULL) and shared_gate[row] times the shared
+ * expert's row; x += norm(m) under w_after; h =
  * norm(x) under w_next.  lcu_group_norm: h[i] = norm(x[row_index[i]]). */
 int lcu_embed_pos_norm(void* x_dev, void* h_dev, const void* ids_i32_dev, int n_ids, const void* table_dev, int n_vocab,
                        const void* pos_table_dev, int n_pos, const void* start_dev, const void* w_embed_dev,
@@ -416,18 +417,17 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
                                   const void* pos_dev, int max_positions, const lcu_window_params* window, void* arrived_dev,
                                   void* stream);
 
-/* One new token, bfloat16, fused.  x is normalised already.  arrived_dev: LCU_ARRIVAL_BYTES of counters that
- * are zero before the call and after it (the workgroup that arrives last goes on with what follows; nobody
- * waits).
+/* One new token, bfloat16, fused.  x is normalised already.
  *   lcu_decode_linear: fp32 out = w . x + bias
  *   lcu_decode_recurrent_in: rows y (GELU) and x of a recurrent block, the latter through the convolution
  *   lcu_decode_recurrent_step: gates and state of lcu_gated_recurrence for one token
  *   lcu_decode_kv: rows q | k | v, then lcu_kv_store at position *pos
- *   lcu_decode_router: lcu_router for one token (workspace)
  *   lcu_decode_experts_up: hidden activations of the chosen experts (w at up + choice * up_stride bytes,
  *     packed as for lcu_linear_gated, K columns; ld hidden units each) and of the shared one
- *   lcu_decode_project_norm: m = sum over slots of w[choice] . lhs[slot] (+ bias) + shared_gate times the shared
- *     product, then lcu_residual_norm of the row (workspace) */
+ *   lcu_decode_experts_down: slot s: fp32 row out + s * ldo = w[choice[s]] . hidden[s]; the shared product is
+ *     slot `slots`
+ *   lcu_decode_residual_router: lcu_residual_norm of the row (the sum of `top` rows of out and the gated shared
+ *     row), then lcu_router of it when router_w is given */
 int lcu_decode_linear(void* out_f32_dev, const void* x_dev, const void* w_dev, const void* bias_dev, int K, int N, void* stream);
 int lcu_decode_recurrent_in(void* y_dev, void* u_dev, void* conv_state_dev, const void* x_dev, const void* w_dev,
                             const void* bias_dev, const void* conv_dev, const void* conv_bias_dev, int taps, int K, int ld,
@@ -438,16 +438,17 @@ int lcu_decode_recurrent_step(void* out_dev, const void* u_dev, const void* y_de
 int lcu_decode_kv(void* q_out_dev, void* k_cache_dev, void* v_cache_dev, const void* x_dev, const void* w_dev, const void* bias_dev,
                   int q_cols, int k_cols, int v_cols, void* v_first_dev, int v_mode, const void* lambda_dev, const void* pos_dev,
                   int max_positions, int K, void* stream);
-int lcu_decode_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const void* h_dev, const void* w_dev, int n_experts,
-                      int top, void* arrived_dev, int K, void* stream);
 int lcu_decode_experts_up(void* hidden_dev, void* shared_hidden_dev, const void* h_dev, const void* choice_dev,
                           const void* weight_dev, const void* up_dev, size_t up_stride, const lcu_gate_params* gate,
                           const void* shared_up_dev, const lcu_gate_params* shared_gate, int top, int ld, int shared_ld, int K,
                           void* stream);
-int lcu_decode_project_norm(void* x_dev, void* h_dev, const void* lhs_dev, const void* w_dev, const void* bias_dev, int K,
-                            const void* choice_dev, size_t stride, int slots, const void* shared_lhs_dev, const void* shared_w_dev,
-                            int shared_K, const void* shared_gate_dev, const void* w_after_dev, const void* w_next_dev,
-                            void* arrived_dev, int width, int ld, int groups, float eps, void* stream);
+int lcu_decode_experts_down(void* out_f32_dev, int ldo, const void* hidden_dev, const void* choice_dev, const void* w_dev,
+                            size_t stride, int slots, int K, const void* shared_hidden_dev, const void* shared_w_dev, int shared_K,
+                            int N, void* stream);
+int lcu_decode_residual_router(void* x_dev, void* h_dev, const void* out_f32_dev, int top, const void* shared_f32_dev,
+                               const void* shared_gate_dev, const void* w_after_dev, const void* w_next_dev, int width, int ld,
+                               int groups, float eps, const void* router_w_dev, int n_experts, int choose, void* expert_dev,
+                               void* weight_dev, void* router_gate_dev, void* stream);
 
 /* pseudo-random matrix (synthetic weights): mean + std * N(0, 1) (the hash of lcu_fill_normal_f16) into
  * columns 0 .. cols - 1 of rows of ld elements */

@@ -113,9 +113,9 @@ SIGNATURES = {
     "lcu_decode_recurrent_in": (i32, [vp] * 8 + [i32, i32, i32, vp]),
     "lcu_decode_recurrent_step": (i32, [vp] * 9 + [i32, i32, vp]),
     "lcu_decode_kv": (i32, [vp, vp, vp, vp, vp, vp, i32, i32, i32, vp, i32, vp, vp, i32, i32, vp]),
-    "lcu_decode_router": (i32, [vp, vp, vp, vp, vp, i32, i32, vp, i32, vp]),
     "lcu_decode_experts_up": (i32, [vp] * 6 + [sz, vp, vp, vp, i32, i32, i32, i32, vp]),
-    "lcu_decode_project_norm": (i32, [vp, vp, vp, vp, vp, i32, vp, sz, i32, vp, vp, i32, vp, vp, vp, vp, i32, i32, i32, f32, vp]),
+    "lcu_decode_experts_down": (i32, [vp, i32, vp, vp, vp, sz, i32, i32, vp, vp, i32, i32, vp]),
+    "lcu_decode_residual_router": (i32, [vp, vp, vp, i32] + [vp] * 4 + [i32, i32, i32, f32, vp, i32, i32, vp, vp, vp, vp]),
     "lcu_fill_normal_matrix": (i32, [vp, sz, i32, i32, i32, u64, u64, f32, f32, vp]),
     # llama_cu_c.h
     "lcu_model_open": (vp, [C.c_char_p, i32, i32]),

@@ -1,47 +1,12 @@
 // Mixture of experts: router (scores, choice of the largest, gate of the shared expert) and the
 // plan that sorts the tokens' choices by expert for the grouped products (linear.hip).
-#include "linear.hpp"
-#include "rownorm.hpp"
+#include "router.hpp"
 
 using namespace lcu;
 
 namespace {
 
-constexpr int MAX_EXPERTS = 512;
-
-// One wavefront: the `top` largest of z (LDS; ties: the smaller index), with their scores.  z is used up.
-__device__ __forceinline__ void choose(float* z, int n_experts, int top, int* __restrict__ expert, float* __restrict__ weight) {
-  const int lane = threadIdx.x & 63;
-  for (int k = 0; k < top; ++k) {
-    float best = -INFINITY;
-    int idx = 0x7fffffff;
-    for (int e = lane; e < n_experts; e += WAVE) {
-      const float v = z[e];
-      if (v > best || (v == best && e < idx)) {
-        best = v;
-        idx = e;
-      }
-    }
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) {
-      const float ob = __shfl_xor(best, off, WAVE);
-      const int oi = __shfl_xor(idx, off, WAVE);
-      if (ob > best || (ob == best && oi < idx)) {
-        best = ob;
-        idx = oi;
-      }
-    }
-    if (idx >= n_experts) idx = k;  // no finite logit left
-    if (lane == 0) {
-      expert[k] = idx;
-      weight[k] = sigmoid_f32(best);
-      z[idx] = -INFINITY;
-    }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-  }
-}
+constexpr int MAX_EXPERTS = ROUTER_MAX_ROWS - 1;
 
 // One workgroup per token: logit e = row e of w . h in fp32, then the `top` largest (ties: the smaller
 // index), their scores sigmoid(z), and sigmoid of the row behind the experts' (the shared gate).
@@ -63,13 +28,26 @@ __global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, f
   __syncthreads();
   if (wave != 0) return;
   if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
-  choose(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
+  choose_experts(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
 }
 
 // The same for bfloat16 operands on the matrix cores: one workgroup takes 16 tokens and all rows of w, its
 // wavefronts a quarter of K each, four tiles of 16 rows of w at a time; the quarters are added in LDS in
 // wavefront order, and every wavefront chooses for four of the tokens.
 constexpr int ROUTER_TOKENS = 16;
+template <int TILES>
+__device__ __forceinline__ void router_tiles(float4_t (&acc)[4], const bf16_t* a, const bf16_t* const (&b)[4], int s0, int s1) {
+#pragma unroll 4
+  for (int s = s0; s < s1; ++s) {
+    const bf16x8_t fa = *reinterpret_cast<const bf16x8_t*>(a + s * 32);
+#pragma unroll
+    for (int j = 0; j < TILES; ++j) {
+      const bf16x8_t fb = *reinterpret_cast<const bf16x8_t*>(b[j] + s * 32);
+      acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, fb, acc[j], 0, 0, 0);
+    }
+  }
+}
+
 __global__ __launch_bounds__(256) void router_tile_kernel(int* __restrict__ expert, float* __restrict__ weight,
                                                           float* __restrict__ shared_gate, const bf16_t* __restrict__ h,
                                                           const bf16_t* __restrict__ w, int n, int n_experts, int top, int K) {
@@ -88,16 +66,11 @@ __global__ __launch_bounds__(256) void router_tile_kernel(int* __restrict__ expe
       b[j] = w + (size_t)min(e0 + j * 16 + col, n_rows - 1) * K + quad * 8;
     }
     const int tiles = min(4, (n_rows - e0 + 15) / 16);
-#pragma unroll 4
-    for (int s = s0; s < s1; ++s) {
-      const bf16x8_t fa = *reinterpret_cast<const bf16x8_t*>(a + s * 32);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        if (j < tiles) {
-          const bf16x8_t fb = *reinterpret_cast<const bf16x8_t*>(b[j] + s * 32);
-          acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, fb, acc[j], 0, 0, 0);
-        }
-      }
+    switch (tiles) {
+      case 1: router_tiles<1>(acc, a, b, s0, s1); break;
+      case 2: router_tiles<2>(acc, a, b, s0, s1); break;
+      case 3: router_tiles<3>(acc, a, b, s0, s1); break;
+      default: router_tiles<4>(acc, a, b, s0, s1); break;
     }
     for (int turn = 0; turn < 4; ++turn) {
       if (wave == turn) {
@@ -120,42 +93,8 @@ __global__ __launch_bounds__(256) void router_tile_kernel(int* __restrict__ expe
     if (t >= n) continue;
     float* z = zs + (t - t0) * ldz;
     if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
-    choose(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
+    choose_experts(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
   }
-}
-
-// One new token: a workgroup per row of w; the one that arrives last chooses.
-__global__ __launch_bounds__(256) void router_step_kernel(int* __restrict__ expert, float* __restrict__ weight,
-                                                          float* __restrict__ shared_gate, const bf16_t* __restrict__ h,
-                                                          const bf16_t* __restrict__ w, int n_experts, int top, int K,
-                                                          float* __restrict__ logits, uint32_t* __restrict__ arrived) {
-  __shared__ float z[MAX_EXPERTS + 1];
-  __shared__ float part[4];
-  __shared__ bool last;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n_rows = gridDim.x;
-  const bf16_t* we = w + (size_t)blockIdx.x * K;
-  float s = 0.0f;
-#pragma unroll 4
-  for (int k = tid * 8; k < K; k += 256 * 8) {
-    const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(h + k), wv = *reinterpret_cast<const bf16x8_t*>(we + k);
-#pragma unroll
-    for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
-  }
-  s = wave_sum(s);
-  if (lane == 0) part[wave] = s;
-  __syncthreads();
-  if (tid == 0) {
-    __hip_atomic_store(logits + blockIdx.x, (part[0] + part[1]) + (part[2] + part[3]), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the logit is out before the count goes up
-    last = arrives_last(arrived, blockIdx.x, gridDim.x);
-  }
-  __syncthreads();
-  if (!last) return;
-  for (int i = tid; i < n_rows; i += 256) z[i] = __hip_atomic_load(logits + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  __syncthreads();
-  if (wave != 0) return;
-  if (shared_gate && lane == 0) *shared_gate = sigmoid_f32(z[n_experts]);
-  choose(z, n_experts, top, expert, weight);
 }
 
 // One workgroup: counts per expert, their prefix sums, each choice's sorted row, and the row tiles.
@@ -218,21 +157,6 @@ int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const 
     router_tile_kernel<<<(n + ROUTER_TOKENS - 1) / ROUTER_TOKENS, 256, lds, st>>>(
         (int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev, (const bf16_t*)w_dev, n, n_experts, top, K);
   }
-  LCU_LAUNCH_CHECK();
-  return LCU_OK;
-}
-
-int lcu_decode_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const void* h_dev, const void* w_dev, int n_experts,
-                      int top, void* arrived_dev, int K, void* stream) {
-  LCU_REQUIRE(expert_dev && weight_dev && h_dev && w_dev && arrived_dev, "lcu_decode_router: null pointer");
-  LCU_REQUIRE(n_experts > 0 && n_experts <= MAX_EXPERTS && top > 0 && top <= n_experts && K > 0 && K % 64 == 0,
-              "lcu_decode_router: experts %d (at most %d), top %d, K %d", n_experts, MAX_EXPERTS, top, K);
-  hipStream_t st = as_stream(stream);
-  const workspace_t ws = workspace_for(st);
-  if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_decode_router: lcu_init has not run on this device");
-  router_step_kernel<<<n_experts + (shared_gate_dev ? 1 : 0), 256, 0, st>>>((int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev,
-                                                              (const bf16_t*)h_dev, (const bf16_t*)w_dev, n_experts, top, K,
-                                                              (float*)ws.ptr, (uint32_t*)arrived_dev);
   LCU_LAUNCH_CHECK();
   return LCU_OK;
 }

@@ -361,7 +361,7 @@ __device__ __forceinline__ void wait_vmcnt() {
 // v_mfma_f32_32x32x16_bf16, and end in a bias, a GELU, or a clamped gate; GROUPED ones take the
 // rows of a tile and its weight matrix from a tile list on the device (experts_plan in experts.hip).
 struct f16_epilogue {
-  static constexpr bool BF16 = false, GROUPED = false, GATED = false;
+  static constexpr bool BF16 = false, GROUPED = false;
 };
 
 template <int BM, int BN, int WM, int WN, int KS, int NS, bool U8, bool SPLIT = false, class EP = f16_epilogue>

@@ -27,7 +27,6 @@
 
 #include "common.hpp"
 #include "linear.hpp"
-#include "rownorm.hpp"
 
 using namespace lcu;
 
@@ -863,120 +862,34 @@ __global__ __launch_bounds__(GEMV_THREADS) void decode_experts_up_kernel(const b
   st.run(nullptr, 1.0f, part);
 }
 
-// ---- a projection and what follows it: x += norm(projection), h = norm(x) ---------------------------
-// Workgroups compute rows of one or several products (slots: one for a mixer's output; the chosen experts
-// and the shared one for a feed-forward) and store them as fp32 at device scope.  The workgroup that arrives
-// last (arrives_last) adds the slots, normalises the sum, adds it to
-// the residual row, and normalises that for the next sublayer.  Nobody waits for anybody.
+// Second products: rows of one or several matrices (slots: the chosen experts and the shared one), fp32 results
+// of slot s at out + s * ldo
 struct projection_slots {
   const bf16_t* W;
   const bf16_t* lhs;          // row of slot s at lhs + s * K
-  const int* choice;          // slot s multiplies W + choice[s] * stride; NULL: W itself
+  const int* choice;          // slot s multiplies W + choice[s] * stride
   size_t stride;              // elements
   int K, slots;
   const bf16_t* shared_W;     // one more slot, or NULL
   const bf16_t* shared_lhs;
   int shared_K;
-  const float* shared_gate;   // its factor
-  const float* bias;
-  float* part;                // [slots + 1][ld]
-};
-struct residual_step {
-  float* x;
-  bf16_t* h;
-  const float* w_after;
-  const float* w_next;  // NULL: no next sublayer
-  uint32_t* arrived;
-  row_shape rs;
-};
-
-struct store_part_row {
   float* out;
-  const float* bias;
-  __device__ __forceinline__ void operator()(int n, float v) const {
-    __hip_atomic_store(out + n, bias ? v + bias[n] : v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  }
+  int N, ldo;
 };
 
-template <int R, int U, int NV>
-__global__ __launch_bounds__(GEMV_THREADS) void decode_project_kernel(projection_slots p, residual_step r) {
-  static_assert(GEMV_THREADS == ROW_THREADS, "the last workgroup normalises the row");
-  extern __shared__ __attribute__((aligned(16))) float lds[];
+template <int R, int U>
+__global__ __launch_bounds__(GEMV_THREADS) void decode_experts_down_kernel(projection_slots p) {
   __shared__ float part[GEMV_WAVES * R];
-  __shared__ bool last;
-  const int per_slot = (r.rs.width + R - 1) / R;
+  const int per_slot = (p.N + R - 1) / R;
   const int slot = blockIdx.x / per_slot, task = blockIdx.x - slot * per_slot;
-  {
-    const bool shared = slot == p.slots;
-    const int K = shared ? p.shared_K : p.K;
-    const bf16_t* W = shared ? p.shared_W : p.choice ? p.W + (size_t)p.choice[slot] * p.stride : p.W;
-    const bf16_t* x = shared ? p.shared_lhs : p.lhs + (size_t)slot * p.K;
-    const bf16_tasks<R, store_part_row> tk{W, K, r.rs.width, store_part_row{p.part + (size_t)slot * r.rs.ld, p.bias}};
-    stream_t<false, R, U, false, bf16_tasks<R, store_part_row>, 0, true> st(tk, reinterpret_cast<const half_t*>(x), nullptr, K, 0, task);
-    st.begin();
-    st.run(nullptr, 1.0f, part);
-  }
-  if (threadIdx.x == 0) {
-    // this thread stored the workgroup's rows, write-through; they are complete before the count goes up
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    last = arrives_last(r.arrived, blockIdx.x, gridDim.x);
-  }
-  __syncthreads();
-  if (!last) return;
-  const int total = p.slots + (p.shared_W ? 1 : 0);
-  row_t<NV> m, t;
-  load_row(t, r.w_after, r.rs);
-#pragma unroll
-  for (int j = 0; j < NV; ++j) m.v[j] = (float4_t)(0.0f);
-  for (int s = 0; s < total; ++s) {
-    // device scope, 16 bytes per request, four requests per statement
-    const float* src = p.part + (size_t)s * r.rs.ld;
-    const float f = s == p.slots ? *p.shared_gate : 1.0f;
-#pragma unroll
-    for (int j = 0; j < NV; j += 4) {
-      uint4_t v[4];
-      const auto word = [&](int k) {
-        const int c = m.column(j + k);
-        return reinterpret_cast<const uint64_t*>(src + (j + k < NV && c < r.rs.width ? c : 0));
-      };
-      load_word_pairs_device_scope(v, word(0), word(1), word(2), word(3));
-#pragma unroll
-      for (int k = 0; k < 4; ++k) {
-        if (j + k < NV) {
-          const float4_t x = __builtin_bit_cast(float4_t, v[k]);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            if (m.column(j + k) + e < r.rs.width) m.v[j + k][e] += f * x[e];
-          }
-        }
-      }
-    }
-  }
-  scale_row(m, r.rs, lds, t);
-  load_row(t, r.x, r.rs);
-#pragma unroll
-  for (int j = 0; j < NV; ++j) m.v[j] += t.v[j];
-  store_row(r.x, m, r.rs);
-  if (r.w_next) {
-    load_row(t, r.w_next, r.rs);
-    scale_row(m, r.rs, lds, t);
-    store_row(r.h, m, r.rs);
-  }
-}
-
-int launch_project(const projection_slots& p, const residual_step& r, hipStream_t st) {
-  const int n = p.slots + (p.shared_W ? 1 : 0);
-  const size_t lds = row_lds_bytes(r.rs);
-  const int K = p.shared_W && p.shared_K > p.K ? p.shared_K : p.K;
-  with_row_pieces(r.rs.ld, [&](auto nv) {
-    if (K > 2048) {
-      decode_project_kernel<2, 2, decltype(nv)::value><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
-    } else {
-      decode_project_kernel<2, 1, decltype(nv)::value><<<n * ((r.rs.width + 1) / 2), GEMV_THREADS, lds, st>>>(p, r);
-    }
-  });
-  LCU_LAUNCH_CHECK();
-  return LCU_OK;
+  const bool shared = slot == p.slots;
+  const int K = shared ? p.shared_K : p.K;
+  const bf16_t* W = shared ? p.shared_W : p.W + (size_t)p.choice[slot] * p.stride;
+  const bf16_t* x = shared ? p.shared_lhs : p.lhs + (size_t)slot * p.K;
+  const bf16_tasks<R, store_f32_row> tk{W, K, p.N, store_f32_row{p.out + (size_t)slot * p.ldo, nullptr}};
+  stream_t<false, R, U, false, bf16_tasks<R, store_f32_row>, 0, true> st(tk, reinterpret_cast<const half_t*>(x), nullptr, K, 0, task);
+  st.begin();
+  st.run(nullptr, 1.0f, part);
 }
 
 // calls f with the number of 16-byte pieces of x per thread (x_stage_t) that covers dim <= 24576
@@ -1293,29 +1206,24 @@ int lcu_decode_experts_up(void* hidden_dev, void* shared_hidden_dev, const void*
   return LCU_OK;
 }
 
-int lcu_decode_project_norm(void* x_dev, void* h_dev, const void* lhs_dev, const void* w_dev, const void* bias_dev, int K,
-                            const void* choice_dev, size_t stride, int slots, const void* shared_lhs_dev, const void* shared_w_dev,
-                            int shared_K, const void* shared_gate_dev, const void* w_after_dev, const void* w_next_dev,
-                            void* arrived_dev, int width, int ld, int groups, float eps, void* stream) {
-  LCU_REQUIRE(x_dev && lhs_dev && w_dev && w_after_dev && arrived_dev && (h_dev || !w_next_dev) &&
-                  (!shared_w_dev || (shared_lhs_dev && shared_gate_dev)),
-              "lcu_decode_project_norm: null pointer");
-  LCU_REQUIRE(K > 0 && K % 64 == 0 && slots > 0 && (slots == 1 || choice_dev) && (!shared_w_dev || (shared_K > 0 && shared_K % 64 == 0)) &&
+int lcu_decode_experts_down(void* out_f32_dev, int ldo, const void* hidden_dev, const void* choice_dev, const void* w_dev,
+                            size_t stride, int slots, int K, const void* shared_hidden_dev, const void* shared_w_dev, int shared_K,
+                            int N, void* stream) {
+  LCU_REQUIRE(out_f32_dev && hidden_dev && choice_dev && w_dev && (!shared_w_dev || shared_hidden_dev),
+              "lcu_decode_experts_down: null pointer");
+  LCU_REQUIRE(K > 0 && K % 64 == 0 && slots > 0 && N > 0 && ldo >= N && (!shared_w_dev || (shared_K > 0 && shared_K % 64 == 0)) &&
                   stride % 2 == 0,
-              "lcu_decode_project_norm: bad shape K %d %d slots %d", K, shared_K, slots);
-  LCU_REQUIRE(width > 0 && width <= ROW_MAX_WIDTH && ld >= width && ld % 64 == 0 && groups > 0 && width % groups == 0 &&
-                  groups <= ROW_MAX_GROUPS,
-              "lcu_decode_project_norm: bad row width %d ld %d groups %d", width, ld, groups);
-  hipStream_t st = as_stream(stream);
-  const workspace_t ws = workspace_for(st);
-  if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_decode_project_norm: lcu_init has not run on this device");
-  LCU_REQUIRE((size_t)(slots + 1) * ld * sizeof(float) <= ws.bytes, "lcu_decode_project_norm: %d slots do not fit the workspace", slots);
-  const projection_slots p{(const bf16_t*)w_dev, (const bf16_t*)lhs_dev, (const int*)choice_dev, stride / 2, K, slots,
-                           (const bf16_t*)shared_w_dev, (const bf16_t*)shared_lhs_dev, shared_K, (const float*)shared_gate_dev,
-                           (const float*)bias_dev, (float*)ws.ptr};
-  const residual_step r{(float*)x_dev, (bf16_t*)h_dev, (const float*)w_after_dev, (const float*)w_next_dev, (uint32_t*)arrived_dev,
-                        row_shape{width, ld, groups, eps}};
-  return launch_project(p, r, st);
+              "lcu_decode_experts_down: bad shape K %d %d slots %d N %d", K, shared_K, slots, N);
+  const projection_slots p{(const bf16_t*)w_dev, (const bf16_t*)hidden_dev, (const int*)choice_dev, stride / 2, K, slots,
+                           (const bf16_t*)shared_w_dev, (const bf16_t*)shared_hidden_dev, shared_K, (float*)out_f32_dev, N, ldo};
+  const int grid = (slots + (shared_w_dev ? 1 : 0)) * ((N + 1) / 2);
+  if ((shared_w_dev && shared_K > K ? shared_K : K) > 2048) {
+    decode_experts_down_kernel<2, 2><<<grid, GEMV_THREADS, 0, as_stream(stream)>>>(p);
+  } else {
+    decode_experts_down_kernel<2, 1><<<grid, GEMV_THREADS, 0, as_stream(stream)>>>(p);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
 }
 
 #ifdef LCU_PHASE_TIMELINE

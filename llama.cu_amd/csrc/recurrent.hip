@@ -81,33 +81,29 @@ struct gate_args {
   int n, bw, ld;
 };
 
-// One workgroup: 64 tokens x 32 channels of both gates.  Wavefront w multiplies 32 tokens (w & 1) by the
+// The map S -> A S + B of consecutive tokens
+struct state_map {
+  float A{1.0f}, B{0.0f};
+  __device__ __forceinline__ void then(float a, float b) {
+    B = fmaf(a, B, b);
+    A = a * A;
+  }
+};
+
+// fp32.  One workgroup: 64 tokens x 32 channels of both gates.  Wavefront w multiplies 32 tokens (w & 1) by the
 // channels of gate w >> 1; both gates of a channel then meet in LDS, and every thread turns eight
 // consecutive tokens of one channel into a, b and their composite map.
-template <class T>
-__global__ __launch_bounds__(256) void gates_kernel(const T* __restrict__ u, gate_args p) {
+__global__ __launch_bounds__(256) void gates_f32_kernel(const float* __restrict__ u, gate_args p) {
   __shared__ float gate[2][CHUNK][GATE_N + 1];
   __shared__ float seg[2][8][GATE_N];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int t0 = blockIdx.y * CHUNK, c0 = blockIdx.x * GATE_N;  // c0: first channel of the tile, inside one block
   const int blk = c0 / p.bw, j0 = c0 - blk * p.bw;
   const int which = wave >> 1, rows0 = (wave & 1) * 32;
-  const T* W = (const T*)(which ? p.wi : p.wr) + ((size_t)blk * p.bw + j0) * p.bw;
-  const T* ub = u + (size_t)blk * p.bw;
-  if constexpr (sizeof(T) == 2) {
-    float16_t acc = (float16_t)(0.0f);
-    const T* ua = ub + (size_t)min(t0 + rows0 + (lane & 31), p.n - 1) * p.ld + (lane >> 5) * 8;
-    const T* wa = W + (size_t)(lane & 31) * p.bw + (lane >> 5) * 8;
-#pragma unroll 4
-    for (int k = 0; k < p.bw; k += 16) {
-      const bf16x8_t fa = *reinterpret_cast<const bf16x8_t*>(ua + k);
-      const bf16x8_t fb = *reinterpret_cast<const bf16x8_t*>(wa + k);
-      acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa, fb, acc, 0, 0, 0);
-    }
-#pragma unroll
-    for (int v = 0; v < 16; ++v) gate[which][rows0 + (v >> 2) * 8 + (lane >> 5) * 4 + (v & 3)][lane & 31] = acc[v];
-  } else {
-    // fp32: lane (channel lane & 31, half lane >> 5) sums 16 tokens of its wavefront's 32
+  const float* W = (const float*)(which ? p.wi : p.wr) + ((size_t)blk * p.bw + j0) * p.bw;
+  const float* ub = u + (size_t)blk * p.bw;
+  {
+    // lane (channel lane & 31, half lane >> 5) sums 16 tokens of its wavefront's 32
     float acc[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) acc[i] = 0.0f;
@@ -124,40 +120,100 @@ __global__ __launch_bounds__(256) void gates_kernel(const T* __restrict__ u, gat
   __syncthreads();
   const int ch = tid & 31, s8 = tid >> 5, c = c0 + ch;
   const float br = p.br[c], bi = p.bi[c], decay = p.decay[c];
-  float A = 1.0f, B = 0.0f;
+  state_map map;
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
     const int lt = s8 * 8 + e, t = t0 + lt;
     if (t < p.n) {
-      float a, b;
-      if constexpr (sizeof(T) == 2) {
-        const float log_a = decay * sigmoid_fast(gate[0][lt][ch] + br);
-        a = __expf(log_a);
-        b = drive_factor(log_a, a) * sigmoid_fast(gate[1][lt][ch] + bi) * to_f32(u[(size_t)t * p.ld + c]);
-      } else {
-        const float log_a = decay * sigmoid_f32(gate[0][lt][ch] + br);
-        a = expf(log_a);
-        b = sqrtf(-expm1f(2.0f * log_a)) * sigmoid_f32(gate[1][lt][ch] + bi) * to_f32(u[(size_t)t * p.ld + c]);
-      }
+      const float log_a = decay * sigmoid_f32(gate[0][lt][ch] + br);
+      const float a = expf(log_a);
+      const float b = sqrtf(-expm1f(2.0f * log_a)) * sigmoid_f32(gate[1][lt][ch] + bi) * u[(size_t)t * p.ld + c];
       p.a[(size_t)t * p.ld + c] = a;
       p.b[(size_t)t * p.ld + c] = b;
-      A = a * A;
-      B = fmaf(a, B, b);
+      map.then(a, b);
     }
   }
-  seg[0][s8][ch] = A;
-  seg[1][s8][ch] = B;
+  seg[0][s8][ch] = map.A;
+  seg[1][s8][ch] = map.B;
   __syncthreads();
   if (tid < GATE_N) {
-    A = 1.0f;
-    B = 0.0f;
+    state_map whole;
 #pragma unroll
-    for (int s = 0; s < 8; ++s) {
-      B = fmaf(seg[0][s][tid], B, seg[1][s][tid]);
-      A = seg[0][s][tid] * A;
+    for (int s = 0; s < 8; ++s) whole.then(seg[0][s][tid], seg[1][s][tid]);
+    p.chunk_a[(size_t)blockIdx.y * p.ld + c0 + tid] = whole.A;
+    p.chunk_b[(size_t)blockIdx.y * p.ld + c0 + tid] = whole.B;
+  }
+}
+
+// bfloat16.  One wavefront: a chunk of 64 tokens x 32 channels, both gates, so that a lane holds r and i of
+// the same tokens of one channel: of every 8 tokens, the four from 4 (lane >> 5).  Four wavefronts of a
+// workgroup take neighbouring channel tiles and share the rows of u.
+__global__ __launch_bounds__(256) void gates_bf16_kernel(const bf16_t* __restrict__ u, gate_args p, int channels) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int t0 = blockIdx.y * CHUNK, c0 = (blockIdx.x * 4 + wave) * GATE_N;
+  if (c0 >= channels) return;
+  const int blk = c0 / p.bw, j0 = c0 - blk * p.bw, col = lane & 31, half = lane >> 5, c = c0 + col;
+  const bf16_t* ua = u + (size_t)blk * p.bw + half * 8;
+  const bf16_t* u0 = ua + (size_t)min(t0 + col, p.n - 1) * p.ld;
+  const bf16_t* u1 = ua + (size_t)min(t0 + 32 + col, p.n - 1) * p.ld;
+  const size_t w_at = ((size_t)blk * p.bw + j0 + col) * p.bw + half * 8;
+  const bf16_t* wr = (const bf16_t*)p.wr + w_at;
+  const bf16_t* wi = (const bf16_t*)p.wi + w_at;
+  float16_t r[2], g[2];
+#pragma unroll
+  for (int m = 0; m < 2; ++m) {
+    r[m] = (float16_t)(0.0f);
+    g[m] = (float16_t)(0.0f);
+  }
+  const auto piece = [](const bf16_t* q, int k) { return *reinterpret_cast<const bf16x8_t*>(q + k); };
+#pragma unroll 2
+  for (int k = 0; k < p.bw; k += 32) {  // block widths are multiples of 32
+    const bf16x8_t a0 = piece(u0, k), a1 = piece(u1, k), b0 = piece(wr, k), b1 = piece(wi, k);
+    const bf16x8_t a2 = piece(u0, k + 16), a3 = piece(u1, k + 16), b2 = piece(wr, k + 16), b3 = piece(wi, k + 16);
+    r[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b0, r[0], 0, 0, 0);
+    r[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b0, r[1], 0, 0, 0);
+    g[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b1, g[0], 0, 0, 0);
+    g[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b1, g[1], 0, 0, 0);
+    r[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a2, b2, r[0], 0, 0, 0);
+    r[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a3, b2, r[1], 0, 0, 0);
+    g[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a2, b3, g[0], 0, 0, 0);
+    g[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a3, b3, g[1], 0, 0, 0);
+  }
+  const float br = p.br[c], bi = p.bi[c], decay = p.decay[c];
+  state_map whole;
+#pragma unroll
+  for (int m = 0; m < 2; ++m) {
+    // token of element v: t0 + 32 m + (v >> 2) * 8 + half * 4 + (v & 3)
+    float uv[16];
+#pragma unroll
+    for (int v = 0; v < 16; ++v) {
+      const int t = t0 + m * 32 + (v >> 2) * 8 + half * 4 + (v & 3);
+      uv[v] = (float)u[(size_t)min(t, p.n - 1) * p.ld + c];
     }
-    p.chunk_a[(size_t)blockIdx.y * p.ld + c0 + tid] = A;
-    p.chunk_b[(size_t)blockIdx.y * p.ld + c0 + tid] = B;
+#pragma unroll
+    for (int o = 0; o < 4; ++o) {
+      state_map map;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int v = o * 4 + e, t = t0 + m * 32 + o * 8 + half * 4 + e;
+        const float log_a = decay * sigmoid_fast(r[m][v] + br);
+        const float a = __expf(log_a);
+        const float b = drive_factor(log_a, a) * sigmoid_fast(g[m][v] + bi) * uv[v];
+        if (t < p.n) {
+          p.a[(size_t)t * p.ld + c] = a;
+          p.b[(size_t)t * p.ld + c] = b;
+          map.then(a, b);
+        }
+      }
+      // the lane 32 further holds the neighbouring four tokens of the eight
+      const float oA = __shfl_xor(map.A, 32, WAVE), oB = __shfl_xor(map.B, 32, WAVE);
+      whole.then(half ? oA : map.A, half ? oB : map.B);
+      whole.then(half ? map.A : oA, half ? map.B : oB);
+    }
+  }
+  if (half == 0) {
+    p.chunk_a[(size_t)blockIdx.y * p.ld + c] = whole.A;
+    p.chunk_b[(size_t)blockIdx.y * p.ld + c] = whole.B;
   }
 }
 
@@ -302,11 +358,11 @@ int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, in
   float* cb = ca + (size_t)chunks * ld;
   const gate_args p{wr_dev, wi_dev, (const float*)br_dev, (const float*)bi_dev, (const float*)decay_dev, a, b, ca, cb, n,
                     block_width, ld};
-  const dim3 tiles(channels / GATE_N, chunks), rows((channels + 255) / 256, chunks);
+  const dim3 rows((channels + 255) / 256, chunks);
   if (dtype == LCU_F32) {
-    gates_kernel<float><<<tiles, 256, 0, st>>>((const float*)u_dev, p);
+    gates_f32_kernel<<<dim3(channels / GATE_N, chunks), 256, 0, st>>>((const float*)u_dev, p);
   } else {
-    gates_kernel<bf16_t><<<tiles, 256, 0, st>>>((const bf16_t*)u_dev, p);
+    gates_bf16_kernel<<<dim3((channels / GATE_N + 3) / 4, chunks), 256, 0, st>>>((const bf16_t*)u_dev, p, channels);
   }
   carry_kernel<<<(channels + 63) / 64, 64, 0, st>>>(ca, cb, (float*)state_dev, chunks, channels, ld);
   if (dtype == LCU_F32) {

@@ -5,6 +5,7 @@
 #include <type_traits>
 
 #include "linear.hpp"
+#include "router.hpp"
 #include "rownorm.hpp"
 
 using namespace lcu;
@@ -12,8 +13,8 @@ using namespace lcu;
 namespace {
 
 // x[row] = norm(table[token] + pos_table[start + row]) under w0; h[row] = norm(x[row]) under w1 when given
-template <class T, int NV>
-__global__ __launch_bounds__(ROW_THREADS) void embed_pos_norm_kernel(float* __restrict__ x, T* __restrict__ h,
+template <class T, int NV, int TH>
+__global__ __launch_bounds__(TH) void embed_pos_norm_kernel(float* __restrict__ x, T* __restrict__ h,
                                                                      const int* __restrict__ ids, const T* __restrict__ table,
                                                                      const T* __restrict__ pos_table, const float* __restrict__ w0,
                                                                      const float* __restrict__ w1, const int* __restrict__ start,
@@ -21,46 +22,51 @@ __global__ __launch_bounds__(ROW_THREADS) void embed_pos_norm_kernel(float* __re
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = blockIdx.x;
   const int id = min(max(ids[r], 0), n_vocab - 1), p = min(max(*start + r, 0), n_pos - 1);
-  row_t<NV> row, at, w;
+  row_t<NV, TH> row, at, w, next;
+  load_row(w, w0, rs);
+  if (w1) load_row(next, w1, rs);
   load_row(row, table + (size_t)id * rs.ld, rs);
   load_row(at, pos_table + (size_t)p * rs.ld, rs);
-  load_row(w, w0, rs);
 #pragma unroll
   for (int j = 0; j < NV; ++j) row.v[j] += at.v[j];
   scale_row(row, rs, lds, w);
   store_row(x + (size_t)r * rs.ld, row, rs);
   if (w1) {
-    load_row(w, w1, rs);
-    scale_row(row, rs, lds, w);
+    scale_row(row, rs, lds, next);
     store_row(h + (size_t)r * rs.ld, row, rs);
   }
 }
 
-// m[row] = out[row], or the sum of a token's expert rows (inverse[row * top + k] is where the k-th of them
-// lies) plus its shared expert's row times shared_gate[row]; x += norm(m) under w_after; h = norm(x) under w_next.
-template <class T, int NV>
-__global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(float* __restrict__ x, T* __restrict__ h,
+// what sublayers left for row r: its rows of src.out, and the shared expert's row times its gate
+template <int NV, int TH>
+__device__ __forceinline__ void load_sum(row_t<NV, TH>& m, row_t<NV, TH>& t, const sublayer_rows& src, int r, const row_shape& rs) {
+  const auto from = [&](int k) {
+    const size_t at = (size_t)r * src.top + k;
+    return src.out + (src.inverse ? (size_t)src.inverse[at] : at) * rs.ld;
+  };
+  load_row(m, from(0), rs);
+  for (int k = 1; k < src.top; ++k) {
+    load_row(t, from(k), rs);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) m.v[j] += t.v[j];
+  }
+  if (src.shared) {
+    const float f = src.shared_gate[r];
+    load_row(t, src.shared + (size_t)r * rs.ld, rs);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) m.v[j] += f * t.v[j];
+  }
+}
+
+// m = the sublayer's result; x += norm(m) under w_after; h = norm(x) under w_next.
+template <class T, int NV, int TH>
+__global__ __launch_bounds__(TH) void residual_norm_kernel(float* __restrict__ x, T* __restrict__ h,
                                                                     sublayer_rows src, const float* __restrict__ w_after,
                                                                     const float* __restrict__ w_next, row_shape rs) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = blockIdx.x;
-  row_t<NV> m, t, old;
-  if (src.inverse) {
-    load_row(m, src.out + (size_t)src.inverse[(size_t)r * src.top] * rs.ld, rs);
-    for (int k = 1; k < src.top; ++k) {
-      load_row(t, src.out + (size_t)src.inverse[(size_t)r * src.top + k] * rs.ld, rs);
-#pragma unroll
-      for (int j = 0; j < NV; ++j) m.v[j] += t.v[j];
-    }
-    if (src.shared) {
-      const float f = src.shared_gate[r];
-      load_row(t, src.shared + (size_t)r * rs.ld, rs);
-#pragma unroll
-      for (int j = 0; j < NV; ++j) m.v[j] += f * t.v[j];
-    }
-  } else {
-    load_row(m, src.out + (size_t)r * rs.ld, rs);
-  }
+  row_t<NV, TH> m, t, old;
+  load_sum(m, t, src, r, rs);
   float* xr = x + (size_t)r * rs.ld;
   load_row(old, xr, rs);
   load_row(t, w_after, rs);
@@ -75,30 +81,95 @@ __global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(float* __res
   }
 }
 
+// The step between two sublayers for one row, and the router behind it when there is one: every wavefront
+// takes rows of the router's matrix (its first one asked for before the norms are worked out), the first one
+// then chooses.
+template <int NV>
+__global__ __launch_bounds__(STEP_THREADS) void residual_step_kernel(float* __restrict__ x, bf16_t* __restrict__ h, sublayer_rows src,
+                                                                     const float* __restrict__ w_after,
+                                                                     const float* __restrict__ w_next, row_shape rs, router_step rt) {
+  constexpr int TH = STEP_THREADS, AHEAD = 8;  // 16-byte pieces of a router row a lane asks for ahead: 4096 columns
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float z[ROUTER_MAX_ROWS];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  row_t<NV, TH> m, t, old, after, next;
+  load_row(after, w_after, rs);
+  load_row(old, x, rs);
+  if (w_next) load_row(next, w_next, rs);
+  load_sum(m, t, src, 0, rs);
+  bf16x8_t ahead[AHEAD];
+  const bf16_t* first = rt.w + (size_t)min(wave, rt.rows - 1) * rs.ld;
+  if (rt.w) {
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a) ahead[a] = *reinterpret_cast<const bf16x8_t*>(first + min((a * WAVE + lane) * 8, rs.ld - 8));
+  }
+  scale_row(m, rs, lds, after);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) m.v[j] += old.v[j];
+  store_row(x, m, rs);
+  if (!w_next) return;
+  scale_row(m, rs, lds, next);
+  store_row(h, m, rs);
+  if (!rt.w) return;
+  bf16_t* hs = reinterpret_cast<bf16_t*>(lds);  // scale_row is done with it
+  store_row(hs, m, rs);
+  __syncthreads();
+  for (int e = wave; e < rt.rows; e += TH / WAVE) {
+    const bf16_t* we = rt.w + (size_t)e * rs.ld;
+    float s = 0.0f;
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a) {
+      const int c = (a * WAVE + lane) * 8;
+      if (c < rs.ld) {
+        const bf16x8_t wv = e == wave ? ahead[a] : *reinterpret_cast<const bf16x8_t*>(we + c);
+        const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(hs + c);
+#pragma unroll
+        for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
+      }
+    }
+    for (int c = (AHEAD * WAVE + lane) * 8; c < rs.ld; c += WAVE * 8) {
+      const bf16x8_t wv = *reinterpret_cast<const bf16x8_t*>(we + c), hv = *reinterpret_cast<const bf16x8_t*>(hs + c);
+#pragma unroll
+      for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
+    }
+    s = wave_sum(s);
+    if (lane == 0) z[e] = s;
+  }
+  __syncthreads();
+  if (wave != 0) return;
+  if (rt.shared_gate && lane == 0) *rt.shared_gate = sigmoid_f32(z[rt.experts]);
+  choose_experts(z, rt.experts, rt.top, rt.expert, rt.weight);
+}
+
 // h[i] = norm(x[rows[i]]) under w (rows NULL: row i)
-template <class T, int NV>
-__global__ __launch_bounds__(ROW_THREADS) void group_norm_kernel(T* __restrict__ h, const float* __restrict__ x,
+template <class T, int NV, int TH>
+__global__ __launch_bounds__(TH) void group_norm_kernel(T* __restrict__ h, const float* __restrict__ x,
                                                                  const int* __restrict__ rows, const float* __restrict__ w,
                                                                  row_shape rs) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = rows ? rows[blockIdx.x] : blockIdx.x;
-  row_t<NV> row, wr;
+  row_t<NV, TH> row, wr;
   load_row(row, x + (size_t)r * rs.ld, rs);
   load_row(wr, w, rs);
   scale_row(row, rs, lds, wr);
   store_row(h + (size_t)blockIdx.x * rs.ld, row, rs);
 }
 
-// calls f with a null pointer of the element type and the pieces of a row
+// calls f with a null pointer of the element type, the pieces of a row and the threads that share it
 template <class F>
-void with_row_kind(int dtype, int ld, F&& f) {
-  with_row_pieces(ld, [&](auto nv) {
+void with_row_kind(int dtype, int ld, bool single, F&& f) {
+  const auto typed = [&](auto nv, auto th) {
     if (dtype == LCU_F32) {
-      f((float*)nullptr, nv);
+      f((float*)nullptr, nv, th);
     } else {
-      f((bf16_t*)nullptr, nv);
+      f((bf16_t*)nullptr, nv, th);
     }
-  });
+  };
+  if (single) {
+    with_step_pieces(ld, [&](auto nv) { typed(nv, std::integral_constant<int, STEP_THREADS>{}); });
+  } else {
+    with_row_pieces(ld, [&](auto nv) { typed(nv, std::integral_constant<int, ROW_THREADS>{}); });
+  }
 }
 
 // index = the first maximum of n fp32 values
@@ -211,9 +282,9 @@ int lcu_embed_pos_norm(void* x_dev, void* h_dev, const void* ids_dev, int n_ids,
   LCU_REQUIRE(n_vocab > 0 && n_pos > 0, "lcu_embed_pos_norm: bad table sizes %d %d", n_vocab, n_pos);
   if (n_ids == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
-  with_row_kind(dtype, ld, [&](auto* kind, auto nv) {
+  with_row_kind(dtype, ld, n_ids == 1, [&](auto* kind, auto nv, auto th) {
     using T = std::remove_pointer_t<decltype(kind)>;
-    embed_pos_norm_kernel<T, decltype(nv)::value><<<n_ids, ROW_THREADS, row_lds_bytes(rs), st>>>(
+    embed_pos_norm_kernel<T, decltype(nv)::value, decltype(th)::value><<<n_ids, decltype(th)::value, row_lds_bytes(rs), st>>>(
         (float*)x_dev, (T*)h_dev, (const int*)ids_dev, (const T*)table_dev, (const T*)pos_table_dev, (const float*)w_embed_dev,
         (const float*)w_next_dev, (const int*)start_dev, n_vocab, n_pos, rs);
   });
@@ -230,13 +301,43 @@ int lcu_residual_norm(void* x_dev, void* h_dev, const void* out_f32_dev, const v
   const int rc = check_rows("lcu_residual_norm", dtype, rows, rs);
   if (rc) return rc;
   if (rows == 0) return LCU_OK;
+  LCU_REQUIRE(top >= 1, "lcu_residual_norm: %d rows per token", top);
   const sublayer_rows src{(const float*)out_f32_dev, (const int*)inverse_dev, top, (const float*)shared_f32_dev,
                           (const float*)shared_gate_dev};
   hipStream_t st = as_stream(stream);
-  with_row_kind(dtype, ld, [&](auto* kind, auto nv) {
+  with_row_kind(dtype, ld, rows == 1, [&](auto* kind, auto nv, auto th) {
     using T = std::remove_pointer_t<decltype(kind)>;
-    residual_norm_kernel<T, decltype(nv)::value><<<rows, ROW_THREADS, row_lds_bytes(rs), st>>>(
+    residual_norm_kernel<T, decltype(nv)::value, decltype(th)::value><<<rows, decltype(th)::value, row_lds_bytes(rs), st>>>(
         (float*)x_dev, (T*)h_dev, src, (const float*)w_after_dev, (const float*)w_next_dev, rs);
+  });
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+int lcu_decode_residual_router(void* x_dev, void* h_dev, const void* out_f32_dev, int top, const void* shared_f32_dev,
+                               const void* shared_gate_dev, const void* w_after_dev, const void* w_next_dev, int width, int ld,
+                               int groups, float eps, const void* router_w_dev, int n_experts, int choose, void* expert_dev,
+                               void* weight_dev, void* router_gate_dev, void* stream) {
+  LCU_REQUIRE(x_dev && out_f32_dev && w_after_dev && (h_dev || !w_next_dev) && (!shared_f32_dev || shared_gate_dev) &&
+                  (!router_w_dev || (w_next_dev && expert_dev && weight_dev)),
+              "lcu_decode_residual_router: null pointer");
+  const row_shape rs{width, ld, groups, eps};
+  const int rc = check_rows("lcu_decode_residual_router", LCU_BF16, 1, rs);
+  if (rc) return rc;
+  router_step rt{};
+  if (router_w_dev) {
+    rt = router_step{(const bf16_t*)router_w_dev, n_experts + (router_gate_dev ? 1 : 0), n_experts, choose, (int*)expert_dev,
+                     (float*)weight_dev, (float*)router_gate_dev};
+    LCU_REQUIRE(n_experts > 0 && rt.rows <= ROUTER_MAX_ROWS && choose > 0 && choose <= n_experts,
+                "lcu_decode_residual_router: experts %d (at most %d), top %d", n_experts, ROUTER_MAX_ROWS - 1, choose);
+  }
+  LCU_REQUIRE(top >= 1, "lcu_decode_residual_router: %d rows", top);
+  const sublayer_rows src{(const float*)out_f32_dev, nullptr, top, (const float*)shared_f32_dev, (const float*)shared_gate_dev};
+  size_t lds = row_lds_bytes(rs);
+  if (router_w_dev && lds < (size_t)ld * 2) lds = (size_t)ld * 2;
+  with_step_pieces(ld, [&](auto nv) {
+    residual_step_kernel<decltype(nv)::value><<<1, STEP_THREADS, lds, as_stream(stream)>>>(
+        (float*)x_dev, (bf16_t*)h_dev, src, (const float*)w_after_dev, (const float*)w_next_dev, rs, rt);
   });
   LCU_LAUNCH_CHECK();
   return LCU_OK;
@@ -250,9 +351,9 @@ int lcu_group_norm(void* h_dev, const void* x_f32_dev, const void* row_index_dev
   if (rc) return rc;
   if (rows == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
-  with_row_kind(dtype, ld, [&](auto* kind, auto nv) {
+  with_row_kind(dtype, ld, rows == 1, [&](auto* kind, auto nv, auto th) {
     using T = std::remove_pointer_t<decltype(kind)>;
-    group_norm_kernel<T, decltype(nv)::value><<<rows, ROW_THREADS, row_lds_bytes(rs), st>>>(
+    group_norm_kernel<T, decltype(nv)::value, decltype(th)::value><<<rows, decltype(th)::value, row_lds_bytes(rs), st>>>(
         (T*)h_dev, (const float*)x_f32_dev, (const int*)row_index_dev, (const float*)w_dev, rs);
   });
   LCU_LAUNCH_CHECK();

@@ -1,11 +1,11 @@
-// Grouped RMS norm of one row by one 256-thread workgroup.
+// Grouped RMS norm of one row by one workgroup, the row in registers.
 #pragma once
 #include "common.hpp"
 
 namespace lcu {
 
-constexpr int ROW_THREADS = 256;
-constexpr int ROW_WAVES = ROW_THREADS / WAVE;
+constexpr int ROW_THREADS = 256;    // many rows: a workgroup each
+constexpr int STEP_THREADS = 1024;  // a single row: the launch is nothing but latency
 constexpr int ROW_MAX_WIDTH = 12288;
 constexpr int ROW_MAX_GROUPS = 2048;
 constexpr int ROW_PIECE = WAVE * 4;  // columns a wavefront holds per register piece
@@ -18,18 +18,18 @@ struct row_shape {
 // where a sublayer left its result
 struct sublayer_rows {
   const float* out;
-  const int* inverse;  // NULL: row r of out; else top rows of out per token
+  const int* inverse;  // top rows of out per token: rows inverse[r * top + k], or r * top + k when NULL
   int top;
   const float* shared;
   const float* shared_gate;
 };
 
 // A row spread over the workgroup's registers: piece j of thread t holds the four columns from
-// (t + 256 j) * 4.  Columns at or beyond the width hold zeros.
-template <int NV>
+// (t + TH j) * 4 (TH threads).  Columns at or beyond the width hold zeros.
+template <int NV, int TH>
 struct row_t {
   float4_t v[NV];
-  static __device__ __forceinline__ int column(int j) { return (int)(threadIdx.x + ROW_THREADS * j) * 4; }
+  static __device__ __forceinline__ int column(int j) { return (int)(threadIdx.x + TH * j) * 4; }
 };
 
 __device__ __forceinline__ float4_t load4(const float* p) { return *reinterpret_cast<const float4_t*>(p); }
@@ -51,16 +51,16 @@ __device__ __forceinline__ void store4(bf16_t* p, float4_t v) {
 
 // Rows have a padded stride (a multiple of 64 elements), so whole pieces up to ld may be read and written;
 // vectors of the width (norm weights) are padded by their owners to ld too.
-template <int NV, class T>
-__device__ __forceinline__ void load_row(row_t<NV>& r, const T* p, const row_shape& rs) {
+template <int NV, int TH, class T>
+__device__ __forceinline__ void load_row(row_t<NV, TH>& r, const T* p, const row_shape& rs) {
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int c = r.column(j);
     r.v[j] = c < rs.ld ? load4(p + c) : (float4_t)(0.0f);
   }
 }
-template <int NV, class T>
-__device__ __forceinline__ void store_row(T* p, const row_t<NV>& r, const row_shape& rs) {
+template <int NV, int TH, class T>
+__device__ __forceinline__ void store_row(T* p, const row_t<NV, TH>& r, const row_shape& rs) {
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int c = r.column(j);
@@ -79,8 +79,9 @@ inline size_t row_lds_bytes(const row_shape& rs) {
 // row <- row / sqrt(mean of its part's squares + eps) * w.  Parts that are whole pieces of a wavefront (256
 // columns) are summed in registers; other sizes go through LDS column by column.  `lds` may be reused right
 // after an earlier call.
-template <int NV>
-__device__ __forceinline__ void scale_row(row_t<NV>& r, const row_shape& rs, float* lds, const row_t<NV>& w) {
+template <int NV, int TH>
+__device__ __forceinline__ void scale_row(row_t<NV, TH>& r, const row_shape& rs, float* lds, const row_t<NV, TH>& w) {
+  constexpr int WAVES = TH / WAVE;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, part = rs.width / rs.groups;
   if (part % ROW_PIECE == 0) {
     float* piece = lds;
@@ -88,13 +89,13 @@ __device__ __forceinline__ void scale_row(row_t<NV>& r, const row_shape& rs, flo
     for (int j = 0; j < NV; ++j) {
       const float4_t q = r.v[j] * r.v[j];
       const float s = wave_sum((q[0] + q[1]) + (q[2] + q[3]));
-      if (lane == 0 && r.column(j) < rs.ld) piece[j * ROW_WAVES + wave] = s;
+      if (lane == 0 && r.column(j) < rs.ld) piece[j * WAVES + wave] = s;
     }
     __syncthreads();
     const int per = part / ROW_PIECE;
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
-      const int g = __builtin_amdgcn_readfirstlane((j * ROW_WAVES + wave) / per);
+      const int g = __builtin_amdgcn_readfirstlane((j * WAVES + wave) / per);
       if (g < rs.groups) {
         float total = 0.0f;
         for (int k = 0; k < per; ++k) total += piece[g * per + k];
@@ -112,7 +113,7 @@ __device__ __forceinline__ void scale_row(row_t<NV>& r, const row_shape& rs, flo
     if (c < rs.ld) store4(sq + c, r.v[j] * r.v[j]);
   }
   __syncthreads();
-  for (int g = wave; g < rs.groups; g += ROW_WAVES) {
+  for (int g = wave; g < rs.groups; g += WAVES) {
     float s = 0.0f;
     for (int i = lane; i < part; i += WAVE) s += sq[g * part + i];
     s = wave_sum(s);
@@ -145,6 +146,17 @@ void with_row_pieces(int ld, F&& f) {
     f(std::integral_constant<int, 12>{});
   }
 }
+// the same for STEP_THREADS threads
+template <class F>
+void with_step_pieces(int ld, F&& f) {
+  if (ld <= 4096) {
+    f(std::integral_constant<int, 1>{});
+  } else if (ld <= 8192) {
+    f(std::integral_constant<int, 2>{});
+  } else {
+    f(std::integral_constant<int, 3>{});
+  }
+}
 
 // ---- which workgroup arrives last -------------------------------------------------------------------
 // Counters of a launch whose last workgroup goes on with the others' results: ARRIVAL_LANES first-level
@@ -156,14 +168,18 @@ constexpr int ARRIVAL_WORDS = (ARRIVAL_LANES + 1) * ARRIVAL_STRIDE;
 
 // Called by one thread after the workgroup's device-scope stores are complete.
 __device__ __forceinline__ bool arrives_last(uint32_t* counters, uint32_t block, uint32_t blocks) {
+  uint32_t* top = counters + ARRIVAL_LANES * ARRIVAL_STRIDE;
+  if (blocks <= ARRIVAL_LANES) {  // few enough for one word
+    if (__hip_atomic_fetch_add(top, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != blocks - 1) return false;
+    __hip_atomic_store(top, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    return true;
+  }
   const uint32_t lane = block % ARRIVAL_LANES;
   const uint32_t mine = blocks / ARRIVAL_LANES + (lane < blocks % ARRIVAL_LANES ? 1u : 0u);
   uint32_t* c = counters + lane * ARRIVAL_STRIDE;
   if (__hip_atomic_fetch_add(c, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != mine - 1) return false;
   __hip_atomic_store(c, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  uint32_t* top = counters + ARRIVAL_LANES * ARRIVAL_STRIDE;
-  const uint32_t full = blocks < ARRIVAL_LANES ? blocks : ARRIVAL_LANES;
-  if (__hip_atomic_fetch_add(top, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != full - 1) return false;
+  if (__hip_atomic_fetch_add(top, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != ARRIVAL_LANES - 1) return false;
   __hip_atomic_store(top, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   return true;
 }

@@ -8,6 +8,7 @@
 // to 32, 64, 128 or 256; the padding holds zeros.  A head's visible keys are the first ones, [0, kept), and
 // the window [lo, i]: every kernel walks exactly these.
 #include <algorithm>
+#include <type_traits>
 
 #include "linear.hpp"
 #include "rownorm.hpp"
@@ -32,29 +33,31 @@ __device__ __forceinline__ int window_begin(const window_args& p, int i) { retur
 // v_first when MIX_WITH: (1 - lambda) v + lambda v_first; KEEP_AS_FIRST leaves the projected v in v_first.
 enum v_mode { V_PLAIN = 0, V_KEEP_AS_FIRST = 1, V_MIX_WITH_FIRST = 2 };
 
-template <class T>
-__device__ __forceinline__ float mixed_value(float v, T* v_first, int mode, float lambda) {
-  if (mode == V_KEEP_AS_FIRST) *v_first = (T)v;
-  if (mode == V_MIX_WITH_FIRST) v = (1.0f - lambda) * v + lambda * to_f32(*v_first);
-  return v;
-}
-
+// four columns per thread (column counts are multiples of 32)
 template <class T>
 __global__ __launch_bounds__(256) void kv_store_kernel(T* __restrict__ k_cache, T* __restrict__ v_cache, const T* __restrict__ qkv,
                                                        int ldq, int q_cols, int k_cols, int v_cols, T* __restrict__ v_first,
                                                        int mode, const float* __restrict__ lambda, const int* __restrict__ start,
-                                                       int max_pos) {
-  const int c = blockIdx.x * 256 + threadIdx.x, t = blockIdx.y;
-  if (c >= k_cols + v_cols) return;
+                                                       int max_pos, int n) {
+  const int per = (k_cols + v_cols) / 4, i = blockIdx.x * 256 + threadIdx.x;
+  if (i >= n * per) return;
+  const int t = i / per, c = (i - t * per) * 4;
   const size_t pos = min(max(*start + t, 0), max_pos - 1);
-  const T* row = qkv + (size_t)t * ldq + q_cols;
+  float4_t v = load4(qkv + (size_t)t * ldq + q_cols + c);
   if (c < k_cols) {
-    k_cache[pos * k_cols + c] = row[c];
-  } else {
-    const int vc = c - k_cols;
-    const float v = mixed_value(to_f32(row[c]), v_first + (size_t)t * v_cols + vc, mode, mode == V_MIX_WITH_FIRST ? *lambda : 0.0f);
-    v_cache[pos * v_cols + vc] = (T)v;
+    store4(k_cache + pos * k_cols + c, v);
+    return;
   }
+  const int vc = c - k_cols;
+  T* first = v_first + (size_t)t * v_cols + vc;
+  if (mode == V_KEEP_AS_FIRST) store4(first, v);
+  if (mode == V_MIX_WITH_FIRST) {
+    const float l = *lambda;
+    const float4_t f = load4(first);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = (1.0f - l) * v[e] + l * f[e];
+  }
+  store4(v_cache + pos * v_cols + vc, v);
 }
 
 // ---- one workgroup per (query row, head), plain fp32 arithmetic: the fp32 element type -----------------
@@ -251,159 +254,205 @@ int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, 
 }
 
 // ---- one new token, bfloat16 ----------------------------------------------------------------------------
-// Workgroup (kv head, slice of the visible keys): 16 lanes share a key row and score it for every query
-// head of the group (the row is read once for all of them); then the slice's maximum, sum and weighted
-// values per head go to part[kv head][slice][head][dv + 2], and the last workgroup of a kv head to arrive
-// adds the slices up (arrives_last).  Nobody waits.
-__device__ __forceinline__ float load_device(const float* p) {
-  return __hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-}
-// eight loads at device scope in flight together (see load_words_device_scope)
-__device__ __forceinline__ void load8_device(float (&o)[8], const float* const (&p)[8]) {
-  asm volatile(
-      "global_load_dword %0, %8, off sc0 sc1\n\tglobal_load_dword %1, %9, off sc0 sc1\n\t"
-      "global_load_dword %2, %10, off sc0 sc1\n\tglobal_load_dword %3, %11, off sc0 sc1\n\t"
-      "global_load_dword %4, %12, off sc0 sc1\n\tglobal_load_dword %5, %13, off sc0 sc1\n\t"
-      "global_load_dword %6, %14, off sc0 sc1\n\tglobal_load_dword %7, %15, off sc0 sc1\n\ts_waitcnt vmcnt(0)"
-      : "=&v"(o[0]), "=&v"(o[1]), "=&v"(o[2]), "=&v"(o[3]), "=&v"(o[4]), "=&v"(o[5]), "=&v"(o[6]), "=&v"(o[7])
-      : "v"(p[0]), "v"(p[1]), "v"(p[2]), "v"(p[3]), "v"(p[4]), "v"(p[5]), "v"(p[6]), "v"(p[7])
-      : "memory");
-}
-constexpr int DEC_MAX_SLICE = 256;   // keys of a slice
-constexpr int DEC_MAX_GROUP = 16;    // query heads per kv head
+// Workgroup (kv head, slice of the visible keys): 16 lanes share a key, eight columns each (DKP / DVP passes of
+// 128 columns), and score it for every query head of the group, so that a cache row is read once for all of
+// them; keys and values of DEC_FLIGHT rows per lane group are requested together, before anything is
+// computed.  Each of the 16 groups keeps a running maximum, sum and weighted values per head; the groups
+// meet in LDS, the slice's result goes to part[kv head][slice][head][dv + 4] (values, maximum, sum), and the
+// last workgroup of a kv head to arrive adds the slices up (arrives_last).  Nobody waits.
+constexpr int DEC_FLIGHT = 4;
+constexpr int DEC_MAX_SLICES = 64;
+constexpr int DEC_MAX_GROUP = 16;  // query heads per kv head
 
+template <int RMAX, int DKP, int DVP>
 __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                                                                const bf16_t* __restrict__ k, const bf16_t* __restrict__ v,
                                                                const int* __restrict__ pos_dev, int max_pos,
                                                                float* __restrict__ part, uint32_t* __restrict__ arrived,
                                                                window_args p) {
-  extern __shared__ float dec_lds[];
-  const int R = p.heads / p.kv_heads;
-  float* qs = dec_lds;                   // [R][dk]
-  float* sc = qs + R * p.dk;             // [R][DEC_MAX_SLICE]
-  float* ov = sc + R * DEC_MAX_SLICE;    // [4][R][dv]
+  extern __shared__ __attribute__((aligned(16))) float dec_lds[];  // [16 groups][R][dv], then [16][R][2]
   __shared__ bool last;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int R = p.heads / p.kv_heads;
+  const int tid = threadIdx.x, sub = tid & 15, grp = tid >> 4;
   const int g = blockIdx.x, slice = blockIdx.y, slices = gridDim.y;
   const int i = min(max(*pos_dev, 0), max_pos - 1);
   const int lo = window_begin(p, i), kept = min(p.keep, lo), n_keys = kept + i - lo + 1;
   const int per = (n_keys + slices - 1) / slices;
-  const int x0 = slice * per, cnt = max(0, min(per, n_keys - x0));
-  for (int c = tid; c < R * p.dk; c += 256) qs[c] = (float)q[(size_t)g * R * p.dk + c];
-  __syncthreads();
-  const int sub = lane & 15, grp = tid >> 4;
-  for (int x = grp; x < cnt; x += 16) {
-    const int xi = x0 + x, j = xi < kept ? xi : lo + xi - kept;
-    const bf16_t* kr = k + ((size_t)j * p.kv_heads + g) * p.dk;
-    float s[DEC_MAX_GROUP];
+  const int x0 = slice * per, x1 = min(x0 + per, n_keys);
+  const bool k_lane[2] = {sub * 8 < p.dk, 128 + sub * 8 < p.dk}, v_lane[2] = {sub * 8 < p.dv, 128 + sub * 8 < p.dv};
+  bf16x8_t qv[RMAX][DKP];
 #pragma unroll
-    for (int r = 0; r < DEC_MAX_GROUP; ++r) s[r] = 0.0f;
-    for (int c = sub * 8; c < p.dk; c += 128) {
-      const bf16x8_t kv = *reinterpret_cast<const bf16x8_t*>(kr + c);
+  for (int r = 0; r < RMAX; ++r) {
 #pragma unroll
-      for (int r = 0; r < DEC_MAX_GROUP; ++r) {
-        if (r < R) {
+    for (int d = 0; d < DKP; ++d) {
+      qv[r][d] = r < R && k_lane[d] ? *reinterpret_cast<const bf16x8_t*>(q + ((size_t)g * R + r) * p.dk + d * 128 + sub * 8) : (bf16x8_t)(0.0f);
+    }
+  }
+  float m[RMAX], l[RMAX], o[RMAX][DVP][8], r1[RMAX], r2[RMAX];
 #pragma unroll
-          for (int e = 0; e < 8; ++e) s[r] = fmaf(qs[r * p.dk + c + e], (float)kv[e], s[r]);
+  for (int r = 0; r < RMAX; ++r) {
+    m[r] = -1e30f;
+    l[r] = 0.0f;
+    r1[r] = p.r1[g * R + min(r, R - 1)];
+    r2[r] = p.r2[g * R + min(r, R - 1)];
+#pragma unroll
+    for (int d = 0; d < DVP; ++d) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[r][d][e] = 0.0f;
+    }
+  }
+  for (int xb = x0; xb < x1; xb += 16 * DEC_FLIGHT) {
+    bf16x8_t kv[DEC_FLIGHT][DKP], vv[DEC_FLIGHT][DVP];
+    int j[DEC_FLIGHT];
+#pragma unroll
+    for (int f = 0; f < DEC_FLIGHT; ++f) {
+      const int x = min(xb + f * 16 + grp, x1 - 1);
+      j[f] = x < kept ? x : lo + x - kept;
+      const bf16_t* kr = k + ((size_t)j[f] * p.kv_heads + g) * p.dk + sub * 8;
+#pragma unroll
+      for (int d = 0; d < DKP; ++d) kv[f][d] = k_lane[d] ? *reinterpret_cast<const bf16x8_t*>(kr + d * 128) : (bf16x8_t)(0.0f);
+    }
+#pragma unroll
+    for (int f = 0; f < DEC_FLIGHT; ++f) {
+      const bf16_t* vr = v + ((size_t)j[f] * p.kv_heads + g) * p.dv + sub * 8;
+#pragma unroll
+      for (int d = 0; d < DVP; ++d) vv[f][d] = v_lane[d] ? *reinterpret_cast<const bf16x8_t*>(vr + d * 128) : (bf16x8_t)(0.0f);
+    }
+#pragma unroll
+    for (int r = 0; r < RMAX; ++r) {
+      if (r < R) {
+        float s[DEC_FLIGHT], top = m[r];
+#pragma unroll
+        for (int f = 0; f < DEC_FLIGHT; ++f) {
+          float d0 = 0.0f;
+#pragma unroll
+          for (int d = 0; d < DKP; ++d) {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) d0 = fmaf((float)qv[r][d][e], (float)kv[f][d][e], d0);
+          }
+          s[f] = row16_sum(d0) * p.scale - r1[r] * log1pf(r2[r] * (float)(i - j[f]));
+          if (xb + f * 16 + grp < x1) top = fmaxf(top, s[f]);
+        }
+        const float shrink = expf(m[r] - top);
+        m[r] = top;
+        l[r] *= shrink;
+#pragma unroll
+        for (int d = 0; d < DVP; ++d) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) o[r][d][e] *= shrink;
+        }
+#pragma unroll
+        for (int f = 0; f < DEC_FLIGHT; ++f) {
+          const float w = xb + f * 16 + grp < x1 ? expf(s[f] - top) : 0.0f;
+          l[r] += w;
+#pragma unroll
+          for (int d = 0; d < DVP; ++d) {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[r][d][e] = fmaf(w, (float)vv[f][d][e], o[r][d][e]);
+          }
         }
       }
     }
+  }
+  float* ml = dec_lds + 16 * R * p.dv;
 #pragma unroll
-    for (int r = 0; r < DEC_MAX_GROUP; ++r) {
-      if (r < R) {
-        const float d = row16_sum(s[r]);
-        if (sub == 0) sc[r * DEC_MAX_SLICE + x] = d * p.scale - p.r1[g * R + r] * log1pf(p.r2[g * R + r] * (float)(i - j));
+  for (int r = 0; r < RMAX; ++r) {
+    if (r < R) {
+#pragma unroll
+      for (int d = 0; d < DVP; ++d) {
+        if (v_lane[d]) {
+          float* dst = dec_lds + ((size_t)grp * R + r) * p.dv + d * 128 + sub * 8;
+          store4(dst, (float4_t){o[r][d][0], o[r][d][1], o[r][d][2], o[r][d][3]});
+          store4(dst + 4, (float4_t){o[r][d][4], o[r][d][5], o[r][d][6], o[r][d][7]});
+        }
+      }
+      if (sub == 0) {
+        ml[(grp * R + r) * 2] = m[r];
+        ml[(grp * R + r) * 2 + 1] = l[r];
       }
     }
   }
   __syncthreads();
-  float* pg = part + (size_t)(g * slices + slice) * R * (p.dv + 2);
-  for (int r = wave; r < R; r += 4) {
-    float m = -1e30f;
-    for (int x = lane; x < cnt; x += WAVE) m = fmaxf(m, sc[r * DEC_MAX_SLICE + x]);
-    m = wave_max_dpp(m);
-    float l = 0.0f;
-    for (int x = lane; x < cnt; x += WAVE) {
-      const float e = expf(sc[r * DEC_MAX_SLICE + x] - m);
-      sc[r * DEC_MAX_SLICE + x] = e;
-      l += e;
-    }
-    l = wave_sum(l);
-    if (lane == 0) {
-      __hip_atomic_store(pg + r * (p.dv + 2) + p.dv, m, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      __hip_atomic_store(pg + r * (p.dv + 2) + p.dv + 1, l, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    }
-  }
-  __syncthreads();
-  // weighted values: wavefront w takes keys w, w + 4, ...; a lane owns columns lane, lane + 64, ...
-  for (int c = lane; c < p.dv; c += WAVE) {
-    float o[DEC_MAX_GROUP];
-#pragma unroll
-    for (int r = 0; r < DEC_MAX_GROUP; ++r) o[r] = 0.0f;
-#pragma unroll 4
-    for (int x = wave; x < cnt; x += 4) {
-      const int xi = x0 + x, j = xi < kept ? xi : lo + xi - kept;
-      const float vv = (float)v[((size_t)j * p.kv_heads + g) * p.dv + c];
-#pragma unroll
-      for (int r = 0; r < DEC_MAX_GROUP; ++r) {
-        if (r < R) o[r] = fmaf(sc[r * DEC_MAX_SLICE + x], vv, o[r]);
-      }
-    }
-#pragma unroll
-    for (int r = 0; r < DEC_MAX_GROUP; ++r) {
-      if (r < R) ov[(wave * R + r) * p.dv + c] = o[r];
-    }
-  }
-  __syncthreads();
+  const int ldp = p.dv + 4;
+  float* pg = part + (size_t)(g * slices + slice) * R * ldp;
   for (int c = tid; c < R * p.dv; c += 256) {
-    const int rd = R * p.dv;
-    const float o = (ov[c] + ov[rd + c]) + (ov[2 * rd + c] + ov[3 * rd + c]);
-    __hip_atomic_store(pg + (c / p.dv) * (p.dv + 2) + c % p.dv, o, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    const int r = c / p.dv, e = c - r * p.dv;
+    float mx = -1e30f;
+#pragma unroll
+    for (int w = 0; w < 16; ++w) mx = fmaxf(mx, ml[(w * R + r) * 2]);
+    float sum = 0.0f, val = 0.0f;
+#pragma unroll
+    for (int w = 0; w < 16; ++w) {
+      const float f = expf(ml[(w * R + r) * 2] - mx);
+      sum = fmaf(f, ml[(w * R + r) * 2 + 1], sum);
+      val = fmaf(f, dec_lds[((size_t)w * R + r) * p.dv + e], val);
+    }
+    __hip_atomic_store(pg + r * ldp + e, val, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (e == 0) {
+      __hip_atomic_store(pg + r * ldp + p.dv, mx, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      __hip_atomic_store(pg + r * ldp + p.dv + 1, sum, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    }
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // every wavefront's stores are out before the count goes up
   __syncthreads();
   if (tid == 0) last = arrives_last(arrived + (size_t)g * ARRIVAL_WORDS, slice, slices);
   __syncthreads();
   if (!last) return;
-  // factor and share of every slice, per head; then the columns
-  const float* all = part + (size_t)g * slices * R * (p.dv + 2);
-  float* sm = sc;              // [R][slices]: maxima, then factors (a slice is at most DEC_MAX_SLICE keys, and so are the slices)
-  float* sl = dec_lds;         // [R]: sums (q is done with)
-  for (int c = tid; c < R * slices; c += 256) {
-    const int r = c / slices, s = c % slices;
-    sm[r * DEC_MAX_SLICE + s] = load_device(all + ((size_t)s * R + r) * (p.dv + 2) + p.dv);
-  }
-  __syncthreads();
-  for (int r = wave; r < R; r += 4) {
-    float m = -1e30f;
-    for (int s = lane; s < slices; s += WAVE) m = fmaxf(m, sm[r * DEC_MAX_SLICE + s]);
-    m = wave_max_dpp(m);
-    float l = 0.0f;
-    for (int s = lane; s < slices; s += WAVE) {
-      const float f = expf(sm[r * DEC_MAX_SLICE + s] - m);
-      l += f * load_device(all + ((size_t)s * R + r) * (p.dv + 2) + p.dv + 1);
-      sm[r * DEC_MAX_SLICE + s] = f;
-    }
-    l = wave_sum(l);
-    if (lane == 0) sl[r] = l;
-  }
-  __syncthreads();
-  for (int c = tid; c < R * p.dv; c += 256) {
-    const int r = c / p.dv, e = c % p.dv;
-    float o = 0.0f;
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");  // ordinary loads from here on see the other workgroups' stores
+  const float* all = part + (size_t)g * slices * R * ldp;
+  const int quads = p.dv / 4;
+  for (int c = tid; c < R * quads; c += 256) {
+    const int r = c / quads, e = (c - r * quads) * 4;
+    float mx = -1e30f, sum = 0.0f;
+    float4_t val = (float4_t)(0.0f);
     for (int s0 = 0; s0 < slices; s0 += 8) {
-      float v[8];
-      const float* at[8];
+      float4_t pv[8];
+      float pm[8], pl[8];
 #pragma unroll
-      for (int k = 0; k < 8; ++k) at[k] = all + ((size_t)min(s0 + k, slices - 1) * R + r) * (p.dv + 2) + e;
-      load8_device(v, at);
+      for (int b = 0; b < 8; ++b) {
+        const float* src = all + ((size_t)min(s0 + b, slices - 1) * R + r) * ldp;
+        pv[b] = load4(src + e);
+        pm[b] = src[p.dv];
+        pl[b] = src[p.dv + 1];
+      }
 #pragma unroll
-      for (int k = 0; k < 8; ++k) {
-        if (s0 + k < slices) o = fmaf(sm[r * DEC_MAX_SLICE + s0 + k], v[k], o);
+      for (int b = 0; b < 8; ++b) {
+        if (s0 + b < slices) {
+          const float now = fmaxf(mx, pm[b]), was = expf(mx - now), f = expf(pm[b] - now);
+          sum = sum * was + f * pl[b];
+          val = val * was + f * pv[b];
+          mx = now;
+        }
       }
     }
-    out[(size_t)(g * R + r) * p.dv + e] = (bf16_t)(o / sl[r]);
+    store4(out + ((size_t)g * R + r) * p.dv + e, val * (1.0f / sum));
   }
+}
+
+template <int DKP, int DVP>
+int launch_decode(bf16_t* out, const bf16_t* q, const bf16_t* k, const bf16_t* v, const int* pos, int max_pos, float* part,
+                  uint32_t* arrived, const window_args& p, int slices, hipStream_t st) {
+  const int R = p.heads / p.kv_heads;
+  const size_t lds = (size_t)16 * R * (p.dv + 2) * sizeof(float);
+  const auto go = [&](auto rmax) -> int {
+    auto kernel = attention_decode_kernel<decltype(rmax)::value, DKP, DVP>;
+    if (lds > 64 * 1024) {
+      static bool raised[16] = {};  // per device, once
+      int dev = 0;
+      LCU_HIP(hipGetDevice(&dev));
+      if (!raised[dev & 15]) {
+        LCU_HIP(hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024));
+        raised[dev & 15] = true;
+      }
+    }
+    kernel<<<dim3(p.kv_heads, slices), 256, lds, st>>>(out, q, k, v, pos, max_pos, part, arrived, p);
+    LCU_LAUNCH_CHECK();
+    return LCU_OK;
+  };
+  if (R <= 1) return go(std::integral_constant<int, 1>{});
+  if (R <= 4) return go(std::integral_constant<int, 4>{});
+  if (R <= 8) return go(std::integral_constant<int, 8>{});
+  return go(std::integral_constant<int, DEC_MAX_GROUP>{});
 }
 
 int check_window(const char* who, const lcu_window_params* w, int dtype) {
@@ -436,16 +485,17 @@ int lcu_kv_store(void* k_cache_dev, void* v_cache_dev, const void* qkv_dev, int 
                   ldq >= q_cols + k_cols + v_cols && (dtype == LCU_BF16 || dtype == LCU_F32),
               "lcu_kv_store: bad shape n %d of %d, columns %d %d %d of %d", n, max_positions, q_cols, k_cols, v_cols, ldq);
   if (n == 0) return LCU_OK;
-  const dim3 grid((k_cols + v_cols + 255) / 256, n);
+  LCU_REQUIRE(k_cols % 4 == 0 && v_cols % 4 == 0 && q_cols % 4 == 0 && ldq % 4 == 0, "lcu_kv_store: columns in groups of four");
+  const unsigned grid = (unsigned)(((size_t)n * ((k_cols + v_cols) / 4) + 255) / 256);
   hipStream_t st = as_stream(stream);
   if (dtype == LCU_F32) {
     kv_store_kernel<float><<<grid, 256, 0, st>>>((float*)k_cache_dev, (float*)v_cache_dev, (const float*)qkv_dev, ldq, q_cols, k_cols,
                                                  v_cols, (float*)v_first_dev, v_mode, (const float*)lambda_dev,
-                                                 (const int*)start_dev, max_positions);
+                                                 (const int*)start_dev, max_positions, n);
   } else {
     kv_store_kernel<bf16_t><<<grid, 256, 0, st>>>((bf16_t*)k_cache_dev, (bf16_t*)v_cache_dev, (const bf16_t*)qkv_dev, ldq, q_cols,
                                                   k_cols, v_cols, (bf16_t*)v_first_dev, v_mode, (const float*)lambda_dev,
-                                                  (const int*)start_dev, max_positions);
+                                                  (const int*)start_dev, max_positions, n);
   }
   LCU_LAUNCH_CHECK();
   return LCU_OK;
@@ -499,27 +549,22 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
   if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_attention_windowed_decode: lcu_init has not run on this device");
   const long seen = (long)window->window + window->keep;
   const int most = (int)(seen < max_positions ? seen : max_positions);  // visible keys of any position
-  // slices: enough workgroups for the chip, at least 32 keys each, never more keys than a slice holds
-  int slices = std::min((most + 31) / 32, (256 + window->kv_heads - 1) / window->kv_heads);
-  slices = std::max(slices, (most + DEC_MAX_SLICE - 1) / DEC_MAX_SLICE);
-  const size_t need = (size_t)window->heads * slices * (window->dv + 2) * sizeof(float);
-  const size_t lds = ((size_t)R * (window->dk + DEC_MAX_SLICE + 4 * window->dv)) * sizeof(float);
-  LCU_REQUIRE(need <= ws.bytes && slices <= DEC_MAX_SLICE, "lcu_attention_windowed_decode: %d slices do not fit the workspace", slices);
-  LCU_REQUIRE(lds <= 128 * 1024, "lcu_attention_windowed_decode: %d heads of %d / %d per kv head", R, window->dk, window->dv);
-  static bool raised[16] = {};
-  int dev = 0;
-  LCU_HIP(hipGetDevice(&dev));
-  if (!raised[dev & 15]) {
-    LCU_HIP(hipFuncSetAttribute((const void*)attention_decode_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024));
-    raised[dev & 15] = true;
-  }
+  // a slice for every 64 keys, while that does not take more than one workgroup per compute unit
+  const int slices = std::min(std::min((most + 63) / 64, (256 + window->kv_heads - 1) / window->kv_heads), DEC_MAX_SLICES);
+  const size_t need = (size_t)window->heads * slices * (window->dv + 4) * sizeof(float);
+  LCU_REQUIRE(need <= ws.bytes, "lcu_attention_windowed_decode: %d slices do not fit the workspace", slices);
+  LCU_REQUIRE((size_t)16 * R * (window->dv + 2) * sizeof(float) <= 150 * 1024,
+              "lcu_attention_windowed_decode: %d query heads per kv head with value size %d", R, window->dv);
   const window_args p = make_window(window, window->heads * window->dk, window->heads * window->dv);
-  attention_decode_kernel<<<dim3(window->kv_heads, slices), 256, lds, st>>>((bf16_t*)out_dev, (const bf16_t*)q_dev,
-                                                                           (const bf16_t*)k_cache_dev, (const bf16_t*)v_cache_dev,
-                                                                           (const int*)pos_dev, max_positions, (float*)ws.ptr,
-                                                                           (uint32_t*)arrived_dev, p);
-  LCU_LAUNCH_CHECK();
-  return LCU_OK;
+  const auto run = [&](auto dkp, auto dvp) {
+    return launch_decode<decltype(dkp)::value, decltype(dvp)::value>(
+        (bf16_t*)out_dev, (const bf16_t*)q_dev, (const bf16_t*)k_cache_dev, (const bf16_t*)v_cache_dev, (const int*)pos_dev,
+        max_positions, (float*)ws.ptr, (uint32_t*)arrived_dev, p, slices, st);
+  };
+  const std::integral_constant<int, 1> one;
+  const std::integral_constant<int, 2> two;
+  if (window->dk <= 128) return window->dv <= 128 ? run(one, one) : run(one, two);
+  return window->dv <= 128 ? run(two, one) : run(two, two);
 }
 
 }  // extern "C"

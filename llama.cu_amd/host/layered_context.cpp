@@ -60,7 +60,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   t_scratch_ = zeroed(scratch);
   t_hidden_ = zeroed(hidden * e);
   t_shared_hidden_ = zeroed(shared * e);
-  t_expert_out_ = zeroed(expert_rows * ld * 4);
+  t_expert_out_ = zeroed((expert_rows + 1) * ld * 4);  // a one-token step keeps the shared expert's row behind the others
   t_shared_out_ = zeroed(R * ld * 4);
   t_v_first_ = zeroed(R * v_first * e);
   for (gpu_buffer* b : {&t_choice_, &t_weight_, &t_row_token_, &t_row_weight_, &t_inverse_}) *b = zeroed(expert_rows * 4);
@@ -69,9 +69,12 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   t_tile_row_ = zeroed(tiles * 4);
   t_expert_end_ = zeroed(experts * 4);
   t_n_tiles_ = zeroed(4);
-  // the one-token attention kernel holds the heads of a group in registers
-  for (layer_params const& p : m.shape.layers) {
-    if (p.mixer == mixer_type::attention && p.attention.heads / p.attention.kv_heads > 16) fused_step_ = false;
+  // the one-token attention kernel holds the heads of a group in registers and LDS
+  for (size_t l = 0; l < m.layers.size(); ++l) {
+    attention_params const& a = m.shape.layers[l].attention;
+    if (m.shape.layers[l].mixer != mixer_type::attention) continue;
+    const int group = a.heads / a.kv_heads;
+    if (group > 16 || group * (m.layers[l].attention.dv + 2) > 2400) fused_step_ = false;
   }
   t_arrived_ = zeroed(counters * LCU_ARRIVAL_BYTES);
   t_step_ = zeroed((1 + R) * 4);
@@ -151,7 +154,7 @@ void layered_context_impl::attention(attention_weights const& w, attention_param
 void layered_context_impl::experts(experts_weights const& w, experts_params const& p, int n) {
   layered_model_impl const& m = *model_;
   const int rows = n * p.top, W = m.shape.width;
-  plan_.tile_rows = m.dtype == LCU_F32 ? 32 : (rows >= 96 * p.experts ? 128 : 64);
+  plan_.tile_rows = m.dtype == LCU_F32 ? 32 : (rows >= 192 * p.experts ? 256 : rows >= 96 * p.experts ? 128 : 64);
   plan_.max_tiles = rows / plan_.tile_rows + std::min(p.experts, rows);
   LCU_CHECK(lcu_router(t_choice_.data(), t_weight_.data(), p.shared_ff > 0 ? t_shared_gate_.data() : nullptr, t_h_.data(),
                        w.router.data(), p.experts, p.top, m.dtype, n, m.ld, stream_));
@@ -182,7 +185,7 @@ void layered_context_impl::enqueue_rows(int n) {
     } else {
       attention(w.attention, q.attention, state_[l], n);
     }
-    LCU_CHECK(lcu_residual_norm(t_x_.data(), t_h_.data(), t_m_.data(), nullptr, 0, nullptr, nullptr, w.norm1b.data(),
+    LCU_CHECK(lcu_residual_norm(t_x_.data(), t_h_.data(), t_m_.data(), nullptr, 1, nullptr, nullptr, w.norm1b.data(),
                                 q.has_mlp ? w.norm2.data() : next_norm(l + 1), m.dtype, n, p.width, m.ld, p.norm_groups, p.norm_eps,
                                 stream_));
     if (q.has_mlp) {
@@ -202,59 +205,55 @@ void layered_context_impl::enqueue_rows(int n) {
   }
 }
 
-// x += norm(w . lhs + bias) and the next norm, one launch
-void layered_context_impl::project(const void* lhs, const void* w, const void* bias, int K, const void* w_after, const void* w_next) {
-  layered_params const& p = model_->shape;
-  LCU_CHECK(lcu_decode_project_norm(t_x_.data(), t_h_.data(), lhs, w, bias, K, nullptr, 0, 1, nullptr, nullptr, 0, nullptr, w_after,
-                                    w_next, t_arrived_.data(), p.width, model_->ld, p.norm_groups, p.norm_eps, stream_));
-}
-
-// One token: the launches of enqueue_rows fused around the weight streams.  A recurrent layer takes three
-// (both branches with the convolution, gates with the state, output with the norms), an attention layer three
-// (projections with the cache rows, attention, output with the norms), a feed-forward three (router, first
-// products, second products with the norms).  The last layer's norms end in the final one.
+// One token: launches fused around the weight streams.  A recurrent layer's mixer takes three (both branches
+// with the convolution, gates with the state, output product), an attention layer's too (projections with the
+// cache rows, attention, output product), a feed-forward two (first products, second products); between
+// sublayers one launch adds the result, takes both norms and, in front of a feed-forward, routes.  The last
+// layer's norms end in the final one.
 void layered_context_impl::enqueue_one() {
   layered_model_impl const& m = *model_;
   layered_params const& p = m.shape;
   const size_t n_layers = m.layers.size();
   const auto norm_ahead = [&](size_t l) { return l < n_layers ? m.layers[l].norm1.data() : m.final_norm.data(); };
-  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), 1, m.embed.data(), p.vocab, m.pos.data(), p.max_positions,
-                               start(), m.embed_norm.data(), norm_ahead(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps,
-                               stream_));
+  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), 1, m.embed.data(), p.vocab, m.pos.data(), p.max_positions, start(),
+                               m.embed_norm.data(), norm_ahead(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps, stream_));
   for (size_t l = 0; l < n_layers; ++l) {
     layer_params const& q = p.layers[l];
     layer_weights const& L = m.layers[l];
     layer_state& s = state_[l];
-    const void* after_mixer = q.has_mlp ? L.norm2.data() : norm_ahead(l + 1);
     if (q.mixer == mixer_type::rglru) {
       recurrence_weights const& w = L.recurrence;
       LCU_CHECK(lcu_decode_recurrent_in(t_wide_.data(), t_u_.data(), s.conv.data(), t_h_.data(), w.yx.data(), w.yx_bias.data(),
                                         w.conv.data(), w.conv_bias.data(), q.recurrence.taps, m.ld, w.ld, stream_));
       LCU_CHECK(lcu_decode_recurrent_step(t_rec_.data(), t_u_.data(), t_wide_.data(), w.gate_r.data(), w.gate_i.data(), w.bias_r.data(),
                                           w.bias_i.data(), w.decay.data(), s.s.data(), w.channels, w.block, stream_));
-      project(t_rec_.data(), w.out.data(), nullptr, w.ld, L.norm1b.data(), after_mixer);
+      LCU_CHECK(lcu_decode_linear(t_m_.data(), t_rec_.data(), w.out.data(), nullptr, w.ld, p.width, stream_));
     } else {
       attention_weights const& w = L.attention;
       attention_params const& a = q.attention;
       const lcu_window_params window{a.heads, a.kv_heads, w.dk, w.dv, a.window, a.keep_first, a.scale, w.r1.data(), w.r2.data()};
       LCU_CHECK(lcu_decode_kv(t_wide_.data(), s.k.data(), s.v.data(), t_h_.data(), w.qkv.data(), w.qkv_bias.data(), w.q_cols, w.k_cols,
                               w.v_cols, t_v_first_.data(), w.v_mode, w.v_mix.data(), start(), context_len_, m.ld, stream_));
-      LCU_CHECK(lcu_attention_windowed_decode(t_rec_.data(), t_wide_.data(), s.k.data(), s.v.data(), start(), context_len_,
-                                              &window, t_arrived_.data(), stream_));
-      project(t_rec_.data(), w.out.data(), w.out_bias.data(), w.ldo, L.norm1b.data(), after_mixer);
+      LCU_CHECK(lcu_attention_windowed_decode(t_rec_.data(), t_wide_.data(), s.k.data(), s.v.data(), start(), context_len_, &window,
+                                              t_arrived_.data(), stream_));
+      LCU_CHECK(lcu_decode_linear(t_m_.data(), t_rec_.data(), w.out.data(), w.out_bias.data(), w.ldo, p.width, stream_));
     }
+    experts_weights const& w = L.mlp;
+    const bool shared = q.has_mlp && q.mlp.shared_ff > 0;
+    LCU_CHECK(lcu_decode_residual_router(t_x_.data(), t_h_.data(), t_m_.data(), 1, nullptr, nullptr, L.norm1b.data(),
+                                         q.has_mlp ? L.norm2.data() : norm_ahead(l + 1), p.width, m.ld, p.norm_groups, p.norm_eps,
+                                         w.router.data(), q.mlp.experts, q.mlp.top, t_choice_.data(), t_weight_.data(),
+                                         shared ? t_shared_gate_.data() : nullptr, stream_));
     if (q.has_mlp) {
-      experts_weights const& w = L.mlp;
-      const bool shared = q.mlp.shared_ff > 0;
-      LCU_CHECK(lcu_decode_router(t_choice_.data(), t_weight_.data(), shared ? t_shared_gate_.data() : nullptr, t_h_.data(),
-                                  w.router.data(), q.mlp.experts, q.mlp.top, t_arrived_.data(), m.ld, stream_));
       LCU_CHECK(lcu_decode_experts_up(t_hidden_.data(), t_shared_hidden_.data(), t_h_.data(), t_choice_.data(), t_weight_.data(),
                                       w.up.data(), w.up_stride, &q.mlp.gate, w.shared_up.data(), &q.mlp.shared_gate, q.mlp.top, w.ld,
                                       w.shared_ld, m.ld, stream_));
-      LCU_CHECK(lcu_decode_project_norm(t_x_.data(), t_h_.data(), t_hidden_.data(), w.down.data(), nullptr, w.ld, t_choice_.data(),
-                                        w.down_stride, q.mlp.top, t_shared_hidden_.data(), w.shared_down.data(), w.shared_ld,
-                                        t_shared_gate_.data(), L.norm2b.data(), norm_ahead(l + 1), t_arrived_.data(), p.width, m.ld,
-                                        p.norm_groups, p.norm_eps, stream_));
+      LCU_CHECK(lcu_decode_experts_down(t_expert_out_.data(), m.ld, t_hidden_.data(), t_choice_.data(), w.down.data(), w.down_stride,
+                                        q.mlp.top, w.ld, t_shared_hidden_.data(), w.shared_down.data(), w.shared_ld, p.width, stream_));
+      const float* shared_row = (float*)t_expert_out_.data() + (size_t)q.mlp.top * m.ld;
+      LCU_CHECK(lcu_decode_residual_router(t_x_.data(), t_h_.data(), t_expert_out_.data(), q.mlp.top, shared ? shared_row : nullptr,
+                                           shared ? t_shared_gate_.data() : nullptr, L.norm2b.data(), norm_ahead(l + 1), p.width, m.ld,
+                                           p.norm_groups, p.norm_eps, nullptr, 0, 0, nullptr, nullptr, nullptr, stream_));
     }
   }
   LCU_CHECK(lcu_decode_linear(t_logits_.data(), t_h_.data(), m.head.data(), nullptr, m.ld, p.vocab, stream_));

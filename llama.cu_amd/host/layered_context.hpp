@@ -31,7 +31,6 @@ struct layered_context_impl final : public llama_context {
   void enqueue_one();                              // one token in bfloat16: fused launches, position from t_step_
   void step_one();                                 // enqueue_one, captured and replayed
   void drop_graph();
-  void project(const void* lhs, const void* w, const void* bias, int K, const void* w_after, const void* w_next);
   void recurrence(recurrence_weights const& w, recurrence_params const& p, layer_state& s, int n);
   void attention(attention_weights const& w, attention_params const& p, layer_state& s, int n);
   void experts(experts_weights const& w, experts_params const& p, int n);
