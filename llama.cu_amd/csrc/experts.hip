@@ -31,13 +31,13 @@ __global__ __launch_bounds__(256) void router_kernel(int* __restrict__ expert, f
   choose_experts(z, n_experts, top, expert + (size_t)t * top, weight + (size_t)t * top);
 }
 
-// The same for bfloat16 operands on the matrix cores: one workgroup takes 16 tokens and all rows of w, its
-// wavefronts a quarter of K each, four tiles of 16 rows of w at a time; the quarters are added in LDS in
-// wavefront order, and every wavefront chooses for four of the tokens.
-constexpr int ROUTER_TOKENS = 16;
+// The same for bfloat16 operands on the matrix cores: one workgroup takes 16 tokens and all rows of w, its eight
+// wavefronts an eighth of K each, four tiles of 16 rows of w at a time; the eighths meet in LDS and are added
+// in wavefront order, and every wavefront chooses for two of the tokens.
+constexpr int ROUTER_TOKENS = 16, ROUTER_WAVES = 8;
 template <int TILES>
 __device__ __forceinline__ void router_tiles(float4_t (&acc)[4], const bf16_t* a, const bf16_t* const (&b)[4], int s0, int s1) {
-#pragma unroll 4
+#pragma unroll 8
   for (int s = s0; s < s1; ++s) {
     const bf16x8_t fa = *reinterpret_cast<const bf16x8_t*>(a + s * 32);
 #pragma unroll
@@ -48,14 +48,15 @@ __device__ __forceinline__ void router_tiles(float4_t (&acc)[4], const bf16_t* a
   }
 }
 
-__global__ __launch_bounds__(256) void router_tile_kernel(int* __restrict__ expert, float* __restrict__ weight,
+__global__ __launch_bounds__(64 * ROUTER_WAVES) void router_tile_kernel(int* __restrict__ expert, float* __restrict__ weight,
                                                           float* __restrict__ shared_gate, const bf16_t* __restrict__ h,
                                                           const bf16_t* __restrict__ w, int n, int n_experts, int top, int K) {
   extern __shared__ float zs[];  // [ROUTER_TOKENS][ldz]
+  __shared__ float part[ROUTER_WAVES][ROUTER_TOKENS][64 + 1];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, t0 = blockIdx.x * ROUTER_TOKENS;
   const int n_rows = n_experts + (shared_gate ? 1 : 0), ldz = (n_rows + 15) / 16 * 16 + 1;
   const int col = lane & 15, quad = lane >> 4;
-  const int steps = K / 32, s0 = wave * steps / 4, s1 = (wave + 1) * steps / 4;
+  const int steps = K / 32, s0 = wave * steps / ROUTER_WAVES, s1 = (wave + 1) * steps / ROUTER_WAVES;
   const bf16_t* a = h + (size_t)min(t0 + col, n - 1) * K + quad * 8;
   for (int e0 = 0; e0 < n_rows; e0 += 64) {
     float4_t acc[4];
@@ -72,24 +73,23 @@ __global__ __launch_bounds__(256) void router_tile_kernel(int* __restrict__ expe
       case 3: router_tiles<3>(acc, a, b, s0, s1); break;
       default: router_tiles<4>(acc, a, b, s0, s1); break;
     }
-    for (int turn = 0; turn < 4; ++turn) {
-      if (wave == turn) {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          if (j < tiles) {
+    for (int j = 0; j < 4; ++j) {
 #pragma unroll
-            for (int v = 0; v < 4; ++v) {
-              float* z = zs + (quad * 4 + v) * ldz + e0 + j * 16 + col;
-              *z = turn == 0 ? acc[j][v] : *z + acc[j][v];
-            }
-          }
-        }
-      }
-      __syncthreads();
+      for (int v = 0; v < 4; ++v) part[wave][quad * 4 + v][j * 16 + col] = acc[j][v];
     }
+    __syncthreads();
+    for (int i = tid; i < ROUTER_TOKENS * 64; i += 64 * ROUTER_WAVES) {
+      const int t = i / 64, e = i % 64;
+      float z = 0.0f;
+#pragma unroll
+      for (int x = 0; x < ROUTER_WAVES; ++x) z += part[x][t][e];
+      if (e0 + e < n_rows) zs[t * ldz + e0 + e] = z;
+    }
+    __syncthreads();
   }
-  for (int k = 0; k < ROUTER_TOKENS / 4; ++k) {
-    const int t = t0 + wave * (ROUTER_TOKENS / 4) + k;
+  for (int k = 0; k < ROUTER_TOKENS / ROUTER_WAVES; ++k) {
+    const int t = t0 + wave * (ROUTER_TOKENS / ROUTER_WAVES) + k;
     if (t >= n) continue;
     float* z = zs + (t - t0) * ldz;
     if (shared_gate && lane == 0) shared_gate[t] = sigmoid_f32(z[n_experts]);
@@ -154,7 +154,7 @@ int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const 
                                             (const float*)w_dev, n_experts, top, K);
   } else {
     const size_t lds = (size_t)ROUTER_TOKENS * ((n_experts + 1 + 15) / 16 * 16 + 1) * sizeof(float);
-    router_tile_kernel<<<(n + ROUTER_TOKENS - 1) / ROUTER_TOKENS, 256, lds, st>>>(
+    router_tile_kernel<<<(n + ROUTER_TOKENS - 1) / ROUTER_TOKENS, 64 * ROUTER_WAVES, lds, st>>>(
         (int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev, (const bf16_t*)w_dev, n, n_experts, top, K);
   }
   LCU_LAUNCH_CHECK();

@@ -145,76 +145,133 @@ __global__ __launch_bounds__(256) void gates_f32_kernel(const float* __restrict_
   }
 }
 
-// bfloat16.  One wavefront: a chunk of 64 tokens x 32 channels, both gates, so that a lane holds r and i of
-// the same tokens of one channel: of every 8 tokens, the four from 4 (lane >> 5).  Four wavefronts of a
-// workgroup take neighbouring channel tiles and share the rows of u.
-__global__ __launch_bounds__(256) void gates_bf16_kernel(const bf16_t* __restrict__ u, gate_args p, int channels) {
+// bfloat16.  A wavefront takes a chunk of 64 tokens x 32 channels of both gates in two halves of 32 tokens, so
+// that a lane holds r and i of the same tokens of one channel: element v of half m belongs to token
+// t0 + 32 m + (v >> 2) * 8 + 4 (lane >> 5) + (v & 3).
+__device__ __forceinline__ void finish_gates(const gate_args& p, const bf16_t* __restrict__ u, const float16_t& r, const float16_t& g,
+                                             int t0, int c, state_map& whole) {
+  const int half = (threadIdx.x & 63) >> 5;
+  const float br = p.br[c], bi = p.bi[c], decay = p.decay[c];
+  float uv[16];
+#pragma unroll
+  for (int v = 0; v < 16; ++v) {
+    uv[v] = (float)u[(size_t)min(t0 + (v >> 2) * 8 + half * 4 + (v & 3), p.n - 1) * p.ld + c];
+  }
+#pragma unroll
+  for (int o = 0; o < 4; ++o) {
+    state_map map;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int v = o * 4 + e, t = t0 + o * 8 + half * 4 + e;
+      const float log_a = decay * sigmoid_fast(r[v] + br);
+      const float a = __expf(log_a);
+      const float b = drive_factor(log_a, a) * sigmoid_fast(g[v] + bi) * uv[v];
+      if (t < p.n) {
+        p.a[(size_t)t * p.ld + c] = a;
+        p.b[(size_t)t * p.ld + c] = b;
+        map.then(a, b);
+      }
+    }
+    // the lane 32 further holds the neighbouring four tokens of the eight
+    const float oA = __shfl_xor(map.A, 32, WAVE), oB = __shfl_xor(map.B, 32, WAVE);
+    whole.then(half ? oA : map.A, half ? oB : map.B);
+    whole.then(half ? map.A : oA, half ? map.B : oB);
+  }
+}
+
+__device__ __forceinline__ void store_chunk_map(const gate_args& p, const state_map& whole, int c) {
+  if ((threadIdx.x & 32) == 0) {
+    p.chunk_a[(size_t)blockIdx.y * p.ld + c] = whole.A;
+    p.chunk_b[(size_t)blockIdx.y * p.ld + c] = whole.B;
+  }
+}
+
+// any block width: operands straight from memory
+__global__ __launch_bounds__(256, 4) void gates_bf16_kernel(const bf16_t* __restrict__ u, gate_args p, int channels) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int t0 = blockIdx.y * CHUNK, c0 = (blockIdx.x * 4 + wave) * GATE_N;
   if (c0 >= channels) return;
   const int blk = c0 / p.bw, j0 = c0 - blk * p.bw, col = lane & 31, half = lane >> 5, c = c0 + col;
   const bf16_t* ua = u + (size_t)blk * p.bw + half * 8;
-  const bf16_t* u0 = ua + (size_t)min(t0 + col, p.n - 1) * p.ld;
-  const bf16_t* u1 = ua + (size_t)min(t0 + 32 + col, p.n - 1) * p.ld;
   const size_t w_at = ((size_t)blk * p.bw + j0 + col) * p.bw + half * 8;
   const bf16_t* wr = (const bf16_t*)p.wr + w_at;
   const bf16_t* wi = (const bf16_t*)p.wi + w_at;
+  const auto piece = [](const bf16_t* q, int k) { return *reinterpret_cast<const bf16x8_t*>(q + k); };
+  state_map whole;
+  for (int m = 0; m < 2; ++m) {
+    const bf16_t* um = ua + (size_t)min(t0 + 32 * m + col, p.n - 1) * p.ld;
+    float16_t r = (float16_t)(0.0f), g = (float16_t)(0.0f);
+#pragma unroll 2
+    for (int k = 0; k < p.bw; k += 32) {  // block widths are multiples of 32
+      const bf16x8_t a0 = piece(um, k), b0 = piece(wr, k), c0v = piece(wi, k);
+      const bf16x8_t a1 = piece(um, k + 16), b1 = piece(wr, k + 16), c1v = piece(wi, k + 16);
+      r = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b0, r, 0, 0, 0);
+      g = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, c0v, g, 0, 0, 0);
+      r = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b1, r, 0, 0, 0);
+      g = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, c1v, g, 0, 0, 0);
+    }
+    finish_gates(p, u, r, g, t0 + 32 * m, c, whole);
+  }
+  store_chunk_map(p, whole, c);
+}
+
+// block widths that are multiples of 128: four wavefronts share a chunk's rows of u and 128 channels' gate rows
+// in LDS, 64 columns of K at a time, the next ones in registers meanwhile
+constexpr int TILE_C = 128, TILE_K = 64, LDG = TILE_K + 8;
+__global__ __launch_bounds__(256, 2) void gates_tile_kernel(const bf16_t* __restrict__ u, gate_args p) {
+  __shared__ __attribute__((aligned(16))) bf16_t us[CHUNK * LDG];
+  __shared__ __attribute__((aligned(16))) bf16_t ws[2][TILE_C * LDG];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int t0 = blockIdx.y * CHUNK, c0 = blockIdx.x * TILE_C, blk = c0 / p.bw;
+  const int row = tid >> 3, col8 = (tid & 7) * 8;  // eight threads per row of 64 columns, 32 rows per pass
+  const bf16_t* ug = u + (size_t)blk * p.bw + col8;
+  const bf16_t* wg[2] = {(const bf16_t*)p.wr + (size_t)c0 * p.bw + col8, (const bf16_t*)p.wi + (size_t)c0 * p.bw + col8};
+  uint4_t ru[2], rw[2][4];
+  const auto load = [&](int k) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) ru[i] = *reinterpret_cast<const uint4_t*>(ug + (size_t)min(t0 + row + 32 * i, p.n - 1) * p.ld + k);
+#pragma unroll
+    for (int w = 0; w < 2; ++w) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) rw[w][i] = *reinterpret_cast<const uint4_t*>(wg[w] + (size_t)(row + 32 * i) * p.bw + k);
+    }
+  };
   float16_t r[2], g[2];
 #pragma unroll
   for (int m = 0; m < 2; ++m) {
     r[m] = (float16_t)(0.0f);
     g[m] = (float16_t)(0.0f);
   }
-  const auto piece = [](const bf16_t* q, int k) { return *reinterpret_cast<const bf16x8_t*>(q + k); };
-#pragma unroll 2
-  for (int k = 0; k < p.bw; k += 32) {  // block widths are multiples of 32
-    const bf16x8_t a0 = piece(u0, k), a1 = piece(u1, k), b0 = piece(wr, k), b1 = piece(wi, k);
-    const bf16x8_t a2 = piece(u0, k + 16), a3 = piece(u1, k + 16), b2 = piece(wr, k + 16), b3 = piece(wi, k + 16);
-    r[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b0, r[0], 0, 0, 0);
-    r[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b0, r[1], 0, 0, 0);
-    g[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b1, g[0], 0, 0, 0);
-    g[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b1, g[1], 0, 0, 0);
-    r[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a2, b2, r[0], 0, 0, 0);
-    r[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a3, b2, r[1], 0, 0, 0);
-    g[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a2, b3, g[0], 0, 0, 0);
-    g[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a3, b3, g[1], 0, 0, 0);
+  load(0);
+  for (int k = 0; k < p.bw; k += TILE_K) {
+    __syncthreads();  // the previous tile has been read
+#pragma unroll
+    for (int i = 0; i < 2; ++i) *reinterpret_cast<uint4_t*>(us + (row + 32 * i) * LDG + col8) = ru[i];
+#pragma unroll
+    for (int w = 0; w < 2; ++w) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) *reinterpret_cast<uint4_t*>(ws[w] + (row + 32 * i) * LDG + col8) = rw[w][i];
+    }
+    __syncthreads();
+    if (k + TILE_K < p.bw) load(k + TILE_K);
+    const int frag = (lane & 31) * LDG + (lane >> 5) * 8;
+#pragma unroll
+    for (int s = 0; s < TILE_K; s += 16) {
+      const bf16x8_t a0 = *reinterpret_cast<const bf16x8_t*>(us + frag + s);
+      const bf16x8_t a1 = *reinterpret_cast<const bf16x8_t*>(us + 32 * LDG + frag + s);
+      const bf16x8_t b0 = *reinterpret_cast<const bf16x8_t*>(ws[0] + wave * 32 * LDG + frag + s);
+      const bf16x8_t b1 = *reinterpret_cast<const bf16x8_t*>(ws[1] + wave * 32 * LDG + frag + s);
+      r[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b0, r[0], 0, 0, 0);
+      r[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b0, r[1], 0, 0, 0);
+      g[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, b1, g[0], 0, 0, 0);
+      g[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a1, b1, g[1], 0, 0, 0);
+    }
   }
-  const float br = p.br[c], bi = p.bi[c], decay = p.decay[c];
+  const int c = c0 + wave * 32 + (lane & 31);
   state_map whole;
-#pragma unroll
-  for (int m = 0; m < 2; ++m) {
-    // token of element v: t0 + 32 m + (v >> 2) * 8 + half * 4 + (v & 3)
-    float uv[16];
-#pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      const int t = t0 + m * 32 + (v >> 2) * 8 + half * 4 + (v & 3);
-      uv[v] = (float)u[(size_t)min(t, p.n - 1) * p.ld + c];
-    }
-#pragma unroll
-    for (int o = 0; o < 4; ++o) {
-      state_map map;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int v = o * 4 + e, t = t0 + m * 32 + o * 8 + half * 4 + e;
-        const float log_a = decay * sigmoid_fast(r[m][v] + br);
-        const float a = __expf(log_a);
-        const float b = drive_factor(log_a, a) * sigmoid_fast(g[m][v] + bi) * uv[v];
-        if (t < p.n) {
-          p.a[(size_t)t * p.ld + c] = a;
-          p.b[(size_t)t * p.ld + c] = b;
-          map.then(a, b);
-        }
-      }
-      // the lane 32 further holds the neighbouring four tokens of the eight
-      const float oA = __shfl_xor(map.A, 32, WAVE), oB = __shfl_xor(map.B, 32, WAVE);
-      whole.then(half ? oA : map.A, half ? oB : map.B);
-      whole.then(half ? map.A : oA, half ? map.B : oB);
-    }
-  }
-  if (half == 0) {
-    p.chunk_a[(size_t)blockIdx.y * p.ld + c] = whole.A;
-    p.chunk_b[(size_t)blockIdx.y * p.ld + c] = whole.B;
-  }
+  finish_gates(p, u, r[0], g[0], t0, c, whole);
+  finish_gates(p, u, r[1], g[1], t0 + 32, c, whole);
+  store_chunk_map(p, whole, c);
 }
 
 // chunk_a[k] <- the state that enters chunk k; state <- the state after the last chunk
@@ -362,7 +419,11 @@ int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, in
   if (dtype == LCU_F32) {
     gates_f32_kernel<<<dim3(channels / GATE_N, chunks), 256, 0, st>>>((const float*)u_dev, p);
   } else {
-    gates_bf16_kernel<<<dim3((channels / GATE_N + 3) / 4, chunks), 256, 0, st>>>((const bf16_t*)u_dev, p, channels);
+    if (block_width % TILE_C == 0) {
+      gates_tile_kernel<<<dim3(channels / TILE_C, chunks), 256, 0, st>>>((const bf16_t*)u_dev, p);
+    } else {
+      gates_bf16_kernel<<<dim3((channels / GATE_N + 3) / 4, chunks), 256, 0, st>>>((const bf16_t*)u_dev, p, channels);
+    }
   }
   carry_kernel<<<(channels + 63) / 64, 64, 0, st>>>(ca, cb, (float*)state_dev, chunks, channels, ld);
   if (dtype == LCU_F32) {

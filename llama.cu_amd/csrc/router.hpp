@@ -43,9 +43,7 @@ __device__ __forceinline__ void choose_experts(float* z, int n_experts, int top,
       weight[k] = sigmoid_f32(best);
       z[idx] = -INFINITY;
     }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // z is LDS of this wavefront: its accesses are in order
   }
 }
 

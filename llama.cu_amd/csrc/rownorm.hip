@@ -82,7 +82,7 @@ __global__ __launch_bounds__(TH) void residual_norm_kernel(float* __restrict__ x
 }
 
 // The step between two sublayers for one row, and the router behind it when there is one: every wavefront
-// takes rows of the router's matrix (its first one asked for before the norms are worked out), the first one
+// takes rows of the router's matrix (its first two asked for before the norms are worked out), the first one
 // then chooses.
 template <int NV>
 __global__ __launch_bounds__(STEP_THREADS) void residual_step_kernel(float* __restrict__ x, bf16_t* __restrict__ h, sublayer_rows src,
@@ -97,11 +97,14 @@ __global__ __launch_bounds__(STEP_THREADS) void residual_step_kernel(float* __re
   load_row(old, x, rs);
   if (w_next) load_row(next, w_next, rs);
   load_sum(m, t, src, 0, rs);
-  bf16x8_t ahead[AHEAD];
-  const bf16_t* first = rt.w + (size_t)min(wave, rt.rows - 1) * rs.ld;
+  bf16x8_t ahead[2][AHEAD];
   if (rt.w) {
 #pragma unroll
-    for (int a = 0; a < AHEAD; ++a) ahead[a] = *reinterpret_cast<const bf16x8_t*>(first + min((a * WAVE + lane) * 8, rs.ld - 8));
+    for (int turn = 0; turn < 2; ++turn) {
+      const bf16_t* we = rt.w + (size_t)min(wave + turn * TH / WAVE, rt.rows - 1) * rs.ld;
+#pragma unroll
+      for (int a = 0; a < AHEAD; ++a) ahead[turn][a] = *reinterpret_cast<const bf16x8_t*>(we + min((a * WAVE + lane) * 8, rs.ld - 8));
+    }
   }
   scale_row(m, rs, lds, after);
 #pragma unroll
@@ -114,26 +117,30 @@ __global__ __launch_bounds__(STEP_THREADS) void residual_step_kernel(float* __re
   bf16_t* hs = reinterpret_cast<bf16_t*>(lds);  // scale_row is done with it
   store_row(hs, m, rs);
   __syncthreads();
-  for (int e = wave; e < rt.rows; e += TH / WAVE) {
-    const bf16_t* we = rt.w + (size_t)e * rs.ld;
+  const auto dot = [&](float s, bf16x8_t wv, int c) {
+    const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(hs + c);
+#pragma unroll
+    for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
+    return s;
+  };
+  const auto row = [&](int e, auto&& held) {
+    if (e >= rt.rows) return;
     float s = 0.0f;
 #pragma unroll
     for (int a = 0; a < AHEAD; ++a) {
       const int c = (a * WAVE + lane) * 8;
-      if (c < rs.ld) {
-        const bf16x8_t wv = e == wave ? ahead[a] : *reinterpret_cast<const bf16x8_t*>(we + c);
-        const bf16x8_t hv = *reinterpret_cast<const bf16x8_t*>(hs + c);
-#pragma unroll
-        for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
-      }
+      if (c < rs.ld) s = dot(s, held(a, c), c);
     }
     for (int c = (AHEAD * WAVE + lane) * 8; c < rs.ld; c += WAVE * 8) {
-      const bf16x8_t wv = *reinterpret_cast<const bf16x8_t*>(we + c), hv = *reinterpret_cast<const bf16x8_t*>(hs + c);
-#pragma unroll
-      for (int b = 0; b < 8; ++b) s = fmaf((float)hv[b], (float)wv[b], s);
+      s = dot(s, *reinterpret_cast<const bf16x8_t*>(rt.w + (size_t)e * rs.ld + c), c);
     }
     s = wave_sum(s);
     if (lane == 0) z[e] = s;
+  };
+  row(wave, [&](int a, int) { return ahead[0][a]; });
+  row(wave + TH / WAVE, [&](int a, int) { return ahead[1][a]; });
+  for (int e = wave + 2 * TH / WAVE; e < rt.rows; e += TH / WAVE) {
+    row(e, [&](int, int c) { return *reinterpret_cast<const bf16x8_t*>(rt.w + (size_t)e * rs.ld + c); });
   }
   __syncthreads();
   if (wave != 0) return;

@@ -261,7 +261,7 @@ int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, 
 // meet in LDS, the slice's result goes to part[kv head][slice][head][dv + 4] (values, maximum, sum), and the
 // last workgroup of a kv head to arrive adds the slices up (arrives_last).  Nobody waits.
 constexpr int DEC_FLIGHT = 4;
-constexpr int DEC_MAX_SLICES = 64;
+constexpr int DEC_MAX_SLICES = 64, DEC_TOGETHER = 16;  // slices; those whose results are asked for together
 constexpr int DEC_MAX_GROUP = 16;  // query heads per kv head
 
 template <int RMAX, int DKP, int DVP>
@@ -330,10 +330,10 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restric
 #pragma unroll
             for (int e = 0; e < 8; ++e) d0 = fmaf((float)qv[r][d][e], (float)kv[f][d][e], d0);
           }
-          s[f] = row16_sum(d0) * p.scale - r1[r] * log1pf(r2[r] * (float)(i - j[f]));
+          s[f] = row16_sum(d0) * p.scale - r1[r] * __logf(1.0f + r2[r] * (float)(i - j[f]));
           if (xb + f * 16 + grp < x1) top = fmaxf(top, s[f]);
         }
-        const float shrink = expf(m[r] - top);
+        const float shrink = __expf(m[r] - top);
         m[r] = top;
         l[r] *= shrink;
 #pragma unroll
@@ -343,7 +343,7 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restric
         }
 #pragma unroll
         for (int f = 0; f < DEC_FLIGHT; ++f) {
-          const float w = xb + f * 16 + grp < x1 ? expf(s[f] - top) : 0.0f;
+          const float w = xb + f * 16 + grp < x1 ? __expf(s[f] - top) : 0.0f;
           l[r] += w;
 #pragma unroll
           for (int d = 0; d < DVP; ++d) {
@@ -383,7 +383,7 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restric
     float sum = 0.0f, val = 0.0f;
 #pragma unroll
     for (int w = 0; w < 16; ++w) {
-      const float f = expf(ml[(w * R + r) * 2] - mx);
+      const float f = __expf(ml[(w * R + r) * 2] - mx);
       sum = fmaf(f, ml[(w * R + r) * 2 + 1], sum);
       val = fmaf(f, dec_lds[((size_t)w * R + r) * p.dv + e], val);
     }
@@ -405,20 +405,20 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restric
     const int r = c / quads, e = (c - r * quads) * 4;
     float mx = -1e30f, sum = 0.0f;
     float4_t val = (float4_t)(0.0f);
-    for (int s0 = 0; s0 < slices; s0 += 8) {
-      float4_t pv[8];
-      float pm[8], pl[8];
+    for (int s0 = 0; s0 < slices; s0 += DEC_TOGETHER) {
+      float4_t pv[DEC_TOGETHER];
+      float pm[DEC_TOGETHER], pl[DEC_TOGETHER];
 #pragma unroll
-      for (int b = 0; b < 8; ++b) {
+      for (int b = 0; b < DEC_TOGETHER; ++b) {
         const float* src = all + ((size_t)min(s0 + b, slices - 1) * R + r) * ldp;
         pv[b] = load4(src + e);
         pm[b] = src[p.dv];
         pl[b] = src[p.dv + 1];
       }
 #pragma unroll
-      for (int b = 0; b < 8; ++b) {
+      for (int b = 0; b < DEC_TOGETHER; ++b) {
         if (s0 + b < slices) {
-          const float now = fmaxf(mx, pm[b]), was = expf(mx - now), f = expf(pm[b] - now);
+          const float now = fmaxf(mx, pm[b]), was = __expf(mx - now), f = __expf(pm[b] - now);
           sum = sum * was + f * pl[b];
           val = val * was + f * pv[b];
           mx = now;
@@ -549,8 +549,9 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
   if (ws.ptr == nullptr) return set_error(LCU_E_NOINIT, "lcu_attention_windowed_decode: lcu_init has not run on this device");
   const long seen = (long)window->window + window->keep;
   const int most = (int)(seen < max_positions ? seen : max_positions);  // visible keys of any position
-  // a slice for every 64 keys, while that does not take more than one workgroup per compute unit
-  const int slices = std::min(std::min((most + 63) / 64, (256 + window->kv_heads - 1) / window->kv_heads), DEC_MAX_SLICES);
+  // a slice for every 64 keys, sixteen of them while that gives half the compute units a workgroup
+  const int even = std::max(DEC_TOGETHER, 128 / window->kv_heads);
+  const int slices = std::min(std::min((most + 63) / 64, even), DEC_MAX_SLICES);
   const size_t need = (size_t)window->heads * slices * (window->dv + 4) * sizeof(float);
   LCU_REQUIRE(need <= ws.bytes, "lcu_attention_windowed_decode: %d slices do not fit the workspace", slices);
   LCU_REQUIRE((size_t)16 * R * (window->dv + 2) * sizeof(float) <= 150 * 1024,
