@@ -8,10 +8,14 @@
 // ignored.  A model name is looked up as models/<name>; a name containing '/' is the directory.
 // max_tokens and context_len are additions for testing with small contexts; with sample_seed the
 // tokens are drawn from the probabilities (the sampler the reference leaves commented out,
-// llama_cu.cu:1202-1203) instead of taking the most probable one.
+// llama_cu.cu:1202-1203) instead of taking the most probable one.  A directory with a config.json holds a model
+// of another family (llama_model::open); without a vocab file its prompt is token ids, and so is the output.
+#include <algorithm>
 #include <chrono>
 #include <cstdio>
 #include <cstdlib>
+#include <cstring>
+#include <memory>
 #include <string>
 #include <vector>
 
@@ -45,11 +49,68 @@ void print_model_facts(llama_params const& p, size_t context_len) {
          p.shared_context_memory_size(context_len) / mb, p.kv_cache_size(context_len) / mb);
 }
 
+// A LLaMA in the reference's format; nullptr after a message.
+std::unique_ptr<llama_model> load_llama(std::string const& dir, size_t context_len) {
+  mapped_buffer params_buf(dir + "/params");
+  if (!params_buf.is_ok()) {
+    fprintf(stderr, "Could not load params file\n");
+    return nullptr;
+  }
+  if (!mapped_buffer(dir + "/vocab").is_ok()) {
+    fprintf(stderr, "Could not load vocab file\n");
+    return nullptr;
+  }
+  llama_params params;
+  if (!params.load(params_buf)) {
+    fprintf(stderr, "Invalid model parameters\n");
+    return nullptr;
+  }
+  llama_partition partition;
+  partition.autopipe(params, context_len);
+  partition.debug_print();
+  if (!partition.is_valid()) {
+    fprintf(stderr, "Could not partition model\n");
+    return nullptr;
+  }
+  print_model_facts(params, context_len);
+  auto model = llama_model::load(params, partition, dir);
+  if (!model) {
+    fprintf(stderr, "Could not load model\n");
+  }
+  return model;
+}
+
+// A model with a config.json; nullptr after a message.
+std::unique_ptr<llama_model> load_configured(std::string const& dir, size_t context_len) {
+  auto model = llama_model::open(dir, (int)context_len);
+  if (!model) {
+    fprintf(stderr, "Could not load model\n");
+    return nullptr;
+  }
+  llama_params const& p = model->params;
+  printf("Dimension: %d\nLayers: %d\nHeads: %d\nVocab: %d\nNorm Epsilon: %f\n", p.dim, p.n_layers, p.n_heads, p.n_vocab, p.norm_eps);
+  return model;
+}
+
+// token ids written as numbers; false on anything else
+bool parse_ids(std::string const& text, std::vector<int32_t>& ids) {
+  const char* at = text.c_str();
+  while (true) {
+    at += strspn(at, " ,\t\n");
+    if (*at == '\0') return !ids.empty();
+    char* end = nullptr;
+    const long id = strtol(at, &end, 10);
+    if (end == at || id < 0 || id > INT32_MAX) return false;
+    ids.push_back((int32_t)id);
+    at = end;
+  }
+}
+
 // Generates up to max_tokens tokens after the prompt; returns the per-token wall times.
-std::vector<float> generate(llama_context& context, llama_vocabulary& vocab, std::vector<short> const& prompt,
+std::vector<float> generate(llama_context& context, llama_vocabulary* vocab, std::vector<int32_t> const& prompt,
                             options const& opt, int& generated) {
-  std::vector<short> history = prompt;  // everything fed or produced so far
-  std::vector<short> feed = prompt;     // what the next call consumes
+  std::vector<int32_t> history = prompt;  // everything fed or produced so far
+  std::vector<int32_t> feed = prompt;     // what the next call consumes
   std::vector<float> times;
   generated = 0;
   while (generated < opt.max_tokens) {
@@ -60,16 +121,20 @@ std::vector<float> generate(llama_context& context, llama_vocabulary& vocab, std
       const size_t keep = std::min(history.size(), opt.context_len / 2);
       feed.assign(history.end() - keep, history.end());
     }
-    const short token = context.next_token(feed);
+    const int token = context.forward(feed.data(), (int)feed.size(), nullptr, 0, nullptr);
     const float dt = (float)seconds_since(t0);
     if (token < 0) {
-      fprintf(stderr, "\nnext_token failed: %zu tokens do not fit the context\n", feed.size());
+      fprintf(stderr, "\nnext_token failed: %zu tokens do not fit the context or the vocabulary\n", feed.size());
       break;
     }
-    if (token == 2) {  // end of sequence
+    if (vocab && token == 2) {  // end of sequence
       break;
     }
-    fputs(vocab.tokens[token].text.c_str(), stdout);
+    if (vocab) {
+      fputs(vocab->tokens[token].text.c_str(), stdout);
+    } else {
+      printf("%s%d", generated > 0 ? " " : "", token);
+    }
     fflush(stdout);
     feed.assign(1, token);
     history.push_back(token);
@@ -98,53 +163,42 @@ int main(int argc, char const** argv) {
   }
   initialize();
   const std::string dir = model_dir(opt.model);
-  mapped_buffer params_buf(dir + "/params");
+  const bool configured = mapped_buffer(dir + "/config.json").is_ok();
   mapped_buffer vocab_buf(dir + "/vocab");
-  if (!params_buf.is_ok()) {
-    fprintf(stderr, "Could not load params file\n");
-    return 1;
-  }
-  if (!vocab_buf.is_ok()) {
-    fprintf(stderr, "Could not load vocab file\n");
-    return 1;
-  }
-  llama_params params;
-  if (!params.load(params_buf)) {
-    fprintf(stderr, "Invalid model parameters\n");
-    return 1;
-  }
-  llama_vocabulary vocab(vocab_buf);
-  if (vocab.tokens.size() != params.n_vocab) {
-    fprintf(stderr, "Vocab size mismatch\n");
-    return 1;
-  }
-  llama_partition partition;
-  partition.autopipe(params, opt.context_len);
-  partition.debug_print();
-  if (!partition.is_valid()) {
-    fprintf(stderr, "Could not partition model\n");
-    return 1;
-  }
-  print_model_facts(params, opt.context_len);
-  auto model = llama_model::load(params, partition, dir);
+  auto model = configured ? load_configured(dir, opt.context_len) : load_llama(dir, opt.context_len);
   if (!model) {
-    fprintf(stderr, "Could not load model\n");
     return 1;
   }
+  std::unique_ptr<llama_vocabulary> vocab;
+  if (vocab_buf.is_ok()) {
+    vocab = std::make_unique<llama_vocabulary>(vocab_buf);
+    if (vocab->tokens.size() != model->params.n_vocab) {
+      fprintf(stderr, "Vocab size mismatch\n");
+      return 1;
+    }
+  }
+  opt.context_len = std::min(opt.context_len, (size_t)model->max_context());
   auto context = llama_context::create(model.get(), (int)opt.context_len, 0.8f);
   printf("Context memory: %f MB\n", context->context_memory_usage() / 1024.0 / 1024.0);
   if (opt.sample) {
     context->sample_with_seed(opt.sample_seed);
   }
 
-  const std::vector<short> prompt = vocab.tokenize(opt.prompt, true);
+  std::vector<int32_t> prompt;
+  if (vocab) {
+    const std::vector<short> ids = vocab->tokenize(opt.prompt, true);
+    prompt.assign(ids.begin(), ids.end());
+  } else if (!parse_ids(opt.prompt, prompt)) {
+    fprintf(stderr, "The model has no vocab file: the prompt must be token ids\n");
+    return 1;
+  }
   if (prompt.size() > opt.context_len) {
     fprintf(stderr, "Prompt of %zu tokens exceeds the context of %zu\n", prompt.size(), opt.context_len);
     return 1;
   }
   int generated = 0;
   const auto start = steady::now();
-  const std::vector<float> times = generate(*context, vocab, prompt, opt, generated);
+  const std::vector<float> times = generate(*context, vocab.get(), prompt, opt, generated);
   printf("\ntokens: %d time: %f\n", generated, seconds_since(start));
   // times.txt: prompt length, then one wall time per generated token (plot_times.py reads it)
   FILE* fp = fopen("times.txt", "w");
