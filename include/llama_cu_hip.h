@@ -410,9 +410,9 @@ int lcu_kv_store(void* k_cache_dev, void* v_cache_dev, const void* qkv_dev, int 
                  void* stream);
 int lcu_attention_windowed(void* out_dev, int ldo, const void* q_dev, int ldq, const void* k_cache_dev, const void* v_cache_dev,
                            int start, const lcu_window_params* window, int dtype, int n, void* stream);
-/* one new token at position *pos_dev (bfloat16), the visible keys spread over the chip; arrived_dev:
- * kv_heads times LCU_ARRIVAL_BYTES, zero before the first call (and left zero).  Uses the stream's workspace. */
-#define LCU_ARRIVAL_BYTES (65 * 128)
+/* one new token at position *pos_dev (bfloat16), the visible keys spread over the chip; arrived_dev: kv_heads
+ * uint32, zero before the call and after it (the workgroup that arrives last adds the parts up; nobody waits).
+ * Uses the stream's workspace. */
 int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* k_cache_dev, const void* v_cache_dev,
                                   const void* pos_dev, int max_positions, const lcu_window_params* window, void* arrived_dev,
                                   void* stream);

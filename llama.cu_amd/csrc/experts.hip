@@ -154,6 +154,13 @@ int lcu_router(void* expert_dev, void* weight_dev, void* shared_gate_dev, const 
                                             (const float*)w_dev, n_experts, top, K);
   } else {
     const size_t lds = (size_t)ROUTER_TOKENS * ((n_experts + 1 + 15) / 16 * 16 + 1) * sizeof(float);
+    static bool raised[16] = {};  // per device, once: hundreds of experts take more than 64 KB
+    int dev = 0;
+    LCU_HIP(hipGetDevice(&dev));
+    if (!raised[dev & 15]) {
+      LCU_HIP(hipFuncSetAttribute((const void*)router_tile_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024));
+      raised[dev & 15] = true;
+    }
     router_tile_kernel<<<(n + ROUTER_TOKENS - 1) / ROUTER_TOKENS, 64 * ROUTER_WAVES, lds, st>>>(
         (int*)expert_dev, (float*)weight_dev, (float*)shared_gate_dev, (const bf16_t*)h_dev, (const bf16_t*)w_dev, n, n_experts, top, K);
   }

@@ -359,7 +359,7 @@ __device__ __forceinline__ void wait_vmcnt() {
 // EP: what the accumulators become.  f16_epilogue is the fp16 output described above.  The bfloat16
 // epilogues (linear.hpp) take bfloat16 operands, which travel exactly like the fp16 ones, through
 // v_mfma_f32_32x32x16_bf16, and end in a bias, a GELU, or a clamped gate; GROUPED ones take the
-// rows of a tile and its weight matrix from a tile list on the device (experts_plan in experts.hip).
+// rows of a tile and its weight matrix from a tile list on the device (lcu_experts_plan).
 struct f16_epilogue {
   static constexpr bool BF16 = false, GROUPED = false;
 };
@@ -1343,7 +1343,7 @@ int gemm_bf16(linear_epilogue<false, GATED> const& ep, const void* A, const void
   const auto tn = [&](int bn) { return (long)((N + bn - 1) / bn); };
   if (M <= 64) return launch_bf16<64, 64, 2, GATED ? 1 : 2, 1, 3>(ep, A, W, tm(64), M, K, N, st);
   if (tm(256) * tn(128) >= 160) return launch_bf16<256, 128, 4, 2, 1, 3>(ep, A, W, tm(256), M, K, N, st);
-  if (tm(128) * tn(128) >= 256) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, tm(128), M, K, N, st);
+  if (tm(128) * tn(128) > 256) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, tm(128), M, K, N, st);
   if (tm(128) * tn(128) >= 160) return launch_bf16<128, 128, 4, 2, 1, 3>(ep, A, W, tm(128), M, K, N, st);
   if constexpr (GATED) {
     if (tm(128) * tn(64) > 128) return launch_bf16<128, 64, 4, 1, 1, 3>(ep, A, W, tm(128), M, K, N, st);
@@ -1365,7 +1365,7 @@ template <bool GATED>
 int gemm_bf16_grouped(linear_epilogue<true, GATED> const& ep, const void* A, const void* W, int max_tiles, int K, int N,
                       hipStream_t st) {
   if (ep.tile_rows == 256) return launch_bf16<256, 128, 4, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
-  if (ep.tile_rows == 128) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, max_tiles, 0, K, N, st);
+  if (ep.tile_rows == 128) return launch_bf16<128, 128, 4, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
   return launch_bf16<64, 128, 2, 2, 1, 3>(ep, A, W, max_tiles, 0, K, N, st);
 }
 template int gemm_bf16_grouped<false>(linear_epilogue<true, false> const&, const void*, const void*, int, int, int, hipStream_t);

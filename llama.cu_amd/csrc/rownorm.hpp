@@ -158,30 +158,4 @@ void with_step_pieces(int ld, F&& f) {
   }
 }
 
-// ---- which workgroup arrives last -------------------------------------------------------------------
-// Counters of a launch whose last workgroup goes on with the others' results: ARRIVAL_LANES first-level
-// counters, 128 bytes apart, and one behind them that counts full ones (thousands of workgroups adding to one
-// word would queue for it).  All are zero before the launch and after it.
-constexpr int ARRIVAL_LANES = 64;
-constexpr int ARRIVAL_STRIDE = 32;  // words
-constexpr int ARRIVAL_WORDS = (ARRIVAL_LANES + 1) * ARRIVAL_STRIDE;
-
-// Called by one thread after the workgroup's device-scope stores are complete.
-__device__ __forceinline__ bool arrives_last(uint32_t* counters, uint32_t block, uint32_t blocks) {
-  uint32_t* top = counters + ARRIVAL_LANES * ARRIVAL_STRIDE;
-  if (blocks <= ARRIVAL_LANES) {  // few enough for one word
-    if (__hip_atomic_fetch_add(top, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != blocks - 1) return false;
-    __hip_atomic_store(top, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    return true;
-  }
-  const uint32_t lane = block % ARRIVAL_LANES;
-  const uint32_t mine = blocks / ARRIVAL_LANES + (lane < blocks % ARRIVAL_LANES ? 1u : 0u);
-  uint32_t* c = counters + lane * ARRIVAL_STRIDE;
-  if (__hip_atomic_fetch_add(c, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != mine - 1) return false;
-  __hip_atomic_store(c, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  if (__hip_atomic_fetch_add(top, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) != ARRIVAL_LANES - 1) return false;
-  __hip_atomic_store(top, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  return true;
-}
-
 }  // namespace lcu

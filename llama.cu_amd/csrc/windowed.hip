@@ -259,7 +259,8 @@ int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, 
 // them; keys and values of DEC_FLIGHT rows per lane group are requested together, before anything is
 // computed.  Each of the 16 groups keeps a running maximum, sum and weighted values per head; the groups
 // meet in LDS, the slice's result goes to part[kv head][slice][head][dv + 4] (values, maximum, sum), and the
-// last workgroup of a kv head to arrive adds the slices up (arrives_last).  Nobody waits.
+// last workgroup of a kv head to arrive adds the slices up: a counter says which it is, and that workgroup sets
+// it back to zero.  Nobody waits.
 constexpr int DEC_FLIGHT = 4;
 constexpr int DEC_MAX_SLICES = 64, DEC_TOGETHER = 16;  // slices; those whose results are asked for together
 constexpr int DEC_MAX_GROUP = 16;  // query heads per kv head
@@ -395,7 +396,10 @@ __global__ __launch_bounds__(256) void attention_decode_kernel(bf16_t* __restric
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // every wavefront's stores are out before the count goes up
   __syncthreads();
-  if (tid == 0) last = arrives_last(arrived + (size_t)g * ARRIVAL_WORDS, slice, slices);
+  if (tid == 0) {
+    last = __hip_atomic_fetch_add(arrived + g, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (uint32_t)slices - 1;
+    if (last) __hip_atomic_store(arrived + g, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
   __syncthreads();
   if (!last) return;
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");  // ordinary loads from here on see the other workgroups' stores

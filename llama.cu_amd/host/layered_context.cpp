@@ -76,7 +76,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
     const int group = a.heads / a.kv_heads;
     if (group > 16 || group * (m.layers[l].attention.dv + 2) > 2400) fused_step_ = false;
   }
-  t_arrived_ = zeroed(counters * LCU_ARRIVAL_BYTES);
+  t_arrived_ = zeroed(counters * 4);
   t_step_ = zeroed((1 + R) * 4);
   t_probs_ = zeroed((size_t)m.shape.vocab * 2);
   t_index_ = zeroed(4);
@@ -154,7 +154,8 @@ void layered_context_impl::attention(attention_weights const& w, attention_param
 void layered_context_impl::experts(experts_weights const& w, experts_params const& p, int n) {
   layered_model_impl const& m = *model_;
   const int rows = n * p.top, W = m.shape.width;
-  plan_.tile_rows = m.dtype == LCU_F32 ? 32 : (rows >= 192 * p.experts ? 256 : rows >= 96 * p.experts ? 128 : 64);
+  // tiles of about half an expert's rows: larger ones multiply faster, but every expert ends in a part of one
+  plan_.tile_rows = m.dtype == LCU_F32 ? 32 : (rows >= 384 * p.experts ? 256 : rows >= 96 * p.experts ? 128 : 64);
   plan_.max_tiles = rows / plan_.tile_rows + std::min(p.experts, rows);
   LCU_CHECK(lcu_router(t_choice_.data(), t_weight_.data(), p.shared_ff > 0 ? t_shared_gate_.data() : nullptr, t_h_.data(),
                        w.router.data(), p.experts, p.top, m.dtype, n, m.ld, stream_));

@@ -59,7 +59,7 @@ struct layered_context_impl final : public llama_context {
   uint64_t sample_seed_{0}, samples_drawn_{0};
   void* decode_graph_{nullptr};
   int decode_calls_{0};
-  gpu_buffer t_arrived_;                           // counters of the fused launches, zero between launches
+  gpu_buffer t_arrived_;                           // counters of the attention step, zero between launches
   void* stream_{nullptr};
 };
 
