@@ -366,7 +366,7 @@ def layered_leg(P, name, steps, warmup, vocab=32000, families=("rirulix", "llama
     B = P.binding
     s = LAYERED[name]
     out = {"layers": s["layers"], "width": s["width"]}
-    prompts = (512, 2048)
+    prompts = (512, 2048, 32)
     if "rirulix" in families:
         model = P.Model(config=layered_config(s, vocab), seed=1)
         ctx = P.Context(model, context_len=4096, temperature=0.8)

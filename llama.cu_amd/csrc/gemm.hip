@@ -768,7 +768,7 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
     }
   }
   if constexpr (EP::BF16) {
-    static_assert(!SPLIT && !U8, "bfloat16 operands: whole K range per workgroup");
+    static_assert(!U8, "bfloat16 operands are not quantised");
     if (group == 0) {
 #pragma unroll
       for (int i = 0; i < TM; ++i) {
@@ -776,7 +776,13 @@ __global__ __launch_bounds__(64 * WM * WN * KS, WM * WN * KS <= 4 ? 2 : 1) void 
         for (int v = 0; v < 16; ++v) {
           const int gm = m0 + wm + i * 32 + (v >> 2) * 8 + (lane >> 5) * 4 + (v & 3);
           if (gm >= M) continue;
-          if constexpr (EP::GATED) {
+          if constexpr (SPLIT) {  // the epilogue belongs to the launch that adds the splits
+#pragma unroll
+            for (int j = 0; j < TN; ++j) {
+              const int gn = n0 + wn + j * 32 + (lane & 31);
+              if (gn < N) part[((size_t)split * M + gm) * N + gn] = acc[i][j][v];
+            }
+          } else if constexpr (EP::GATED) {
             // 32 columns of gate rows, then the 32 of the up rows they belong to: one lane holds both
             static_assert(TN == 2, "a wavefront's columns are one gate / up pair of blocks");
             const int hc = (n0 + wn) / 2 + (lane & 31);
@@ -1307,13 +1313,15 @@ int dispatch_gemm(operands_t op, const half_t* A, int M, int K, int N, int block
 }
 
 // ---- bfloat16 operands ----
-template <int BM, int BN, int WM, int WN, int KS, int NS, class EP>
-int launch_bf16(EP const& ep, const void* A, const void* W, int tiles_m, int M, int K, int N, hipStream_t st) {
+// splits > 1: the K stages of every tile dealt to that many workgroups, fp32 sums to part (no epilogue)
+template <int BM, int BN, int WM, int WN, int KS, int NS, bool SPLIT = false, class EP>
+int launch_bf16(EP const& ep, const void* A, const void* W, int tiles_m, int M, int K, int N, hipStream_t st, int splits = 1,
+                float* part = nullptr) {
   constexpr int ROWB = BK * KS * 2;
   constexpr size_t lds = (size_t)NS * (BM + BN) * ROWB;
   static_assert(lds <= 160 * 1024, "rings do not fit LDS");
   static_assert(KS == 1 || lds >= (size_t)BM * BN * 4 / 2, "LDS must hold one group's accumulators");
-  auto kernel = gemm_dl_kernel<BM, BN, WM, WN, KS, NS, false, false, EP>;
+  auto kernel = gemm_dl_kernel<BM, BN, WM, WN, KS, NS, false, SPLIT, EP>;
   if constexpr (lds > 64 * 1024) {
     static bool raised[16] = {};  // per device, once
     int dev = 0;
@@ -1325,9 +1333,52 @@ int launch_bf16(EP const& ep, const void* A, const void* W, int tiles_m, int M, 
   }
   const int tiles_n = (N + BN - 1) / BN;
   const more_matrices_t none{{nullptr, nullptr}, {nullptr, nullptr}, {nullptr, nullptr}, 0};
-  kernel<<<tiles_m * tiles_n, 64 * WM * WN * KS, lds, st>>>(nullptr, (const half_t*)A, W, nullptr, M, K, N, 0, 0.0f, tiles_m,
-                                                            tiles_n, nullptr, 1, none, ep);
+  kernel<<<tiles_m * tiles_n * splits, 64 * WM * WN * KS, lds, st>>>(nullptr, (const half_t*)A, W, nullptr, M, K, N, 0, 0.0f,
+                                                                     tiles_m, tiles_n, part, splits, none, ep);
   LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+// the splits' sums in split order, then the epilogue; a thread per output
+template <bool GATED>
+__global__ __launch_bounds__(256) void splitk_epilogue_kernel(linear_epilogue<false, GATED> ep, const float* __restrict__ part, int M,
+                                                              int N, int splits) {
+  const int outs = GATED ? N / 2 : N, i = blockIdx.x * 256 + threadIdx.x;
+  if (i >= M * outs) return;
+  const int m = i / outs, n = i - m * outs;
+  const auto sum = [&](int c) {
+    float s = 0.0f;
+    for (int k = 0; k < splits; ++k) s += part[((size_t)k * M + m) * N + c];
+    return s;
+  };
+  if constexpr (GATED) {
+    const int c = n / 32 * 64 + n % 32;
+    ep.store_gated(m, n, sum(c), sum(c + 32));
+  } else {
+    ep.store(m, n, sum(n));
+  }
+}
+
+// Few rows: the weight stream is what counts (see launch_skinny).  *done = false when the shape gives no second
+// workgroup to a tile.
+template <bool GATED>
+int bf16_skinny(linear_epilogue<false, GATED> const& ep, const void* A, const void* W, int M, int K, int N, hipStream_t st, bool* done) {
+  *done = false;
+  device_state* ds = current_device_state();
+  const workspace_t ws = workspace_for(st);
+  if (ds == nullptr || ws.ptr == nullptr) return LCU_OK;
+  const int tiles = (N + 127) / 128;
+  int splits = std::min((ds->compute_units + tiles - 1) / tiles, K / BK / 4);
+  while (splits > 1 && (size_t)splits * M * N * sizeof(float) > ws.bytes) --splits;
+  if (splits < 2) return LCU_OK;
+  float* part = (float*)ws.ptr;
+  const int rc = M <= 32 ? launch_bf16<32, 128, 1, 4, 1, 3, true>(ep, A, W, 1, M, K, N, st, splits, part)
+                         : launch_bf16<64, 128, 1, 4, 1, 3, true>(ep, A, W, 1, M, K, N, st, splits, part);
+  if (rc != LCU_OK) return rc;
+  const int outs = M * (GATED ? N / 2 : N);
+  splitk_epilogue_kernel<GATED><<<(outs + 255) / 256, 256, 0, st>>>(ep, part, M, N, splits);
+  LCU_LAUNCH_CHECK();
+  *done = true;
   return LCU_OK;
 }
 
@@ -1341,7 +1392,12 @@ template <bool GATED>
 int gemm_bf16(linear_epilogue<false, GATED> const& ep, const void* A, const void* W, int M, int K, int N, hipStream_t st) {
   const auto tm = [&](int bm) { return (M + bm - 1) / bm; };
   const auto tn = [&](int bn) { return (long)((N + bn - 1) / bn); };
-  if (M <= 64) return launch_bf16<64, 64, 2, GATED ? 1 : 2, 1, 3>(ep, A, W, tm(64), M, K, N, st);
+  if (M <= 64) {
+    bool done = false;
+    const int rc = bf16_skinny<GATED>(ep, A, W, M, K, N, st, &done);
+    if (rc != LCU_OK || done) return rc;
+    return launch_bf16<64, 64, 2, GATED ? 1 : 2, 1, 3>(ep, A, W, tm(64), M, K, N, st);
+  }
   if (tm(256) * tn(128) >= 160) return launch_bf16<256, 128, 4, 2, 1, 3>(ep, A, W, tm(256), M, K, N, st);
   if (tm(128) * tn(128) > 256) return launch_bf16<128, 128, 2, 2, 1, 2>(ep, A, W, tm(128), M, K, N, st);
   if (tm(128) * tn(128) >= 160) return launch_bf16<128, 128, 4, 2, 1, 3>(ep, A, W, tm(128), M, K, N, st);

@@ -81,7 +81,7 @@ def call(G, name, *args):
 # ---- linear ---------------------------------------------------------------------------------------------
 @BOTH
 @pytest.mark.parametrize("M,K,N", [(1, 64, 5), (3, 192, 70), (37, 320, 100), (64, 128, 129), (130, 256, 200), (300, 448, 2048),
-                                   (513, 128, 4100)])
+                                   (513, 128, 4100), (2, 1024, 300), (31, 2048, 1100), (48, 1536, 65), (64, 512, 3000)])
 def test_linear_with_bias_and_gelu_columns(gpu, dt, M, K, N):
     rng = np.random.default_rng(M * 7 + N)
     x, w, b = rounded(rng.standard_normal((M, K))), rounded(rng.standard_normal((N, K)) / K ** 0.5), rng.standard_normal(N)
@@ -100,7 +100,7 @@ def test_linear_with_bias_and_gelu_columns(gpu, dt, M, K, N):
 
 
 @BOTH
-@pytest.mark.parametrize("M,K,ff", [(1, 64, 32), (5, 128, 40), (66, 192, 100), (200, 128, 640), (700, 64, 1000)])
+@pytest.mark.parametrize("M,K,ff", [(1, 64, 32), (5, 128, 40), (66, 192, 100), (200, 128, 640), (700, 64, 1000), (2, 1024, 70), (40, 768, 500)])
 def test_gated_linear_clamps(gpu, dt, M, K, ff):
     rng = np.random.default_rng(ff)
     x, gw, uw = rounded(2 * rng.standard_normal((M, K))), rounded(rng.standard_normal((ff, K)) / K ** 0.5), \
