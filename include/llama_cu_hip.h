@@ -323,6 +323,10 @@ int lcu_error_stats(void* out3_dev, const void* a_dev, const void* b_dev, size_t
 int lcu_linear(void* out_dev, int out_f32, int ldo, const void* lhs_dev, const void* w_dev, const void* bias_dev,
                int gelu_cols, int dtype, int M, int K, int N, void* stream);
 
+/* the same without bias; columns from tail_from on go to fp32 rows tail [M][ld_tail] instead */
+int lcu_linear_tail(void* out_dev, int ldo, void* tail_f32_dev, int ld_tail, int tail_from, const void* lhs_dev, const void* w_dev,
+                    int dtype, int M, int K, int N, void* stream);
+
 /* clamped gated unit: g = min(gate, limit), u = clamp(up, +-limit), g sigmoid(alpha g) (u + up_shift) */
 typedef struct lcu_gate_params {
   float limit, alpha, up_shift;
@@ -367,10 +371,13 @@ int lcu_experts_down(void* out_f32_dev, int ldo, const void* lhs_dev, const void
  * (NULL: none).  lcu_residual_norm: m = per token the sum of `top` fp32 rows of out (rows
  * inverse[token * top + k], or token * top + k when inverse is NULL) and shared_gate[row] times the shared
  * expert's row; x += norm(m) under w_after; h =
- * norm(x) under w_next.  lcu_group_norm: h[i] = norm(x[row_index[i]]). */
+ * norm(x) under w_next.  Where w_next is NULL and h is given, h = x as it is.  lcu_embed_scaled: x = scale *
+ * table[id], h likewise.  lcu_group_norm: h[i] = norm(x[row_index[i]]). */
 int lcu_embed_pos_norm(void* x_dev, void* h_dev, const void* ids_i32_dev, int n_ids, const void* table_dev, int n_vocab,
                        const void* pos_table_dev, int n_pos, const void* start_dev, const void* w_embed_dev,
                        const void* w_next_dev, int dtype, int width, int ld, int groups, float eps, void* stream);
+int lcu_embed_scaled(void* x_dev, void* h_dev, const void* ids_i32_dev, int n_ids, const void* table_dev, int n_vocab, float scale,
+                     const void* w_next_dev, int dtype, int width, int ld, int groups, float eps, void* stream);
 int lcu_residual_norm(void* x_dev, void* h_dev, const void* out_f32_dev, const void* inverse_dev, int top,
                       const void* shared_f32_dev, const void* shared_gate_dev, const void* w_after_dev,
                       const void* w_next_dev, int dtype, int rows, int width, int ld, int groups, float eps, void* stream);
@@ -382,12 +389,12 @@ int lcu_softmax_f32(void* probs_f16_dev, const void* logits_dev, int n, float te
 
 /* Gated linear recurrence.  Channels lie block by block, each block padded to a multiple of 32.
  * lcu_conv_causal: u[t] = bias + sum over taps of w[k] z[t - (taps - 1) + k] per channel (w fp32
- * [taps][ld]); inputs before this call come from state [taps - 1][ld] (element type), which is then
+ * [taps][ld], bias NULL: none), then silu when asked; inputs before this call come from state [taps - 1][ld] (element type), which is then
  * brought up to date.  lcu_gated_recurrence: r, i = sigmoid of the block-diagonal products of u (w
  * [blocks][block_width][block_width]) plus bias, log a = decay r, S = a S + sqrt(1 - a^2) i u from the fp32
  * state [ld], which is brought up to date; out = S * y.  scratch: lcu_gated_recurrence_scratch bytes. */
 int lcu_conv_causal(void* u_dev, const void* z_dev, int ldz, const void* w_dev, const void* bias_dev, void* state_dev, int taps,
-                    int dtype, int n, int channels, int ld, void* stream);
+                    int silu, int dtype, int n, int channels, int ld, void* stream);
 size_t lcu_gated_recurrence_scratch(int n, int ld);
 int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, int ldy, const void* wr_dev, const void* wi_dev,
                          const void* br_dev, const void* bi_dev, const void* decay_dev, void* state_dev, void* scratch_dev,
@@ -400,8 +407,18 @@ int lcu_gated_recurrence(void* out_dev, const void* u_dev, const void* y_dev, in
 typedef struct lcu_window_params {
   int heads, kv_heads, dk, dv, window, keep;
   float scale;
-  const void* r1_dev; /* fp32 [heads] */
+  const void* r1_dev; /* fp32 [heads]; NULL: no distance bias */
   const void* r2_dev;
+  /* lcu_attention_windowed only; zeros: nothing of this.  The last dk_shared columns of a key come from
+   * k_shared [position][dk_shared], the same for all heads; k_ld, v_ld: elements from position to position (0:
+   * kv_heads times the own columns); first_position: that of row 0 of k, v and k_shared, at or before the first
+   * window's begin; sink: fp32 [heads], exp(sink) is added to the denominator; gate [n][ldg]: the result is
+   * multiplied with sigmoid(gate). */
+  int dk_shared, k_ld, v_ld, first_position;
+  const void* k_shared_dev;
+  const void* sink_dev;
+  const void* gate_dev;
+  int ldg;
 } lcu_window_params;
 /* Rows q | k | v of a projection: k and v of row t into cache row *start + t.  v_mode 0: v as it is; 1: and
  * a copy into v_first [n][v_cols]; 2: (1 - lambda) v + lambda v_first. */
@@ -417,8 +434,69 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
                                   const void* pos_dev, int max_positions, const lcu_window_params* window, void* arrived_dev,
                                   void* stream);
 
+/* Latent attention: keys and values of all heads are products of one normed latent c per token (and a rotated key
+ * part that the heads share).  Head parts are padded to multiples of 32 (dn unrotated, dr rotated of which the
+ * first rot are turned in pairs (2i, 2i + 1); dr 0: no rotated part), values to dv, the latent to ldc (a multiple
+ * of 64); window INT_MAX: every key before.  A query head is [dn | dr]. */
+typedef struct lcu_latent_params {
+  int heads, dn, dr, rot, dv, rank, ldc, window;
+  float scale;
+} lcu_latent_params;
+/* Projected rows [n][ld] of tokens *start ...: c (rank columns from latent_at) is normed into row *start + t of
+ * latents [max_positions][ldc]; the shared key part (from key_at) is rotated into keys [max_positions][dr]; when
+ * rotate_queries, the rotated part of head h (from query_at + h (dn + dr)) is rotated in place; when low_rank > 0 the
+ * first low_rank columns are normed into low [n][low_ld].  Angle of pair i at position p: p freq[i]; gain: factor
+ * on cosine and sine.  Norm weights are fp32, padded like what they scale. */
+typedef struct lcu_latent_rows_args {
+  void* rows_dev;
+  int ld, n, latent_at, key_at, query_at, rotate_queries, low_rank, low_ld, max_positions;
+  const void* latent_norm_dev;
+  const void* low_norm_dev;
+  void* low_dev;
+  void* latents_dev;
+  void* keys_dev;
+  const void* freq_dev; /* fp32 [rot / 2] */
+  float gain, eps;
+  const void* start_dev;
+} lcu_latent_rows_args;
+int lcu_latent_rows(const lcu_latent_rows_args* rows, const lcu_latent_params* p, int dtype, void* stream);
+/* Few tokens, bfloat16, without keys and values multiplied out.  lcu_latent_queries: out [n][heads * ldc], head h =
+ * uk_t[h] [ldc][dn] times the unrotated part of the query; with rows, lcu_latent_rows in the same launch (the
+ * unrotated parts do not depend on it).  lcu_latent_attention: scores and softmax over the latents (sink as above,
+ * NULL: none), then uv [heads * dv][ldc] and the gate (NULL: none).  scratch: lcu_latent_attention_scratch bytes;
+ * lcu_latent_attention_fits: 0 where the sizes are too large for its kernels (ldc above 512). */
+int lcu_latent_queries(void* out_dev, const void* q_dev, int ldq, const void* uk_t_dev, const lcu_latent_params* p,
+                       const lcu_latent_rows_args* rows, int n, void* stream);
+int lcu_latent_attention_fits(const lcu_latent_params* p);
+int lcu_latent_slices(const lcu_latent_params* p, int n, int max_positions);
+size_t lcu_latent_attention_scratch(const lcu_latent_params* p, int n, int max_positions);
+int lcu_latent_attention(void* out_dev, int ldo, const void* q_latent_dev, const void* q_rot_dev, int ldq, const void* latents_dev,
+                         const void* keys_dev, const void* start_dev, int max_positions, const void* uv_dev, const void* sink_dev,
+                         const void* gate_dev, int ldg, const lcu_latent_params* p, void* scratch_dev, int n, void* stream);
+
+/* Gated delta rule.  Channels q [kv_heads * dk] | k [kv_heads * dk] | v [heads * dv] of a token (after their convolution,
+ * rows of ld), dim in dk (32, 64, 128 or 256) and vdim in dv (a multiple of 32, at most 256), padding zero; query/key
+ * head h / (heads / kv_heads).  q and k are made unit vectors (eps 1e-6), q times dim^-1/2; beta = sigmoid(b), g =
+ * exp(-exp(a_log) softplus(a + dt_bias)), from fp32 rows [b | a]; S = g S, S += k (beta (v - S^T k))^T, o = S^T q; out
+ * = rms norm of o over vdim, times norm, times silu(gate).  state: fp32 [heads][dk][dv], brought up to date. */
+typedef struct lcu_delta_params {
+  int heads, kv_heads, dk, dv, dim, vdim;
+  float eps;
+  const void* a_log_dev;   /* fp32 [heads] */
+  const void* dt_bias_dev; /* fp32 [heads] */
+  const void* norm_dev;    /* fp32 [vdim] */
+} lcu_delta_params;
+size_t lcu_delta_rule_scratch(const lcu_delta_params* d, int n);
+int lcu_delta_rule(void* out_dev, int ldo, const void* qkv_dev, int ld, const void* gate_dev, int ldg, const void* ba_f32_dev, int ld_ba,
+                   const lcu_delta_params* d, void* state_dev, void* scratch_dev, int dtype, int n, void* stream);
+
 /* One new token, bfloat16, fused.  x is normalised already.
  *   lcu_decode_linear: fp32 out = w . x + bias
+ *   lcu_decode_linear_bf16: the same without bias, bfloat16 out
+ *   lcu_decode_delta_in: the first `channels` rows through the step of the convolution and silu (w [taps][channels],
+ *     state [taps - 1][channels]) to u, `plain` rows to plain, the rest to tail in fp32
+ *   lcu_decode_delta_step: lcu_delta_rule for one token
+ *   lcu_decode_gated: lcu_linear_gated for one token (ld hidden units)
  *   lcu_decode_recurrent_in: rows y (GELU) and x of a recurrent block, the latter through the convolution
  *   lcu_decode_recurrent_step: gates and state of lcu_gated_recurrence for one token
  *   lcu_decode_kv: rows q | k | v, then lcu_kv_store at position *pos
@@ -429,6 +507,12 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
  *   lcu_decode_residual_router: lcu_residual_norm of the row (the sum of `top` rows of out and the gated shared
  *     row), then lcu_router of it when router_w is given */
 int lcu_decode_linear(void* out_f32_dev, const void* x_dev, const void* w_dev, const void* bias_dev, int K, int N, void* stream);
+int lcu_decode_linear_bf16(void* out_dev, const void* x_dev, const void* w_dev, int K, int N, void* stream);
+int lcu_decode_delta_in(void* u_dev, void* plain_dev, void* tail_f32_dev, void* conv_state_dev, const void* x_dev, const void* w_dev,
+                        const void* conv_dev, int taps, int K, int channels, int plain, int N, void* stream);
+int lcu_decode_delta_step(void* out_dev, const void* qkv_dev, const void* gate_dev, const void* ba_f32_dev, const lcu_delta_params* d,
+                          void* state_dev, void* stream);
+int lcu_decode_gated(void* hidden_dev, const void* h_dev, const void* w_dev, const lcu_gate_params* gate, int ld, int K, void* stream);
 int lcu_decode_recurrent_in(void* y_dev, void* u_dev, void* conv_state_dev, const void* x_dev, const void* w_dev,
                             const void* bias_dev, const void* conv_dev, const void* conv_bias_dev, int taps, int K, int ld,
                             void* stream);

@@ -7,6 +7,7 @@
 // Each entry continues the sequence of its id; the logits at the places of `want` go to DIR/<step>.f32 (fp32,
 // in order), and "done <step>" follows on standard output.  A sequence named in `end` gives its context
 // back, which the next new id takes over.  At the end of the input the program returns 0.
+#include <algorithm>
 #include <cstdio>
 #include <cstdlib>
 #include <cstring>
@@ -99,7 +100,7 @@ int main(int argc, char const** argv) {
   }
   auto model = llama_model::open(opt.model, opt.max_tokens > 0 ? opt.max_tokens : 2048, opt.type);
   if (!model) return fail("could not load the model");
-  const int most = model->max_context();
+  const int most = opt.max_tokens > 0 ? model->max_context() : std::min(model->max_context(), 8192);
   sequences seqs{*model, opt.max_tokens > 0 && opt.max_tokens < most ? opt.max_tokens : most, {}, {}};
   const size_t vocab = model->params.n_vocab;
   std::string line, error;

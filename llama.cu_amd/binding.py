@@ -93,22 +93,36 @@ SIGNATURES = {
     "lcu_fill_f16": (i32, [vp, sz, u16, vp]),
     "lcu_error_stats": (i32, [vp, vp, vp, sz, vp]),
     "lcu_linear": (i32, [vp, i32, i32, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "lcu_linear_tail": (i32, [vp, i32, vp, i32, i32, vp, vp, i32, i32, i32, i32, vp]),
     "lcu_linear_gated": (i32, [vp, i32, vp, vp, vp, i32, i32, i32, i32, vp]),
     "lcu_router": (i32, [vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
     "lcu_experts_plan": (i32, [vp, vp, vp, i32, i32, i32, vp]),
     "lcu_experts_up": (i32, [vp, i32, vp, vp, sz, vp, vp, i32, i32, i32, i32, vp]),
     "lcu_experts_down": (i32, [vp, i32, vp, vp, sz, vp, i32, i32, i32, i32, vp]),
     "lcu_embed_pos_norm": (i32, [vp, vp, vp, i32, vp, i32, vp, i32, vp, vp, vp, i32, i32, i32, i32, f32, vp]),
+    "lcu_embed_scaled": (i32, [vp, vp, vp, i32, vp, i32, f32, vp, i32, i32, i32, i32, f32, vp]),
     "lcu_residual_norm": (i32, [vp, vp, vp, vp, i32, vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
     "lcu_group_norm": (i32, [vp, vp, vp, vp, i32, i32, i32, i32, i32, f32, vp]),
     "lcu_argmax_f32": (i32, [vp, vp, i32, vp]),
     "lcu_softmax_f32": (i32, [vp, vp, i32, f32, vp]),
-    "lcu_conv_causal": (i32, [vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
+    "lcu_conv_causal": (i32, [vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32, i32, vp]),
     "lcu_gated_recurrence_scratch": (sz, [i32, i32]),
     "lcu_gated_recurrence": (i32, [vp, vp, vp, i32, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp]),
     "lcu_kv_store": (i32, [vp, vp, vp, i32, i32, i32, i32, vp, i32, vp, vp, i32, i32, i32, vp]),
     "lcu_attention_windowed": (i32, [vp, i32, vp, i32, vp, vp, i32, vp, i32, i32, vp]),
     "lcu_attention_windowed_decode": (i32, [vp, vp, vp, vp, vp, i32, vp, vp, vp]),
+    "lcu_latent_rows": (i32, [vp, vp, i32, vp]),
+    "lcu_latent_queries": (i32, [vp, vp, i32, vp, vp, vp, i32, vp]),
+    "lcu_latent_attention_fits": (i32, [vp]),
+    "lcu_latent_slices": (i32, [vp, i32, i32]),
+    "lcu_latent_attention_scratch": (sz, [vp, i32, i32]),
+    "lcu_latent_attention": (i32, [vp, i32, vp, vp, i32, vp, vp, vp, i32, vp, vp, vp, i32, vp, vp, i32, vp]),
+    "lcu_delta_rule_scratch": (sz, [vp, i32]),
+    "lcu_delta_rule": (i32, [vp, i32, vp, i32, vp, i32, vp, i32, vp, vp, vp, i32, i32, vp]),
+    "lcu_decode_delta_in": (i32, [vp] * 7 + [i32] * 5 + [vp]),
+    "lcu_decode_delta_step": (i32, [vp] * 7),
+    "lcu_decode_gated": (i32, [vp, vp, vp, vp, i32, i32, vp]),
+    "lcu_decode_linear_bf16": (i32, [vp, vp, vp, i32, i32, vp]),
     "lcu_decode_linear": (i32, [vp, vp, vp, vp, i32, i32, vp]),
     "lcu_decode_recurrent_in": (i32, [vp] * 8 + [i32, i32, i32, vp]),
     "lcu_decode_recurrent_step": (i32, [vp] * 9 + [i32, i32, vp]),
@@ -208,7 +222,26 @@ class ExpertPlan(C.Structure):
 class WindowParams(C.Structure):
     """lcu_window_params"""
     _fields_ = [("heads", i32), ("kv_heads", i32), ("dk", i32), ("dv", i32), ("window", i32), ("keep", i32), ("scale", f32),
-                ("r1", vp), ("r2", vp)]
+                ("r1", vp), ("r2", vp), ("dk_shared", i32), ("k_ld", i32), ("v_ld", i32), ("first_position", i32), ("k_shared", vp),
+                ("sink", vp), ("gate", vp), ("ldg", i32)]
+
+
+class LatentParams(C.Structure):
+    """lcu_latent_params"""
+    _fields_ = [(n, i32) for n in ("heads", "dn", "dr", "rot", "dv", "rank", "ldc", "window")] + [("scale", f32)]
+
+
+class LatentRows(C.Structure):
+    """lcu_latent_rows_args"""
+    _fields_ = [("rows", vp)] + [(n, i32) for n in ("ld", "n", "latent_at", "key_at", "query_at", "rotate_queries", "low_rank", "low_ld",
+                                                    "max_positions")] + \
+        [(n, vp) for n in ("latent_norm", "low_norm", "low", "latents", "keys", "freq")] + [("gain", f32), ("eps", f32), ("start", vp)]
+
+
+class DeltaParams(C.Structure):
+    """lcu_delta_params"""
+    _fields_ = [(n, i32) for n in ("heads", "kv_heads", "dk", "dv", "dim", "vdim")] + [("eps", f32)] + \
+        [(n, vp) for n in ("a_log", "dt_bias", "norm")]
 
 
 class DeviceBuffer:

@@ -11,10 +11,11 @@ LIB = os.path.join(PKG, "libllama_cu_amd.so")
 TIMELINE_LIB = os.path.join(PKG, "libllama_cu_amd_timeline.so")
 
 HIP_SOURCES = ["csrc/runtime.hip", "csrc/elementwise.hip", "csrc/gemv.hip", "csrc/gemm.hip", "csrc/attention.hip",
-               "csrc/linear.hip", "csrc/rownorm.hip", "csrc/recurrent.hip", "csrc/windowed.hip", "csrc/experts.hip"]
+               "csrc/linear.hip", "csrc/rownorm.hip", "csrc/recurrent.hip", "csrc/windowed.hip", "csrc/experts.hip", "csrc/latent.hip",
+               "csrc/delta.hip"]
 HOST_SOURCES = ["host/buffers.cpp", "host/params.cpp", "host/model.cpp", "host/batch.cpp", "host/tokenizer.cpp", "host/capi.cpp",
-                "host/json.cpp", "host/safetensors.cpp", "host/registry.cpp", "host/rirulix.cpp", "host/layered_model.cpp",
-                "host/layered_context.cpp"]
+                "host/json.cpp", "host/safetensors.cpp", "host/registry.cpp", "host/rirulix.cpp", "host/logivik.cpp",
+                "host/layered_model.cpp", "host/layered_context.cpp"]
 # command line programs linked against the library (found at run time next to bin/ through $ORIGIN)
 APPS = {"transform": "apps/transform.cpp", "llama_cu": "apps/llama_cu.cpp", "trace_run": "apps/trace_run.cpp"}
 BIN = os.path.join(PKG, "bin")

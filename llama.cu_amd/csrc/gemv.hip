@@ -757,6 +757,42 @@ struct conv_step_row {
   }
 };
 
+// bfloat16 rows
+struct store_bf16_row {
+  bf16_t* out;
+  __device__ __forceinline__ void operator()(int n, float v) const { out[n] = (bf16_t)v; }
+};
+
+// The rows of a delta-rule layer: the first `channels` are inputs of the convolution, whose step and silu are taken
+// here (one thread owns a channel's row and its last inputs); then `plain` rows as they are; the rest in fp32.
+struct delta_in_row {
+  bf16_t* u;
+  bf16_t* out;
+  float* tail;
+  bf16_t* state;      // [taps - 1][channels], oldest first
+  const float* conv;  // [taps][channels]
+  int taps, channels, plain;
+  __device__ __forceinline__ void operator()(int n, float v) const {
+    if (n >= channels) {
+      n -= channels;
+      if (n < plain) {
+        out[n] = (bf16_t)v;
+      } else {
+        tail[n - plain] = v;
+      }
+      return;
+    }
+    const bf16_t z = (bf16_t)v;
+    float acc = 0.0f;
+    for (int k = 0; k + 1 < taps; ++k) {
+      acc = fmaf(conv[(size_t)k * channels + n], (float)state[(size_t)k * channels + n], acc);
+      state[(size_t)k * channels + n] = k + 2 < taps ? state[(size_t)(k + 1) * channels + n] : z;
+    }
+    acc = fmaf(conv[(size_t)(taps - 1) * channels + n], (float)z, acc);
+    u[n] = (bf16_t)(acc * sigmoid_f32(acc));
+  }
+};
+
 // q | k | v rows of an attention layer: q to q_out, k and the (mixed) v to the caches' row of this position
 struct qkv_row {
   bf16_t* q_out;
@@ -1156,6 +1192,41 @@ int lcu_decode_logits(void* logits_dev, const void* x_dev, const void* norm_w_de
 int lcu_decode_linear(void* out_f32_dev, const void* x_dev, const void* w_dev, const void* bias_dev, int K, int N, void* stream) {
   LCU_REQUIRE(out_f32_dev && x_dev && w_dev && K > 0 && K % 64 == 0 && N > 0, "lcu_decode_linear: bad arguments");
   return launch_decode_rows(x_dev, w_dev, K, N, store_f32_row{(float*)out_f32_dev, (const float*)bias_dev}, as_stream(stream));
+}
+
+int lcu_decode_linear_bf16(void* out_dev, const void* x_dev, const void* w_dev, int K, int N, void* stream) {
+  LCU_REQUIRE(out_dev && x_dev && w_dev && K > 0 && K % 64 == 0 && N > 0, "lcu_decode_linear_bf16: bad arguments");
+  return launch_decode_rows(x_dev, w_dev, K, N, store_bf16_row{(bf16_t*)out_dev}, as_stream(stream));
+}
+
+int lcu_decode_delta_in(void* u_dev, void* plain_dev, void* tail_f32_dev, void* conv_state_dev, const void* x_dev, const void* w_dev,
+                        const void* conv_dev, int taps, int K, int channels, int plain, int N, void* stream) {
+  LCU_REQUIRE(u_dev && plain_dev && tail_f32_dev && x_dev && w_dev && conv_dev && (conv_state_dev || taps == 1) && taps >= 1 && K > 0 &&
+                  K % 64 == 0 && channels > 0 && plain >= 0 && N >= channels + plain,
+              "lcu_decode_delta_in: bad arguments");
+  return launch_decode_rows(x_dev, w_dev, K, N,
+                            delta_in_row{(bf16_t*)u_dev, (bf16_t*)plain_dev, (float*)tail_f32_dev, (bf16_t*)conv_state_dev,
+                                         (const float*)conv_dev, taps, channels, plain},
+                            as_stream(stream));
+}
+
+int lcu_decode_gated(void* hidden_dev, const void* h_dev, const void* w_dev, const lcu_gate_params* gate, int ld, int K, void* stream) {
+  LCU_REQUIRE(hidden_dev && h_dev && w_dev && gate, "lcu_decode_gated: null pointer");
+  LCU_REQUIRE(ld > 0 && ld % 32 == 0 && K > 0 && K % 64 == 0, "lcu_decode_gated: bad shape ld %d K %d", ld, K);
+  const clamped_gate g{gate->limit, gate->alpha, gate->up_shift};
+  expert_slots p{};  // no chosen expert: the matrix takes the place of the shared one
+  p.shared_up = (const bf16_t*)w_dev;
+  p.shared_hidden = (bf16_t*)hidden_dev;
+  p.gate = p.shared_gate = g;
+  p.ld = p.shared_ld = ld;
+  p.K = K;
+  if (K > 2048) {
+    decode_experts_up_kernel<2><<<ld, GEMV_THREADS, 0, as_stream(stream)>>>((const bf16_t*)h_dev, p);
+  } else {
+    decode_experts_up_kernel<1><<<ld, GEMV_THREADS, 0, as_stream(stream)>>>((const bf16_t*)h_dev, p);
+  }
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
 }
 
 int lcu_decode_recurrent_in(void* y_dev, void* u_dev, void* conv_state_dev, const void* x_dev, const void* w_dev,

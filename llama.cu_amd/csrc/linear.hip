@@ -137,6 +137,23 @@ int lcu_linear(void* out_dev, int out_f32, int ldo, const void* lhs_dev, const v
   return run_linear<false>(ep, dtype, lhs_dev, w_dev, M, K, N, as_stream(stream));
 }
 
+int lcu_linear_tail(void* out_dev, int ldo, void* tail_f32_dev, int ld_tail, int tail_from, const void* lhs_dev, const void* w_dev,
+                    int dtype, int M, int K, int N, void* stream) {
+  LCU_REQUIRE(out_dev && tail_f32_dev && lhs_dev && w_dev, "lcu_linear_tail: null pointer");
+  const int rc = check_linear("lcu_linear_tail", dtype, M, K, N, ldo);
+  if (rc) return rc;
+  LCU_REQUIRE(tail_from > 0 && tail_from < N && ldo >= tail_from && ld_tail >= N - tail_from,
+              "lcu_linear_tail: columns from %d of %d, row strides %d %d", tail_from, N, ldo, ld_tail);
+  linear_epilogue<false, false> ep{};
+  ep.out = out_dev;
+  ep.ldo = ldo;
+  ep.out_f32 = dtype == LCU_F32;
+  ep.tail = (float*)tail_f32_dev;
+  ep.tail_from = tail_from;
+  ep.ld_tail = ld_tail;
+  return run_linear<false>(ep, dtype, lhs_dev, w_dev, M, K, N, as_stream(stream));
+}
+
 int lcu_linear_gated(void* out_dev, int ldo, const void* lhs_dev, const void* w_dev, const lcu_gate_params* gate, int dtype,
                      int M, int K, int N, void* stream) {
   LCU_REQUIRE(out_dev && lhs_dev && w_dev && gate, "lcu_linear_gated: null pointer");

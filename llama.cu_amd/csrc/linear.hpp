@@ -39,6 +39,8 @@ struct linear_epilogue {
   bool out_f32;
   const float* bias;         // [N] or nullptr
   int gelu_cols;             // columns below this one pass through the GELU
+  float* tail;               // fp32 rows [ld_tail] of the columns from tail_from on, or nullptr
+  int tail_from, ld_tail;
   clamped_gate gate;
   const float* row_scale;    // factor of row r of lhs, or nullptr (gated products only)
   const int* tile_group;
@@ -60,6 +62,10 @@ struct linear_epilogue {
   __device__ __forceinline__ void store(int m, int n, float v) const {
     if (bias) v += bias[n];
     if (n < gelu_cols) v = gelu_tanh(v);
+    if (tail && n >= tail_from) {
+      tail[(size_t)m * ld_tail + n - tail_from] = v;
+      return;
+    }
     put(m, n, v);
   }
   __device__ __forceinline__ void store_gated(int m, int n, float g, float u) const {

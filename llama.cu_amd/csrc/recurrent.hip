@@ -8,6 +8,8 @@
 // kernel leaves a_t and the drive b_t of every token and, per chunk, the chunk's map S -> A S + B; one
 // thread per channel runs over the chunks' maps (carry), and then every chunk runs through its own
 // tokens from its incoming state (apply).
+#include <type_traits>
+
 #include "linear.hpp"
 #include "rownorm.hpp"
 
@@ -18,17 +20,17 @@ namespace {
 constexpr int CHUNK = 64;   // tokens per chunk and per gate tile
 constexpr int GATE_N = 32;  // channels per gate tile
 
-// u[t][c] = bias[c] + sum_k w[k][c] z[t - (taps - 1) + k]; inputs before this call come from state
-// [taps - 1][ld], oldest first.  A thread takes four channels of CONV_T tokens.
+// u[t][c] = bias[c] + sum_k w[k][c] z[t - (taps - 1) + k], then silu where asked; inputs before this call come from
+// state [taps - 1][ld], oldest first.  A thread takes four channels of CONV_T tokens.
 constexpr int CONV_T = 8;
-template <class T>
+template <class T, bool SILU>
 __global__ __launch_bounds__(256) void conv_causal_kernel(T* __restrict__ u, const T* __restrict__ z, int ldz,
                                                           const float* __restrict__ w, const float* __restrict__ bias,
                                                           const T* __restrict__ state, int taps, int n, int channels, int ld) {
   const int c = (blockIdx.x * 256 + threadIdx.x) * 4, t0 = blockIdx.y * CONV_T;
   if (c >= channels) return;
   float4_t acc[CONV_T];
-  const float4_t b = load4(bias + c);
+  const float4_t b = bias ? load4(bias + c) : (float4_t)(0.0f);
 #pragma unroll
   for (int e = 0; e < CONV_T; ++e) acc[e] = b;
   for (int k = 0; k < taps; ++k) {
@@ -43,6 +45,10 @@ __global__ __launch_bounds__(256) void conv_causal_kernel(T* __restrict__ u, con
   }
 #pragma unroll
   for (int e = 0; e < CONV_T; ++e) {
+    if constexpr (SILU) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[e][i] *= sigmoid_f32(acc[e][i]);
+    }
     if (t0 + e < n) store4(u + (size_t)(t0 + e) * ld + c, acc[e]);
   }
 }
@@ -371,26 +377,25 @@ int check_channels(const char* who, int dtype, int n, int channels, int ld) {
 extern "C" {
 
 int lcu_conv_causal(void* u_dev, const void* z_dev, int ldz, const void* w_dev, const void* bias_dev, void* state_dev, int taps,
-                    int dtype, int n, int channels, int ld, void* stream) {
-  LCU_REQUIRE(u_dev && z_dev && w_dev && bias_dev && (state_dev || taps == 1), "lcu_conv_causal: null pointer");
+                    int silu, int dtype, int n, int channels, int ld, void* stream) {
+  LCU_REQUIRE(u_dev && z_dev && w_dev && (state_dev || taps == 1), "lcu_conv_causal: null pointer");
   const int rc = check_channels("lcu_conv_causal", dtype, n, channels, ld);
   if (rc) return rc;
   LCU_REQUIRE(taps >= 1 && ldz >= channels && ldz % 4 == 0 && channels % 4 == 0, "lcu_conv_causal: taps %d, input stride %d", taps, ldz);
   if (n == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
   const dim3 grid((channels / 4 + 255) / 256, (n + CONV_T - 1) / CONV_T), columns((channels + 255) / 256);
+  const auto run = [&](auto* kind, auto act) {
+    using T = std::remove_pointer_t<decltype(kind)>;
+    conv_causal_kernel<T, decltype(act)::value><<<grid, 256, 0, st>>>((T*)u_dev, (const T*)z_dev, ldz, (const float*)w_dev,
+                                                                      (const float*)bias_dev, (const T*)state_dev, taps, n, channels, ld);
+    if (taps > 1) conv_state_kernel<T><<<columns, 256, 0, st>>>((T*)state_dev, (const T*)z_dev, ldz, n, taps, channels, ld);
+  };
+  const auto typed = [&](auto* kind) { silu ? run(kind, std::true_type{}) : run(kind, std::false_type{}); };
   if (dtype == LCU_F32) {
-    conv_causal_kernel<float><<<grid, 256, 0, st>>>((float*)u_dev, (const float*)z_dev, ldz, (const float*)w_dev,
-                                                    (const float*)bias_dev, (const float*)state_dev, taps, n, channels, ld);
-    if (taps > 1) {
-      conv_state_kernel<float><<<columns, 256, 0, st>>>((float*)state_dev, (const float*)z_dev, ldz, n, taps, channels, ld);
-    }
+    typed((float*)nullptr);
   } else {
-    conv_causal_kernel<bf16_t><<<grid, 256, 0, st>>>((bf16_t*)u_dev, (const bf16_t*)z_dev, ldz, (const float*)w_dev,
-                                                     (const float*)bias_dev, (const bf16_t*)state_dev, taps, n, channels, ld);
-    if (taps > 1) {
-      conv_state_kernel<bf16_t><<<columns, 256, 0, st>>>((bf16_t*)state_dev, (const bf16_t*)z_dev, ldz, n, taps, channels, ld);
-    }
+    typed((bf16_t*)nullptr);
   }
   LCU_LAUNCH_CHECK();
   return LCU_OK;

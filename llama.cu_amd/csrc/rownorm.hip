@@ -12,29 +12,33 @@ using namespace lcu;
 
 namespace {
 
-// x[row] = norm(table[token] + pos_table[start + row]) under w0; h[row] = norm(x[row]) under w1 when given
+// x[row] = scale table[token] + pos_table[start + row] (when given), its norm under w0 (when given); h[row] = x[row],
+// its norm under w1 when given
 template <class T, int NV, int TH>
 __global__ __launch_bounds__(TH) void embed_pos_norm_kernel(float* __restrict__ x, T* __restrict__ h,
-                                                                     const int* __restrict__ ids, const T* __restrict__ table,
+                                                                     const int* __restrict__ ids, const T* __restrict__ table, float scale,
                                                                      const T* __restrict__ pos_table, const float* __restrict__ w0,
                                                                      const float* __restrict__ w1, const int* __restrict__ start,
                                                                      int n_vocab, int n_pos, row_shape rs) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = blockIdx.x;
-  const int id = min(max(ids[r], 0), n_vocab - 1), p = min(max(*start + r, 0), n_pos - 1);
+  const int id = min(max(ids[r], 0), n_vocab - 1);
   row_t<NV, TH> row, at, w, next;
-  load_row(w, w0, rs);
+  if (w0) load_row(w, w0, rs);
   if (w1) load_row(next, w1, rs);
   load_row(row, table + (size_t)id * rs.ld, rs);
-  load_row(at, pos_table + (size_t)p * rs.ld, rs);
 #pragma unroll
-  for (int j = 0; j < NV; ++j) row.v[j] += at.v[j];
-  scale_row(row, rs, lds, w);
-  store_row(x + (size_t)r * rs.ld, row, rs);
-  if (w1) {
-    scale_row(row, rs, lds, next);
-    store_row(h + (size_t)r * rs.ld, row, rs);
+  for (int j = 0; j < NV; ++j) row.v[j] *= scale;
+  if (pos_table) {
+    load_row(at, pos_table + (size_t)min(max(*start + r, 0), n_pos - 1) * rs.ld, rs);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) row.v[j] += at.v[j];
   }
+  if (w0) scale_row(row, rs, lds, w);
+  store_row(x + (size_t)r * rs.ld, row, rs);
+  if (!h) return;
+  if (w1) scale_row(row, rs, lds, next);
+  store_row(h + (size_t)r * rs.ld, row, rs);
 }
 
 // what sublayers left for row r: its rows of src.out, and the shared expert's row times its gate
@@ -58,7 +62,7 @@ __device__ __forceinline__ void load_sum(row_t<NV, TH>& m, row_t<NV, TH>& t, con
   }
 }
 
-// m = the sublayer's result; x += norm(m) under w_after; h = norm(x) under w_next.
+// m = the sublayer's result; x += norm(m) under w_after; h = x, its norm under w_next when given.
 template <class T, int NV, int TH>
 __global__ __launch_bounds__(TH) void residual_norm_kernel(float* __restrict__ x, T* __restrict__ h,
                                                                     sublayer_rows src, const float* __restrict__ w_after,
@@ -74,11 +78,12 @@ __global__ __launch_bounds__(TH) void residual_norm_kernel(float* __restrict__ x
 #pragma unroll
   for (int j = 0; j < NV; ++j) m.v[j] += old.v[j];
   store_row(xr, m, rs);
+  if (!h) return;
   if (w_next) {
     load_row(t, w_next, rs);
     scale_row(m, rs, lds, t);
-    store_row(h + (size_t)r * rs.ld, m, rs);
   }
+  store_row(h + (size_t)r * rs.ld, m, rs);
 }
 
 // The step between two sublayers for one row, and the router behind it when there is one: every wavefront
@@ -110,8 +115,8 @@ __global__ __launch_bounds__(STEP_THREADS) void residual_step_kernel(float* __re
 #pragma unroll
   for (int j = 0; j < NV; ++j) m.v[j] += old.v[j];
   store_row(x, m, rs);
-  if (!w_next) return;
-  scale_row(m, rs, lds, next);
+  if (!h) return;
+  if (w_next) scale_row(m, rs, lds, next);
   store_row(h, m, rs);
   if (!rt.w) return;
   bf16_t* hs = reinterpret_cast<bf16_t*>(lds);  // scale_row is done with it
@@ -292,8 +297,27 @@ int lcu_embed_pos_norm(void* x_dev, void* h_dev, const void* ids_dev, int n_ids,
   with_row_kind(dtype, ld, n_ids == 1, [&](auto* kind, auto nv, auto th) {
     using T = std::remove_pointer_t<decltype(kind)>;
     embed_pos_norm_kernel<T, decltype(nv)::value, decltype(th)::value><<<n_ids, decltype(th)::value, row_lds_bytes(rs), st>>>(
-        (float*)x_dev, (T*)h_dev, (const int*)ids_dev, (const T*)table_dev, (const T*)pos_table_dev, (const float*)w_embed_dev,
+        (float*)x_dev, (T*)h_dev, (const int*)ids_dev, (const T*)table_dev, 1.0f, (const T*)pos_table_dev, (const float*)w_embed_dev,
         (const float*)w_next_dev, (const int*)start_dev, n_vocab, n_pos, rs);
+  });
+  LCU_LAUNCH_CHECK();
+  return LCU_OK;
+}
+
+int lcu_embed_scaled(void* x_dev, void* h_dev, const void* ids_dev, int n_ids, const void* table_dev, int n_vocab, float scale,
+                     const void* w_next_dev, int dtype, int width, int ld, int groups, float eps, void* stream) {
+  LCU_REQUIRE(x_dev && ids_dev && table_dev && (h_dev || !w_next_dev), "lcu_embed_scaled: null pointer");
+  const row_shape rs{width, ld, groups, eps};
+  const int rc = check_rows("lcu_embed_scaled", dtype, n_ids, rs);
+  if (rc) return rc;
+  LCU_REQUIRE(n_vocab > 0, "lcu_embed_scaled: bad table size %d", n_vocab);
+  if (n_ids == 0) return LCU_OK;
+  hipStream_t st = as_stream(stream);
+  with_row_kind(dtype, ld, n_ids == 1, [&](auto* kind, auto nv, auto th) {
+    using T = std::remove_pointer_t<decltype(kind)>;
+    embed_pos_norm_kernel<T, decltype(nv)::value, decltype(th)::value><<<n_ids, decltype(th)::value, row_lds_bytes(rs), st>>>(
+        (float*)x_dev, (T*)h_dev, (const int*)ids_dev, (const T*)table_dev, scale, nullptr, nullptr, (const float*)w_next_dev, nullptr,
+        n_vocab, 0, rs);
   });
   LCU_LAUNCH_CHECK();
   return LCU_OK;

@@ -1,7 +1,9 @@
 // Attention over a key/value cache with a sliding window, kept first tokens, grouped heads and a
 // per-head distance bias:
 //   score(i, j) = scale q_i.k_j - r1 ln(1 + r2 (i - j)),  visible when j <= i and (i - j < window or j < keep)
-// followed by an ordinary softmax.  Scores, softmax and weighted sums are fp32.
+// followed by a softmax, whose denominator may hold one more term per head, exp(sink).  Scores, softmax and weighted
+// sums are fp32.  The last columns of a key may come from an array that all heads share, and the result may be
+// multiplied with the sigmoid of a gate (neither in the one-token kernel).
 //
 // Layouts: q rows of heads x dk inside rows of ldq elements; caches k [positions][kv_heads * dk] and
 // v [positions][kv_heads * dv].  dk is the head size padded to a multiple of 32, dv the value size padded
@@ -21,8 +23,15 @@ struct window_args {
   int heads, kv_heads, dk, dv, ldq, ldo;
   int window, keep;
   float scale;
-  const float* r1;
+  const float* r1;     // NULL: no distance bias
   const float* r2;
+  int k_ld, v_ld;      // elements from position to position
+  int base;            // position of the first row of k, v and k_shared
+  int dk_shared;       // the last dk_shared columns of a key are k_shared [position][dk_shared]
+  const void* k_shared;
+  const float* sink;   // [heads] or NULL
+  const void* gate;    // [row][ldg], heads x dv, or NULL
+  int ldg;
 };
 
 // first key of the window of position i, and how many kept keys lie below it
@@ -68,15 +77,16 @@ __global__ __launch_bounds__(256) void attention_row_kernel(T* __restrict__ out,
   __shared__ float red[4];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int t = blockIdx.x, h = blockIdx.y, g = h / (p.heads / p.kv_heads), i = start + t;
-  const int lo = window_begin(p, i), kept = min(p.keep, lo), n_keys = kept + i - lo + 1;
+  const int lo = window_begin(p, i), kept = min(p.keep, lo), n_keys = kept + i - lo + 1, own = p.dk - p.dk_shared;
   const T* qr = q + (size_t)t * p.ldq + (size_t)h * p.dk;
-  const float r1 = p.r1[h], r2 = p.r2[h];
-  float m = -INFINITY;
+  const float r1 = p.r1 ? p.r1[h] : 0.0f, r2 = p.r1 ? p.r2[h] : 0.0f;
+  float m = p.sink ? p.sink[h] : -INFINITY;
   for (int x = wave; x < n_keys; x += 4) {
     const int j = x < kept ? x : lo + x - kept;
-    const T* kr = k + ((size_t)j * p.kv_heads + g) * p.dk;
+    const T* kr = k + (size_t)(j - p.base) * p.k_ld + (size_t)g * own;
+    const T* ks = (const T*)p.k_shared + (size_t)(j - p.base) * p.dk_shared;
     float s = 0.0f;
-    for (int c = lane; c < p.dk; c += WAVE) s = fmaf(to_f32(qr[c]), to_f32(kr[c]), s);
+    for (int c = lane; c < p.dk; c += WAVE) s = fmaf(to_f32(qr[c]), to_f32(c < own ? kr[c] : ks[c - own]), s);
     s = wave_sum(s) * p.scale - r1 * log1pf(r2 * (float)(i - j));
     if (lane == 0) sc[x] = s;
     m = fmaxf(m, s);
@@ -95,13 +105,16 @@ __global__ __launch_bounds__(256) void attention_row_kernel(T* __restrict__ out,
   if (lane == 0) red[wave] = l;
   __syncthreads();
   l = (red[0] + red[1]) + (red[2] + red[3]);
+  if (p.sink) l += expf(p.sink[h] - m);
   for (int c = tid; c < p.dv; c += 256) {
     float o = 0.0f;
     for (int x = 0; x < n_keys; ++x) {
       const int j = x < kept ? x : lo + x - kept;
-      o = fmaf(sc[x], to_f32(v[((size_t)j * p.kv_heads + g) * p.dv + c]), o);
+      o = fmaf(sc[x], to_f32(v[(size_t)(j - p.base) * p.v_ld + (size_t)g * p.dv + c]), o);
     }
-    out[(size_t)t * p.ldo + (size_t)h * p.dv + c] = (T)(o / l);
+    o /= l;
+    if (p.gate) o *= sigmoid_f32(to_f32(((const T*)p.gate)[(size_t)t * p.ldg + (size_t)h * p.dv + c]));
+    out[(size_t)t * p.ldo + (size_t)h * p.dv + c] = (T)o;
   }
 }
 
@@ -112,7 +125,7 @@ __global__ __launch_bounds__(256) void attention_row_kernel(T* __restrict__ out,
 // remainder), so that they keep 16 significant bits.
 constexpr int QT = 64, KT = 64;
 
-template <int DV>
+template <int DV, bool BIAS>
 __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                                                              const bf16_t* __restrict__ k, const bf16_t* __restrict__ v, int n,
                                                              int start, window_args p) {
@@ -132,7 +145,8 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict_
     *reinterpret_cast<uint4_t*>(Qs + r * ldk + e) =
         *reinterpret_cast<const uint4_t*>(q + (size_t)min(q0 + r, n - 1) * p.ldq + (size_t)h * p.dk + e);
   }
-  const float r1 = p.r1[h], r2 = p.r2[h];
+  const float r1 = BIAS ? p.r1[h] : 0.0f, r2 = BIAS ? p.r2[h] : 0.0f;
+  const int own8 = (p.dk - p.dk_shared) / 8;
   const int first = start + q0, last = start + min(q0 + QT, n) - 1;  // positions of the tile's rows
   const int win_tile = window_begin(p, first) / KT, kept_tiles = (min(p.keep, first + QT) + KT - 1) / KT;
   const int col = lane & 15, quad = lane >> 4;
@@ -140,8 +154,8 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict_
   float4_t o[NT];
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
-    m[e] = -1e30f;
-    l[e] = 0.0f;
+    m[e] = p.sink ? p.sink[h] : -1e30f;  // the sink counts as a key of value zero
+    l[e] = p.sink ? 1.0f : 0.0f;
   }
 #pragma unroll
   for (int t = 0; t < NT; ++t) o[t] = (float4_t)(0.0f);
@@ -152,13 +166,16 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict_
     const int k0 = kt * KT;
     __syncthreads();  // the previous tile has been read
     for (int c = tid; c < KT * dk8; c += 256) {
-      const int r = c / dk8, e = (c % dk8) * 8;
-      *reinterpret_cast<uint4_t*>(Ks + r * ldk + e) =
-          *reinterpret_cast<const uint4_t*>(k + ((size_t)min(k0 + r, last) * p.kv_heads + g) * p.dk + e);
+      const int r = c / dk8, e = c % dk8;
+      const size_t row = max(min(k0 + r, last) - p.base, 0);
+      const bf16_t* src = e < own8 ? k + row * p.k_ld + ((size_t)g * own8 + e) * 8
+                                   : (const bf16_t*)p.k_shared + row * p.dk_shared + (e - own8) * 8;
+      *reinterpret_cast<uint4_t*>(Ks + r * ldk + e * 8) = *reinterpret_cast<const uint4_t*>(src);
     }
     for (int c = tid; c < KT * (DV / 8); c += 256) {
       const int r = c % KT, e = (c / KT) * 8;
-      const bf16x8_t x = *reinterpret_cast<const bf16x8_t*>(v + ((size_t)min(k0 + r, last) * p.kv_heads + g) * DV + e);
+      const size_t row = max(min(k0 + r, last) - p.base, 0);
+      const bf16x8_t x = *reinterpret_cast<const bf16x8_t*>(v + row * p.v_ld + (size_t)g * DV + e);
 #pragma unroll
       for (int b = 0; b < 8; ++b) Vt[(e + b) * LDP + r] = x[b];
     }
@@ -184,7 +201,8 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict_
       for (int t = 0; t < 4; ++t) {
         const int j = k0 + t * 16 + col, d = i - j;
         see[t] = d >= 0 && (d < p.window || j < p.keep);
-        s[t][e] = s[t][e] * p.scale - r1 * __logf(1.0f + r2 * (float)max(d, 0));
+        s[t][e] *= p.scale;
+        if constexpr (BIAS) s[t][e] -= r1 * __logf(1.0f + r2 * (float)max(d, 0));
         if (see[t]) top = fmaxf(top, s[t][e]);
       }
       top = fmaxf(top, dpp_f32<0xB1>(top));
@@ -226,7 +244,11 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict_
     if (r < n) {
       const float inv = 1.0f / l[e];
 #pragma unroll
-      for (int t = 0; t < NT; ++t) out[(size_t)r * p.ldo + (size_t)h * DV + t * 16 + col] = (bf16_t)(o[t][e] * inv);
+      for (int t = 0; t < NT; ++t) {
+        float x = o[t][e] * inv;
+        if (p.gate) x *= sigmoid_f32((float)((const bf16_t*)p.gate)[(size_t)r * p.ldg + (size_t)h * DV + t * 16 + col]);
+        out[(size_t)r * p.ldo + (size_t)h * DV + t * 16 + col] = (bf16_t)x;
+      }
     }
   }
 }
@@ -235,11 +257,11 @@ size_t tile_lds(int dk, int dv) {
   return ((size_t)(QT + KT) * (dk + 8) + (size_t)dv * (KT + 8) + (size_t)4 * 2 * 16 * (KT + 8)) * 2;
 }
 
-template <int DV>
+template <int DV, bool BIAS>
 int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, int start, const window_args& p, hipStream_t st) {
   const size_t lds = tile_lds(p.dk, DV);
   LCU_REQUIRE(lds <= 160 * 1024, "lcu_attention_windowed: head size %d with value size %d", p.dk, DV);
-  auto kernel = attention_tile_kernel<DV>;
+  auto kernel = attention_tile_kernel<DV, BIAS>;
   static bool raised[16] = {};  // per device, once
   int dev = 0;
   LCU_HIP(hipGetDevice(&dev));
@@ -460,19 +482,42 @@ int launch_decode(bf16_t* out, const bf16_t* q, const bf16_t* k, const bf16_t* v
 }
 
 int check_window(const char* who, const lcu_window_params* w, int dtype) {
-  LCU_REQUIRE(w && w->r1_dev && w->r2_dev, "%s: null pointer", who);
+  LCU_REQUIRE(w && (!w->r1_dev || w->r2_dev), "%s: null pointer", who);
   LCU_REQUIRE(dtype == LCU_BF16 || dtype == LCU_F32, "%s: element type %d", who, dtype);
   LCU_REQUIRE(w->heads > 0 && w->kv_heads > 0 && w->heads % w->kv_heads == 0 && w->dk > 0 && w->dk % 32 == 0 && w->dk <= 256 &&
                   (w->dv == 32 || w->dv == 64 || w->dv == 128 || w->dv == 256),
               "%s: heads %d / %d, head size %d (a multiple of 32, at most 256), value size %d (32, 64, 128, 256)", who, w->heads,
               w->kv_heads, w->dk, w->dv);
   LCU_REQUIRE(w->window > 0 && w->keep >= 0 && w->heads <= 65535, "%s: window %d keep %d", who, w->window, w->keep);
+  LCU_REQUIRE(w->dk_shared >= 0 && w->dk_shared % 8 == 0 && w->dk_shared < w->dk && (w->dk_shared == 0 || w->k_shared_dev),
+              "%s: %d shared columns of a key of %d", who, w->dk_shared, w->dk);
+  LCU_REQUIRE((w->k_ld == 0 || (w->k_ld >= w->kv_heads * (w->dk - w->dk_shared) && w->k_ld % 8 == 0)) &&
+                  (w->v_ld == 0 || (w->v_ld >= w->kv_heads * w->dv && w->v_ld % 8 == 0)),
+              "%s: position strides %d %d", who, w->k_ld, w->v_ld);
+  LCU_REQUIRE(!w->gate_dev || w->ldg >= w->heads * w->dv, "%s: gate rows of %d", who, w->ldg);
   return LCU_OK;
 }
 
 window_args make_window(const lcu_window_params* w, int ldq, int ldo) {
-  return window_args{w->heads, w->kv_heads, w->dk, w->dv, ldq, ldo, w->window, w->keep, w->scale, (const float*)w->r1_dev,
-                     (const float*)w->r2_dev};
+  return window_args{w->heads,
+                     w->kv_heads,
+                     w->dk,
+                     w->dv,
+                     ldq,
+                     ldo,
+                     w->window,
+                     w->keep,
+                     w->scale,
+                     (const float*)w->r1_dev,
+                     (const float*)w->r2_dev,
+                     w->k_ld ? w->k_ld : w->kv_heads * (w->dk - w->dk_shared),
+                     w->v_ld ? w->v_ld : w->kv_heads * w->dv,
+                     w->first_position,
+                     w->dk_shared,
+                     w->k_shared_dev,
+                     (const float*)w->sink_dev,
+                     w->gate_dev,
+                     w->ldg};
 }
 
 }  // namespace
@@ -512,6 +557,10 @@ int lcu_attention_windowed(void* out_dev, int ldo, const void* q_dev, int ldq, c
   if (rc) return rc;
   LCU_REQUIRE(n >= 0 && start >= 0 && ldq >= window->heads * window->dk && ldo >= window->heads * window->dv && ldq % 8 == 0,
               "lcu_attention_windowed: bad shape n %d start %d strides %d %d", n, start, ldq, ldo);
+  LCU_REQUIRE(window->first_position >= 0 &&
+                  (window->first_position == 0 ||
+                   (window->keep == 0 && (long)window->first_position <= std::max(0L, (long)start - window->window + 1))),
+              "lcu_attention_windowed: keys from position %d on do not hold the window of position %d", window->first_position, start);
   if (n == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
   const window_args p = make_window(window, ldq, ldo);
@@ -531,11 +580,16 @@ int lcu_attention_windowed(void* out_dev, int ldo, const void* q_dev, int ldq, c
     LCU_LAUNCH_CHECK();
     return LCU_OK;
   }
+  const auto run = [&](auto size) {
+    constexpr int DV = decltype(size)::value;
+    return p.r1 ? launch_tiles<DV, true>(out_dev, q_dev, k_cache_dev, v_cache_dev, n, start, p, st)
+                : launch_tiles<DV, false>(out_dev, q_dev, k_cache_dev, v_cache_dev, n, start, p, st);
+  };
   switch (window->dv) {
-    case 32: return launch_tiles<32>(out_dev, q_dev, k_cache_dev, v_cache_dev, n, start, p, st);
-    case 64: return launch_tiles<64>(out_dev, q_dev, k_cache_dev, v_cache_dev, n, start, p, st);
-    case 128: return launch_tiles<128>(out_dev, q_dev, k_cache_dev, v_cache_dev, n, start, p, st);
-    default: return launch_tiles<256>(out_dev, q_dev, k_cache_dev, v_cache_dev, n, start, p, st);
+    case 32: return run(std::integral_constant<int, 32>{});
+    case 64: return run(std::integral_constant<int, 64>{});
+    case 128: return run(std::integral_constant<int, 128>{});
+    default: return run(std::integral_constant<int, 256>{});
   }
 }
 
@@ -546,6 +600,9 @@ int lcu_attention_windowed_decode(void* out_dev, const void* q_dev, const void* 
   const int rc = check_window("lcu_attention_windowed_decode", window, LCU_BF16);
   if (rc) return rc;
   const int R = window->heads / window->kv_heads;
+  LCU_REQUIRE(window->r1_dev && window->dk_shared == 0 && !window->sink_dev && !window->gate_dev && window->first_position == 0 &&
+                  window->k_ld == 0 && window->v_ld == 0,
+              "lcu_attention_windowed_decode: only the distance bias and caches of its own layout");
   LCU_REQUIRE(R <= DEC_MAX_GROUP && max_positions > 0, "lcu_attention_windowed_decode: %d query heads per kv head (at most %d)", R,
               DEC_MAX_GROUP);
   hipStream_t st = as_stream(stream);

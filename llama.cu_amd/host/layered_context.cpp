@@ -1,17 +1,27 @@
-// The step of a layered decoder.  A layer is x += norm1b(mixer(norm1(x))), x += norm2b(ff(norm2(x))); the
-// launch that adds a sublayer's result also normalises the next sublayer's input.
+// The step of a layered decoder.  A layer is x += norm1b(mixer(norm1(x))), x += norm2b(ff(norm2(x))), without norm1
+// and norm2 where sublayers read x itself; the launch that adds a sublayer's result also leaves the next
+// sublayer's input.
 #include "layered_context.hpp"
 
 #include <stdlib.h>
 #include <string.h>
 
 #include <algorithm>
+#include <limits>
 
 namespace llama_cu {
 
 namespace {
 constexpr int MAX_ROWS = 2048;  // tokens of one pass: bounds the activations, not the prompt
+// Calls of at most this many tokens attend over the latents; longer ones multiply keys and values out, which
+// costs the visible keys once but makes every row's sums several times shorter.
+constexpr int FEW_ROWS = 32;
+
+lcu_latent_params latent_shape(latent_weights const& w, latent_params const& p) {
+  return lcu_latent_params{p.heads, w.dn, w.dr, p.rot.dims, w.dv, p.kv_rank, w.ldc, p.window > 0 ? p.window : std::numeric_limits<int>::max(),
+                           p.scale};
 }
+}  // namespace
 
 layered_context_impl::layered_context_impl(layered_model_impl* model, int context_len, float temperature)
     : llama_context(context_len, temperature), model_(model), rows_(std::min(context_len, MAX_ROWS)) {
@@ -20,6 +30,7 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   LCU_CHECK(lcu_stream_create(&stream_));
   layered_model_impl const& m = *model_;
   const size_t R = rows_, e = m.elem, ctx = context_len_;
+  size_t low = 0, queries = 0, latent_queries = 0, keys_values = 0, tail = 0;
   size_t counters = 1, wide = 0, u = 0, rec = 0, scratch = 0, hidden = 0, shared = 0, expert_rows = 0, v_first = 0, experts = 0, tiles = 0;
   state_.resize(m.layers.size());
   for (size_t l = 0; l < m.layers.size(); ++l) {
@@ -33,6 +44,35 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
       scratch = std::max(scratch, lcu_gated_recurrence_scratch((int)R, (int)ld));
       if (p.recurrence.taps > 1) state_[l].conv = zeroed((p.recurrence.taps - 1) * ld * e);
       state_[l].s = zeroed(ld * 4);
+    } else if (p.mixer == mixer_type::latent) {
+      latent_weights const& a = w.latent;
+      const lcu_latent_params lp = latent_shape(a, p.latent);
+      wide = std::max(wide, (size_t)a.ldw);
+      rec = std::max(rec, (size_t)a.ldo);
+      if (p.latent.q_rank > 0) {
+        low = std::max(low, (size_t)a.low_ld);
+        queries = std::max(queries, (size_t)a.q_cols);
+      }
+      if (a.few) {
+        latent_queries = std::max(latent_queries, (size_t)p.latent.heads * a.ldc);
+        for (size_t n = 1; n <= std::min<size_t>(FEW_ROWS, R); ++n) {
+          scratch = std::max(scratch, lcu_latent_attention_scratch(&lp, (int)n, (int)ctx));
+        }
+      }
+      const size_t seen = p.latent.window > 0 ? std::min(ctx, (size_t)p.latent.window + R) : ctx;
+      keys_values = std::max(keys_values, seen * p.latent.heads * (a.dn + a.dv));
+      state_[l].k = zeroed(ctx * a.ldc * e);
+      if (a.dr > 0) state_[l].v = zeroed(ctx * a.dr * e);
+    } else if (p.mixer == mixer_type::delta) {
+      delta_weights const& d = w.delta;
+      const lcu_delta_params dp = delta_shape(d, p.delta);
+      wide = std::max(wide, (size_t)d.channels + d.plain);
+      u = std::max(u, (size_t)d.channels);
+      tail = std::max(tail, (size_t)2 * p.delta.heads);
+      rec = std::max(rec, (size_t)d.ldo);
+      scratch = std::max(scratch, lcu_delta_rule_scratch(&dp, (int)R));
+      if (p.delta.taps > 1) state_[l].conv = zeroed((size_t)(p.delta.taps - 1) * d.channels * e);
+      state_[l].s = zeroed((size_t)p.delta.heads * d.dk * d.dv * 4);
     } else {
       wide = std::max(wide, (size_t)w.attention.ldq);
       rec = std::max(rec, (size_t)w.attention.ldo);
@@ -41,7 +81,8 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
       state_[l].k = zeroed(ctx * w.attention.k_cols * e);
       state_[l].v = zeroed(ctx * w.attention.v_cols * e);
     }
-    if (p.has_mlp) {
+    if (p.dense.ff > 0) shared = std::max(shared, R * (size_t)w.dense.ld);
+    if (p.has_mlp && p.dense.ff == 0) {
       const size_t top = p.mlp.top, E = p.mlp.experts;
       expert_rows = std::max(expert_rows, R * top);
       hidden = std::max(hidden, R * top * (size_t)w.mlp.ld);
@@ -58,6 +99,11 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
   t_u_ = zeroed(R * u * e);
   t_rec_ = zeroed(R * rec * e);
   t_scratch_ = zeroed(scratch);
+  t_low_ = zeroed(R * low * e);
+  t_queries_ = zeroed(R * queries * e);
+  t_latent_queries_ = zeroed(std::min<size_t>(FEW_ROWS, R) * latent_queries * e);
+  t_keys_values_ = zeroed(keys_values * e);
+  t_tail_ = zeroed(R * tail * 4);
   t_hidden_ = zeroed(hidden * e);
   t_shared_hidden_ = zeroed(shared * e);
   t_expert_out_ = zeroed((expert_rows + 1) * ld * 4);  // a one-token step keeps the shared expert's row behind the others
@@ -75,6 +121,9 @@ layered_context_impl::layered_context_impl(layered_model_impl* model, int contex
     if (m.shape.layers[l].mixer != mixer_type::attention) continue;
     const int group = a.heads / a.kv_heads;
     if (group > 16 || group * (m.layers[l].attention.dv + 2) > 2400) fused_step_ = false;
+  }
+  for (size_t l = 0; l < m.layers.size(); ++l) {
+    if (m.shape.layers[l].mixer == mixer_type::latent && !m.layers[l].latent.few) fused_step_ = false;
   }
   t_arrived_ = zeroed(counters * 4);
   t_step_ = zeroed((1 + R) * 4);
@@ -114,7 +163,7 @@ size_t layered_context_impl::context_memory_usage() {
   size_t count = 0;
   for (layer_state const& s : state_) count += s.k.size() + s.v.size() + s.conv.size() + s.s.size();
   for (gpu_buffer const* b :
-       {&t_x_, &t_h_, &t_m_, &t_wide_, &t_u_, &t_rec_, &t_scratch_, &t_hidden_, &t_shared_hidden_, &t_expert_out_, &t_shared_out_,
+       {&t_low_, &t_queries_, &t_latent_queries_, &t_keys_values_, &t_tail_, &t_x_, &t_h_, &t_m_, &t_wide_, &t_u_, &t_rec_, &t_scratch_, &t_hidden_, &t_shared_hidden_, &t_expert_out_, &t_shared_out_,
         &t_v_first_, &t_choice_, &t_weight_, &t_shared_gate_, &t_row_token_, &t_row_weight_, &t_inverse_, &t_tile_expert_,
         &t_tile_row_, &t_expert_end_, &t_n_tiles_, &t_arrived_, &t_step_, &t_want_, &t_head_in_, &t_logits_, &t_probs_, &t_index_}) {
     count += b->size();
@@ -131,7 +180,7 @@ void layered_context_impl::recurrence(recurrence_weights const& w, recurrence_pa
   const size_t e = m.elem;
   char* y = (char*)t_wide_.data();
   LCU_CHECK(lcu_linear(y, 0, 2 * w.ld, t_h_.data(), w.yx.data(), w.yx_bias.data(), w.ld, m.dtype, n, m.ld, 2 * w.ld, stream_));
-  LCU_CHECK(lcu_conv_causal(t_u_.data(), y + (size_t)w.ld * e, 2 * w.ld, w.conv.data(), w.conv_bias.data(), s.conv.data(), p.taps,
+  LCU_CHECK(lcu_conv_causal(t_u_.data(), y + (size_t)w.ld * e, 2 * w.ld, w.conv.data(), w.conv_bias.data(), s.conv.data(), p.taps, 0,
                             m.dtype, n, w.channels, w.ld, stream_));
   LCU_CHECK(lcu_gated_recurrence(t_rec_.data(), t_u_.data(), y, 2 * w.ld, w.gate_r.data(), w.gate_i.data(), w.bias_r.data(),
                                  w.bias_i.data(), w.decay.data(), s.s.data(), t_scratch_.data(), m.dtype, n, w.channels, w.block,
@@ -149,6 +198,123 @@ void layered_context_impl::attention(attention_weights const& w, attention_param
                                    m.dtype, n, stream_));
   LCU_CHECK(lcu_linear(t_m_.data(), 1, m.ld, t_rec_.data(), w.out.data(), w.out_bias.data(), 0, m.dtype, n, w.ldo, m.shape.width,
                        stream_));
+}
+
+// `fused`: one token in bfloat16, products as weight streams.
+void layered_context_impl::latent(latent_weights const& w, latent_params const& p, layer_state& s, int n, bool fused) {
+  layered_model_impl const& m = *model_;
+  const lcu_latent_params lp = latent_shape(w, p);
+  const auto product = [&](gpu_buffer& out, gpu_buffer const& x, gpu_buffer const& weight, int K, int N) {
+    if (fused) {
+      LCU_CHECK(lcu_decode_linear_bf16(out.data(), x.data(), weight.data(), K, N, stream_));
+    } else {
+      LCU_CHECK(lcu_linear(out.data(), 0, N, x.data(), weight.data(), nullptr, 0, m.dtype, n, K, N, stream_));
+    }
+  };
+  lcu_latent_rows_args rows{};
+  rows.rows_dev = t_wide_.data();
+  rows.ld = w.ldw;
+  rows.n = n;
+  rows.latent_at = w.latent_at;
+  rows.key_at = w.key_at;
+  rows.query_at = w.dn;
+  rows.rotate_queries = w.dr > 0 && p.q_rank == 0;
+  rows.low_rank = p.q_rank;
+  rows.low_ld = w.low_ld;
+  rows.max_positions = context_len_;
+  rows.latent_norm_dev = w.latent_norm.data();
+  rows.low_norm_dev = w.low_norm.data();
+  rows.low_dev = t_low_.data();
+  rows.latents_dev = s.k.data();
+  rows.keys_dev = s.v.data();
+  rows.freq_dev = w.freq.data();
+  rows.gain = w.gain;
+  rows.eps = m.shape.norm_eps;
+  rows.start_dev = start();
+  const bool few = w.few && n <= FEW_ROWS, low = p.q_rank > 0;
+  product(t_wide_, t_h_, w.in, m.ld, w.ldw);
+  if (low || !few) LCU_CHECK(lcu_latent_rows(&rows, &lp, m.dtype, stream_));
+  if (low) product(t_queries_, t_low_, w.uq, w.low_ld, w.q_cols);
+  const char* q = (char*)(low ? t_queries_ : t_wide_).data();
+  const int ldq = low ? w.q_cols : w.ldw;
+  const void* gate = p.gate ? (char*)t_wide_.data() + (size_t)w.gate_at * m.elem : nullptr;
+  char* values = (char*)w.ukv.data() + (size_t)p.heads * w.dn * w.ldc * m.elem;
+  if (few) {
+    LCU_CHECK(lcu_latent_queries(t_latent_queries_.data(), q, ldq, w.uk_t.data(), &lp, low ? nullptr : &rows, n, stream_));
+    LCU_CHECK(lcu_latent_attention(t_rec_.data(), w.ldo, t_latent_queries_.data(), q + (size_t)w.dn * m.elem, ldq, s.k.data(), s.v.data(),
+                                   start(), context_len_, values, p.sink ? w.sink.data() : nullptr, gate, w.ldw, &lp, t_scratch_.data(), n,
+                                   stream_));
+  } else {
+    // keys and values of every position the call sees
+    const int first = p.window > 0 ? std::max(0, start_pos_ - p.window + 1) : 0, seen = start_pos_ + n - first;
+    const int keys = p.heads * w.dn, cols = keys + p.heads * w.dv;
+    LCU_CHECK(lcu_linear(t_keys_values_.data(), 0, cols, (char*)s.k.data() + (size_t)first * w.ldc * m.elem, w.ukv.data(), nullptr, 0,
+                         m.dtype, seen, w.ldc, cols, stream_));
+    lcu_window_params window{};
+    window.heads = window.kv_heads = p.heads;
+    window.dk = w.dn + w.dr;
+    window.dv = w.dv;
+    window.window = lp.window;
+    window.scale = p.scale;
+    window.dk_shared = w.dr;
+    window.k_ld = window.v_ld = cols;
+    window.first_position = first;
+    window.k_shared_dev = w.dr > 0 ? (char*)s.v.data() + (size_t)first * w.dr * m.elem : nullptr;
+    window.sink_dev = p.sink ? w.sink.data() : nullptr;
+    window.gate_dev = gate;
+    window.ldg = w.ldw;
+    LCU_CHECK(lcu_attention_windowed(t_rec_.data(), w.ldo, q, ldq, t_keys_values_.data(),
+                                     (char*)t_keys_values_.data() + (size_t)keys * m.elem, start_pos_, &window, m.dtype, n, stream_));
+  }
+  if (fused) {
+    LCU_CHECK(lcu_decode_linear(t_m_.data(), t_rec_.data(), w.out.data(), nullptr, w.ldo, m.shape.width, stream_));
+  } else {
+    LCU_CHECK(lcu_linear(t_m_.data(), 1, m.ld, t_rec_.data(), w.out.data(), nullptr, 0, m.dtype, n, w.ldo, m.shape.width, stream_));
+  }
+}
+
+lcu_delta_params layered_context_impl::delta_shape(delta_weights const& w, delta_params const& p) const {
+  return lcu_delta_params{p.heads, p.kv_heads, w.dk, w.dv, p.dim, p.vdim, model_->shape.norm_eps, w.a_log.data(), w.dt_bias.data(),
+                          w.norm.data()};
+}
+
+void layered_context_impl::delta(delta_weights const& w, delta_params const& p, layer_state& s, int n) {
+  layered_model_impl const& m = *model_;
+  const lcu_delta_params d = delta_shape(w, p);
+  const int ld = w.channels + w.plain, tail = 2 * p.heads;
+  LCU_CHECK(lcu_linear_tail(t_wide_.data(), ld, t_tail_.data(), tail, ld, t_h_.data(), w.in.data(), m.dtype, n, m.ld, w.rows, stream_));
+  LCU_CHECK(lcu_conv_causal(t_u_.data(), t_wide_.data(), ld, w.conv.data(), nullptr, s.conv.data(), p.taps, 1, m.dtype, n, w.channels,
+                            w.channels, stream_));
+  LCU_CHECK(lcu_delta_rule(t_rec_.data(), w.ldo, t_u_.data(), w.channels, (char*)t_wide_.data() + (size_t)w.channels * m.elem, ld,
+                           t_tail_.data(), tail, &d, s.s.data(), t_scratch_.data(), m.dtype, n, stream_));
+  LCU_CHECK(lcu_linear(t_m_.data(), 1, m.ld, t_rec_.data(), w.out.data(), nullptr, 0, m.dtype, n, w.ldo, m.shape.width, stream_));
+}
+
+void layered_context_impl::decode_delta(delta_weights const& w, delta_params const& p, layer_state& s) {
+  layered_model_impl const& m = *model_;
+  const lcu_delta_params d = delta_shape(w, p);
+  LCU_CHECK(lcu_decode_delta_in(t_u_.data(), t_wide_.data(), t_tail_.data(), s.conv.data(), t_h_.data(), w.in.data(), w.conv.data(), p.taps,
+                                m.ld, w.channels, w.plain, w.rows, stream_));
+  LCU_CHECK(lcu_decode_delta_step(t_rec_.data(), t_u_.data(), t_wide_.data(), t_tail_.data(), &d, s.s.data(), stream_));
+  LCU_CHECK(lcu_decode_linear(t_m_.data(), t_rec_.data(), w.out.data(), nullptr, w.ldo, m.shape.width, stream_));
+}
+
+void layered_context_impl::dense(dense_weights const& w, dense_params const& p, int n) {
+  layered_model_impl const& m = *model_;
+  LCU_CHECK(lcu_linear_gated(t_shared_hidden_.data(), w.ld, t_h_.data(), w.up.data(), &p.gate, m.dtype, n, m.ld, 2 * w.ld, stream_));
+  LCU_CHECK(lcu_linear(t_m_.data(), 1, m.ld, t_shared_hidden_.data(), w.down.data(), nullptr, 0, m.dtype, n, w.ld, m.shape.width, stream_));
+}
+
+void layered_context_impl::embed(int n, void* w_next) {
+  layered_model_impl const& m = *model_;
+  layered_params const& p = m.shape;
+  if (p.learned_positions && p.embed_norm) {
+    LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), n, m.embed.data(), p.vocab, m.pos.data(), p.max_positions, start(),
+                                 m.embed_norm.data(), w_next, m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps, stream_));
+  } else {
+    LCU_CHECK(lcu_embed_scaled(t_x_.data(), t_h_.data(), ids(), n, m.embed.data(), p.vocab, p.embed_scale, w_next, m.dtype, p.width, m.ld,
+                               p.norm_groups, p.norm_eps, stream_));
+  }
 }
 
 void layered_context_impl::experts(experts_weights const& w, experts_params const& p, int n) {
@@ -175,24 +341,28 @@ void layered_context_impl::experts(experts_weights const& w, experts_params cons
 void layered_context_impl::enqueue_rows(int n) {
   layered_model_impl const& m = *model_;
   layered_params const& p = m.shape;
-  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), n, m.embed.data(), p.vocab, m.pos.data(), p.max_positions,
-                               start(), m.embed_norm.data(), next_norm(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps,
-                               stream_));
+  embed(n, next_norm(0));
   for (size_t l = 0; l < m.layers.size(); ++l) {
     layer_params const& q = p.layers[l];
     layer_weights const& w = m.layers[l];
-    if (q.mixer == mixer_type::rglru) {
-      recurrence(w.recurrence, q.recurrence, state_[l], n);
-    } else {
-      attention(w.attention, q.attention, state_[l], n);
+    const bool last = l + 1 == m.layers.size();  // nobody reads t_h_ after it
+    switch (q.mixer) {
+      case mixer_type::rglru: recurrence(w.recurrence, q.recurrence, state_[l], n); break;
+      case mixer_type::attention: attention(w.attention, q.attention, state_[l], n); break;
+      case mixer_type::latent: latent(w.latent, q.latent, state_[l], n, false); break;
+      case mixer_type::delta: delta(w.delta, q.delta, state_[l], n); break;
     }
-    LCU_CHECK(lcu_residual_norm(t_x_.data(), t_h_.data(), t_m_.data(), nullptr, 1, nullptr, nullptr, w.norm1b.data(),
-                                q.has_mlp ? w.norm2.data() : next_norm(l + 1), m.dtype, n, p.width, m.ld, p.norm_groups, p.norm_eps,
-                                stream_));
-    if (q.has_mlp) {
+    LCU_CHECK(lcu_residual_norm(t_x_.data(), last && !q.has_mlp ? nullptr : t_h_.data(), t_m_.data(), nullptr, 1, nullptr, nullptr,
+                                w.norm1b.data(), q.has_mlp ? w.norm2.data() : next_norm(l + 1), m.dtype, n, p.width, m.ld, p.norm_groups,
+                                p.norm_eps, stream_));
+    if (q.dense.ff > 0) {
+      dense(w.dense, q.dense, n);
+      LCU_CHECK(lcu_residual_norm(t_x_.data(), last ? nullptr : t_h_.data(), t_m_.data(), nullptr, 1, nullptr, nullptr, w.norm2b.data(),
+                                  next_norm(l + 1), m.dtype, n, p.width, m.ld, p.norm_groups, p.norm_eps, stream_));
+    } else if (q.has_mlp) {
       experts(w.mlp, q.mlp, n);
       const bool shared = q.mlp.shared_ff > 0;
-      LCU_CHECK(lcu_residual_norm(t_x_.data(), t_h_.data(), t_expert_out_.data(), t_inverse_.data(), q.mlp.top,
+      LCU_CHECK(lcu_residual_norm(t_x_.data(), last ? nullptr : t_h_.data(), t_expert_out_.data(), t_inverse_.data(), q.mlp.top,
                                   shared ? t_shared_out_.data() : nullptr, shared ? t_shared_gate_.data() : nullptr, w.norm2b.data(),
                                   next_norm(l + 1), m.dtype, n, p.width, m.ld, p.norm_groups, p.norm_eps, stream_));
     }
@@ -206,18 +376,18 @@ void layered_context_impl::enqueue_rows(int n) {
   }
 }
 
-// One token: launches fused around the weight streams.  A recurrent layer's mixer takes three (both branches
+// One token: launches fused around the weight streams.  A recurrent layer's mixer takes three (projections
 // with the convolution, gates with the state, output product), an attention layer's too (projections with the
-// cache rows, attention, output product), a feed-forward two (first products, second products); between
-// sublayers one launch adds the result, takes both norms and, in front of a feed-forward, routes.  The last
+// cache rows, attention, output product), a latent layer's five (projections; keys applied to the queries, with norm,
+// rotations and cache rows; scores; values; output product; two more with a queries' latent), a feed-forward two
+// (first products, second products); between sublayers one launch adds the result, takes both norms and, in front of a feed-forward, routes.  The last
 // layer's norms end in the final one.
 void layered_context_impl::enqueue_one() {
   layered_model_impl const& m = *model_;
   layered_params const& p = m.shape;
   const size_t n_layers = m.layers.size();
   const auto norm_ahead = [&](size_t l) { return l < n_layers ? m.layers[l].norm1.data() : m.final_norm.data(); };
-  LCU_CHECK(lcu_embed_pos_norm(t_x_.data(), t_h_.data(), ids(), 1, m.embed.data(), p.vocab, m.pos.data(), p.max_positions, start(),
-                               m.embed_norm.data(), norm_ahead(0), m.dtype, p.width, m.ld, p.norm_groups, p.norm_eps, stream_));
+  embed(1, norm_ahead(0));
   for (size_t l = 0; l < n_layers; ++l) {
     layer_params const& q = p.layers[l];
     layer_weights const& L = m.layers[l];
@@ -229,6 +399,10 @@ void layered_context_impl::enqueue_one() {
       LCU_CHECK(lcu_decode_recurrent_step(t_rec_.data(), t_u_.data(), t_wide_.data(), w.gate_r.data(), w.gate_i.data(), w.bias_r.data(),
                                           w.bias_i.data(), w.decay.data(), s.s.data(), w.channels, w.block, stream_));
       LCU_CHECK(lcu_decode_linear(t_m_.data(), t_rec_.data(), w.out.data(), nullptr, w.ld, p.width, stream_));
+    } else if (q.mixer == mixer_type::latent) {
+      latent(L.latent, q.latent, s, 1, true);
+    } else if (q.mixer == mixer_type::delta) {
+      decode_delta(L.delta, q.delta, s);
     } else {
       attention_weights const& w = L.attention;
       attention_params const& a = q.attention;
@@ -245,7 +419,12 @@ void layered_context_impl::enqueue_one() {
                                          q.has_mlp ? L.norm2.data() : norm_ahead(l + 1), p.width, m.ld, p.norm_groups, p.norm_eps,
                                          w.router.data(), q.mlp.experts, q.mlp.top, t_choice_.data(), t_weight_.data(),
                                          shared ? t_shared_gate_.data() : nullptr, stream_));
-    if (q.has_mlp) {
+    if (q.dense.ff > 0) {
+      LCU_CHECK(lcu_decode_gated(t_shared_hidden_.data(), t_h_.data(), L.dense.up.data(), &q.dense.gate, L.dense.ld, m.ld, stream_));
+      LCU_CHECK(lcu_decode_linear(t_m_.data(), t_shared_hidden_.data(), L.dense.down.data(), nullptr, L.dense.ld, p.width, stream_));
+      LCU_CHECK(lcu_decode_residual_router(t_x_.data(), t_h_.data(), t_m_.data(), 1, nullptr, nullptr, L.norm2b.data(), norm_ahead(l + 1),
+                                           p.width, m.ld, p.norm_groups, p.norm_eps, nullptr, 0, 0, nullptr, nullptr, nullptr, stream_));
+    } else if (q.has_mlp) {
       LCU_CHECK(lcu_decode_experts_up(t_hidden_.data(), t_shared_hidden_.data(), t_h_.data(), t_choice_.data(), t_weight_.data(),
                                       w.up.data(), w.up_stride, &q.mlp.gate, w.shared_up.data(), &q.mlp.shared_gate, q.mlp.top, w.ld,
                                       w.shared_ld, m.ld, stream_));

@@ -23,8 +23,8 @@ struct layered_context_impl final : public llama_context {
  private:
   // what a layer carries from token to token
   struct layer_state {
-    gpu_buffer k, v;         // attention: [context][kv_heads * dk], [context][kv_heads * dv]
-    gpu_buffer conv, s;      // recurrence: the convolution's last inputs [taps - 1][ld], the fp32 state [ld]
+    gpu_buffer k, v;         // attention: [context][kv_heads * dk], [context][kv_heads * dv]; latent: [context][ldc], [context][dr]
+    gpu_buffer conv, s;      // recurrences: the convolution's last inputs [taps - 1][ld], the fp32 state
   };
   gpu_buffer zeroed(size_t bytes);
   void enqueue_rows(int n);                        // n tokens, launch by launch
@@ -33,7 +33,13 @@ struct layered_context_impl final : public llama_context {
   void drop_graph();
   void recurrence(recurrence_weights const& w, recurrence_params const& p, layer_state& s, int n);
   void attention(attention_weights const& w, attention_params const& p, layer_state& s, int n);
+  void latent(latent_weights const& w, latent_params const& p, layer_state& s, int n, bool fused);
+  void delta(delta_weights const& w, delta_params const& p, layer_state& s, int n);
+  void decode_delta(delta_weights const& w, delta_params const& p, layer_state& s);
+  void dense(dense_weights const& w, dense_params const& p, int n);
   void experts(experts_weights const& w, experts_params const& p, int n);
+  void embed(int n, void* w_next);
+  lcu_delta_params delta_shape(delta_weights const& w, delta_params const& p) const;
   void enqueue_head(int n_rows);
   void* next_norm(size_t layer) const;             // weights of the norm in front of layer `layer`, or NULL
 
@@ -41,6 +47,7 @@ struct layered_context_impl final : public llama_context {
   int rows_;                                       // tokens of one pass; longer calls run in several
   std::vector<layer_state> state_;
   gpu_buffer t_x_, t_h_, t_m_, t_wide_, t_u_, t_rec_, t_scratch_, t_hidden_, t_shared_hidden_, t_expert_out_, t_shared_out_;
+  gpu_buffer t_low_, t_queries_, t_latent_queries_, t_keys_values_, t_tail_;  // latent attention, delta rule
   gpu_buffer t_v_first_, t_choice_, t_weight_, t_shared_gate_, t_row_token_, t_row_weight_, t_inverse_, t_tile_expert_,
       t_tile_row_, t_expert_end_, t_n_tiles_;
   gpu_buffer t_step_, t_want_, t_head_in_, t_logits_, t_probs_, t_index_;

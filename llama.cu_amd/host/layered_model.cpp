@@ -3,6 +3,8 @@
 #include <math.h>
 #include <string.h>
 
+#include <algorithm>
+
 #include "layered.hpp"
 #include "safetensors.hpp"
 
@@ -74,6 +76,26 @@ size_t gate_row(size_t j) { return j / 32 * 64 + j % 32; }
 
 int padded_value_size(int vdim) { return vdim <= 32 ? 32 : vdim <= 64 ? 64 : vdim <= 128 ? 128 : 256; }
 
+// [heads][ldc][dn] from the keys' rows of a latent layer's ukv
+std::vector<char> transposed_keys(latent_weights const& w, int heads, const char* ukv, size_t elem) {
+  std::vector<char> t((size_t)heads * w.ldc * w.dn * elem);
+  for (size_t h = 0; h < (size_t)heads; ++h) {
+    for (size_t d = 0; d < (size_t)w.dn; ++d) {
+      for (size_t r = 0; r < (size_t)w.ldc; ++r) {
+        memcpy(&t[((h * w.ldc + r) * w.dn + d) * elem], ukv + ((h * w.dn + d) * w.ldc + r) * elem, elem);
+      }
+    }
+  }
+  return t;
+}
+
+gpu_buffer upload_bytes(std::vector<char> const& v) {
+  gpu_buffer b(v.size());
+  b.copy_from(v.data(), v.size());
+  LCU_CHECK(lcu_sync(nullptr));
+  return b;
+}
+
 struct loader {
   layered_model_impl& m;
   safetensors_file const& file;
@@ -88,11 +110,13 @@ struct loader {
     }
     return t;
   }
-  gpu_buffer vector(std::string const& name, size_t n) {
+  gpu_buffer vector(std::string const& name, size_t n, float shift = 0.0f) {
     std::vector<float> v(round_up(n, 64), 0.0f);  // padded like the rows they scale
     put_vector(v, *get(name, {n}), [](size_t i) { return i; });
+    for (size_t i = 0; i < n; ++i) v[i] += shift;
     return upload_vector(v);
   }
+  gpu_buffer norm(std::string const& name) { return vector(name, m.shape.width, m.shape.norm_shift); }
   gpu_buffer matrix(std::string const& name, size_t rows, size_t cols, size_t ld) {
     packed_matrix p(m.dtype, rows, ld);
     stored_tensor const& t = *get(name, {rows, cols});
@@ -167,6 +191,85 @@ struct loader {
     }
   }
 
+  void latent(latent_weights& w, latent_params const& p, std::string const& at) {
+    const size_t W = m.shape.width, H = p.heads, D = p.dim, X = p.rot_dim, E = p.vdim, R = p.kv_rank, Q = p.q_rank;
+    const auto same = [](size_t c) { return c; };
+    packed_matrix in(m.dtype, w.ldw, m.ld), ukv(m.dtype, H * (w.dn + w.dv), w.ldc), out(m.dtype, W, w.ldo);
+    // a query head is [unrotated | rotated], each part padded
+    const auto query_row = [&](size_t r) {
+      const size_t d = r % (D + X);
+      return r / (D + X) * (w.dn + w.dr) + (d < D ? d : w.dn + d - D);
+    };
+    if (Q > 0) {
+      stored_tensor const *dq = get(at + "dq", {Q, W}), *uq = get(at + "uq", {H * (D + X), Q});
+      packed_matrix up(m.dtype, w.q_cols, w.low_ld);
+      if (ok) in.put(*dq, Q, W);
+      if (ok) up.put(*uq, H * (D + X), Q, query_row, same);
+      w.uq = up.upload();
+      w.low_norm = vector(at + "dq.norm", Q);
+    } else {
+      stored_tensor const* q = get(at + "q", {H * (D + X), W});
+      if (ok) in.put(*q, H * (D + X), W, query_row, same);
+    }
+    stored_tensor const *dkv = get(at + "dkv", {R + X, W}), *uk = get(at + "uk", {H * D, R}), *uv = get(at + "uv", {H * E, R});
+    stored_tensor const* o = get(at + "o", {W, H * E});
+    if (!ok) return;
+    in.put(*dkv, R + X, W, [&](size_t r) { return r < R ? w.latent_at + r : w.key_at + r - R; }, same);
+    ukv.put(*uk, H * D, R, [&](size_t r) { return r / D * w.dn + r % D; }, same);
+    const auto value = [&](size_t c) { return c / E * w.dv + c % E; };
+    ukv.put(*uv, H * E, R, [&](size_t r) { return H * w.dn + value(r); }, same);
+    out.put(*o, W, H * E, same, value);
+    if (p.gate) {
+      stored_tensor const* g = get(at + "g", {H * E, W});
+      if (ok) in.put(*g, H * E, W, [&](size_t r) { return w.gate_at + value(r); }, same);
+    }
+    w.in = in.upload();
+    w.ukv = ukv.upload();
+    if (w.few) w.uk_t = upload_bytes(transposed_keys(w, p.heads, (const char*)ukv.h.data(), m.elem));
+    w.out = out.upload();
+    w.latent_norm = vector(at + "dkv.norm", R);
+    if (p.sink) w.sink = vector(at + "sink", H);
+  }
+
+  void delta(delta_weights& w, delta_params const& p, std::string const& at) {
+    const size_t W = m.shape.width, H = p.heads, G = p.kv_heads, D = p.dim, E = p.vdim, T = p.taps;
+    const auto same = [](size_t c) { return c; };
+    packed_matrix in(m.dtype, w.rows, m.ld), out(m.dtype, W, w.ldo);
+    std::vector<float> conv(T * w.channels, 0.0f);
+    const auto part = [&](const char* name, size_t heads, size_t dim, size_t padded, size_t first) {
+      stored_tensor const *t = get(at + name, {heads * dim, W}), *c = get(at + name + ".conv", {heads * dim, T});
+      if (!ok) return;
+      const auto row = [&](size_t r) { return first + r / dim * padded + r % dim; };
+      in.put(*t, heads * dim, W, row, same);
+      for (size_t r = 0; r < heads * dim; ++r) {
+        for (size_t k = 0; k < T; ++k) conv[k * w.channels + row(r)] = c->at(r * T + k);
+      }
+    };
+    part("q", G, D, w.dk, 0);
+    part("k", G, D, w.dk, G * w.dk);
+    part("v", H, E, w.dv, 2 * G * w.dk);
+    stored_tensor const *g = get(at + "g", {H * E, W}), *b = get(at + "b", {H, W}), *a = get(at + "a", {H, W}), *o = get(at + "o", {W, H * E});
+    if (!ok) return;
+    const auto value = [&](size_t c) { return c / E * w.dv + c % E; };
+    in.put(*g, H * E, W, [&](size_t r) { return w.channels + value(r); }, same);
+    in.put(*b, H, W, w.channels + w.plain);
+    in.put(*a, H, W, w.channels + w.plain + H);
+    out.put(*o, W, H * E, same, value);
+    w.in = in.upload();
+    w.conv = upload_vector(conv);
+    w.out = out.upload();
+    w.a_log = vector(at + "A_log", H);
+    w.dt_bias = vector(at + "dt_bias", H);
+    w.norm = vector(at + "norm", E);
+  }
+
+  void dense(dense_weights& w, dense_params const& p, std::string const& at) {
+    packed_matrix up(m.dtype, 2 * w.ld, m.ld), down(m.dtype, m.shape.width, w.ld);
+    expert(up, 0, down, 0, at, p.ff);
+    w.up = up.upload();
+    w.down = down.upload();
+  }
+
   // one expert's matrices into rows of a packed pair
   void expert(packed_matrix& up, size_t up_row, packed_matrix& down, size_t down_row, std::string const& at, size_t ff) {
     const size_t W = m.shape.width;
@@ -201,25 +304,32 @@ struct loader {
   bool run() {
     layered_params const& s = m.shape;
     m.embed = matrix("embed", s.vocab, s.width, m.ld);
-    m.pos = matrix("pos", s.max_positions, s.width, m.ld);
-    m.embed_norm = vector("embed.norm", s.width);
-    m.final_norm = vector("final.norm", s.width);
+    if (s.learned_positions) m.pos = matrix("pos", s.max_positions, s.width, m.ld);
+    if (s.embed_norm) m.embed_norm = norm("embed.norm");
+    m.final_norm = norm("final.norm");
     m.head = matrix("head", s.vocab, s.width, m.ld);
     for (size_t l = 0; ok && l < s.layers.size(); ++l) {
       layer_params const& p = s.layers[l];
       layer_weights& w = m.layers[l];
       const std::string at = "l" + std::to_string(l) + ".";
-      w.norm1 = vector(at + "norm1", s.width);
-      w.norm1b = vector(at + "norm1b", s.width);
-      if (p.mixer == mixer_type::rglru) {
-        recurrence(w.recurrence, p.recurrence, at + "mix.");
-      } else {
-        attention(w.attention, p.attention, at + "mix.");
+      // the norm on a sublayer's result has the plain name where there is none ahead of it
+      const std::string after = s.norm_ahead ? "b" : "";
+      if (s.norm_ahead) w.norm1 = norm(at + "norm1");
+      w.norm1b = norm(at + "norm1" + after);
+      switch (p.mixer) {
+        case mixer_type::rglru: recurrence(w.recurrence, p.recurrence, at + "mix."); break;
+        case mixer_type::attention: attention(w.attention, p.attention, at + "mix."); break;
+        case mixer_type::latent: latent(w.latent, p.latent, at + "mix."); break;
+        case mixer_type::delta: delta(w.delta, p.delta, at + "mix."); break;
       }
       if (p.has_mlp) {
-        w.norm2 = vector(at + "norm2", s.width);
-        w.norm2b = vector(at + "norm2b", s.width);
-        experts(w.mlp, p.mlp, at + "mlp.");
+        if (s.norm_ahead) w.norm2 = norm(at + "norm2");
+        w.norm2b = norm(at + "norm2" + after);
+        if (p.dense.ff > 0) {
+          dense(w.dense, p.dense, at + "mlp.");
+        } else {
+          experts(w.mlp, p.mlp, at + "mlp.");
+        }
       }
     }
     return ok;
@@ -238,7 +348,9 @@ static llama_params outline(layered_params const& s) {
   p.n_vocab = (uint32_t)s.vocab;
   p.norm_eps = s.norm_eps;
   for (layer_params const& l : s.layers) {
-    if (l.mixer == mixer_type::attention && (uint32_t)l.attention.heads > p.n_heads) p.n_heads = (uint32_t)l.attention.heads;
+    for (int heads : {l.attention.heads, l.latent.heads, l.delta.heads}) {
+      if ((uint32_t)heads > p.n_heads) p.n_heads = (uint32_t)heads;
+    }
   }
   return p;
 }
@@ -259,6 +371,30 @@ void layered_model_impl::lay_out() {
       w.block = (int)round_up(p.recurrence.width / p.recurrence.blocks, 32);
       w.channels = w.block * p.recurrence.blocks;
       w.ld = (int)round_up(w.channels, 64);
+    } else if (p.mixer == mixer_type::latent) {
+      latent_weights& w = layers[l].latent;
+      latent_params const& a = p.latent;
+      w.dn = (int)round_up(a.dim, 32);
+      w.dr = (int)round_up(a.rot_dim, 32);
+      w.dv = padded_value_size(a.vdim);
+      w.ldc = (int)round_up(a.kv_rank, 64);
+      w.low_ld = (int)round_up(a.q_rank, 64);
+      w.q_cols = a.heads * (w.dn + w.dr);
+      w.latent_at = a.q_rank > 0 ? w.low_ld : w.q_cols;
+      w.key_at = w.latent_at + w.ldc;
+      w.gate_at = w.key_at + w.dr;
+      w.ldw = (int)round_up(w.gate_at + (a.gate ? a.heads * w.dv : 0), 64);
+      w.ldo = (int)round_up(a.heads * w.dv, 64);
+      const lcu_latent_params lp{a.heads, w.dn, w.dr, a.rot.dims, w.dv, a.kv_rank, w.ldc, 1, a.scale};
+      w.few = dtype == LCU_BF16 && lcu_latent_attention_fits(&lp) != 0;
+    } else if (p.mixer == mixer_type::delta) {
+      delta_weights& w = layers[l].delta;
+      w.dk = padded_value_size(p.delta.dim);
+      w.dv = (int)round_up(p.delta.vdim, 32);
+      w.channels = (int)round_up(2 * p.delta.kv_heads * w.dk + p.delta.heads * w.dv, 64);
+      w.plain = p.delta.heads * w.dv;
+      w.rows = w.channels + w.plain + 2 * p.delta.heads;
+      w.ldo = (int)round_up(w.plain, 64);
     } else {
       attention_weights& w = layers[l].attention;
       w.dk = (int)round_up(p.attention.dim, 32);
@@ -273,7 +409,8 @@ void layered_model_impl::lay_out() {
         first_mix = false;
       }
     }
-    if (p.has_mlp) {
+    if (p.dense.ff > 0) layers[l].dense.ld = (int)round_up(p.dense.ff, 64);
+    if (p.has_mlp && p.dense.ff == 0) {
       experts_weights& w = layers[l].mlp;
       w.ld = (int)round_up(p.mlp.ff, 64);
       w.shared_ld = (int)round_up(p.mlp.shared_ff, 64);
@@ -304,9 +441,50 @@ bool layered_model_impl::shapes_supported() const {
         first_v = &a;
       }
     }
+    if (p.mixer == mixer_type::latent && (layers[l].latent.dn + layers[l].latent.dr > 256 || p.latent.vdim > 256)) {
+      return bad(at + "head size " + std::to_string(p.latent.dim) + " + " + std::to_string(p.latent.rot_dim) + " / " +
+                 std::to_string(p.latent.vdim) + " (at most 256, parts in multiples of 32)");
+    }
+    if (p.mixer == mixer_type::delta && (p.delta.dim > 256 || p.delta.vdim > 256)) {
+      return bad(at + "head size " + std::to_string(p.delta.dim) + " / " + std::to_string(p.delta.vdim) + " (at most 256)");
+    }
     if (p.has_mlp && p.mlp.experts > 512) return bad(at + std::to_string(p.mlp.experts) + " experts (at most 512)");
   }
   return true;
+}
+
+int layered_model_impl::max_context() const {
+  // the fp32 attention kernel keeps the scores of every visible key
+  if (dtype == LCU_F32) {
+    for (layer_params const& p : shape.layers) {
+      if (p.mixer == mixer_type::latent && (p.latent.window == 0 || p.latent.window > 32768)) return std::min(shape.max_positions, 32768);
+    }
+  }
+  return shape.max_positions;
+}
+
+std::vector<float> rotation_params::frequencies(float& gain) const {
+  const double pi = 3.14159265358979323846;
+  std::vector<float> f(dims / 2);
+  // the pair that turns t times within `original` positions
+  const auto pair_of = [&](double t) { return dims * log(original / (2.0 * pi * t)) / (2.0 * log(base)); };
+  const double lo = std::max(floor(pair_of(fast)), 0.0), hi = std::min(ceil(pair_of(slow)), dims - 1.0);
+  for (int i = 0; i < dims / 2; ++i) {
+    const double plain = pow(base, -2.0 * i / dims);
+    const double ramp = scaled ? std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0) : 0.0;
+    f[i] = (float)(plain / factor * ramp + plain * (1.0 - ramp));
+  }
+  gain = scaled ? (float)(0.1 * log(factor) + 1.0) : 1.0f;
+  return f;
+}
+
+// the rotation's table, which no weight file holds
+void layered_model_impl::make_tables() {
+  for (size_t l = 0; l < layers.size(); ++l) {
+    if (shape.layers[l].latent.rot.dims == 0) continue;
+    latent_weights& w = layers[l].latent;
+    w.freq = upload_vector(shape.layers[l].latent.rot.frequencies(w.gain));
+  }
 }
 
 /* static */ std::unique_ptr<llama_model> layered_model_impl::load(layered_params const& p, element_type type,
@@ -318,6 +496,7 @@ bool layered_model_impl::shapes_supported() const {
   LCU_CHECK(lcu_init(0));
   loader l{*m, file};
   if (!l.run()) return nullptr;
+  m->make_tables();
   return m;
 }
 
@@ -340,9 +519,21 @@ bool layered_model_impl::shapes_supported() const {
     LCU_CHECK(lcu_fill_normal_matrix(b.data(), 1, (int)n, (int)n, LCU_F32, seed, ++stream, mean, std, nullptr));
     return b;
   };
+  // `count` blocks of `rows` rows, `apart` rows from one to the next, from row `first` of b on: padding rows stay zero
+  const auto blocks = [&](gpu_buffer& b, size_t first, size_t count, size_t rows, size_t apart, size_t cols, size_t row_ld) {
+    for (size_t k = 0; k < count; ++k) {
+      LCU_CHECK(lcu_fill_normal_matrix((char*)b.data() + (first + k * apart) * row_ld * m->elem, rows, (int)cols, (int)row_ld, dtype, seed,
+                                       ++stream, 0.0f, 1.0f / sqrtf((float)cols), nullptr));
+    }
+  };
+  const auto zeros = [&](size_t rows, size_t row_ld) {
+    gpu_buffer b(rows * row_ld * m->elem);
+    LCU_CHECK(lcu_memset(b.data(), 0, b.size(), nullptr));
+    return b;
+  };
   const size_t W = p.width, V = p.vocab, ld = m->ld;
-  m->embed = matrix(V, W, ld, 1.0f);
-  m->pos = matrix(p.max_positions, W, ld, 0.5f);
+  m->embed = matrix(V, W, ld, 1.0f / p.embed_scale);
+  if (p.learned_positions) m->pos = matrix(p.max_positions, W, ld, 0.5f);
   m->embed_norm = vector(W, 1.0f, 0.1f);
   m->final_norm = vector(W, 1.0f, 0.1f);
   m->head = linear(V, W, ld);
@@ -363,6 +554,52 @@ bool layered_model_impl::shapes_supported() const {
       w.bias_i = vector(C, 0.0f, 0.1f);
       w.decay = vector(C, q.recurrence.decay * 0.1f, 0.05f);
       w.out = linear(W, C, C);
+    } else if (q.mixer == mixer_type::latent) {
+      latent_weights& w = L.latent;
+      latent_params const& a = q.latent;
+      const size_t H = a.heads, D = a.dim, X = a.rot_dim, E = a.vdim;
+      const auto queries = [&](gpu_buffer& b, size_t cols, size_t row_ld) {
+        blocks(b, 0, H, D, w.dn + w.dr, cols, row_ld);
+        if (X > 0) blocks(b, w.dn, H, X, w.dn + w.dr, cols, row_ld);
+      };
+      w.in = zeros(w.ldw, ld);
+      if (a.q_rank > 0) {
+        blocks(w.in, 0, 1, a.q_rank, 0, W, ld);
+        w.uq = zeros(w.q_cols, w.low_ld);
+        queries(w.uq, a.q_rank, w.low_ld);
+        w.low_norm = vector(a.q_rank, 1.0f, 0.1f);
+      } else {
+        queries(w.in, W, ld);
+      }
+      blocks(w.in, w.latent_at, 1, a.kv_rank, 0, W, ld);
+      if (X > 0) blocks(w.in, w.key_at, 1, X, 0, W, ld);
+      if (a.gate) blocks(w.in, w.gate_at, H, E, w.dv, W, ld);
+      w.ukv = zeros(H * (w.dn + w.dv), w.ldc);
+      blocks(w.ukv, 0, H, D, w.dn, a.kv_rank, w.ldc);
+      blocks(w.ukv, H * w.dn, H, E, w.dv, a.kv_rank, w.ldc);
+      if (w.few) {
+        std::vector<char> keys(H * w.dn * w.ldc * m->elem);
+        LCU_CHECK(lcu_d2h(keys.data(), w.ukv.data(), keys.size(), nullptr));
+        LCU_CHECK(lcu_sync(nullptr));
+        w.uk_t = upload_bytes(transposed_keys(w, a.heads, keys.data(), m->elem));
+      }
+      w.latent_norm = vector(a.kv_rank, 1.0f, 0.1f);
+      if (a.sink) w.sink = vector(H, 0.5f, 1.0f);
+      w.out = linear(W, w.ldo, w.ldo);
+    } else if (q.mixer == mixer_type::delta) {
+      delta_weights& w = L.delta;
+      delta_params const& d = q.delta;
+      const size_t H = d.heads, G = d.kv_heads;
+      w.in = zeros(w.rows, ld);
+      blocks(w.in, 0, 2 * G, d.dim, w.dk, W, ld);
+      blocks(w.in, 2 * G * w.dk, H, d.vdim, w.dv, W, ld);
+      blocks(w.in, w.channels, H, d.vdim, w.dv, W, ld);
+      blocks(w.in, w.channels + w.plain, 1, 2 * H, 0, W, ld);
+      w.conv = vector((size_t)d.taps * w.channels, 0.0f, 0.5f);
+      w.a_log = vector(H, -1.0f, 1.0f);
+      w.dt_bias = vector(H, -1.0f, 0.5f);
+      w.norm = vector(d.vdim, 1.0f, 0.1f);
+      w.out = linear(W, w.ldo, w.ldo);
     } else {
       attention_weights& w = L.attention;
       w.qkv = linear(w.ldq, W, ld);
@@ -373,7 +610,11 @@ bool layered_model_impl::shapes_supported() const {
       w.r2 = vector(q.attention.heads, 0.3f, 0.02f);
       w.v_mix = vector(1, 0.3f, 0.0f);
     }
-    if (q.has_mlp) {
+    if (q.dense.ff > 0) {
+      dense_weights& w = L.dense;
+      w.up = linear(2 * w.ld, W, ld);
+      w.down = linear(W, w.ld, w.ld);
+    } else if (q.has_mlp) {
       experts_weights& w = L.mlp;
       const size_t E = q.mlp.experts;
       w.router = linear(E + 1, W, ld);
@@ -386,6 +627,7 @@ bool layered_model_impl::shapes_supported() const {
     }
   }
   LCU_CHECK(lcu_sync(nullptr));
+  m->make_tables();
   return m;
 }
 

@@ -2,6 +2,7 @@
 // reference's format (main.cpp:24-57).
 #include "registry.hpp"
 
+#include "logivik.hpp"
 #include "rirulix.hpp"
 
 namespace llama_cu {
@@ -9,6 +10,7 @@ namespace llama_cu {
 namespace {
 const model_family FAMILIES[] = {
     {"Rirulix", rirulix_load, rirulix_synthesize},
+    {"Logivik", logivik_load, logivik_synthesize},
 };
 
 bool parse_config(std::string_view text, json& config, model_family const*& family) {

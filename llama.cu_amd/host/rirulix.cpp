@@ -1,6 +1,6 @@
 #include "rirulix.hpp"
 
-#include <cmath>
+#include "config_reader.hpp"
 
 namespace llama_cu {
 
@@ -10,23 +10,6 @@ namespace {
 constexpr float DECAY = -8.0f;         // log a = DECAY r softplus(lam)
 constexpr float GATE_ALPHA = 1.702f;   // g sigmoid(GATE_ALPHA g) (u + GATE_SHIFT)
 constexpr float GATE_SHIFT = 1.0f;
-
-struct config_reader {
-  bool ok{true};
-  void complain(std::string const& where, const char* key) {
-    if (ok) fprintf(stderr, "Invalid config.json: %s\"%s\" is missing or out of range\n", where.c_str(), key);
-    ok = false;
-  }
-  int integer(json const& v, const char* key, std::string const& where, int64_t lo = 1, int64_t hi = 1 << 28) {
-    int64_t n = lo;
-    if (!v[key].get_int(lo, hi, n)) complain(where, key);
-    return (int)n;
-  }
-  float real(json const& v, const char* key, std::string const& where) {
-    if (!v[key].is(json::number) || !std::isfinite(v[key].num)) complain(where, key);
-    return (float)v[key].num;
-  }
-};
 
 }  // namespace
 

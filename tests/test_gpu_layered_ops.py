@@ -226,7 +226,7 @@ def test_recurrence_in_portions(gpu, dt, width, blocks, taps, cuts):
     for n in cuts:
         dz, dy = put(gpu, spread(z[at:at + n], (n, ld)), dt), put(gpu, spread(y[at:at + n], (n, ld)), dt)
         u, out = zeros(gpu, (n, ld), dt), zeros(gpu, (n, ld), dt)
-        call(gpu, "lcu_conv_causal", u, dz, ld, args["conv"], args["convb"], conv_state, taps, dt, n, channels, ld)
+        call(gpu, "lcu_conv_causal", u, dz, ld, args["conv"], args["convb"], conv_state, taps, 0, dt, n, channels, ld)
         if n == 1 and dt == BF16:
             call(gpu, "lcu_decode_recurrent_step", out, u, dy, args["wr"], args["wi"], args["br"], args["bi"], args["decay"], state,
                  channels, bw)
