@@ -304,15 +304,37 @@ def batched_leg(P, model, cfg, sizes=(8, 32), prompt=64, steps=32, warmup=4):
     return out
 
 
-# Layered decoders (Rirulix) beside the LLaMA of the same width and active feed-forward width: two recurrent
-# layers to one attention layer, 16 experts of which a token uses two, and a shared expert.
+# Layered decoders beside the LLaMA of the same width and active feed-forward width.  Rirulix: two recurrent layers to
+# one attention layer, 16 experts of which a token uses two, and a shared expert.  Logivik: latent attention over
+# everything, latent attention with a window and the delta rule in turn, dense feed-forwards.
 LAYERED = {
-    "w2048": dict(width=2048, layers=6, heads=16, kv_heads=4, ff=1408, shared_ff=2816, multiple_of=256),
-    "w4096": dict(width=4096, layers=6, heads=32, kv_heads=8, ff=2816, shared_ff=5376, multiple_of=256),
+    "w2048": dict(width=2048, layers=6, heads=16, kv_heads=4, ff=1408, shared_ff=2816, multiple_of=256, kv_rank=512, q_rank=768),
+    "w4096": dict(width=4096, layers=6, heads=32, kv_heads=8, ff=2816, shared_ff=5376, multiple_of=256, kv_rank=512, q_rank=1536),
 }
 
 
-def layered_config(s, vocab=32000, context=4096):
+def logivik_config(s, vocab=32000):
+    h, ff = s["heads"], 2 * s["ff"] + s["shared_ff"]
+    latent = {"heads": h, "dim": 128, "vdim": 128, "kv_rank": s["kv_rank"]}
+    kinds = [("latent_attention", dict(latent, rot_dim=64, scale=192 ** -0.5,
+                                       rot={"dims": 64, "base": 1e4, "scaling": {"factor": 4.0, "original": 1024, "fast": 32.0, "slow": 1.0}})),
+             ("latent_attention_2", dict(latent, q_rank=s["q_rank"], scale=128 ** -0.5, mask={"size": 1024})),
+             ("delta", {"heads": h, "kv_heads": h // 2, "dim": 128, "vdim": 128, "conv": 4})]
+    return {"architecture": "Logivik", "width": s["width"], "vocab": vocab, "embedding": {"scale": s["width"] ** 0.5}, "norm": {"eps": 1e-6},
+            "layers": [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": ff}} for t, m in (kinds[l % 3] for l in range(s["layers"]))]}
+
+
+def logivik_bytes(s, vocab):
+    """Weight bytes a one-token step reads."""
+    w, d, r = s["width"], s["heads"] * 128, s["kv_rank"]
+    up = 2 * d * r                                                     # keys and values out of the latent
+    latent = w * (s["heads"] * 192 + r + 64 + d) + up + d * w
+    second = w * (s["q_rank"] + r) + s["q_rank"] * d + up + d * w
+    delta = w * (3 * d + 2 * s["heads"]) + d * w
+    return 2 * (s["layers"] // 3 * (latent + second + delta) + s["layers"] * 3 * w * (2 * s["ff"] + s["shared_ff"]) + vocab * w)
+
+
+def rirulix_config(s, vocab=32000, context=4096):
     mlp = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": s["ff"], "limit": 7.0},
            "shared": {"ff": s["shared_ff"], "limit": 7.0}}
     rec = {"type": "rglru", "mixer": {"width": s["width"], "blocks": s["width"] // 256, "conv": 4}, "mlp": mlp}
@@ -323,7 +345,7 @@ def layered_config(s, vocab=32000, context=4096):
             "norm": {"eps": 1e-5, "groups": 8}, "layers": [att if l % 3 == 2 else rec for l in range(s["layers"])]}
 
 
-def layered_bytes(s, vocab):
+def rirulix_bytes(s, vocab):
     """Weight bytes a one-token step reads: every matrix but the experts not chosen."""
     w = s["width"]
     n_att = s["layers"] // 3
@@ -362,18 +384,20 @@ def throughput(B, ctx, vocab, prompts, steps, warmup):
     return out
 
 
-def layered_leg(P, name, steps, warmup, vocab=32000, families=("rirulix", "llama")):
+def layered_leg(P, name, steps, warmup, vocab=32000, families=("logivik", "rirulix", "llama")):
     B = P.binding
     s = LAYERED[name]
     out = {"layers": s["layers"], "width": s["width"]}
     prompts = (512, 2048, 32)
-    if "rirulix" in families:
-        model = P.Model(config=layered_config(s, vocab), seed=1)
+    for family, config, weights in (("logivik", logivik_config, logivik_bytes), ("rirulix", rirulix_config, rirulix_bytes)):
+        if family not in families:
+            continue
+        model = P.Model(config=config(s, vocab), seed=1)
         ctx = P.Context(model, context_len=4096, temperature=0.8)
         r = throughput(B, ctx, vocab, prompts, steps, warmup)
-        r["weight_bytes_per_token"] = layered_bytes(s, vocab)
+        r["weight_bytes_per_token"] = weights(s, vocab)
         r["decode"]["weight_gb_s"] = round(r["weight_bytes_per_token"] / r["decode"]["ms_per_step"] / 1e6, 1)
-        out["rirulix_bf16"] = r
+        out[family + "_bf16"] = r
         ctx.close()
         model.close()
     if "llama" in families:
@@ -401,7 +425,7 @@ def main():
     ap.add_argument("--layered", nargs="*", choices=sorted(LAYERED), metavar="SIZE",
                     help="instead of the headline workload: prefill and decode throughput of layered decoders of these sizes "
                          "(default: all) beside the LLaMA of equal width, as one JSON line")
-    ap.add_argument("--family", choices=("rirulix", "llama"), help="with --layered: this family only (for profiles)")
+    ap.add_argument("--family", choices=("logivik", "rirulix", "llama"), help="with --layered: this family only (for profiles)")
     ap.add_argument("--copy-calibration", action="store_true",
                     help="also run one 256 MiB device-to-device copy: a copy kernel of known size, against which "
                          "rocprofv3 FETCH_SIZE / WRITE_SIZE readings of the other kernels are scaled")
@@ -414,7 +438,7 @@ def main():
     B = P.binding
     B.init(0)
     if args.layered is not None:
-        families = (args.family,) if args.family else ("rirulix", "llama")
+        families = (args.family,) if args.family else ("logivik", "rirulix", "llama")
         sizes = args.layered or sorted(LAYERED)
         print(json.dumps({"metric": "layered decoders: prefill and decode throughput", "data": "synthetic", "n_gpus": 1,
                           "steps": args.steps, "warmup": args.warmup,

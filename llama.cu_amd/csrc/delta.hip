@@ -5,16 +5,19 @@
 //
 // Channels of a token: q [kv_heads * D] | k [kv_heads * D] | v [heads * E], after their convolution; D is the head size
 // padded to 32, 64, 128 or 256 and E the value size padded to a multiple of 32, padding zero.  Everything here is fp32
-// but these channels and the result, which have the element type; products run on the fp32 matrix cores, and on the
+// but these channels and the result, which have the element type; products run on the fp32 matrix cores, or on the
 // bfloat16 ones where both operands are channels as stored (their products are exact in fp32).
 //
 // Several tokens: chunks of 64.  With G_t the sum of log g up to t inside the chunk and S the state that enters it,
-//   u_t = beta_t (v_t - e^G_t S^T k_t - sum_(s<t) e^(G_t - G_s) (k_s . k_t) u_s)
+//   u_t + beta_t sum_(s<t) e^(G_t - G_s) (k_s . k_t) u_s = r_t = beta_t (v_t - e^G_t S^T k_t)
 //   o_t = e^G_t S^T q_t + sum_(s<=t) e^(G_t - G_s) (k_s . q_t) u_s
 //   S'  = e^G_64 S + sum_s e^(G_64 - G_s) k_s u_s^T
-// The first is linear in S: u = X - Y S, where X and Y solve one triangular system with right sides beta v and beta e^G k.
-// The chunk kernel solves it for every chunk at once; the scan kernel then runs over the chunks, sixteen columns of S
-// per workgroup.  No exponent is ever positive.
+// or u = T r and o = e^G S^T q + P T r, with T the inverse of the unit triangular matrix of the first line and P the
+// factors of the second.  The chunk kernel leaves T and P T of every chunk at once; the scan kernel runs over the chunks,
+// sixteen columns of S per workgroup.  No exponent is ever positive.
+//
+// Where the channels are bfloat16, the products with S and u have one operand that bfloat16 holds exactly; the fp32 one goes
+// in as three bfloat16 terms, which together hold all of its bits.
 #include <type_traits>
 
 #include "linear.hpp"
@@ -36,12 +39,13 @@ struct delta_args {
   const float* dt_bias;
   const float* norm;                  // [vdim], plain
   float eps;
-  // per (head, chunk): solutions X [64][E] and Y [64][D], decayed q.k [64][64], row factors [64][2] (of o, of k), e^G_64
-  float* X;
-  float* Y;
-  float* P;
+  // per (head, chunk): T and P T [64][64], on and below the diagonal blocks; per row the factors beta, beta e^G / |k|,
+  // e^G / |q|, e^(G_64 - G) / |k| [4][64]; e^G_64.  Per (q/k head, chunk): the keys transposed [D][64], in their own type.
+  float* T;
+  float* PT;
   float* rows;
   float* total;
+  void* Kt;
 };
 
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
@@ -74,18 +78,19 @@ __device__ __forceinline__ float4_t row_products(const float* x, const float* y,
   return acc;
 }
 
-// One workgroup: one chunk of one head.
+// One workgroup: one chunk of one head.  `role`, one per wavefront: a block of sixteen rows, then a block of columns.
 template <class T, int D>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(const T* __restrict__ qkv, delta_args p) {
   constexpr int LDA = CHUNK + 4;
-  __shared__ __attribute__((aligned(16))) float A[CHUNK * LDA];  // beta_t e^(G_t - G_s) k_t . k_s, s < t
+  // A: beta_t e^(G_t - G_s) k_t . k_s, s < t, whose diagonal blocks the inverses of theirs replace; P
+  __shared__ __attribute__((aligned(16))) float A[CHUNK * LDA], P[CHUNK * LDA];
   __shared__ float Gs[CHUNK], beta[CHUNK], inv_q[CHUNK], inv_k[CHUNK];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
-  const int h = blockIdx.x, chunk = blockIdx.y, g = h / (p.heads / p.kv_heads), t0 = chunk * CHUNK;
+  const int role = (wave + blockIdx.x + blockIdx.y) & 3;  // the roles differ in length
+  const int h = blockIdx.x, chunk = blockIdx.y, group = p.heads / p.kv_heads, g = h / group, t0 = chunk * CHUNK;
   const size_t at = (size_t)h * gridDim.y + chunk;
   const T* Q = qkv + (size_t)g * D;
   const T* K = qkv + (size_t)(p.kv_heads + g) * D;
-  const T* V = qkv + (size_t)2 * p.kv_heads * D + (size_t)h * p.E;
   const auto row = [&](int t) { return (size_t)min(t0 + t, p.n - 1) * p.ld; };
   if (wave == 0) {
     const bool real = t0 + lane < p.n;
@@ -121,46 +126,50 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const T* __restrict__ 
       inv_k[tid >> 2] = 1.0f / sqrtf(k2 + UNIT_EPS);
     }
   }
-  __syncthreads();
-  // wavefront w: rows 16 w .. 16 w + 15 of both products
-  float* P = p.P + at * CHUNK * CHUNK;
-#pragma unroll 1
-  for (int ct = 0; ct < 4; ++ct) {
-    float4_t kk = (float4_t)(0.0f), qk = (float4_t)(0.0f);
-    if (ct <= wave) {
-      const T* y = K + row(ct * 16 + col);
-      kk = row_products<D>(K + row(wave * 16 + col), y, kk);
-      qk = row_products<D>(Q + row(wave * 16 + col), y, qk);
+  if (h == g * group) {
+    T* Kt = (T*)p.Kt + ((size_t)g * gridDim.y + chunk) * D * CHUNK;
+    const size_t r = row(lane);
+#pragma unroll 2
+    for (int d = wave * 4; d < D; d += 16) {
+      const float4_t k = load4(K + r + d);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) Kt[(size_t)(d + e) * CHUNK + lane] = (T)k[e];
     }
+  }
+  __syncthreads();
+#pragma unroll 1
+  for (int ct = 0; ct <= role; ++ct) {
+    const T* y = K + row(ct * 16 + col);
+    const float4_t kk = row_products<D>(K + row(role * 16 + col), y, (float4_t)(0.0f));
+    const float4_t qk = row_products<D>(Q + row(role * 16 + col), y, (float4_t)(0.0f));
     const int s = ct * 16 + col;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int t = wave * 16 + quad * 4 + e;
+      const int t = role * 16 + quad * 4 + e;
       const float f = s <= t ? expf(Gs[t] - Gs[s]) * inv_k[s] : 0.0f;
       A[t * LDA + s] = s < t ? beta[t] * inv_k[t] * f * kk[e] : 0.0f;
-      P[t * CHUNK + s] = inv_q[t] * f * qk[e];
+      P[t * LDA + s] = inv_q[t] * f * qk[e];
     }
   }
   if (tid < CHUNK) {
     const float G = Gs[tid], end = Gs[CHUNK - 1];
-    p.rows[(at * CHUNK + tid) * 2] = expf(G) * inv_q[tid];
-    p.rows[(at * CHUNK + tid) * 2 + 1] = expf(end - G) * inv_k[tid];
+    float* rows = p.rows + at * 4 * CHUNK + tid;
+    rows[0] = beta[tid];
+    rows[CHUNK] = beta[tid] * expf(G) * inv_k[tid];
+    rows[2 * CHUNK] = expf(G) * inv_q[tid];
+    rows[3 * CHUNK] = expf(end - G) * inv_k[tid];
     if (tid == 0) p.total[at] = expf(end);
   }
-  __syncthreads();
-  // forward substitution, one column of the right sides per thread
-  for (int c = tid; c < p.E + D; c += 256) {
-    const bool of_v = c < p.E;
-    const T* src = of_v ? V + c : K + (c - p.E);
-    float x[CHUNK];
+  {
+    // the inverse of the role's own diagonal block, written by this wavefront alone; lane = column
+    float* B = A + role * 16 * (LDA + 1);
+    float x[16];
 #pragma unroll
-    for (int t = 0; t < CHUNK; ++t) x[t] = to_f32(src[row(t)]);
-#pragma unroll
-    for (int t = 0; t < CHUNK; ++t) {
-      float acc = x[t] * (of_v ? beta[t] : beta[t] * expf(Gs[t]) * inv_k[t]);
+    for (int t = 0; t < 16; ++t) {
+      float acc = t == col ? 1.0f : 0.0f;
 #pragma unroll
       for (int s4 = 0; s4 < t; s4 += 4) {
-        const float4_t a = load4(A + t * LDA + s4);
+        const float4_t a = load4(B + t * LDA + s4);
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           if (s4 + e < t) acc = fmaf(-a[e], x[s4 + e], acc);
@@ -168,102 +177,250 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const T* __restrict__ 
       }
       x[t] = acc;
     }
-    float* dst = of_v ? p.X + at * CHUNK * p.E + c : p.Y + at * CHUNK * D + (c - p.E);
-    const int ldd = of_v ? p.E : D;
+    if (quad == 0) {
 #pragma unroll
-    for (int t = 0; t < CHUNK; ++t) dst[t * ldd] = x[t];
-  }
-}
-
-// One workgroup: sixteen columns of one head's state through all chunks.  o: fp32 [n][heads * E].
-template <class T, int D>
-__global__ __launch_bounds__(256) void delta_scan_kernel(float* __restrict__ o, float* __restrict__ state, const T* __restrict__ qkv,
-                                                         int chunks, delta_args p) {
-  constexpr int LD = 20, TILES = (D / 16 + 3) / 4;  // state tiles of a wavefront
-  __shared__ float S[D * LD];
-  __shared__ float U[CHUNK * LD], Uk[CHUNK * LD];   // u, and u times the row's factor of k
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
-  const int h = blockIdx.x, c0 = blockIdx.y * 16, g = h / (p.heads / p.kv_heads);
-  float* St = state + (size_t)h * D * p.E + c0;
-  for (int i = tid; i < D * 16; i += 256) S[(i >> 4) * LD + (i & 15)] = St[(size_t)(i >> 4) * p.E + (i & 15)];
-  const T* Q = qkv + (size_t)g * D;
-  const T* K = qkv + (size_t)(p.kv_heads + g) * D;
-  for (int chunk = 0; chunk < chunks; ++chunk) {
-    const size_t at = (size_t)h * chunks + chunk;
-    const int t0 = chunk * CHUNK, r0 = wave * 16 + quad * 4;
-    const float* Y = p.Y + (at * CHUNK + wave * 16 + col) * D;
-    const float* X = p.X + (at * CHUNK + r0) * p.E + c0 + col;
-    const float* rows = p.rows + at * CHUNK * 2;
-    __syncthreads();  // S is whole
-    float4_t ys = (float4_t)(0.0f), qs = (float4_t)(0.0f);
-    const T* q = Q + (size_t)min(t0 + wave * 16 + col, p.n - 1) * p.ld;
-#pragma unroll 4
-    for (int d = 0; d < D; d += 16) {
-      const float4_t a = load4(Y + d + quad * 4), b = load4(q + d + quad * 4);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float s = S[(d + quad * 4 + j) * LD + col];
-        ys = mfma_f32(a[j], s, ys);
-        qs = mfma_f32(b[j], s, qs);
-      }
-    }
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const float u = X[(size_t)e * p.E] - ys[e];
-      U[(r0 + e) * LD + col] = u;
-      Uk[(r0 + e) * LD + col] = u * rows[(r0 + e) * 2 + 1];
-      qs[e] *= rows[(r0 + e) * 2];
-    }
-    __syncthreads();  // everyone has read S and written its part of u
-    const float* P = p.P + (at * CHUNK + wave * 16 + col) * CHUNK;
-    for (int s = 0; s <= wave * 16; s += 16) {
-      const float4_t a = load4(P + s + quad * 4);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) qs = mfma_f32(a[j], U[(s + quad * 4 + j) * LD + col], qs);
-    }
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      if (t0 + r0 + e < p.n) o[(size_t)(t0 + r0 + e) * p.heads * p.E + (size_t)h * p.E + c0 + col] = qs[e];
-    }
-    const float total = p.total[at];
-#pragma unroll
-    for (int i = 0; i < TILES; ++i) {
-      const int d0 = (wave + i * 4) * 16;
-      if (d0 >= D) break;
-      float4_t s;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) s[e] = S[(d0 + quad * 4 + e) * LD + col] * total;
-#pragma unroll
-      for (int t = 0; t < CHUNK; t += 16) {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int r = t + quad * 4 + j;
-          s = mfma_f32(to_f32(K[(size_t)min(t0 + r, p.n - 1) * p.ld + d0 + col]), Uk[r * LD + col], s);
-        }
-      }
-#pragma unroll
-      for (int e = 0; e < 4; ++e) S[(d0 + quad * 4 + e) * LD + col] = s[e];
+      for (int t = 0; t < 16; ++t) B[t * LDA + col] = x[t];
     }
   }
   __syncthreads();
-  for (int i = tid; i < D * 16; i += 256) St[(size_t)(i >> 4) * p.E + (i & 15)] = S[(i >> 4) * LD + (i & 15)];
+  // Block column `role` of T, top to bottom: T_ij = -T_ii sum_m A_im T_mj.  A tile as it leaves the matrix core (four
+  // neighbouring rows per lane) is the second operand of the next product, its rows taken in the order of the lanes.
+  const auto times = [&](const float* M, int i, int m, float4_t b, float4_t acc) {
+    const float4_t a = load4(M + (i * 16 + col) * LDA + m * 16 + quad * 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) acc = mfma_f32(a[e], b[e], acc);
+    return acc;
+  };
+  float4_t t[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    t[i] = (float4_t)(0.0f);
+    if (i == role) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) t[i][e] = A[(i * 16 + quad * 4 + e) * LDA + i * 16 + col];
+    } else if (i > role) {
+      float4_t sum = (float4_t)(0.0f);
+#pragma unroll
+      for (int m = 0; m < i; ++m) {
+        if (m >= role) sum = times(A, i, m, t[m], sum);
+      }
+      t[i] = times(A, i, i, -sum, t[i]);
+    }
+  }
+  float* To = p.T + at * CHUNK * CHUNK + role * 16 + col;
+  float* PTo = p.PT + at * CHUNK * CHUNK + role * 16 + col;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    if (i < role) continue;
+    float4_t sum = (float4_t)(0.0f);
+#pragma unroll
+    for (int m = 0; m <= i; ++m) {
+      if (m >= role) sum = times(P, i, m, t[m], sum);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      To[(i * 16 + quad * 4 + e) * CHUNK] = t[i][e];
+      PTo[(i * 16 + quad * 4 + e) * CHUNK] = sum[e];
+    }
+  }
 }
 
-// out[t][h * E + j] = o / rms(o of the head) * norm[j] * silu(gate): a wavefront per token and head
+// fp32 values as matrix operands: three bfloat16 terms beside bfloat16 channels, one value beside fp32 ones.  An array is
+// [terms][16 columns][LD], along the products' inner dimension.
+template <class T>
+struct terms_of;
+template <>
+struct terms_of<float> {
+  static constexpr int COUNT = 1, STEP = 16, PER = 4, PAD = 4;  // inner extent of a step, elements of a lane
+  typedef float4_t piece;
+};
+template <>
+struct terms_of<bf16_t> {
+  static constexpr int COUNT = 3, STEP = 32, PER = 8, PAD = 8;
+  typedef bf16x8_t piece;
+};
+typedef bf16_t bf16x4_t __attribute__((ext_vector_type(4)));
+
+template <int LD>
+__device__ __forceinline__ void put_terms(float* dst, int c, int at, float4_t v) {
+  store4(dst + c * LD + at, v);
+}
+template <int LD>
+__device__ __forceinline__ void put_terms(bf16_t* dst, int c, int at, float4_t v) {
+#pragma unroll
+  for (int term = 0; term < 3; ++term) {
+    bf16x4_t x;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      x[e] = (bf16_t)v[e];
+      v[e] -= (float)x[e];
+    }
+    *reinterpret_cast<bf16x4_t*>(dst + (term * 16 + c) * LD + at) = x;
+  }
+}
+template <int LD>
+__device__ __forceinline__ float4_t step_product(float4_t a, const float* terms, int col, int at, float4_t acc) {
+  const float4_t b = load4(terms + col * LD + at);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) acc = mfma_f32(a[e], b[e], acc);
+  return acc;
+}
+template <int LD>
+__device__ __forceinline__ float4_t step_product(bf16x8_t a, const bf16_t* terms, int col, int at, float4_t acc) {
+#pragma unroll
+  for (int term = 2; term >= 0; --term) {
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, *reinterpret_cast<const bf16x8_t*>(terms + (term * 16 + col) * LD + at), acc, 0, 0, 0);
+  }
+  return acc;
+}
+
+// One workgroup: sixteen columns of one head's state through all chunks.  A wavefront takes sixteen rows of a chunk and up
+// to TILES blocks of sixteen rows of the state, which it keeps in registers; LDS holds all of the state as operands.  What a
+// chunk needs from memory is asked for one chunk ahead where the registers hold it twice.  o: fp32 [n][heads * E].
+template <class T, int D>
+__global__ __launch_bounds__(256) void delta_scan_kernel(float* __restrict__ o, float* __restrict__ state, const T* __restrict__ qkv,
+                                                         int chunks, delta_args p) {
+  typedef terms_of<T> terms;
+  typedef typename terms::piece piece;
+  constexpr int STEPS = D / terms::STEP, CSTEPS = CHUNK / terms::STEP, TILES = (D / 16 + 3) / 4;
+  constexpr int LDR = CHUNK + 4, LDU = CHUNK + terms::PAD, LDD = D + terms::PAD;
+  constexpr bool AHEAD = D * sizeof(T) <= 512;
+  __shared__ __attribute__((aligned(16))) T S[terms::COUNT * 16 * LDD];
+  __shared__ __attribute__((aligned(16))) T U[terms::COUNT * 16 * LDU];  // u times the row's factor of k
+  __shared__ __attribute__((aligned(16))) float R[16 * LDR];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4, r0 = wave * 16 + quad * 4;
+  const int h = blockIdx.x, c0 = blockIdx.y * 16, g = h / (p.heads / p.kv_heads);
+  const T* Q = qkv + (size_t)g * D;
+  const T* K = qkv + (size_t)(p.kv_heads + g) * D;
+  const T* V = qkv + (size_t)2 * p.kv_heads * D + (size_t)h * p.E + c0 + col;
+  float* St = state + (size_t)h * D * p.E + c0 + col;
+  struct operands {
+    piece k[STEPS], q[STEPS], kt[TILES * CSTEPS];
+    float4_t t[4], pt[4], fac[4];
+    float v[4], total;
+  };
+  const auto fetch = [&](operands& x, int chunk) {
+    const size_t at = (size_t)h * chunks + chunk, r = (size_t)min(chunk * CHUNK + wave * 16 + col, p.n - 1) * p.ld;
+    const T* kt = (const T*)p.Kt + ((size_t)g * chunks + chunk) * D * CHUNK;
+    const size_t m = at * CHUNK * CHUNK + (size_t)(wave * 16 + col) * CHUNK + quad * 4;
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) {
+      x.k[i] = *reinterpret_cast<const piece*>(K + r + i * terms::STEP + quad * terms::PER);
+      x.q[i] = *reinterpret_cast<const piece*>(Q + r + i * terms::STEP + quad * terms::PER);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      x.v[e] = to_f32(V[(size_t)min(chunk * CHUNK + r0 + e, p.n - 1) * p.ld]);
+      x.fac[e] = load4(p.rows + (at * 4 + e) * CHUNK + r0);
+    }
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      if (s <= wave) {
+        x.t[s] = load4(p.T + m + s * 16);
+        x.pt[s] = load4(p.PT + m + s * 16);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < TILES; ++i) {
+#pragma unroll
+      for (int c = 0; c < CSTEPS; ++c) {
+        const int d = min((wave + i * 4) * 16, D - 16) + col;
+        x.kt[i * CSTEPS + c] = *reinterpret_cast<const piece*>(kt + (size_t)d * CHUNK + c * terms::STEP + quad * terms::PER);
+      }
+    }
+    x.total = p.total[at];
+  };
+  operands now, next;
+  if (AHEAD) fetch(now, 0);
+  float4_t s[TILES];
+#pragma unroll
+  for (int i = 0; i < TILES; ++i) {
+    const int d0 = (wave + i * 4) * 16 + quad * 4;
+    if (d0 >= D) break;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s[i][e] = St[(size_t)(d0 + e) * p.E];
+    put_terms<LDD>(S, col, d0, s[i]);
+  }
+  for (int chunk = 0; chunk < chunks; ++chunk) {
+    if (AHEAD) {
+      fetch(next, min(chunk + 1, chunks - 1));
+    } else {
+      fetch(now, chunk);
+    }
+    __syncthreads();  // S is whole
+    float4_t ks = (float4_t)(0.0f), qs = (float4_t)(0.0f);
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) {
+      ks = step_product<LDD>(now.k[i], S, col, i * terms::STEP + quad * terms::PER, ks);
+      qs = step_product<LDD>(now.q[i], S, col, i * terms::STEP + quad * terms::PER, qs);
+    }
+    float4_t r;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r[e] = now.fac[0][e] * now.v[e] - now.fac[1][e] * ks[e];
+    store4(R + col * LDR + r0, r);
+    __syncthreads();  // R is whole, S has been read
+    float4_t u = (float4_t)(0.0f), y = (float4_t)(0.0f);
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+      if (b <= wave) {
+        const float4_t x = load4(R + col * LDR + b * 16 + quad * 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          u = mfma_f32(now.t[b][e], x[e], u);
+          y = mfma_f32(now.pt[b][e], x[e], y);
+        }
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) u[e] *= now.fac[3][e];
+    put_terms<LDU>(U, col, r0, u);
+    __syncthreads();  // U is whole, R has been read
+#pragma unroll
+    for (int i = 0; i < TILES; ++i) {
+      const int d0 = (wave + i * 4) * 16 + quad * 4;
+      if (d0 >= D) break;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s[i][e] *= now.total;
+#pragma unroll
+      for (int c = 0; c < CSTEPS; ++c) {
+        s[i] = step_product<LDU>(now.kt[i * CSTEPS + c], U, col, c * terms::STEP + quad * terms::PER, s[i]);
+      }
+      put_terms<LDD>(S, col, d0, s[i]);
+    }
+    const int t = chunk * CHUNK + r0;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (t + e < p.n) o[(size_t)(t + e) * p.heads * p.E + (size_t)h * p.E + c0 + col] = fmaf(now.fac[2][e], qs[e], y[e]);
+    }
+    if (AHEAD) now = next;
+  }
+#pragma unroll
+  for (int i = 0; i < TILES; ++i) {
+    const int d0 = (wave + i * 4) * 16 + quad * 4;
+    if (d0 >= D) break;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) St[(size_t)(d0 + e) * p.E] = s[i][e];
+  }
+}
+
+// out[t][h * E + j] = o / rms(o of the head) * norm[j] * silu(gate): `lanes` lanes (8 .. 64) per token and head, four
+// values each
 template <class T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out, int ldo, const float* __restrict__ o,
-                                                             const T* __restrict__ gate, int ldg, delta_args p) {
-  const int lane = threadIdx.x & 63, i = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (i >= p.n * p.heads) return;
-  const int t = i / p.heads, h = i - t * p.heads;
-  const float* src = o + (size_t)i * p.E;
-  float s = 0.0f;
-  for (int c = lane; c < p.E; c += WAVE) s = fmaf(src[c], src[c], s);  // padding is zero
-  const float inv = 1.0f / sqrtf(wave_sum(s) / (float)p.vdim + p.eps);
-  for (int c = lane; c < p.E; c += WAVE) {
-    const float z = to_f32(gate[(size_t)t * ldg + (size_t)h * p.E + c]);
-    out[(size_t)t * ldo + (size_t)h * p.E + c] = (T)(c < p.vdim ? src[c] * inv * p.norm[c] * (z * sigmoid_f32(z)) : 0.0f);
-  }
+                                                             const T* __restrict__ gate, int ldg, int lanes, delta_args p) {
+  const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) / lanes;
+  const int c = (threadIdx.x & (lanes - 1)) * 4;
+  const bool has = i < (size_t)p.n * p.heads && c < p.E;
+  const size_t t = i / p.heads, h = i - t * p.heads;
+  const float4_t x = has ? load4(o + i * p.E + c) : (float4_t)(0.0f), z = has ? load4(gate + t * ldg + h * p.E + c) : (float4_t)(0.0f);
+  float s = fmaf(x[0], x[0], fmaf(x[1], x[1], fmaf(x[2], x[2], x[3] * x[3])));  // padding is zero
+  for (int off = lanes >> 1; off > 0; off >>= 1) s += __shfl_xor(s, off, WAVE);
+  const float inv = 1.0f / sqrtf(s / (float)p.vdim + p.eps);
+  if (!has) return;
+  float4_t y;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) y[e] = c + e < p.vdim ? x[e] * inv * p.norm[c + e] * (z[e] * sigmoid_f32(z[e])) : 0.0f;
+  store4(out + t * ldo + h * p.E + c, y);
 }
 
 // One new token: a workgroup per head holds the head's state in registers, ROWS rows of four columns per thread.
@@ -411,7 +568,8 @@ extern "C" {
 size_t lcu_delta_rule_scratch(const lcu_delta_params* d, int n) {
   if (d == nullptr || n <= 0) return 0;
   const size_t chunks = ((size_t)n + CHUNK - 1) / CHUNK;
-  return ((size_t)d->heads * chunks * (CHUNK * ((size_t)d->dk + d->dv + CHUNK + 2) + 1) + (size_t)n * d->heads * d->dv) * sizeof(float);
+  return (chunks * ((size_t)d->heads * (2 * CHUNK * CHUNK + 4 * CHUNK + 1) + (size_t)d->kv_heads * d->dk * CHUNK + 4) +
+          (size_t)n * d->heads * d->dv) * sizeof(float);
 }
 
 int lcu_delta_rule(void* out_dev, int ldo, const void* qkv_dev, int ld, const void* gate_dev, int ldg, const void* ba_f32_dev, int ld_ba,
@@ -427,19 +585,21 @@ int lcu_delta_rule(void* out_dev, int ldo, const void* qkv_dev, int ld, const vo
   delta_args p = make_delta(d, ba_f32_dev, ld_ba, n, ld);
   const int chunks = (n + CHUNK - 1) / CHUNK;
   const size_t units = (size_t)d->heads * chunks;
-  p.X = (float*)scratch_dev;
-  p.Y = p.X + units * CHUNK * d->dv;
-  p.P = p.Y + units * CHUNK * d->dk;
-  p.rows = p.P + units * CHUNK * CHUNK;
-  float* o = p.rows + units * CHUNK * 2;
-  p.total = o + (size_t)n * d->heads * d->dv;
-  const unsigned norms = (unsigned)(((size_t)n * d->heads + 3) / 4);
+  p.T = (float*)scratch_dev;
+  p.PT = p.T + units * CHUNK * CHUNK;
+  p.rows = p.PT + units * CHUNK * CHUNK;
+  float* o = p.rows + units * 4 * CHUNK;
+  float* Kt = o + (size_t)n * d->heads * d->dv;
+  p.Kt = Kt;
+  p.total = Kt + (size_t)d->kv_heads * chunks * d->dk * CHUNK;
+  const int lanes = d->dv <= 32 ? 8 : d->dv <= 64 ? 16 : d->dv <= 128 ? 32 : 64;
+  const unsigned norms = (unsigned)(((size_t)n * d->heads * lanes + 255) / 256);
   const auto run = [&](auto* kind, auto size) {
     using T = std::remove_pointer_t<decltype(kind)>;
     constexpr int D = decltype(size)::value;
     delta_chunk_kernel<T, D><<<dim3(d->heads, chunks), 256, 0, st>>>((const T*)qkv_dev, p);
     delta_scan_kernel<T, D><<<dim3(d->heads, d->dv / 16), 256, 0, st>>>(o, (float*)state_dev, (const T*)qkv_dev, chunks, p);
-    head_norm_gate_kernel<T><<<norms, 256, 0, st>>>((T*)out_dev, ldo, o, (const T*)gate_dev, ldg, p);
+    head_norm_gate_kernel<T><<<norms, 256, 0, st>>>((T*)out_dev, ldo, o, (const T*)gate_dev, ldg, lanes, p);
   };
   with_head_size(d->dk, [&](auto size) {
     if (dtype == LCU_F32) {

@@ -169,6 +169,18 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(latent_args p) {
     }
     return;
   }
+  bf16x8_t kv[2 * NT], rot[2];  // of this lane's key, one tile ahead
+  const auto fetch = [&](int tile) {
+    const size_t j = min(lo + tile * LKEYS + wave * 16 + col, hi);
+    const bf16_t* c = p.c + j * p.ldc + quad * 8;
+#pragma unroll
+    for (int f = 0; f < 2 * NT; ++f) kv[f] = f * 32 < p.ldc ? *reinterpret_cast<const bf16x8_t*>(c + f * 32) : (bf16x8_t)(0.0f);
+#pragma unroll
+    for (int f = 0; f < 2; ++f) {
+      if (f * 32 < p.dr) rot[f] = *reinterpret_cast<const bf16x8_t*>(p.keys + j * p.dr + quad * 8 + f * 32);
+    }
+  };
+  fetch(tile0);
   const int c8 = p.ldc / 8, k8 = (p.ldc + p.dr) / 8;
   for (int i = tid; i < LROWS * k8; i += 256) {
     const int r = i / k8, e = i - r * k8, row = min(r0 + r, rows - 1), t = row / p.heads, h = row - t * p.heads;
@@ -189,13 +201,15 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(latent_args p) {
   __syncthreads();
   for (int tile = tile0; tile < tile1; ++tile) {
     const int j = lo + tile * LKEYS + wave * 16 + col;  // this lane's key
-    const bf16_t* c = p.c + (size_t)min(j, hi) * p.ldc + quad * 8;
-    bf16x8_t kv[2 * NT];
-#pragma unroll
-    for (int f = 0; f < 2 * NT; ++f) kv[f] = f * 32 < p.ldc ? *reinterpret_cast<const bf16x8_t*>(c + f * 32) : (bf16x8_t)(0.0f);
     float4_t s = (float4_t)(0.0f);
     const bf16_t* qr = Qs + col * ldk + quad * 8;
-    for (int k = 0; k < p.dr; k += 32) {
+#pragma unroll
+    for (int f = 0; f < 2; ++f) {
+      if (f * 32 < p.dr) {
+        s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(qr + p.ldc + f * 32), rot[f], s, 0, 0, 0);
+      }
+    }
+    for (int k = 64; k < p.dr; k += 32) {
       s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(qr + p.ldc + k),
                                                   *reinterpret_cast<const bf16x8_t*>(p.keys + (size_t)min(j, hi) * p.dr + quad * 8 + k), s, 0,
                                                   0, 0);
@@ -226,6 +240,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(latent_args p) {
         for (int b = 0; b < 8; ++b) Vt[(f * 32 + quad * 8 + b) * LDV + wave * 16 + col] = kv[f][b];
       }
     }
+    if (tile + 1 < tile1) fetch(tile + 1);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int r = quad * 4 + e;
@@ -298,6 +313,7 @@ __global__ __launch_bounds__(256) void latent_value_kernel(latent_value_args p) 
   extern __shared__ __attribute__((aligned(16))) unsigned char value_lds[];
   bf16_t* C = reinterpret_cast<bf16_t*>(value_lds);  // [16][ldc + 8]
   __shared__ float weight[16][MAX_SLICES];
+  __shared__ int live[16];  // slices up to the last one with keys
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
   const int h = blockIdx.x, t0 = blockIdx.z * 16, tokens = min(16, p.n - t0), rows = p.n * p.heads, ld = p.ldc + 8;
   for (int t = wave; t < tokens; t += 4) {
@@ -311,6 +327,8 @@ __global__ __launch_bounds__(256) void latent_value_kernel(latent_value_args p) 
     float total = wave_sum(f * l);
     if (p.sink) total += __expf(p.sink[h] - top);
     if (has) weight[t][lane] = f / total;
+    const uint64_t with_keys = __ballot(l > 0.0f);
+    if (lane == 0) live[t] = 64 - __clzll(with_keys | 1);
   }
   __syncthreads();
   const int c4 = p.ldc / 4;
@@ -319,11 +337,9 @@ __global__ __launch_bounds__(256) void latent_value_kernel(latent_value_args p) 
     float4_t v = (float4_t)(0.0f);
     if (t < tokens) {
       const float* src = p.part + ((size_t)(t0 + t) * p.heads + h) * p.ldc + c;
+      const int n = live[t];  // those behind have written nothing
 #pragma unroll 8
-      for (int s = 0; s < p.slices; ++s) {
-        const float f = weight[t][s];
-        if (f > 0.0f) v += f * load4(src + (size_t)s * rows * p.ldc);  // slices without keys have written nothing
-      }
+      for (int s = 0; s < n; ++s) v += weight[t][s] * load4(src + (size_t)s * rows * p.ldc);
     }
     store4(C + t * ld + c, v);
   }

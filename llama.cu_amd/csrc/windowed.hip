@@ -121,141 +121,176 @@ __global__ __launch_bounds__(256) void attention_row_kernel(T* __restrict__ out,
 // ---- prompts, bfloat16: matrix cores --------------------------------------------------------------------
 // One workgroup: 64 query rows of one head, 16 per wavefront, against tiles of 64 keys with a running
 // maximum and sum.  Key tiles that hold no visible key of any of the rows (between the kept tokens and the
-// windows) are not visited.  Probabilities go into the second product as two bfloat16 terms (value and
-// remainder), so that they keep 16 significant bits.
+// windows) are not visited; the next tile is asked for while one is worked on.  Scores are computed with the keys as
+// rows, so that a lane holds sixteen of its own query row, which are the second operand of the product with the
+// transposed values as they are: keys of a block of 32 lie in LDS in the order in which lanes hold them.  Probabilities go
+// in as two bfloat16 terms (value and remainder), so that they keep 16 significant bits.  Workgroups of a head differ in id
+// by the number of heads: where that is a multiple of eight they share an L2, and long rows come first.
 constexpr int QT = 64, KT = 64;
+
+// where key r of a tile lies in a row of transposed values
+__device__ __forceinline__ int key_place(int r) { return (r & ~31) + ((r >> 2) & 3) * 8 + ((r >> 4) & 1) * 4 + (r & 3); }
 
 template <int DV, bool BIAS>
 __global__ __launch_bounds__(256) void attention_tile_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ q,
                                                              const bf16_t* __restrict__ k, const bf16_t* __restrict__ v, int n,
                                                              int start, window_args p) {
-  constexpr int NT = DV / 16;
-  constexpr int LDP = KT + 8;
+  constexpr int NT = DV / 16, LDP = KT + 8, KP = 8, VP = (DV + 63) / 64;  // KP, VP: pieces of a tile per thread
   extern __shared__ __attribute__((aligned(16))) unsigned char attn_lds[];
   const int ldk = p.dk + 8;
-  bf16_t* Qs = reinterpret_cast<bf16_t*>(attn_lds);   // [QT][ldk]
-  bf16_t* Ks = Qs + QT * ldk;                         // [KT][ldk]
-  bf16_t* Vt = Ks + KT * ldk;                         // [DV][LDP]: values, transposed
-  bf16_t* Ps = Vt + DV * LDP;                         // [wave][value, remainder][16][LDP]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int q0 = (gridDim.x - 1 - blockIdx.x) * QT, h = blockIdx.y, g = h / (p.heads / p.kv_heads);
-  const int dk8 = p.dk / 8;
-  for (int c = tid; c < QT * dk8; c += 256) {
-    const int r = c / dk8, e = (c % dk8) * 8;
-    *reinterpret_cast<uint4_t*>(Qs + r * ldk + e) =
-        *reinterpret_cast<const uint4_t*>(q + (size_t)min(q0 + r, n - 1) * p.ldq + (size_t)h * p.dk + e);
-  }
+  bf16_t* Ks = reinterpret_cast<bf16_t*>(attn_lds);   // [KT][ldk]
+  bf16_t* Vt = Ks + KT * ldk;                         // [DV][LDP]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
+  const int h = blockIdx.x % p.heads, q0 = ((int)gridDim.x / p.heads - 1 - (int)blockIdx.x / p.heads) * QT;
+  const int g = h / (p.heads / p.kv_heads), dk8 = p.dk / 8, own8 = (p.dk - p.dk_shared) / 8;
   const float r1 = BIAS ? p.r1[h] : 0.0f, r2 = BIAS ? p.r2[h] : 0.0f;
-  const int own8 = (p.dk - p.dk_shared) / 8;
   const int first = start + q0, last = start + min(q0 + QT, n) - 1;  // positions of the tile's rows
   const int win_tile = window_begin(p, first) / KT, kept_tiles = (min(p.keep, first + QT) + KT - 1) / KT;
-  const int col = lane & 15, quad = lane >> 4;
-  float m[4], l[4];
-  float4_t o[NT];
+  uint4_t kr[KP], vr[VP][2];
+  int k_at[KP];  // row and piece of the keys
 #pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    m[e] = p.sink ? p.sink[h] : -1e30f;  // the sink counts as a key of value zero
-    l[e] = p.sink ? 1.0f : 0.0f;
+  for (int x = 0; x < KP; ++x) {
+    const int c = tid + x * 256;
+    k_at[x] = c < KT * dk8 ? c / dk8 << 8 | c % dk8 : -1;
   }
+  const auto fetch = [&](int kt) {
+#pragma unroll
+    for (int x = 0; x < KP; ++x) {
+      if (k_at[x] < 0) continue;
+      const int e = k_at[x] & 255;
+      const size_t row = max(min(kt * KT + (k_at[x] >> 8), last) - p.base, 0);
+      kr[x] = *reinterpret_cast<const uint4_t*>(e < own8 ? k + row * p.k_ld + ((size_t)g * own8 + e) * 8
+                                                         : (const bf16_t*)p.k_shared + row * p.dk_shared + (e - own8) * 8);
+    }
+#pragma unroll
+    for (int x = 0; x < VP; ++x) {
+      const int c = tid + x * 256, r = (c & 31) * 2, e = (c >> 5) * 8;
+      if (e >= DV) continue;
+#pragma unroll
+      for (int y = 0; y < 2; ++y) {
+        const size_t row = max(min(kt * KT + r + y, last) - p.base, 0);
+        vr[x][y] = *reinterpret_cast<const uint4_t*>(v + row * p.v_ld + (size_t)g * DV + e);
+      }
+    }
+  };
+  int kt = kept_tiles > 0 ? 0 : win_tile;
+  fetch(kt);
+  bf16x8_t qf[KP];
+#pragma unroll
+  for (int c = 0; c < KP; ++c) {
+    if (c * 32 >= p.dk) continue;
+    qf[c] = *reinterpret_cast<const bf16x8_t*>(q + (size_t)min(q0 + wave * 16 + col, n - 1) * p.ldq + (size_t)h * p.dk + c * 32 + quad * 8);
+  }
+  const int i = first + wave * 16 + col;             // position of this lane's row
+  float m = p.sink ? p.sink[h] : -1e30f;             // the sink counts as a key of value zero
+  float l = p.sink && quad == 0 ? 1.0f : 0.0f;       // of this lane's keys
+  float4_t o[NT];                                    // values t * 16 + quad * 4 .. + 3 of the row
 #pragma unroll
   for (int t = 0; t < NT; ++t) o[t] = (float4_t)(0.0f);
-  bf16_t* Pw = Ps + wave * 2 * 16 * LDP;
 
-  for (int kt = kept_tiles > 0 ? 0 : win_tile; kt * KT <= last; ++kt) {
-    if (kt >= kept_tiles && kt < win_tile) kt = win_tile;
+  while (kt * KT <= last) {
     const int k0 = kt * KT;
     __syncthreads();  // the previous tile has been read
-    for (int c = tid; c < KT * dk8; c += 256) {
-      const int r = c / dk8, e = c % dk8;
-      const size_t row = max(min(k0 + r, last) - p.base, 0);
-      const bf16_t* src = e < own8 ? k + row * p.k_ld + ((size_t)g * own8 + e) * 8
-                                   : (const bf16_t*)p.k_shared + row * p.dk_shared + (e - own8) * 8;
-      *reinterpret_cast<uint4_t*>(Ks + r * ldk + e * 8) = *reinterpret_cast<const uint4_t*>(src);
-    }
-    for (int c = tid; c < KT * (DV / 8); c += 256) {
-      const int r = c % KT, e = (c / KT) * 8;
-      const size_t row = max(min(k0 + r, last) - p.base, 0);
-      const bf16x8_t x = *reinterpret_cast<const bf16x8_t*>(v + row * p.v_ld + (size_t)g * DV + e);
 #pragma unroll
-      for (int b = 0; b < 8; ++b) Vt[(e + b) * LDP + r] = x[b];
+    for (int x = 0; x < KP; ++x) {
+      if (k_at[x] >= 0) *reinterpret_cast<uint4_t*>(Ks + (k_at[x] >> 8) * ldk + (k_at[x] & 255) * 8) = kr[x];
+    }
+#pragma unroll
+    for (int x = 0; x < VP; ++x) {
+      const int c = tid + x * 256, at = key_place((c & 31) * 2), e = (c >> 5) * 8;
+      if (e >= DV) continue;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) {
+        const uint32_t a = vr[x][0][w], b = vr[x][1][w];
+        *reinterpret_cast<uint32_t*>(Vt + (e + 2 * w) * LDP + at) = (a & 0xFFFFu) | b << 16;
+        *reinterpret_cast<uint32_t*>(Vt + (e + 2 * w + 1) * LDP + at) = a >> 16 | (b & 0xFFFF0000u);
+      }
     }
     __syncthreads();
-    float4_t s[4];
+    ++kt;
+    if (kt >= kept_tiles && kt < win_tile) kt = win_tile;
+    if (kt * KT <= last) fetch(kt);
+    float4_t s[4];  // element e of s[t]: key t * 16 + quad * 4 + e
 #pragma unroll
     for (int t = 0; t < 4; ++t) s[t] = (float4_t)(0.0f);
-    for (int c = 0; c < p.dk; c += 32) {
-      const bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(Qs + (wave * 16 + col) * ldk + c + quad * 8);
+#pragma unroll
+    for (int c = 0; c < KP; ++c) {
+      if (c * 32 >= p.dk) continue;
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
-        const bf16x8_t b = *reinterpret_cast<const bf16x8_t*>(Ks + (t * 16 + col) * ldk + c + quad * 8);
-        s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, s[t], 0, 0, 0);
+        s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            *reinterpret_cast<const bf16x8_t*>(Ks + (t * 16 + col) * ldk + c * 32 + quad * 8), qf[c], s[t], 0, 0, 0);
       }
     }
-    // element e of s[t]: row quad * 4 + e of the wavefront's 16, key t * 16 + col
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int i = first + wave * 16 + quad * 4 + e;
-      float top = -1e30f;
-      bool see[4];
+    for (int t = 0; t < 4; ++t) {
+      s[t] *= p.scale;
+      if constexpr (BIAS) {
 #pragma unroll
-      for (int t = 0; t < 4; ++t) {
-        const int j = k0 + t * 16 + col, d = i - j;
-        see[t] = d >= 0 && (d < p.window || j < p.keep);
-        s[t][e] *= p.scale;
-        if constexpr (BIAS) s[t][e] -= r1 * __logf(1.0f + r2 * (float)max(d, 0));
-        if (see[t]) top = fmaxf(top, s[t][e]);
+        for (int e = 0; e < 4; ++e) s[t][e] -= r1 * __logf(1.0f + r2 * (float)max(i - (k0 + t * 16 + quad * 4 + e), 0));
       }
-      top = fmaxf(top, dpp_f32<0xB1>(top));
-      top = fmaxf(top, dpp_f32<0x4E>(top));
-      top = fmaxf(top, dpp_f32<0x141>(top));
-      top = fmaxf(top, dpp_f32<0x140>(top));
-      const float m_new = fmaxf(m[e], top);
-      const float shrink = __expf(m[e] - m_new);
-      m[e] = m_new;
-      float sum = 0.0f;
-#pragma unroll
-      for (int t = 0; t < 4; ++t) {
-        const float pr = see[t] ? __expf(s[t][e] - m_new) : 0.0f;
-        sum += pr;
-        const bf16_t hi = (bf16_t)pr;
-        Pw[(quad * 4 + e) * LDP + t * 16 + col] = hi;
-        Pw[(16 + quad * 4 + e) * LDP + t * 16 + col] = (bf16_t)(pr - (float)hi);
-      }
-      l[e] = l[e] * shrink + row16_sum(sum);
-#pragma unroll
-      for (int t = 0; t < NT; ++t) o[t][e] *= shrink;
     }
-    __syncthreads();  // P is written and read by the same wavefront; the barrier orders its LDS accesses
+    const int lowest = first + wave * 16;  // of the wavefront's positions
+    if (k0 + KT - 1 > lowest || (lowest + 15 - k0 >= p.window && k0 + KT > p.keep)) {
 #pragma unroll
-    for (int c = 0; c < KT; c += 32) {
-      const bf16x8_t hi = *reinterpret_cast<const bf16x8_t*>(Pw + col * LDP + c + quad * 8);
-      const bf16x8_t rem = *reinterpret_cast<const bf16x8_t*>(Pw + (16 + col) * LDP + c + quad * 8);
+      for (int t = 0; t < 4; ++t) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int j = k0 + t * 16 + quad * 4 + e, d = i - j;
+          if (!(d >= 0 && (d < p.window || j < p.keep))) s[t][e] = -INFINITY;
+        }
+      }
+    }
+    float top = m;
+#pragma unroll
+    for (int t = 0; t < 4; ++t) top = fmaxf(top, fmaxf(fmaxf(s[t][0], s[t][1]), fmaxf(s[t][2], s[t][3])));
+    top = fmaxf(top, __shfl_xor(top, 16, WAVE));
+    top = fmaxf(top, __shfl_xor(top, 32, WAVE));
+    if (__ballot(top != m) != 0) {
+      const float shrink = __expf(m - top);
+      m = top;
+      l *= shrink;
+#pragma unroll
+      for (int t = 0; t < NT; ++t) o[t] *= shrink;
+    }
+#pragma unroll
+    for (int c = 0; c < KT / 32; ++c) {
+      bf16x8_t hi, rem;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float pr = __expf(s[c * 2 + e / 4][e % 4] - m);
+        l += pr;
+        hi[e] = (bf16_t)pr;
+        rem[e] = (bf16_t)(pr - (float)hi[e]);
+      }
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
-        const bf16x8_t b = *reinterpret_cast<const bf16x8_t*>(Vt + (t * 16 + col) * LDP + c + quad * 8);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(rem, b, o[t], 0, 0, 0);
-        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi, b, o[t], 0, 0, 0);
+        const bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(Vt + (t * 16 + col) * LDP + c * 32 + quad * 8);
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, rem, o[t], 0, 0, 0);
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, hi, o[t], 0, 0, 0);
       }
     }
   }
+  l += __shfl_xor(l, 16, WAVE);
+  l += __shfl_xor(l, 32, WAVE);
+  const int r = q0 + wave * 16 + col;
+  if (r < n) {
+    const float inv = 1.0f / l;
 #pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    const int r = q0 + wave * 16 + quad * 4 + e;
-    if (r < n) {
-      const float inv = 1.0f / l[e];
+    for (int t = 0; t < NT; ++t) {
+      const size_t c = (size_t)h * DV + t * 16 + quad * 4;
+      float4_t x = o[t] * inv;
+      if (p.gate) {
+        const float4_t z = load4((const bf16_t*)p.gate + (size_t)r * p.ldg + c);
 #pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        float x = o[t][e] * inv;
-        if (p.gate) x *= sigmoid_f32((float)((const bf16_t*)p.gate)[(size_t)r * p.ldg + (size_t)h * DV + t * 16 + col]);
-        out[(size_t)r * p.ldo + (size_t)h * DV + t * 16 + col] = (bf16_t)x;
+        for (int e = 0; e < 4; ++e) x[e] *= sigmoid_f32(z[e]);
       }
+      store4(out + (size_t)r * p.ldo + c, x);
     }
   }
 }
 
-size_t tile_lds(int dk, int dv) {
-  return ((size_t)(QT + KT) * (dk + 8) + (size_t)dv * (KT + 8) + (size_t)4 * 2 * 16 * (KT + 8)) * 2;
-}
+size_t tile_lds(int dk, int dv) { return ((size_t)KT * (dk + 8) + (size_t)dv * (KT + 8)) * 2; }
 
 template <int DV, bool BIAS>
 int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, int start, const window_args& p, hipStream_t st) {
@@ -269,7 +304,7 @@ int launch_tiles(void* out, const void* q, const void* k, const void* v, int n, 
     LCU_HIP(hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024));
     raised[dev & 15] = true;
   }
-  kernel<<<dim3((n + QT - 1) / QT, p.heads), 256, lds, st>>>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k, (const bf16_t*)v, n,
+  kernel<<<(unsigned)((n + QT - 1) / QT) * p.heads, 256, lds, st>>>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k, (const bf16_t*)v, n,
                                                               start, p);
   LCU_LAUNCH_CHECK();
   return LCU_OK;
@@ -561,6 +596,7 @@ int lcu_attention_windowed(void* out_dev, int ldo, const void* q_dev, int ldq, c
                   (window->first_position == 0 ||
                    (window->keep == 0 && (long)window->first_position <= std::max(0L, (long)start - window->window + 1))),
               "lcu_attention_windowed: keys from position %d on do not hold the window of position %d", window->first_position, start);
+  LCU_REQUIRE(ldo % 4 == 0 && (!window->gate_dev || window->ldg % 4 == 0), "lcu_attention_windowed: row strides %d %d", ldo, window->ldg);
   if (n == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
   const window_args p = make_window(window, ldq, ldo);
