@@ -2,13 +2,23 @@
 one function per mechanism.
 
 The oracle of the tests: loops over tokens, no cache, no shared code with the product.  A model is a config (the
-dict of config.json) and a dict of weight arrays under the names of the weight file.
+dict of config.json) and a dict of weight arrays under the names of the weight file.  `rnd`, where a function has it, is
+applied to every activation that a model in a narrower type would store in it: what it does to the logits is what that
+type's rounding alone can do.
 """
 import numpy as np
 
 from plain_stack import F, bf16_bits, bf16_values, sigmoid, softplus
 
 UNIT_EPS = 1e-6
+
+
+def exact(x):
+    return x
+
+
+def to_bf16(x):
+    return bf16_values(bf16_bits(x)).reshape(np.shape(x)).astype(F)
 
 
 def rms_norm(x, w, eps):
@@ -49,45 +59,45 @@ def rotate_pairs(x, rot, first=0):
 
 
 # ---- latent attention -------------------------------------------------------------------------------
-def masked_attention(q, k, v, scale, size=None, sink=None):
-    """q, k [T, H, D], v [T, H, E] -> [T, H, E].  size: keys 0 <= i - j < size (None: all before).  sink [H]: a term
-    exp(sink) in the denominator only."""
-    T, H, _ = q.shape
-    out = np.zeros((T, H, v.shape[2]))
-    for i in range(T):
+def masked_attention(q, k, v, scale, size=None, sink=None, first=0):
+    """q [n, H, D] at positions first .., k [T, H, D], v [T, H, E] -> [n, H, E].  size: keys 0 <= i - j < size (None: all
+    before).  sink [H]: a term exp(sink) in the denominator only."""
+    n, H, _ = q.shape
+    out = np.zeros((n, H, v.shape[2]))
+    for i in range(first, first + n):
         lo = 0 if size is None else max(0, i - size + 1)
         for h in range(H):
-            s = (k[lo:i + 1, h] @ q[i, h]) * scale
+            s = (k[lo:i + 1, h] @ q[i - first, h]) * scale
             top = s.max() if sink is None else max(s.max(), sink[h])
             e = np.exp(s - top)
             total = e.sum() + (0.0 if sink is None else np.exp(sink[h] - top))
-            out[i, h] = (e / total) @ v[lo:i + 1, h]
+            out[i - first, h] = (e / total) @ v[lo:i + 1, h]
     return out
 
 
-def latent_mixer(h, W, p, m, eps):
+def latent_mixer(h, W, p, m, eps, rnd=exact):
     """Keys and values out of a normed latent; a rotated part shared by the heads, a sink, a gate on the output, a
     latent for the queries and a window where the layer has them."""
     T, H, D, E, R = h.shape[0], m["heads"], m["dim"], m["vdim"], m["kv_rank"]
     rd = m.get("rot_dim", 0)
     if "q_rank" in m:
-        q = rms_norm(h @ W[p + "dq"].T, W[p + "dq.norm"], eps) @ W[p + "uq"].T
+        q = rnd(rnd(rms_norm(rnd(h @ W[p + "dq"].T), W[p + "dq.norm"], eps)) @ W[p + "uq"].T)
     else:
-        q = h @ W[p + "q"].T
+        q = rnd(h @ W[p + "q"].T)
     q = q.reshape(T, H, D + rd)
-    down = h @ W[p + "dkv"].T
-    c = rms_norm(down[:, :R], W[p + "dkv.norm"], eps)
-    k = (c @ W[p + "uk"].T).reshape(T, H, D)
-    v = (c @ W[p + "uv"].T).reshape(T, H, E)
+    down = rnd(h @ W[p + "dkv"].T)
+    c = rnd(rms_norm(down[:, :R], W[p + "dkv.norm"], eps))
+    k = rnd(c @ W[p + "uk"].T).reshape(T, H, D)
+    v = rnd(c @ W[p + "uv"].T).reshape(T, H, E)
     if rd:
-        q = np.concatenate([q[..., :D], rotate_pairs(q[..., D:], m["rot"])], -1)
-        shared = rotate_pairs(down[:, None, R:], m["rot"])
+        q = np.concatenate([q[..., :D], rnd(rotate_pairs(q[..., D:], m["rot"]))], -1)
+        shared = rnd(rotate_pairs(down[:, None, R:], m["rot"]))
         k = np.concatenate([k, np.repeat(shared, H, 1)], -1)
     o = masked_attention(q, k, v, m["scale"], m["mask"]["size"] if "mask" in m else None, W.get(p + "sink"))
     o = o.reshape(T, H * E)
     if p + "g" in W:
-        o = o * sigmoid(h @ W[p + "g"].T)
-    return o @ W[p + "o"].T
+        o = o * sigmoid(rnd(h @ W[p + "g"].T))
+    return rnd(o) @ W[p + "o"].T
 
 
 # ---- gated delta rule -------------------------------------------------------------------------------
@@ -114,38 +124,38 @@ def delta_rule(q, k, v, g, beta, S=None):
     return out, S
 
 
-def delta_mixer(h, W, p, m, eps):
+def delta_mixer(h, W, p, m, eps, rnd=exact):
     T, H, G, D, E = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    branch = lambda n, heads, d: conv_silu(h @ W[p + n].T, W[p + n + ".conv"]).reshape(T, heads, d)
+    branch = lambda n, heads, d: rnd(conv_silu(rnd(h @ W[p + n].T), W[p + n + ".conv"])).reshape(T, heads, d)
     q, k, v = unit(branch("q", G, D)) * D ** -0.5, unit(branch("k", G, D)), branch("v", H, E)
     beta = sigmoid(h @ W[p + "b"].T)
     g = np.exp(-np.exp(W[p + "A_log"]) * softplus(h @ W[p + "a"].T + W[p + "dt_bias"]))
     o = np.stack([delta_rule(q[:, i // (H // G)], k[:, i // (H // G)], v[:, i], g[:, i], beta[:, i])[0] for i in range(H)], 1)
-    o = rms_norm(o, W[p + "norm"], eps) * silu(h @ W[p + "g"].T).reshape(T, H, E)
-    return o.reshape(T, H * E) @ W[p + "o"].T
+    o = rms_norm(o, W[p + "norm"], eps) * silu(rnd(h @ W[p + "g"].T)).reshape(T, H, E)
+    return rnd(o.reshape(T, H * E)) @ W[p + "o"].T
 
 
-def gated_mlp(h, W, p):
-    return (silu(h @ W[p + "gate"].T) * (h @ W[p + "up"].T)) @ W[p + "down"].T
+def gated_mlp(h, W, p, rnd=exact):
+    return rnd(silu(h @ W[p + "gate"].T) * (h @ W[p + "up"].T)) @ W[p + "down"].T
 
 
 # ---- the model --------------------------------------------------------------------------------------
 MIXERS = {"delta": delta_mixer, "latent_attention": latent_mixer, "latent_attention_2": latent_mixer}
 
 
-def forward(cfg, W, tokens, layers=None):
+def forward(cfg, W, tokens, layers=None, rnd=exact):
     """Logits [T, vocab]; `layers`, a list, receives the residual stream after every layer."""
     eps = cfg["norm"]["eps"]
     norm = lambda x, name: rms_norm(x, 1.0 + W[name], eps)
     x = W["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
     for l, spec in enumerate(cfg["layers"]):
         p = "l%d." % l
-        x = x + norm(MIXERS[spec["type"]](x, W, p + "mix.", spec["mixer"], eps), p + "norm1")
+        x = x + norm(MIXERS[spec["type"]](rnd(x), W, p + "mix.", spec["mixer"], eps, rnd), p + "norm1")
         if spec.get("mlp"):
-            x = x + norm(gated_mlp(x, W, p + "mlp."), p + "norm2")
+            x = x + norm(gated_mlp(rnd(x), W, p + "mlp.", rnd), p + "norm2")
         if layers is not None:
             layers.append(x)
-    return norm(x, "final.norm") @ W["head"].T
+    return rnd(norm(x, "final.norm")) @ W["head"].T
 
 
 def tensor_shapes(cfg):

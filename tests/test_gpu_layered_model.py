@@ -11,6 +11,7 @@ import pytest
 
 import lcu
 import plain_stack as S
+from layered_helpers import errors, feed
 
 pytestmark = pytest.mark.gpu
 
@@ -85,12 +86,6 @@ def case(request, tmp_path_factory):
     return dict(cfg=cfg, W=W, path=path, tokens=tokens, logits=logits, layers=layers)
 
 
-def errors(got, want):
-    d = got - want
-    d = d - d.mean(1, keepdims=True)
-    return np.sqrt((d ** 2).mean(1)) / want.std()
-
-
 def held(got, want, dt):
     """fp32: every position; bfloat16: nearly all (a close call between two experts may fall either way, and the
     tokens that attend to that one feel it)."""
@@ -99,15 +94,6 @@ def held(got, want, dt):
         assert e.max() < 1e-4, (e.argmax(), e.max())
     else:
         assert np.quantile(e, 0.92) < 0.05 and np.median(e) < 0.015, (np.quantile(e, 0.92), np.median(e))
-
-
-def feed(ctx, tokens, cuts):
-    out, at = [], 0
-    for n in cuts:
-        out.append(ctx.forward(tokens[at:at + n], range(n))[1])
-        at += n
-    assert at == len(tokens)
-    return np.concatenate(out)
 
 
 CUTS = {"whole": (230,), "tokens": (1,) * 230, "twos": (2,) * 40 + (150,), "decode": (100,) + (1,) * 130,

@@ -10,72 +10,9 @@ import numpy as np
 import pytest
 
 import plain_stack as S
+from layered_helpers import BF16, BOTH, F32, call, close, get, get_ints, gpu, ints, pack_gated, pad, put, rounded, up64, zeros  # noqa: F401
 
 pytestmark = pytest.mark.gpu
-
-F32, BF16 = 1, 0
-BOTH = pytest.mark.parametrize("dt", [BF16, F32], ids=["bf16", "f32"])
-
-
-@pytest.fixture(scope="module")
-def gpu():
-    import gpu_helpers as G
-    G.setup()
-    stream = G.B.vp()
-    G.B.check(G.L().lcu_stream_create(C.byref(stream)))
-    G.stream = stream.value
-    yield G
-    G.release()
-    G.B.check(G.L().lcu_stream_destroy(G.stream))
-
-
-def rounded(a):
-    """Values a bfloat16 holds, as float64 (every input here is one, so that both types see the same numbers)."""
-    return S.bf16_values(S.bf16_bits(a)).reshape(np.shape(a)).astype(np.float64)
-
-
-def up64(n):
-    return (n + 63) // 64 * 64
-
-
-def pad(a, cols):
-    out = np.zeros(a.shape[:-1] + (cols,))
-    out[..., :a.shape[-1]] = a
-    return out
-
-
-def put(G, a, dt=F32):
-    return G.dev_keep(np.asarray(a, np.float32) if dt == F32 else S.bf16_bits(a).reshape(np.shape(a)))
-
-
-def zeros(G, shape, dt=F32):
-    return put(G, np.zeros(shape), dt)
-
-
-def get(G, buf, shape, dt=F32):
-    G.B.check(G.L().lcu_sync(G.stream))
-    if dt == F32:
-        return G.host(buf, shape, np.float32).astype(np.float64)
-    return S.bf16_values(G.host(buf, shape, np.uint16)).astype(np.float64)
-
-
-def get_ints(G, buf, shape):
-    G.B.check(G.L().lcu_sync(G.stream))
-    return G.host(buf, shape, np.int32)
-
-
-def ints(G, a):
-    return G.dev_keep(np.asarray(a, np.int32))
-
-
-def close(got, want, dt, scale=None, f32=2e-5, bf16=2.0 ** -8):
-    scale = np.max(np.abs(want)) if scale is None else scale
-    err = np.max(np.abs(got - want)) / max(scale, 1e-30)
-    assert err <= (f32 if dt == F32 else bf16), err
-
-
-def call(G, name, *args):
-    G.B.check(getattr(G.L(), name)(*[a.ptr if hasattr(a, "ptr") else a for a in args], G.stream), name)
 
 
 # ---- linear ---------------------------------------------------------------------------------------------
@@ -114,15 +51,6 @@ def test_gated_linear_clamps(gpu, dt, M, K, ff):
     assert (x @ gw.T > limit).any() and (np.abs(x @ uw.T) > limit).any()
     close(get(gpu, out, (M, ld), dt)[:, :ff], want, dt)
     gpu.release()
-
-
-def pack_gated(gate, up, ld):
-    """Gate and up rows in blocks of 32 and 32, hidden units padded to ld."""
-    out = np.zeros((2 * ld, gate.shape[1]))
-    j = np.arange(gate.shape[0])
-    out[j // 32 * 64 + j % 32] = gate
-    out[j // 32 * 64 + j % 32 + 32] = up
-    return out
 
 
 # ---- norms and the residual -----------------------------------------------------------------------------
