@@ -113,7 +113,7 @@ __global__ __launch_bounds__(256) void head_products_kernel(bf16_t* __restrict__
   const bf16_t* a = in + (size_t)min(t0 + col, n - 1) * ldi + (size_t)h * in_h + quad * 8;
   const bf16_t* b = w + ((size_t)h * N + j) * K + quad * 8;
   float4_t acc = (float4_t)(0.0f);
-#pragma unroll 4
+#pragma unroll 8
   for (int k = 0; k < K; k += 32) {
     acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a + k), *reinterpret_cast<const bf16x8_t*>(b + k), acc,
                                                   0, 0, 0);
@@ -169,18 +169,6 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(latent_args p) {
     }
     return;
   }
-  bf16x8_t kv[2 * NT], rot[2];  // of this lane's key, one tile ahead
-  const auto fetch = [&](int tile) {
-    const size_t j = min(lo + tile * LKEYS + wave * 16 + col, hi);
-    const bf16_t* c = p.c + j * p.ldc + quad * 8;
-#pragma unroll
-    for (int f = 0; f < 2 * NT; ++f) kv[f] = f * 32 < p.ldc ? *reinterpret_cast<const bf16x8_t*>(c + f * 32) : (bf16x8_t)(0.0f);
-#pragma unroll
-    for (int f = 0; f < 2; ++f) {
-      if (f * 32 < p.dr) rot[f] = *reinterpret_cast<const bf16x8_t*>(p.keys + j * p.dr + quad * 8 + f * 32);
-    }
-  };
-  fetch(tile0);
   const int c8 = p.ldc / 8, k8 = (p.ldc + p.dr) / 8;
   for (int i = tid; i < LROWS * k8; i += 256) {
     const int r = i / k8, e = i - r * k8, row = min(r0 + r, rows - 1), t = row / p.heads, h = row - t * p.heads;
@@ -201,15 +189,13 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(latent_args p) {
   __syncthreads();
   for (int tile = tile0; tile < tile1; ++tile) {
     const int j = lo + tile * LKEYS + wave * 16 + col;  // this lane's key
+    const bf16_t* c = p.c + (size_t)min(j, hi) * p.ldc + quad * 8;
+    bf16x8_t kv[2 * NT];
+#pragma unroll
+    for (int f = 0; f < 2 * NT; ++f) kv[f] = f * 32 < p.ldc ? *reinterpret_cast<const bf16x8_t*>(c + f * 32) : (bf16x8_t)(0.0f);
     float4_t s = (float4_t)(0.0f);
     const bf16_t* qr = Qs + col * ldk + quad * 8;
-#pragma unroll
-    for (int f = 0; f < 2; ++f) {
-      if (f * 32 < p.dr) {
-        s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(qr + p.ldc + f * 32), rot[f], s, 0, 0, 0);
-      }
-    }
-    for (int k = 64; k < p.dr; k += 32) {
+    for (int k = 0; k < p.dr; k += 32) {
       s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(qr + p.ldc + k),
                                                   *reinterpret_cast<const bf16x8_t*>(p.keys + (size_t)min(j, hi) * p.dr + quad * 8 + k), s, 0,
                                                   0, 0);
@@ -240,7 +226,6 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(latent_args p) {
         for (int b = 0; b < 8; ++b) Vt[(f * 32 + quad * 8 + b) * LDV + wave * 16 + col] = kv[f][b];
       }
     }
-    if (tile + 1 < tile1) fetch(tile + 1);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int r = quad * 4 + e;
@@ -309,6 +294,7 @@ struct latent_value_args {
 };
 constexpr int MAX_SLICES = 32;
 
+template <int NT>
 __global__ __launch_bounds__(256) void latent_value_kernel(latent_value_args p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char value_lds[];
   bf16_t* C = reinterpret_cast<bf16_t*>(value_lds);  // [16][ldc + 8]
@@ -316,6 +302,12 @@ __global__ __launch_bounds__(256) void latent_value_kernel(latent_value_args p) 
   __shared__ int live[16];  // slices up to the last one with keys
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4;
   const int h = blockIdx.x, t0 = blockIdx.z * 16, tokens = min(16, p.n - t0), rows = p.n * p.heads, ld = p.ldc + 8;
+  const int j = blockIdx.y * 64 + wave * 16 + col;
+  const bool multiplies = blockIdx.y * 64 + wave * 16 < p.dv;
+  bf16x8_t w[2 * NT];
+  const bf16_t* b = p.w + ((size_t)h * p.dv + (multiplies ? j : 0)) * p.ldc + quad * 8;
+#pragma unroll
+  for (int f = 0; f < 2 * NT; ++f) w[f] = f * 32 < p.ldc ? *reinterpret_cast<const bf16x8_t*>(b + f * 32) : (bf16x8_t)(0.0f);
   for (int t = wave; t < tokens; t += 4) {
     const int row = (t0 + t) * p.heads + h;
     const bool has = lane < p.slices;
@@ -344,15 +336,12 @@ __global__ __launch_bounds__(256) void latent_value_kernel(latent_value_args p) 
     store4(C + t * ld + c, v);
   }
   __syncthreads();
-  const int j = blockIdx.y * 64 + wave * 16 + col;
-  if (blockIdx.y * 64 + wave * 16 >= p.dv) return;
+  if (!multiplies) return;
   const bf16_t* a = C + col * ld + quad * 8;
-  const bf16_t* b = p.w + ((size_t)h * p.dv + j) * p.ldc + quad * 8;
   float4_t acc = (float4_t)(0.0f);
-#pragma unroll 4
-  for (int k = 0; k < p.ldc; k += 32) {
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a + k), *reinterpret_cast<const bf16x8_t*>(b + k), acc,
-                                                  0, 0, 0);
+#pragma unroll
+  for (int f = 0; f < 2 * NT; ++f) {
+    if (f * 32 < p.ldc) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8_t*>(a + f * 32), w[f], acc, 0, 0, 0);
   }
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
@@ -469,6 +458,8 @@ int lcu_latent_attention(void* out_dev, int ldo, const void* q_latent_dev, const
                       p->dn + p->dr, (const bf16_t*)latents_dev, (const bf16_t*)keys_dev, (const int*)start_dev, max_positions, part, ml};
   hipStream_t st = as_stream(stream);
   const size_t lds = attention_lds(p->ldc, p->dr);
+  const latent_value_args v{p->heads, n, p->ldc, p->dv, slices, part, ml, (const float*)sink_dev, (const bf16_t*)uv_dev,
+                            (const bf16_t*)gate_dev, ldg, (bf16_t*)out_dev, ldo};
   const auto go = [&](auto nt) -> int {
     auto kernel = latent_attention_kernel<decltype(nt)::value>;
     static bool raised[16] = {};  // per device, once
@@ -479,20 +470,16 @@ int lcu_latent_attention(void* out_dev, int ldo, const void* q_latent_dev, const
       raised[dev & 15] = true;
     }
     kernel<<<dim3((rows + LROWS - 1) / LROWS, slices), 256, lds, st>>>(a);
+    latent_value_kernel<decltype(nt)::value>
+        <<<dim3(p->heads, (p->dv + 63) / 64, (n + 15) / 16), 256, (size_t)16 * (p->ldc + 8) * 2, st>>>(v);
     LCU_LAUNCH_CHECK();
     return LCU_OK;
   };
   using std::integral_constant;
-  const int rc2 = p->ldc <= 64    ? go(integral_constant<int, 1>{})
-                  : p->ldc <= 128 ? go(integral_constant<int, 2>{})
-                  : p->ldc <= 256 ? go(integral_constant<int, 4>{})
-                                  : go(integral_constant<int, 8>{});
-  if (rc2) return rc2;
-  const latent_value_args v{p->heads, n, p->ldc, p->dv, slices, part, ml, (const float*)sink_dev, (const bf16_t*)uv_dev,
-                            (const bf16_t*)gate_dev, ldg, (bf16_t*)out_dev, ldo};
-  latent_value_kernel<<<dim3(p->heads, (p->dv + 63) / 64, (n + 15) / 16), 256, (size_t)16 * (p->ldc + 8) * 2, st>>>(v);
-  LCU_LAUNCH_CHECK();
-  return LCU_OK;
+  return p->ldc <= 64    ? go(integral_constant<int, 1>{})
+         : p->ldc <= 128 ? go(integral_constant<int, 2>{})
+         : p->ldc <= 256 ? go(integral_constant<int, 4>{})
+                         : go(integral_constant<int, 8>{});
 }
 
 }  // extern "C"
