@@ -274,110 +274,111 @@ __device__ __forceinline__ float4_t step_product(bf16x8_t a, const bf16_t* terms
   return acc;
 }
 
-// One workgroup: sixteen columns of one head's state through all chunks.  A wavefront takes sixteen rows of a chunk and up
-// to TILES blocks of sixteen rows of the state, which it keeps in registers; LDS holds all of the state as operands.  What a
-// chunk needs from memory is asked for one chunk ahead where the registers hold it twice.  o: fp32 [n][heads * E].
+// One workgroup: sixteen columns of one head's state through all chunks.  Wavefronts 0 .. 3 take sixteen rows of a chunk
+// each and work out u, wavefronts 4 .. 7 take the same rows and work out o; each keeps up to TILES blocks of sixteen rows of the
+// state in registers and brings them up to date, and LDS holds all of the state as operands.  What a chunk needs from
+// memory is asked for one chunk ahead where the registers hold it twice.  o: fp32 [n][heads * E].
 template <class T, int D>
-__global__ __launch_bounds__(256) void delta_scan_kernel(float* __restrict__ o, float* __restrict__ state, const T* __restrict__ qkv,
+__global__ __launch_bounds__(512) void delta_scan_kernel(float* __restrict__ o, float* __restrict__ state, const T* __restrict__ qkv,
                                                          int chunks, delta_args p) {
   typedef terms_of<T> terms;
   typedef typename terms::piece piece;
-  constexpr int STEPS = D / terms::STEP, CSTEPS = CHUNK / terms::STEP, TILES = (D / 16 + 3) / 4;
+  constexpr int STEPS = D / terms::STEP, CSTEPS = CHUNK / terms::STEP, TILES = (D / 16 + 7) / 8;
   constexpr int LDR = CHUNK + 4, LDU = CHUNK + terms::PAD, LDD = D + terms::PAD;
   constexpr bool AHEAD = D * sizeof(T) <= 512;
   __shared__ __attribute__((aligned(16))) T S[terms::COUNT * 16 * LDD];
   __shared__ __attribute__((aligned(16))) T U[terms::COUNT * 16 * LDU];  // u times the row's factor of k
   __shared__ __attribute__((aligned(16))) float R[16 * LDR];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, quad = lane >> 4, r0 = wave * 16 + quad * 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, quad = lane >> 4;
+  const int block = wave & 3, r0 = block * 16 + quad * 4;
+  const bool of_u = wave < 4;
   const int h = blockIdx.x, c0 = blockIdx.y * 16, g = h / (p.heads / p.kv_heads);
-  const T* Q = qkv + (size_t)g * D;
-  const T* K = qkv + (size_t)(p.kv_heads + g) * D;
-  const T* V = qkv + (size_t)2 * p.kv_heads * D + (size_t)h * p.E + c0 + col;
+  const T* QK = qkv + (size_t)(of_u ? p.kv_heads + g : g) * D;
+  const T* V = qkv + (size_t)2 * p.kv_heads * D + (size_t)h * p.E + c0;
+  const float* M = of_u ? p.T : p.PT;
   float* St = state + (size_t)h * D * p.E + c0 + col;
   struct operands {
-    piece k[STEPS], q[STEPS], kt[TILES * CSTEPS];
-    float4_t t[4], pt[4], fac[4];
+    piece x[STEPS], kt[TILES * CSTEPS];  // rows of k or q; transposed keys
+    float4_t m[4];                       // rows of T or P T
+    float4_t beta, of_k, of_q, end;      // the rows' factors
     float v[4], total;
   };
+  // offsets of this lane, beside uniform pointers; rows behind the last token are the last one again
+  const unsigned ld = p.ld, last = (unsigned)(p.n - 1) * ld, row = (unsigned)(block * 16 + col) * ld, v_row = (unsigned)r0 * ld;
+  const unsigned m_at = (block * 16 + col) * CHUNK + quad * 4;
+  const unsigned o_ld = p.heads * p.E, o_at = r0 * o_ld + col;
+  unsigned kt_at[TILES];
+#pragma unroll
+  for (int i = 0; i < TILES; ++i) kt_at[i] = (min((wave + i * 8) * 16, D - 16) + col) * CHUNK + quad * terms::PER;
   const auto fetch = [&](operands& x, int chunk) {
-    const size_t at = (size_t)h * chunks + chunk, r = (size_t)min(chunk * CHUNK + wave * 16 + col, p.n - 1) * p.ld;
+    const size_t at = (size_t)h * chunks + chunk;
     const T* kt = (const T*)p.Kt + ((size_t)g * chunks + chunk) * D * CHUNK;
-    const size_t m = at * CHUNK * CHUNK + (size_t)(wave * 16 + col) * CHUNK + quad * 4;
+    const float* m = M + at * CHUNK * CHUNK;
+    const float* rows = p.rows + at * 4 * CHUNK;
+    const unsigned first = (unsigned)chunk * CHUNK * ld, r = min(first + row, last) + quad * terms::PER;
 #pragma unroll
-    for (int i = 0; i < STEPS; ++i) {
-      x.k[i] = *reinterpret_cast<const piece*>(K + r + i * terms::STEP + quad * terms::PER);
-      x.q[i] = *reinterpret_cast<const piece*>(Q + r + i * terms::STEP + quad * terms::PER);
-    }
+    for (int i = 0; i < STEPS; ++i) x.x[i] = *reinterpret_cast<const piece*>(QK + r + i * terms::STEP);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      x.v[e] = to_f32(V[(size_t)min(chunk * CHUNK + r0 + e, p.n - 1) * p.ld]);
-      x.fac[e] = load4(p.rows + (at * 4 + e) * CHUNK + r0);
-    }
+    for (int e = 0; e < 4; ++e) x.v[e] = to_f32(V[min(first + v_row + e * ld, last) + col]);
+    x.beta = load4(rows + (unsigned)r0);
+    x.of_k = load4(rows + CHUNK + (unsigned)r0);
+    x.of_q = load4(rows + 2 * CHUNK + (unsigned)r0);
+    x.end = load4(rows + 3 * CHUNK + (unsigned)r0);
 #pragma unroll
-    for (int s = 0; s < 4; ++s) {
-      if (s <= wave) {
-        x.t[s] = load4(p.T + m + s * 16);
-        x.pt[s] = load4(p.PT + m + s * 16);
-      }
-    }
+    for (int s = 0; s < 4; ++s) x.m[s] = load4(m + min(s, block) * 16 + m_at);
 #pragma unroll
     for (int i = 0; i < TILES; ++i) {
 #pragma unroll
-      for (int c = 0; c < CSTEPS; ++c) {
-        const int d = min((wave + i * 4) * 16, D - 16) + col;
-        x.kt[i * CSTEPS + c] = *reinterpret_cast<const piece*>(kt + (size_t)d * CHUNK + c * terms::STEP + quad * terms::PER);
-      }
+      for (int c = 0; c < CSTEPS; ++c) x.kt[i * CSTEPS + c] = *reinterpret_cast<const piece*>(kt + kt_at[i] + c * terms::STEP);
     }
     x.total = p.total[at];
   };
-  operands now, next;
-  if (AHEAD) fetch(now, 0);
+  operands even, odd;
+  if (AHEAD) fetch(even, 0);
   float4_t s[TILES];
 #pragma unroll
   for (int i = 0; i < TILES; ++i) {
-    const int d0 = (wave + i * 4) * 16 + quad * 4;
+    const int d0 = (wave + i * 8) * 16 + quad * 4;
     if (d0 >= D) break;
 #pragma unroll
     for (int e = 0; e < 4; ++e) s[i][e] = St[(size_t)(d0 + e) * p.E];
     put_terms<LDD>(S, col, d0, s[i]);
   }
-  for (int chunk = 0; chunk < chunks; ++chunk) {
+  const auto step = [&](operands& now, operands& next, int chunk) {
     if (AHEAD) {
       fetch(next, min(chunk + 1, chunks - 1));
     } else {
       fetch(now, chunk);
     }
     __syncthreads();  // S is whole
-    float4_t ks = (float4_t)(0.0f), qs = (float4_t)(0.0f);
+    float4_t xs = (float4_t)(0.0f);
 #pragma unroll
-    for (int i = 0; i < STEPS; ++i) {
-      ks = step_product<LDD>(now.k[i], S, col, i * terms::STEP + quad * terms::PER, ks);
-      qs = step_product<LDD>(now.q[i], S, col, i * terms::STEP + quad * terms::PER, qs);
+    for (int i = 0; i < STEPS; ++i) xs = step_product<LDD>(now.x[i], S, col, i * terms::STEP + quad * terms::PER, xs);
+    if (of_u) {
+      float4_t r;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) r[e] = now.beta[e] * now.v[e] - now.of_k[e] * xs[e];
+      store4(R + col * LDR + r0, r);
     }
-    float4_t r;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) r[e] = now.fac[0][e] * now.v[e] - now.fac[1][e] * ks[e];
-    store4(R + col * LDR + r0, r);
     __syncthreads();  // R is whole, S has been read
-    float4_t u = (float4_t)(0.0f), y = (float4_t)(0.0f);
+    float4_t y = (float4_t)(0.0f);
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
-      if (b <= wave) {
-        const float4_t x = load4(R + col * LDR + b * 16 + quad * 4);
+      if (b <= block) {
+        const float4_t r = load4(R + col * LDR + b * 16 + quad * 4);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          u = mfma_f32(now.t[b][e], x[e], u);
-          y = mfma_f32(now.pt[b][e], x[e], y);
-        }
+        for (int e = 0; e < 4; ++e) y = mfma_f32(now.m[b][e], r[e], y);
       }
     }
+    if (of_u) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) u[e] *= now.fac[3][e];
-    put_terms<LDU>(U, col, r0, u);
+      for (int e = 0; e < 4; ++e) y[e] *= now.end[e];
+      put_terms<LDU>(U, col, r0, y);
+    }
     __syncthreads();  // U is whole, R has been read
 #pragma unroll
     for (int i = 0; i < TILES; ++i) {
-      const int d0 = (wave + i * 4) * 16 + quad * 4;
+      const int d0 = (wave + i * 8) * 16 + quad * 4;
       if (d0 >= D) break;
 #pragma unroll
       for (int e = 0; e < 4; ++e) s[i][e] *= now.total;
@@ -387,16 +388,21 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(float* __restrict__ o, 
       }
       put_terms<LDD>(S, col, d0, s[i]);
     }
-    const int t = chunk * CHUNK + r0;
+    if (!of_u) {
+      float* out = o + (size_t)chunk * CHUNK * o_ld + h * p.E + c0;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      if (t + e < p.n) o[(size_t)(t + e) * p.heads * p.E + (size_t)h * p.E + c0 + col] = fmaf(now.fac[2][e], qs[e], y[e]);
+      for (int e = 0; e < 4; ++e) {
+        if (chunk * CHUNK + r0 + e < p.n) out[o_at + e * o_ld] = fmaf(now.of_q[e], xs[e], y[e]);
+      }
     }
-    if (AHEAD) now = next;
+  };
+  for (int chunk = 0; chunk < chunks; chunk += 2) {
+    step(even, odd, chunk);
+    if (chunk + 1 < chunks) step(odd, even, chunk + 1);
   }
 #pragma unroll
   for (int i = 0; i < TILES; ++i) {
-    const int d0 = (wave + i * 4) * 16 + quad * 4;
+    const int d0 = (wave + i * 8) * 16 + quad * 4;
     if (d0 >= D) break;
 #pragma unroll
     for (int e = 0; e < 4; ++e) St[(size_t)(d0 + e) * p.E] = s[i][e];
@@ -580,6 +586,7 @@ int lcu_delta_rule(void* out_dev, int ldo, const void* qkv_dev, int ld, const vo
   LCU_REQUIRE(n >= 0 && n <= 65535 && ld >= delta_channels(d) && ld % 8 == 0 && ldo >= d->heads * d->dv && ldg >= d->heads * d->dv &&
                   ld_ba >= 2 * d->heads,
               "lcu_delta_rule: bad shape n %d strides %d %d %d %d", n, ld, ldo, ldg, ld_ba);
+  LCU_REQUIRE(((size_t)n + 2 * CHUNK) * ld < ((size_t)1 << 32), "lcu_delta_rule: %d rows of %d", n, ld);
   if (n == 0) return LCU_OK;
   hipStream_t st = as_stream(stream);
   delta_args p = make_delta(d, ba_f32_dev, ld_ba, n, ld);
@@ -598,7 +605,7 @@ int lcu_delta_rule(void* out_dev, int ldo, const void* qkv_dev, int ld, const vo
     using T = std::remove_pointer_t<decltype(kind)>;
     constexpr int D = decltype(size)::value;
     delta_chunk_kernel<T, D><<<dim3(d->heads, chunks), 256, 0, st>>>((const T*)qkv_dev, p);
-    delta_scan_kernel<T, D><<<dim3(d->heads, d->dv / 16), 256, 0, st>>>(o, (float*)state_dev, (const T*)qkv_dev, chunks, p);
+    delta_scan_kernel<T, D><<<dim3(d->heads, d->dv / 16), 512, 0, st>>>(o, (float*)state_dev, (const T*)qkv_dev, chunks, p);
     head_norm_gate_kernel<T><<<norms, 256, 0, st>>>((T*)out_dev, ldo, o, (const T*)gate_dev, ldg, lanes, p);
   };
   with_head_size(d->dk, [&](auto size) {
