@@ -276,8 +276,8 @@ __device__ __forceinline__ float4_t step_product(bf16x8_t a, const bf16_t* terms
 
 // One workgroup: sixteen columns of one head's state through all chunks.  Wavefronts 0 .. 3 take sixteen rows of a chunk
 // each and work out u, wavefronts 4 .. 7 take the same rows and work out o; each keeps up to TILES blocks of sixteen rows of the
-// state in registers and brings them up to date, and LDS holds all of the state as operands.  What a chunk needs from
-// memory is asked for one chunk ahead where the registers hold it twice.  o: fp32 [n][heads * E].
+// state in registers and brings them up to date, and LDS holds all of the state as operands.  What the next chunk needs
+// from memory is asked for as soon as this chunk's has been used.  o: fp32 [n][heads * E].
 template <class T, int D>
 __global__ __launch_bounds__(512) void delta_scan_kernel(float* __restrict__ o, float* __restrict__ state, const T* __restrict__ qkv,
                                                          int chunks, delta_args p) {
@@ -285,7 +285,6 @@ __global__ __launch_bounds__(512) void delta_scan_kernel(float* __restrict__ o, 
   typedef typename terms::piece piece;
   constexpr int STEPS = D / terms::STEP, CSTEPS = CHUNK / terms::STEP, TILES = (D / 16 + 7) / 8;
   constexpr int LDR = CHUNK + 4, LDU = CHUNK + terms::PAD, LDD = D + terms::PAD;
-  constexpr bool AHEAD = D * sizeof(T) <= 512;
   __shared__ __attribute__((aligned(16))) T S[terms::COUNT * 16 * LDD];
   __shared__ __attribute__((aligned(16))) T U[terms::COUNT * 16 * LDU];  // u times the row's factor of k
   __shared__ __attribute__((aligned(16))) float R[16 * LDR];
@@ -295,46 +294,54 @@ __global__ __launch_bounds__(512) void delta_scan_kernel(float* __restrict__ o, 
   const int h = blockIdx.x, c0 = blockIdx.y * 16, g = h / (p.heads / p.kv_heads);
   const T* QK = qkv + (size_t)(of_u ? p.kv_heads + g : g) * D;
   const T* V = qkv + (size_t)2 * p.kv_heads * D + (size_t)h * p.E + c0;
-  const float* M = of_u ? p.T : p.PT;
   float* St = state + (size_t)h * D * p.E + c0 + col;
-  struct operands {
-    piece x[STEPS], kt[TILES * CSTEPS];  // rows of k or q; transposed keys
-    float4_t m[4];                       // rows of T or P T
-    float4_t beta, of_k, of_q, end;      // the rows' factors
-    float v[4], total;
-  };
   // offsets of this lane, beside uniform pointers; rows behind the last token are the last one again
   const unsigned ld = p.ld, last = (unsigned)(p.n - 1) * ld, row = (unsigned)(block * 16 + col) * ld, v_row = (unsigned)r0 * ld;
-  const unsigned m_at = (block * 16 + col) * CHUNK + quad * 4;
-  const unsigned o_ld = p.heads * p.E, o_at = r0 * o_ld + col;
+  const unsigned m_at = (block * 16 + col) * CHUNK + quad * 4, o_ld = p.heads * p.E, o_at = r0 * o_ld + col;
   unsigned kt_at[TILES];
 #pragma unroll
   for (int i = 0; i < TILES; ++i) kt_at[i] = (min((wave + i * 8) * 16, D - 16) + col) * CHUNK + quad * terms::PER;
-  const auto fetch = [&](operands& x, int chunk) {
+
+  piece x[STEPS];  // rows of k or q
+  const auto fetch_rows = [&](int chunk) {
+    const unsigned r = min((unsigned)chunk * CHUNK * ld + row, last) + quad * terms::PER;
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) x[i] = *reinterpret_cast<const piece*>(QK + r + i * terms::STEP);
+  };
+  T v[4];
+  float4_t beta, of_k;
+  const auto fetch_values = [&](int chunk) {
+    const float* rows = p.rows + ((size_t)h * chunks + chunk) * 4 * CHUNK;
+    beta = load4(rows + (unsigned)r0);
+    of_k = load4(rows + CHUNK + (unsigned)r0);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = V[min((unsigned)chunk * CHUNK * ld + v_row + e * ld, last) + col];
+  };
+  float4_t m[4], factor;  // rows of T or P T; e^(G_64 - G) / |k| or e^G / |q|
+  const auto fetch_matrix = [&](int chunk) {
     const size_t at = (size_t)h * chunks + chunk;
-    const T* kt = (const T*)p.Kt + ((size_t)g * chunks + chunk) * D * CHUNK;
-    const float* m = M + at * CHUNK * CHUNK;
-    const float* rows = p.rows + at * 4 * CHUNK;
-    const unsigned first = (unsigned)chunk * CHUNK * ld, r = min(first + row, last) + quad * terms::PER;
+    const float* src = (of_u ? p.T : p.PT) + at * CHUNK * CHUNK;
+    factor = load4(p.rows + at * 4 * CHUNK + (of_u ? 3 : 2) * CHUNK + (unsigned)r0);
 #pragma unroll
-    for (int i = 0; i < STEPS; ++i) x.x[i] = *reinterpret_cast<const piece*>(QK + r + i * terms::STEP);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) x.v[e] = to_f32(V[min(first + v_row + e * ld, last) + col]);
-    x.beta = load4(rows + (unsigned)r0);
-    x.of_k = load4(rows + CHUNK + (unsigned)r0);
-    x.of_q = load4(rows + 2 * CHUNK + (unsigned)r0);
-    x.end = load4(rows + 3 * CHUNK + (unsigned)r0);
-#pragma unroll
-    for (int s = 0; s < 4; ++s) x.m[s] = load4(m + min(s, block) * 16 + m_at);
+    for (int b = 0; b < 4; ++b) {
+      if (b <= block) m[b] = load4(src + b * 16 + m_at);
+    }
+  };
+  piece kt[TILES * CSTEPS];  // transposed keys
+  float total;
+  const auto fetch_keys = [&](int chunk) {
+    const T* src = (const T*)p.Kt + ((size_t)g * chunks + chunk) * D * CHUNK;
 #pragma unroll
     for (int i = 0; i < TILES; ++i) {
 #pragma unroll
-      for (int c = 0; c < CSTEPS; ++c) x.kt[i * CSTEPS + c] = *reinterpret_cast<const piece*>(kt + kt_at[i] + c * terms::STEP);
+      for (int c = 0; c < CSTEPS; ++c) kt[i * CSTEPS + c] = *reinterpret_cast<const piece*>(src + kt_at[i] + c * terms::STEP);
     }
-    x.total = p.total[at];
+    total = p.total[(size_t)h * chunks + chunk];
   };
-  operands even, odd;
-  if (AHEAD) fetch(even, 0);
+  fetch_rows(0);
+  if (of_u) fetch_values(0);
+  fetch_matrix(0);
+  fetch_keys(0);
   float4_t s[TILES];
 #pragma unroll
   for (int i = 0; i < TILES; ++i) {
@@ -344,21 +351,20 @@ __global__ __launch_bounds__(512) void delta_scan_kernel(float* __restrict__ o, 
     for (int e = 0; e < 4; ++e) s[i][e] = St[(size_t)(d0 + e) * p.E];
     put_terms<LDD>(S, col, d0, s[i]);
   }
-  const auto step = [&](operands& now, operands& next, int chunk) {
-    if (AHEAD) {
-      fetch(next, min(chunk + 1, chunks - 1));
-    } else {
-      fetch(now, chunk);
-    }
+#pragma unroll 1
+  for (int chunk = 0; chunk < chunks; ++chunk) {
+    const int next = min(chunk + 1, chunks - 1);
     __syncthreads();  // S is whole
     float4_t xs = (float4_t)(0.0f);
 #pragma unroll
-    for (int i = 0; i < STEPS; ++i) xs = step_product<LDD>(now.x[i], S, col, i * terms::STEP + quad * terms::PER, xs);
+    for (int i = 0; i < STEPS; ++i) xs = step_product<LDD>(x[i], S, col, i * terms::STEP + quad * terms::PER, xs);
+    fetch_rows(next);
     if (of_u) {
       float4_t r;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) r[e] = now.beta[e] * now.v[e] - now.of_k[e] * xs[e];
+      for (int e = 0; e < 4; ++e) r[e] = beta[e] * to_f32(v[e]) - of_k[e] * xs[e];
       store4(R + col * LDR + r0, r);
+      fetch_values(next);
     }
     __syncthreads();  // R is whole, S has been read
     float4_t y = (float4_t)(0.0f);
@@ -367,38 +373,35 @@ __global__ __launch_bounds__(512) void delta_scan_kernel(float* __restrict__ o, 
       if (b <= block) {
         const float4_t r = load4(R + col * LDR + b * 16 + quad * 4);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) y = mfma_f32(now.m[b][e], r[e], y);
+        for (int e = 0; e < 4; ++e) y = mfma_f32(m[b][e], r[e], y);
       }
     }
     if (of_u) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) y[e] *= now.end[e];
+      for (int e = 0; e < 4; ++e) y[e] *= factor[e];
       put_terms<LDU>(U, col, r0, y);
+    } else {
+      float* out = o + (size_t)chunk * CHUNK * o_ld + h * p.E + c0;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if (chunk * CHUNK + r0 + e < p.n) out[o_at + e * o_ld] = fmaf(factor[e], xs[e], y[e]);
+      }
     }
+    fetch_matrix(next);
     __syncthreads();  // U is whole, R has been read
 #pragma unroll
     for (int i = 0; i < TILES; ++i) {
       const int d0 = (wave + i * 8) * 16 + quad * 4;
       if (d0 >= D) break;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) s[i][e] *= now.total;
+      for (int e = 0; e < 4; ++e) s[i][e] *= total;
 #pragma unroll
       for (int c = 0; c < CSTEPS; ++c) {
-        s[i] = step_product<LDU>(now.kt[i * CSTEPS + c], U, col, c * terms::STEP + quad * terms::PER, s[i]);
+        s[i] = step_product<LDU>(kt[i * CSTEPS + c], U, col, c * terms::STEP + quad * terms::PER, s[i]);
       }
       put_terms<LDD>(S, col, d0, s[i]);
     }
-    if (!of_u) {
-      float* out = o + (size_t)chunk * CHUNK * o_ld + h * p.E + c0;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        if (chunk * CHUNK + r0 + e < p.n) out[o_at + e * o_ld] = fmaf(now.of_q[e], xs[e], y[e]);
-      }
-    }
-  };
-  for (int chunk = 0; chunk < chunks; chunk += 2) {
-    step(even, odd, chunk);
-    if (chunk + 1 < chunks) step(odd, even, chunk + 1);
+    fetch_keys(next);
   }
 #pragma unroll
   for (int i = 0; i < TILES; ++i) {
